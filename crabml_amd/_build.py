@@ -23,7 +23,9 @@ HIPCC = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
 LIB = os.path.join(HERE, "libcrabml_hip.so")
 
 HIP_FLAGS = ["--offload-arch=gfx950", "-O3", "-std=c++17", "-ffp-contract=off", "-fPIC", "-Wall",
-             "-Wno-unused-function", "-Wno-unused-result"]
+             "-Wno-unused-function", "-Wno-unused-result",
+             # no packed FP32 instructions (v_pk_{add,mul,fma}_f32): some of their forms have given wrong results on this hardware
+             "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
 # per-file: the MFMA GEMM keeps its accumulators in VGPRs (gfx950's register file is unified; the AGPR form costs a
 # v_accvgpr_read/write per accumulator register and block: 32 of 137 VALU instructions per k-block)
 EXTRA_FLAGS = {"gemm_mfma.hip": ["-mllvm", "-amdgpu-mfma-vgpr-form"]}

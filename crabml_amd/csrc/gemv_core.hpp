@@ -502,23 +502,24 @@ __device__ __forceinline__ void q4k_class_terms(const Q4KPiece<HDR_DPP>& w, cons
 // four LDS banks apart (a stride of 12 nsb floats is a multiple of 64 banks for nsb = 16: every lane on the same banks)
 __host__ __device__ inline int q4k_rec_stride(int nsb) { return nsb * 12 + 4; }
 // the nine chains of one row over its nsb records (12 floats each, 16-byte aligned), in super-block order: buf_q4_k.rs:263-276
+// U: records whose reads are in flight ahead of their adds (the nine chains are independent of each other: one dependent add per record)
+template <int U = 4>
 __device__ __forceinline__ float q4k_ordered_sum(const float* __restrict__ t, int nsb) {
   float sums[8], sumf = 0.0f;
 #pragma unroll
   for (int l = 0; l < 8; l++) sums[l] = 0.0f;
-  // four records' reads in flight ahead of their adds (the nine chains are independent of each other: one dependent add per record)
   int sb = 0;
-  for (; sb + 4 <= nsb; sb += 4) {
-    f32x4 a[4], b[4];
-    float m[4];
+  for (; sb + U <= nsb; sb += U) {
+    f32x4 a[U], b[U];
+    float m[U];
 #pragma unroll
-    for (int u = 0; u < 4; u++) {
+    for (int u = 0; u < U; u++) {
       a[u] = *(const f32x4*)(t + (sb + u) * 12);
       b[u] = *(const f32x4*)(t + (sb + u) * 12 + 4);
       m[u] = t[(sb + u) * 12 + 8];
     }
 #pragma unroll
-    for (int u = 0; u < 4; u++) {
+    for (int u = 0; u < U; u++) {
       sums[0] += a[u][0];
       sums[1] += a[u][1];
       sums[2] += a[u][2];

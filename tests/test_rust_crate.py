@@ -145,7 +145,7 @@ def test_ggml_type_ids_are_passed_as_the_enum_discriminants():
     enum = re.search(r"typedef enum crabml_hip_ggml_type \{(.*?)\}", src, flags=re.S).group(1)
     ids = {m.group(1): int(m.group(2)) for m in re.finditer(r"CRABML_HIP_([A-Z0-9_]+)\s*=\s*(\d+)", enum)}
     assert ids == {"F32": 0, "F16": 1, "Q4_0": 2, "Q4_1": 3, "Q5_0": 6, "Q5_1": 7, "Q8_0": 8, "Q8_1": 9, "Q2_K": 10, "Q3_K": 11, "Q4_K": 12,
-                   "Q5_K": 13, "Q6_K": 14, "Q8_K": 15}
+                   "Q5_K": 13, "Q6_K": 14, "Q8_K": 15, "BF16": 30}
     assert "dtype as u32" in open(os.path.join(CRATE, "src", "hip_tensor.rs")).read()
     if os.path.exists(os.path.join(REFERENCE, "crabml-core", "src", "gguf.rs")):
         g = open(os.path.join(REFERENCE, "crabml-core", "src", "gguf.rs")).read()
@@ -176,14 +176,14 @@ def test_hip_tensor_implements_every_method_of_the_tensor_trait():
         assert os.path.getsize(os.path.join(CRATE, f)) > 200, f
 
 
-@pytest.mark.skipif(not os.path.isdir(REFERENCE) or shutil.which("git") is None, reason="needs the reference checkout (build container)")
+@pytest.mark.skipif(not os.path.exists(os.path.join(REFERENCE, "Cargo.toml")) or shutil.which("git") is None, reason="needs the reference checkout (build container)")
 @pytest.mark.parametrize("patch", ["0001-quantized-device-weights.patch", "0002-cli-device-hip.patch"])
 def test_patches_apply_to_the_reference(patch):
     r = subprocess.run(["git", "apply", "--check", "-p1", os.path.join(ROOT, "patches", patch)], cwd=REFERENCE, capture_output=True, text=True)
     assert r.returncode == 0, r.stderr
 
 
-@pytest.mark.skipif(not os.path.isdir(REFERENCE) or shutil.which("git") is None, reason="needs the reference checkout (build container)")
+@pytest.mark.skipif(not os.path.exists(os.path.join(REFERENCE, "Cargo.toml")) or shutil.which("git") is None, reason="needs the reference checkout (build container)")
 def test_patched_reference_has_the_hip_arm_and_passes_the_stored_type(tmp_path):
     work = tmp_path / "ref"
     shutil.copytree(REFERENCE, work, ignore=shutil.ignore_patterns("testdata", ".git", "target"))
