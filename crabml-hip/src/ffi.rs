@@ -28,6 +28,11 @@ pub const CRABML_HIP_LLAMA_EXACT_NORM: i32 = 8388608;
 /// tensor parallelism: `output_weight` is the rank's vocabulary shard of the classifier (P2P group)
 pub const CRABML_HIP_LLAMA_TP_SPLIT_VOCAB: i32 = 1048576;
 
+/// the hybrid decoder: launch decode steps eagerly
+pub const CRABML_HIP_HYBRID_NO_GRAPH: i32 = 1;
+/// GGML's id of bfloat16 (weights only; crabml's own GGMLType has no such entry)
+pub const CRABML_HIP_BF16: u32 = 30;
+
 #[repr(C)]
 pub struct crabml_hip_device_t {
     _private: [u8; 0],
@@ -90,6 +95,72 @@ pub struct crabml_hip_llama_weights_t {
     pub output_weight: *const crabml_hip_buf_t,
 }
 
+#[repr(C)]
+pub struct crabml_hip_hybrid_t {
+    _private: [u8; 0],
+}
+
+#[repr(C)]
+pub struct crabml_hip_hybrid_config_t {
+    pub width: usize,
+    pub vocab_size: usize,
+    pub n_layers: usize,
+    pub loop_start: usize,
+    pub loop_stop: usize,
+    pub loop_times: usize,
+    pub seq_len: usize,
+    pub pass_rows: usize,
+    pub embed_scale: f32,
+    pub norm_eps: f32,
+    pub logit_softcap: f32,
+    pub compute: u32,
+    pub flags: i32,
+}
+
+#[repr(C)]
+pub struct crabml_hip_hybrid_layer_t {
+    pub attn_heads: usize,
+    pub attn_kv_heads: usize,
+    pub attn_dim: usize,
+    pub attn_vdim: usize,
+    pub attn_chunk: usize,
+    pub lin_heads: usize,
+    pub lin_dim: usize,
+    pub lin_vdim: usize,
+    pub ff: usize,
+    pub attn_score_scale: f32,
+    pub attn_out_scale: f32,
+    pub lin_out_scale: f32,
+    pub lin_decay: *const f64,
+    pub norm1: *const crabml_hip_buf_t,
+    pub attn_q: *const crabml_hip_buf_t,
+    pub attn_k: *const crabml_hip_buf_t,
+    pub attn_v: *const crabml_hip_buf_t,
+    pub attn_gate: *const crabml_hip_buf_t,
+    pub attn_o: *const crabml_hip_buf_t,
+    pub attn_bias_amp: *const crabml_hip_buf_t,
+    pub attn_bias_rate: *const crabml_hip_buf_t,
+    pub attn_sink: *const crabml_hip_buf_t,
+    pub lin_q: *const crabml_hip_buf_t,
+    pub lin_k: *const crabml_hip_buf_t,
+    pub lin_v: *const crabml_hip_buf_t,
+    pub lin_gate: *const crabml_hip_buf_t,
+    pub lin_o: *const crabml_hip_buf_t,
+    pub lin_norm: *const crabml_hip_buf_t,
+    pub norm2: *const crabml_hip_buf_t,
+    pub ff_up: *const crabml_hip_buf_t,
+    pub ff_down: *const crabml_hip_buf_t,
+    pub ff_act: *const crabml_hip_buf_t,
+}
+
+#[repr(C)]
+pub struct crabml_hip_hybrid_weights_t {
+    pub embed: *const crabml_hip_buf_t,
+    pub loop_step: *const crabml_hip_buf_t,
+    pub final_norm: *const crabml_hip_buf_t,
+    pub head: *const crabml_hip_buf_t,
+}
+
 extern "C" {
     // ---- device
     pub fn crabml_hip_abi_version() -> i32;
@@ -136,6 +207,16 @@ extern "C" {
     pub fn crabml_hip_llama_prefill(ctx: *mut crabml_hip_llama_t, tokens: *const u32, n: usize, logits: *mut f32) -> i32;
     pub fn crabml_hip_llama_kv_len(ctx: *const crabml_hip_llama_t) -> usize;
     pub fn crabml_hip_llama_reset(ctx: *mut crabml_hip_llama_t) -> i32;
+
+    // ---- hybrid decoder
+    pub fn crabml_hip_hybrid_create(dev: *mut crabml_hip_device_t, cfg: *const crabml_hip_hybrid_config_t, layers: *const crabml_hip_hybrid_layer_t, w: *const crabml_hip_hybrid_weights_t, out: *mut *mut crabml_hip_hybrid_t) -> i32;
+    pub fn crabml_hip_hybrid_destroy(ctx: *mut crabml_hip_hybrid_t) -> i32;
+    pub fn crabml_hip_hybrid_open(ctx: *mut crabml_hip_hybrid_t, seq: *mut usize) -> i32;
+    pub fn crabml_hip_hybrid_close(ctx: *mut crabml_hip_hybrid_t, seq: usize) -> i32;
+    pub fn crabml_hip_hybrid_len(ctx: *const crabml_hip_hybrid_t, seq: usize) -> usize;
+    pub fn crabml_hip_hybrid_slab_bytes(ctx: *const crabml_hip_hybrid_t) -> usize;
+    pub fn crabml_hip_hybrid_step(ctx: *mut crabml_hip_hybrid_t, n: usize, seqs: *const usize, counts: *const usize, tokens: *const u32, want_counts: *const usize, want: *const u32, logits: *mut f32) -> i32;
+    pub fn crabml_hip_hybrid_decode_greedy(ctx: *mut crabml_hip_hybrid_t, n: usize, seqs: *const usize, tokens: *const u32, n_steps: usize, out_tokens: *mut u32) -> i32;
 
     // ---- tensor-parallel group
     pub fn crabml_hip_tp_get_unique_id(id128: *mut c_void) -> i32;

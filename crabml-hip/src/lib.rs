@@ -10,6 +10,7 @@
 
 mod ffi;
 mod hip_device;
+mod hip_hybrid;
 #[cfg(feature = "llama")]
 mod hip_llama;
 mod hip_tensor;
@@ -17,6 +18,11 @@ mod hip_tensor;
 pub use hip_device::HipTensorDevice;
 pub use hip_device::HipTensorDeviceOptions;
 pub use hip_device::HipTensorDeviceRef;
+pub use hip_hybrid::crabml_hip_hybrid_config_t;
+pub use hip_hybrid::crabml_hip_hybrid_layer_t;
+pub use hip_hybrid::crabml_hip_hybrid_weights_t;
+pub use hip_hybrid::HipHybridRunner;
+pub use hip_hybrid::StepEntry;
 #[cfg(feature = "llama")]
 pub use hip_llama::HipLlamaRunner;
 pub use hip_tensor::HipTensor;

@@ -21,12 +21,12 @@ if not _os.path.exists(LIB_PATH):
 
 from . import _host  # noqa: E402  (raises ImportError loudly if the extension was not built)
 from ._host import (  # noqa: E402,F401
-    CrabmlError, GGMLType, GGUFFile, HipLlamaRunner, HipTensor, HipTensorDevice, Llama2Runner, LlamaConfig, LlamaWeights, RopeMode,
-    TensorStrider, TpComm, abi_version, sample_argmax,
+    CrabmlError, GGMLType, GGUFFile, HipHybridRunner, HipLlamaRunner, HipTensor, HipTensorDevice, Llama2Runner, LlamaConfig, LlamaWeights,
+    ModelRunner, RopeMode, TensorStrider, TpComm, abi_version, known_architectures, load_model, model_architecture, sample_argmax,
 )
 
-__all__ = ["CrabmlError", "GGMLType", "GGUFFile", "HipLlamaRunner", "HipTensor", "HipTensorDevice", "Llama2Runner", "LlamaConfig", "LlamaWeights",
-           "RopeMode", "TensorStrider", "TpComm", "abi_version", "sample_argmax", "pin_host_to_device_node", "LIB_PATH"]
+__all__ = ["CrabmlError", "GGMLType", "GGUFFile", "HipHybridRunner", "HipLlamaRunner", "HipTensor", "HipTensorDevice", "Llama2Runner", "LlamaConfig", "LlamaWeights",
+           "ModelRunner", "RopeMode", "TensorStrider", "TpComm", "abi_version", "known_architectures", "load_model", "model_architecture", "sample_argmax", "pin_host_to_device_node", "LIB_PATH"]
 
 
 def pin_host_to_device_node(device):

@@ -27,7 +27,7 @@ typedef float f32x2 __attribute__((ext_vector_type(2)));
 // ---- GGML block geometry (crabml-core/src/cpu/buf/buf_q*.rs) ---------------------------------
 inline size_t block_elems(uint32_t t) {
   switch (t) {
-    case CRABML_HIP_F32: case CRABML_HIP_F16: return 1;
+    case CRABML_HIP_F32: case CRABML_HIP_F16: case CRABML_HIP_BF16: return 1;
     case CRABML_HIP_Q4_0: case CRABML_HIP_Q4_1: case CRABML_HIP_Q5_0: case CRABML_HIP_Q5_1: case CRABML_HIP_Q8_0: case CRABML_HIP_Q8_1: return 32;
     case CRABML_HIP_Q2_K: case CRABML_HIP_Q3_K: case CRABML_HIP_Q4_K: case CRABML_HIP_Q5_K: case CRABML_HIP_Q6_K: case CRABML_HIP_Q8_K: return 256;
     default: return 0;
@@ -36,7 +36,7 @@ inline size_t block_elems(uint32_t t) {
 inline size_t block_bytes(uint32_t t) {
   switch (t) {
     case CRABML_HIP_F32: return 4;
-    case CRABML_HIP_F16: return 2;
+    case CRABML_HIP_F16: case CRABML_HIP_BF16: return 2;
     case CRABML_HIP_Q4_0: return 18;
     case CRABML_HIP_Q4_1: return 20;
     case CRABML_HIP_Q5_0: return 22;
@@ -55,7 +55,7 @@ inline size_t block_bytes(uint32_t t) {
 // CpuTensorBuf::vec_dot_rhs_dtype, crabml-core/src/cpu/buf/api.rs:142-159
 inline uint32_t vec_dot_rhs_dtype(uint32_t t) {
   switch (t) {
-    case CRABML_HIP_F32: return CRABML_HIP_F32;
+    case CRABML_HIP_F32: case CRABML_HIP_BF16: return CRABML_HIP_F32;
     case CRABML_HIP_F16: return CRABML_HIP_F16;
     case CRABML_HIP_Q8_0: case CRABML_HIP_Q4_0: case CRABML_HIP_Q5_0: return CRABML_HIP_Q8_0;
     case CRABML_HIP_Q8_1: case CRABML_HIP_Q4_1: case CRABML_HIP_Q5_1: return CRABML_HIP_Q8_1;

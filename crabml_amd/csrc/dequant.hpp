@@ -11,6 +11,7 @@ __device__ __forceinline__ float dequant_elem(const char* __restrict__ w, int dt
   switch (dtype) {
     case CRABML_HIP_F32: v = ((const float*)w)[e]; break;
     case CRABML_HIP_F16: v = h2f(((const unsigned short*)w)[e]); break;
+    case CRABML_HIP_BF16: v = bf2f(((const unsigned short*)w)[e]); break;
     case CRABML_HIP_Q8_0: {
       size_t b = e / 32;
       float d = h2f(((const unsigned short*)(w + off_scale))[b]);

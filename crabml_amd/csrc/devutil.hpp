@@ -20,6 +20,12 @@ __device__ __forceinline__ unsigned short f2h(float f) {
   __builtin_memcpy(&h, &x, 2);
   return h;
 }
+// bfloat16: the upper half of an f32 (exact), and back with round-to-nearest-even
+__device__ __forceinline__ float bf2f(unsigned short h) { return __builtin_bit_cast(float, (unsigned)h << 16); }
+__device__ __forceinline__ unsigned short f2bf(float f) {
+  const __bf16 x = (__bf16)f;
+  return __builtin_bit_cast(unsigned short, x);
+}
 // half: `a * b` / `a + b` on f16 = compute in f32, round once to f16
 __device__ __forceinline__ unsigned short h_mul(unsigned short a, unsigned short b) { return f2h(h2f(a) * h2f(b)); }
 __device__ __forceinline__ unsigned short h_add(unsigned short a, unsigned short b) { return f2h(h2f(a) + h2f(b)); }

@@ -231,21 +231,6 @@ TpP2P tp_view(const crabml_hip_llama* c, bool fused_collective) {
   return t;
 }
 
-// hipFuncAttributeMaxDynamicSharedMemorySize is a property of the kernel in this PROCESS, not of a context: a second context
-// with a shorter sequence must not lower the limit an earlier context's launches (and captured graphs) were sized for.
-// Only ever raise it, per device.
-hipError_t raise_dyn_lds(const crabml_hip_device* dev, const void* fn, int bytes) {
-  static std::mutex mu;
-  static std::map<std::pair<int, const void*>, int> have;
-  if (dev->dry) return hipErrorNoDevice;  // record-only test device
-  std::lock_guard<std::mutex> g(mu);
-  int& cur = have[{dev->ordinal, fn}];
-  if (bytes <= cur) return hipSuccess;
-  const hipError_t e = hipFuncSetAttribute(fn, hipFuncAttributeMaxDynamicSharedMemorySize, bytes);
-  if (e == hipSuccess) cur = bytes;
-  return e;
-}
-
 int dalloc(crabml_hip_llama* c, size_t bytes, void** out) {
   size_t cap = 0;
   CH_TRY(pool_alloc(c->dev, bytes, out, &cap));
@@ -427,7 +412,7 @@ int enqueue_classifier_and_sampler(crabml_hip_llama* c, const void* cls_act, cra
     CH_HIP(dev, hipGetLastError());
     return 0;
   }
-  k_argmax_partial<<<ARGMAX_BLOCKS, 256, 0, st>>>(out, c->vocab_l, c->am_val, c->am_idx, c->vocab_off);
+  k_argmax_partial<<<ARGMAX_BLOCKS, 256, 0, st>>>(out, c->vocab_l, c->am_val, c->am_idx, c->vocab_off, 0);
   if (c->split_vocab && c->comm && c->comm->p2p)
     k_argmax_step_tp<<<1, 64, 0, st>>>(c->am_val, c->am_idx, ARGMAX_BLOCKS, token_d, pos_d, step_d, c->out_tokens, c->out_cap, c->state + 4,
                                        tp_view(c, true), n_segments(c));

@@ -3,6 +3,7 @@
 // translation units: the kernels are launched from fused.hip's host code).
 #pragma once
 #include "fused_common.hpp"
+#include "sampler.hpp"
 
 namespace crabml_hip {
 // ---- GEMV + residual: x[row] = W[row].xq + x[row]   (matmul_vec, then add_inplace: arithmetic.rs:27-33) ---
@@ -972,7 +973,8 @@ __global__ __launch_bounds__(1024, 8) void k_gateup_k_lds(Planes wg, Planes wu, 
     rows_terms_q4k<2, false>(wu.q, (const i32x4*)wu.d, la, row0, m, nsb, lane, T + (size_t)(32 + wave * 2) * stride, stride);
     __syncthreads();
     if (wave == 0) {
-      const float s = q4k_ordered_sum(T + (size_t)lane * stride, nsb);  // lane < 32: gate row `lane`; else up row `lane - 32`
+      // (three records ahead: a fourth does not fit the 64 VGPRs that keep two workgroups on a CU)
+      const float s = q4k_ordered_sum<3>(T + (size_t)lane * stride, nsb);  // lane < 32: gate row `lane`; else up row `lane - 32`
       const float u = __shfl(s, (lane & 31) + 32, 64);
       if (lane < 32) {
         const float hval = silu_mul(s, u, exp_tab);
@@ -1189,43 +1191,7 @@ __global__ __launch_bounds__(256) void k_gateup_epi_quant(const float* __restric
 }
 
 // ---- greedy sampler + advance: Iterator::max_by keeps the LAST maximum (sampler.rs:109-116) ------------
-// stage 1: ARGMAX_BLOCKS workgroups, each over a contiguous slice; stage 2: one wave combines and advances.
-#define ARGMAX_BLOCKS 128
-__device__ __forceinline__ void argmax_combine(float& cv, int& ci, float ov, int oi) {
-  // keep the later index among equal maxima; an index of -1 means "empty"
-  bool take = oi >= 0 && (ci < 0 || ov > cv || (!(cv > ov) && oi > ci));
-  if (take) {
-    cv = ov;
-    ci = oi;
-  }
-}
-// base: global index of logits[0] (a vocabulary shard of a tensor-parallel classifier; 0 otherwise)
-__global__ __launch_bounds__(256) void k_argmax_partial(const float* __restrict__ logits, int n, float* __restrict__ pv,
-                                                        int* __restrict__ pi, int base) {
-  __shared__ float sv[4];
-  __shared__ int si[4];
-  const int per = (n + gridDim.x - 1) / gridDim.x;
-  const int lo = blockIdx.x * per, hi = min(n, lo + per);
-  float bv = -INFINITY;
-  int bi = -1;
-  for (int i = lo + threadIdx.x; i < hi; i += blockDim.x) argmax_combine(bv, bi, logits[i], base + i);
-#pragma unroll
-  for (int o = 32; o > 0; o >>= 1) {
-    float ov = __shfl_xor(bv, o, 64);
-    int oi = __shfl_xor(bi, o, 64);
-    argmax_combine(bv, bi, ov, oi);
-  }
-  if ((threadIdx.x & 63) == 0) {
-    sv[threadIdx.x >> 6] = bv;
-    si[threadIdx.x >> 6] = bi;
-  }
-  __syncthreads();
-  if (threadIdx.x == 0) {
-    for (int w = 1; w < 4; w++) argmax_combine(bv, bi, sv[w], si[w]);
-    pv[blockIdx.x] = bv;
-    pi[blockIdx.x] = bi;
-  }
-}
+// stage 1: k_argmax_partial (sampler.hpp); stage 2: one wave combines and advances.
 // best: nullable; {max as f32 bits, index} of THIS context's logits (a tensor-parallel rank's shard: the single-device
 // simulation combines the ranks' pairs afterwards, k_sim_argmax_combine)
 __global__ __launch_bounds__(64) void k_argmax_step(const float* __restrict__ pv, const int* __restrict__ pi, int nparts,

@@ -1,0 +1,79 @@
+// gemm_bf16.hpp -- rows x bfloat16 weights on the matrix cores: the prompt-time linear of the hybrid decoder.
+//
+//   C[row][n] = sum_k A[row][k] W[n][k]     A: bf16 planes, W: bf16 rows, f32 accumulation (v_mfma_f32_16x16x32_bf16)
+//
+// One plane of A is bf16 arithmetic.  Three planes are a row of f32 numbers cut into its upper, middle and lower eight significand
+// bits (split3): every f32 is the exact sum of its planes and every plane times a bf16 weight is exact in f32, so three planes give
+// true f32 products with f32 sums -- the weights ARE bf16 numbers -- at a fifth of the time the f32 matrix instruction would take.
+//
+// Mapping: BM x BN output tile per 256-thread workgroup, k in steps of 64.  A step's tiles go from memory straight into LDS
+// (global_load_lds, 16 bytes per lane), double-buffered: the next step's requests are out before the current one is multiplied.  LDS
+// holds rows of 128 bytes whose 16-byte chunks are permuted by (row / 2) % 8 -- on the SOURCE side, the LDS side of the instruction
+// being linear -- so that the 16 rows a fragment read touches spread over all 64 banks.  Operands are padded by their owners (k to 64,
+// weight rows to 256, activation rows to 128), so the loop has no bounds checks; stores have.  Workgroups are dealt to the eight XCDs
+// in contiguous runs of the tile order, row tiles fastest: an XCD's L2 keeps the weight tile that its row tiles share.
+//
+// The row operations around a linear are folded into it.  In: an RMS norm with a single gain is a factor per row, applied to the
+// accumulators (the producers leave each row's sum of squares in 64-column pieces).  Out: activations by column range, xIELU, soft
+// cap, or the residual add, which also leaves the new row's bf16 planes and square sums for the next linear.
+#pragma once
+#include "gemv_bf16.hpp"
+
+namespace crabml_hip {
+
+typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+typedef unsigned short u16x4 __attribute__((ext_vector_type(4)));
+
+enum {
+  GEMM_OUT_ACT_BF16 = 0,   // rows of bf16 (ActRanges)
+  GEMM_OUT_ACT_F32 = 1,    // rows of f32 (ActRanges)
+  GEMM_OUT_RESIDUAL = 2,   // x += acc (+ add_rows + add_vec); planes of x; square sums
+  GEMM_OUT_XIELU = 3,      // planes of xielu(acc)
+  GEMM_OUT_SOFTCAP = 4,    // f32 rows
+};
+
+// an f32 as bf16 planes: 1 plane = rounded to nearest even; 3 planes = upper / middle / lower bits, their sum exact
+template <int P>
+__device__ __forceinline__ void split_store(float v, unsigned short* p, size_t plane_stride) {
+  if constexpr (P == 1) {
+    *p = f2bf(v);
+  } else {
+    const float hi = __builtin_bit_cast(float, __builtin_bit_cast(unsigned, v) & 0xffff0000u);
+    const float r = v - hi;  // exact: the low 16 bits of the significand
+    const float mid = __builtin_bit_cast(float, __builtin_bit_cast(unsigned, r) & 0xffff0000u);
+    p[0] = (unsigned short)(__builtin_bit_cast(unsigned, hi) >> 16);
+    p[plane_stride] = (unsigned short)(__builtin_bit_cast(unsigned, mid) >> 16);
+    p[2 * plane_stride] = f2bf(r - mid);
+  }
+}
+
+struct GemmBf16 {
+  const unsigned short* a = nullptr;  // [planes][rows padded][k]
+  size_t a_plane = 0;                 // elements between planes
+  const unsigned short* w = nullptr;  // [N padded][k]
+  int M = 0, N = 0, K = 0;            // K % 64 == 0
+  // row factor (nullable sq): gain / sqrt(sum_i sq[row][i] / mean_n + eps)
+  const float* sq_in = nullptr;
+  int n_sq = 0, mean_n = 1;
+  float eps = 0.f;
+  const float* gain = nullptr;
+  // outputs
+  void* out = nullptr;  // ACT / SOFTCAP rows
+  int ldo = 0;
+  ActRanges act;
+  const float* xielu = nullptr;
+  float cap = 0.f;
+  float* x = nullptr;  // RESIDUAL
+  int ldx = 0;
+  const float *add_rows = nullptr, *add_vec = nullptr;
+  unsigned short* planes = nullptr;  // RESIDUAL / XIELU: [planes][rows padded][ldp]
+  size_t p_plane = 0;
+  int ldp = 0;
+  float* sq_out = nullptr;  // [row][n_sq_out]: square sums by 64 columns
+  int n_sq_out = 0;
+};
+
+// planes: 1 or 3 (GEMM_OUT_ACT_BF16 goes with one, GEMM_OUT_ACT_F32 with three)
+void launch_gemm_bf16(crabml_hip_device* dev, crabml_hip_device::ProfRec* rec, int planes, int out, const GemmBf16& g);
+
+}  // namespace crabml_hip

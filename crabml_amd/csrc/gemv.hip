@@ -16,7 +16,7 @@
 // CPU loop (lane-strided partial sums + a 64-lane butterfly), which is why logits carry an fp tolerance.
 // The kernel is HBM-bound (~3.6 flop/byte): no LDS round trip, no MFMA; x is re-read from L1/L2.
 #include "gemv_core.hpp"
-#include "kernels.hpp"
+#include "gemv_bf16.hpp"
 
 namespace crabml_hip {
 
@@ -251,6 +251,19 @@ __global__ __launch_bounds__(256) void k_gemv_f16(const unsigned short* __restri
   if (lane == 0) out[row] = acc;
 }
 
+// bfloat16 rows of any length x f32 (rows whose k the vectorized kernel of gemv_bf16.hpp does not take)
+__global__ __launch_bounds__(256) void k_gemv_bf16_any(const unsigned short* __restrict__ w, const float* __restrict__ x,
+                                                       float* __restrict__ out, int m, int k) {
+  const int lane = threadIdx.x & 63;
+  const int row = blockIdx.x * (blockDim.x >> 6) + wave_in_wg();
+  if (row >= m) return;
+  const unsigned short* wr = w + (size_t)row * k;
+  float acc = 0.f;
+  for (int i = lane; i < k; i += 64) acc = __builtin_fmaf(bf2f(wr[i]), x[i], acc);
+  acc = wave_sum_f32(acc);
+  if (lane == 0) out[row] = acc;
+}
+
 // ---- host launcher -------------------------------------------------------------------------------
 template <typename F>
 static void launch_rows(hipStream_t st, int m, int n_cu, F&& f) {
@@ -275,6 +288,17 @@ int launch_gemv(crabml_hip_device* dev, const crabml_hip_buf* w, size_t m_, size
   // F32 weights take the dense f32 rhs as is (row stride k*4); quantized planes are padded per row
   const size_t act_stride = qt == CRABML_HIP_F32 ? k_ * 4 : al.total;
   // a real batch (prefill): the weights are streamed once through the matrix cores instead of once per row
+  if (w->dtype == CRABML_HIP_BF16 && k % 8 == 0) {  // up to 8 rows of the rhs share one pass over the weights
+    GemvBf16 g;
+    g.w = (const unsigned short*)wp;
+    g.x = (const float*)act;
+    g.out = out;
+    g.N = g.ldo = m;
+    g.K = g.ldw = g.ldx = k;
+    g.nb = (int)b;
+    launch_gemv_bf16<GEMV_IN_PLAIN, GEMV_OUT_STORE>(st, rec0, g);
+    return 0;
+  }
   if (b >= 16 && launch_gemm_mfma(dev, w, m_, k_, act, b, out, rec0, nullptr, fused_add)) return 0;
   for (size_t bi = 0; bi < b; bi++) {
     const char* ap = (const char*)act + bi * act_stride;
@@ -406,6 +430,10 @@ int launch_gemv(crabml_hip_device* dev, const crabml_hip_buf* w, size_t m_, size
       case CRABML_HIP_F16: {
         int grid = (m + 3) / 4;
         launch_k(st, rec, k_gemv_f16, dim3(grid), dim3(256), 0, (const unsigned short*)wp, (const unsigned short*)ap, o, m, k);
+        break;
+      }
+      case CRABML_HIP_BF16: {
+        launch_k(st, rec, k_gemv_bf16_any, dim3((m + 3) / 4), dim3(256), 0, (const unsigned short*)wp, (const float*)ap, o, m, k);
         break;
       }
       default:

@@ -1,0 +1,257 @@
+// gemv_bf16.hpp -- bfloat16 weight rows x f32 activations for up to 8 rows of the rhs at a time, with the neighbouring row
+// operations folded into its two ends: the decode-time linear of the hybrid decoder (hybrid_step.hpp), and matmul_vec on BF16.
+//
+// Mapping: a wave owns R consecutive output rows and strides k 512 elements at a time (8 per lane = one aligned 16-byte request per
+// row); the rhs rows sit in LDS as f32 in two half-octet planes, so the two ds_read_b128 a lane needs are contiguous across the wave.
+// Weights become f32 by a shift / mask, products and sums are f32 fmas: the rhs is never rounded.  The weight requests of a block
+// of steps go out before the activations are staged (the first block) or while the previous block is multiplied.  One pass over the
+// weights serves NB rhs rows; more rows are further grid rows (blockIdx.y) that hit the same weights in L2 / Infinity Cache.
+#pragma once
+#include "devutil.hpp"
+#include "kernels.hpp"
+
+namespace crabml_hip {
+
+// what happens to an rhs row on the way in
+enum {
+  GEMV_IN_PLAIN = 0,
+  GEMV_IN_RMS = 1,    // the row is RMS-normalized with a single gain.  The row factor is taken from the staged row itself and
+                      // applied to the finished dots: W (s x) = s (W x)
+  GEMV_IN_SPLIT = 2,  // elements from k_split on still want their RMS normalization; their sum of squares arrives in pieces (ss)
+};
+// what happens to a dot product on the way out
+enum {
+  GEMV_OUT_STORE = 0,
+  GEMV_OUT_ACT = 1,      // column ranges with their own activation (ActRanges)
+  GEMV_OUT_RESIDUAL = 2, // out += dot (+ add_rows[b] + add_vec)
+  GEMV_OUT_XIELU = 3,    // xielu(dot)
+  GEMV_OUT_SOFTCAP = 4,  // cap * tanh(dot / cap)
+};
+enum { ACT_NONE = 0, ACT_SIGMOID = 1, ACT_SILU = 2 };
+struct ActRanges {  // columns [end[i-1], end[i]) take activation kind[i]
+  int end[4] = {0, 0, 0, 0};
+  int kind[4] = {0, 0, 0, 0};
+};
+
+struct GemvBf16 {
+  const unsigned short* w = nullptr;  // [N][ldw]
+  const float* x = nullptr;           // [nb][ldx]
+  float* out = nullptr;               // [nb][ldo]
+  int N = 0, K = 0, ldw = 0, ldx = 0, ldo = 0, nb = 1;  // K % 8 == 0
+  // GEMV_IN_RMS: elements the mean is over, eps, the gain (device); GEMV_IN_SPLIT: the same for the tail, with ss[b][n_ss] pieces
+  int mean_n = 1;
+  float eps = 0.f;
+  const float* gain = nullptr;
+  int k_split = 0, n_ss = 0;
+  const float* ss = nullptr;
+  ActRanges act;
+  const float* xielu = nullptr;  // {softplus(p), 1/2 + softplus(q)}
+  const float *add_rows = nullptr, *add_vec = nullptr;
+  int ld_add = 0;
+  float cap = 0.f;
+};
+
+__device__ __forceinline__ float act_sigmoid(float z) { return 1.0f / (1.0f + __expf(-z)); }
+__device__ __forceinline__ float act_apply(float z, int kind) {
+  if (kind == ACT_NONE) return z;
+  const float s = act_sigmoid(z);
+  return kind == ACT_SILU ? z * s : s;
+}
+__device__ __forceinline__ float act_ranges(float z, int col, const ActRanges& a) {
+  const int kind = col < a.end[0] ? a.kind[0] : col < a.end[1] ? a.kind[1] : col < a.end[2] ? a.kind[2] : a.kind[3];
+  return act_apply(z, kind);
+}
+// e^z - 1 - z for z <= 0 without the cancellation near zero: its own series below 1/4
+__device__ __forceinline__ float exp_minus_line(float z) {
+  if (z > -0.25f) {
+    float s = 1.0f / 40320.0f;
+    s = __builtin_fmaf(s, z, 1.0f / 5040.0f);
+    s = __builtin_fmaf(s, z, 1.0f / 720.0f);
+    s = __builtin_fmaf(s, z, 1.0f / 120.0f);
+    s = __builtin_fmaf(s, z, 1.0f / 24.0f);
+    s = __builtin_fmaf(s, z, 1.0f / 6.0f);
+    s = __builtin_fmaf(s, z, 0.5f);
+    return s * z * z;
+  }
+  return __expf(z) - 1.0f - z;
+}
+__device__ __forceinline__ float xielu_apply(float z, float right, float left) {
+  const float curved = z > 0.0f ? right * z * z : left * exp_minus_line(z);
+  return __builtin_fmaf(0.5f, z, curved);
+}
+__device__ __forceinline__ float soft_cap(float z, float cap) { return cap > 0.0f ? cap * tanhf(z / cap) : z; }
+
+#define GEMV_BF16_LDS_FLOATS 8192  // rhs elements staged at a time, all rows together: a cut segment is a multiple of the steps in flight
+
+template <int NB, int R, int IN, int OUT>
+__global__ __launch_bounds__(256) void k_gemv_bf16(const GemvBf16 a) {
+  extern __shared__ __attribute__((aligned(16))) float gemv_lds[];  // [NB][2][seg / 2]
+  __shared__ float red[4][NB];
+  const int tid = threadIdx.x, lane = tid & 63, wave = wave_in_wg();
+  const int row0 = (blockIdx.x * 4 + wave) * R, b0 = blockIdx.y * NB;
+  const int seg = a.K < GEMV_BF16_LDS_FLOATS / NB ? a.K : GEMV_BF16_LDS_FLOATS / NB;  // elements per staged segment (512-multiple if cut)
+  const int half = seg / 2;                                                           // floats per half-octet plane
+  constexpr int UN = R >= 4 || NB >= 8 ? 2 : 4;  // steps of 512 in flight
+  const unsigned short* wr[R];
+#pragma unroll
+  for (int r = 0; r < R; r++) {
+    const int row = row0 + r < a.N ? row0 + r : a.N - 1;
+    wr[r] = a.w + (size_t)row * a.ldw;
+  }
+  i32x4 wv[UN][R];
+  auto request = [&](int k0) {
+#pragma unroll
+    for (int u = 0; u < UN; u++) {
+      int k = k0 + u * 512 + lane * 8;
+      k = k < a.K ? k : 0;  // (a lane past the end requests the row's start and never uses it)
+#pragma unroll
+      for (int r = 0; r < R; r++) wv[u][r] = __builtin_nontemporal_load((const i32x4*)(wr[r] + k));
+    }
+  };
+  request(0);
+  float acc[R][NB];
+#pragma unroll
+  for (int r = 0; r < R; r++)
+#pragma unroll
+    for (int b = 0; b < NB; b++) acc[r][b] = 0.f;
+  float tail[NB], sq[NB];
+#pragma unroll
+  for (int b = 0; b < NB; b++) {
+    sq[b] = 0.f;
+    tail[b] = 1.f;
+  }
+  if constexpr (IN == GEMV_IN_SPLIT) {
+#pragma unroll
+    for (int b = 0; b < NB; b++) {
+      const int bb = b0 + b < a.nb ? b0 + b : a.nb - 1;
+      float s = 0.f;
+      for (int i = lane; i < a.n_ss; i += 64) s += a.ss[(size_t)bb * a.n_ss + i];
+      s = wave_sum_f32(s);
+      tail[b] = 1.0f / sqrtf(s / (float)a.mean_n + a.eps);
+    }
+  }
+  for (int s0 = 0; s0 < a.K; s0 += seg) {
+    const int n = a.K - s0 < seg ? a.K - s0 : seg;
+    if (s0 > 0) __syncthreads();  // the previous segment has been read by every wave
+#pragma unroll
+    for (int b = 0; b < NB; b++) {
+      const int bb = b0 + b < a.nb ? b0 + b : a.nb - 1;
+      const float* xr = a.x + (size_t)bb * a.ldx + s0;
+      float* lo = gemv_lds + b * 2 * half;
+      for (int q = tid; q < n / 8; q += 256) {
+        f32x4 v0 = *(const f32x4*)(xr + q * 8), v1 = *(const f32x4*)(xr + q * 8 + 4);
+        if constexpr (IN == GEMV_IN_RMS) {
+#pragma unroll
+          for (int e = 0; e < 4; e++) sq[b] = __builtin_fmaf(v0[e], v0[e], __builtin_fmaf(v1[e], v1[e], sq[b]));
+        }
+        if constexpr (IN == GEMV_IN_SPLIT) {
+          if (s0 + q * 8 >= a.k_split) {
+            v0 *= tail[b];
+            v1 *= tail[b];
+          }
+        }
+        *(f32x4*)(lo + q * 4) = v0;
+        *(f32x4*)(lo + half + q * 4) = v1;
+      }
+    }
+    if constexpr (IN == GEMV_IN_RMS) {
+      if (s0 + seg >= a.K) {
+#pragma unroll
+        for (int b = 0; b < NB; b++) {
+          const float s = wave_sum_f32(sq[b]);
+          if (lane == 0) red[wave][b] = s;
+        }
+      }
+    }
+    __syncthreads();
+    for (int k0 = 0; k0 < n; k0 += UN * 512) {
+      i32x4 cur[UN][R];
+#pragma unroll
+      for (int u = 0; u < UN; u++)
+#pragma unroll
+        for (int r = 0; r < R; r++) cur[u][r] = wv[u][r];
+      if (s0 + k0 + UN * 512 < a.K) request(s0 + k0 + UN * 512);  // (also across a segment's end: seg % (UN * 512) == 0 then)
+#pragma unroll
+      for (int u = 0; u < UN; u++) {
+        const int k = k0 + u * 512 + lane * 8;
+        if (k < n) {
+#pragma unroll
+          for (int b = 0; b < NB; b++) {
+            const float* lo = gemv_lds + b * 2 * half + (k >> 1);
+            const f32x4 x0 = *(const f32x4*)lo, x1 = *(const f32x4*)(lo + half);
+#pragma unroll
+            for (int r = 0; r < R; r++) {
+              float s = acc[r][b];
+#pragma unroll
+              for (int e = 0; e < 2; e++) {
+                const unsigned p = (unsigned)cur[u][r][e], p2 = (unsigned)cur[u][r][e + 2];
+                s = __builtin_fmaf(__builtin_bit_cast(float, p << 16), x0[2 * e], s);
+                s = __builtin_fmaf(__builtin_bit_cast(float, p & 0xffff0000u), x0[2 * e + 1], s);
+                s = __builtin_fmaf(__builtin_bit_cast(float, p2 << 16), x1[2 * e], s);
+                s = __builtin_fmaf(__builtin_bit_cast(float, p2 & 0xffff0000u), x1[2 * e + 1], s);
+              }
+              acc[r][b] = s;
+            }
+          }
+        }
+      }
+    }
+  }
+  float scale[NB];
+#pragma unroll
+  for (int b = 0; b < NB; b++) {
+    scale[b] = 1.f;
+    if constexpr (IN == GEMV_IN_RMS) {
+      const float s = (red[0][b] + red[1][b]) + (red[2][b] + red[3][b]);
+      scale[b] = *a.gain / sqrtf(s / (float)a.mean_n + a.eps);
+    }
+  }
+#pragma unroll
+  for (int r = 0; r < R; r++)
+#pragma unroll
+    for (int b = 0; b < NB; b++) {
+      const float v = wave_sum_f32(acc[r][b]) * scale[b];
+      const int row = row0 + r, bb = b0 + b;
+      if (lane == ((r * NB + b) & 63) && row < a.N && bb < a.nb) {
+        float* o = a.out + (size_t)bb * a.ldo + row;
+        if constexpr (OUT == GEMV_OUT_STORE) *o = v;
+        if constexpr (OUT == GEMV_OUT_ACT) *o = act_ranges(v, row, a.act);
+        if constexpr (OUT == GEMV_OUT_RESIDUAL) {
+          float s = *o + v;
+          if (a.add_rows) s += a.add_rows[(size_t)bb * a.ld_add + row];
+          if (a.add_vec) s += a.add_vec[row];
+          *o = s;
+        }
+        if constexpr (OUT == GEMV_OUT_XIELU) *o = xielu_apply(v, a.xielu[0], a.xielu[1]);
+        if constexpr (OUT == GEMV_OUT_SOFTCAP) *o = soft_cap(v, a.cap);
+      }
+    }
+}
+
+template <int NB, int R, int IN, int OUT>
+inline void launch_gemv_bf16_t(hipStream_t st, crabml_hip_device::ProfRec* rec, const GemvBf16& a) {
+  const int cap = GEMV_BF16_LDS_FLOATS / NB, seg = a.K < cap ? a.K : cap;
+  launch_k(st, rec, k_gemv_bf16<NB, R, IN, OUT>, dim3((a.N + 4 * R - 1) / (4 * R), (a.nb + NB - 1) / NB), dim3(256),
+           (size_t)NB * seg * sizeof(float), a);
+}
+// rows of the rhs that share one pass over the weights: as many as there are, up to 8
+template <int IN, int OUT>
+inline void launch_gemv_bf16(hipStream_t st, crabml_hip_device::ProfRec* rec, const GemvBf16& a) {
+  const bool wide = a.N >= 16384;  // enough rows to give a wave four and still fill the chip
+  if (a.nb <= 1) {
+    if (wide)
+      launch_gemv_bf16_t<1, 4, IN, OUT>(st, rec, a);
+    else if (a.N >= 2048)
+      launch_gemv_bf16_t<1, 2, IN, OUT>(st, rec, a);
+    else
+      launch_gemv_bf16_t<1, 1, IN, OUT>(st, rec, a);
+  } else if (a.nb <= 2) {
+    launch_gemv_bf16_t<2, 2, IN, OUT>(st, rec, a);
+  } else if (a.nb <= 4) {
+    launch_gemv_bf16_t<4, 2, IN, OUT>(st, rec, a);
+  } else {
+    launch_gemv_bf16_t<8, 2, IN, OUT>(st, rec, a);
+  }
+}
+
+}  // namespace crabml_hip

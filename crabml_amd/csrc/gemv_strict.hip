@@ -284,6 +284,12 @@ __global__ __launch_bounds__(64) void k_gemv_strict(const char* __restrict__ w, 
       for (int i = 0; i < k; i++) sumf += h2f(wr[i]) * h2f(x[i]);
       break;
     }
+    case CRABML_HIP_BF16: {
+      const unsigned short* wr = (const unsigned short*)w + (size_t)row * k;
+      const float* x = (const float*)act;
+      for (int i = 0; i < k; i++) sumf += bf2f(wr[i]) * x[i];
+      break;
+    }
     default: break;
   }
   out[row] = add ? sumf + add[row] : sumf;  // (add: the residual, x = matmul_out + x)

@@ -332,6 +332,7 @@ inline bool ggml_block_geometry(uint32_t t, size_t* block_bytes, size_t* block_e
     case 13: *block_bytes = 176; *block_elems = 256; return true;  // Q5_K (the reference's field order, buf_q5_k.rs:13-21)
     case 14: *block_bytes = 210; *block_elems = 256; return true;  // Q6_K
     case 15: *block_bytes = 292; *block_elems = 256; return true;  // Q8_K
+    case 30: *block_bytes = 2; *block_elems = 1; return true;      // BF16 (ggml's id; crabml itself has no such type)
     default: return false;
   }
 }

@@ -8,6 +8,7 @@
 
 #include "hip_tensor.hpp"
 #include "llama2_runner.hpp"
+#include "model_runner.hpp"
 
 namespace crabml_host {
 
@@ -59,7 +60,7 @@ class TpComm {
   int nranks_, rank_;
 };
 
-class HipLlamaRunner {
+class HipLlamaRunner : public ModelRunner {
  public:
   HipLlamaRunner(const LlamaConfig& conf, std::shared_ptr<LlamaWeights<HipTensor>> w, HipTensorDeviceRef device,
                  size_t seq_len, bool use_f16_kv_cache, bool use_graph = true, bool prefetch = true, int tp_size = 1,
@@ -109,31 +110,36 @@ class HipLlamaRunner {
     cw.output_weight = W.output_weight ? W.output_weight->raw() : nullptr;
     device_->check(crabml_hip_llama_create(device_->raw(), &c, &cw, &ctx_));
   }
-  ~HipLlamaRunner() {
+  ~HipLlamaRunner() override {
     if (ctx_) crabml_hip_llama_destroy(ctx_);
   }
   HipLlamaRunner(const HipLlamaRunner&) = delete;
   HipLlamaRunner& operator=(const HipLlamaRunner&) = delete;
 
-  size_t kv_cache_len() const { return crabml_hip_llama_kv_len(ctx_); }
+  const std::string& architecture() const override {
+    static const std::string name = "llama";
+    return name;
+  }
+  size_t vocab_size() const override { return conf_.vocab_size; }
+  size_t kv_cache_len() const override { return crabml_hip_llama_kv_len(ctx_); }
   crabml_hip_llama_t* raw() const { return ctx_; }
   const LlamaConfig& conf() const { return conf_; }
   const HipTensorDeviceRef& device() const { return device_; }
-  void reset() { device_->check(crabml_hip_llama_reset(ctx_)); }
+  void reset() override { device_->check(crabml_hip_llama_reset(ctx_)); }
   // Llama2Runner::forward (llama2.rs:184-211) for one token; returns the logits
-  std::vector<float> forward(size_t token, size_t pos) {
+  std::vector<float> forward(size_t token, size_t pos) override {
     std::vector<float> logits(conf_.vocab_size);
     device_->check(crabml_hip_llama_forward(ctx_, token, pos, logits.data()));
     return logits;
   }
   // the token loop of Llama2Runner::prefill (llama2.rs:111-129) as batched passes; returns the last token's logits
-  std::vector<float> prefill(const std::vector<uint32_t>& tokens) {
+  std::vector<float> prefill(const std::vector<uint32_t>& tokens) override {
     std::vector<float> logits(conf_.vocab_size);
     device_->check(crabml_hip_llama_prefill(ctx_, tokens.data(), tokens.size(), logits.data()));
     return logits;
   }
   void forward_async(size_t token, size_t pos) { device_->check(crabml_hip_llama_forward(ctx_, token, pos, nullptr)); }
-  std::vector<uint32_t> decode_greedy(size_t token, size_t steps) {
+  std::vector<uint32_t> decode_greedy(size_t token, size_t steps) override {
     std::vector<uint32_t> ids(steps);
     device_->check(crabml_hip_llama_decode_greedy(ctx_, token, steps, ids.data()));
     return ids;

@@ -10,6 +10,8 @@
 
 #include "gguf.hpp"
 #include "hip_llama.hpp"
+#include "hybrid.hpp"
+#include "model_registry.hpp"
 #include "hip_tensor.hpp"
 #include "llama2_runner.hpp"
 
@@ -50,7 +52,8 @@ PYBIND11_MODULE(_host, m) {
       .value("F32", GGMLType::F32).value("F16", GGMLType::F16).value("Q4_0", GGMLType::Q4_0)
       .value("Q4_1", GGMLType::Q4_1).value("Q8_0", GGMLType::Q8_0).value("Q8_1", GGMLType::Q8_1)
       .value("Q5_0", GGMLType::Q5_0).value("Q5_1", GGMLType::Q5_1).value("Q2K", GGMLType::Q2K).value("Q3K", GGMLType::Q3K)
-      .value("Q4K", GGMLType::Q4K).value("Q5K", GGMLType::Q5K).value("Q6K", GGMLType::Q6K).value("Q8K", GGMLType::Q8K);
+      .value("Q4K", GGMLType::Q4K).value("Q5K", GGMLType::Q5K).value("Q6K", GGMLType::Q6K).value("Q8K", GGMLType::Q8K)
+      .value("BF16", GGMLType::BF16);
   py::enum_<RopeMode>(m, "RopeMode").value("Llama", RopeMode::Llama).value("Neox", RopeMode::Neox);
 
   py::class_<TensorStrider>(m, "TensorStrider")
@@ -391,7 +394,37 @@ PYBIND11_MODULE(_host, m) {
       .def_property_readonly("rank", &TpComm::rank)
       .def("all_reduce", &TpComm::all_reduce, py::call_guard<py::gil_scoped_release>());
 
-  py::class_<HipLlamaRunner>(m, "HipLlamaRunner")
+  // what every served model can do (model_runner.hpp)
+  py::class_<ModelRunner>(m, "ModelRunner")
+      .def_property_readonly("architecture", &ModelRunner::architecture)
+      .def_property_readonly("vocab_size", &ModelRunner::vocab_size)
+      .def("prefill",
+           [](ModelRunner& r, const std::vector<uint32_t>& tokens) {
+             std::vector<float> lg;
+             {
+               py::gil_scoped_release rel;
+               lg = r.prefill(tokens);
+             }
+             return py::array_t<float>(lg.size(), lg.data());
+           })
+      .def("kv_cache_len", &ModelRunner::kv_cache_len)
+      .def("reset", &ModelRunner::reset)
+      .def("forward",
+           [](ModelRunner& r, size_t token, size_t pos) {
+             std::vector<float> lg;
+             {
+               py::gil_scoped_release rel;
+               lg = r.forward(token, pos);
+             }
+             return py::array_t<float>(lg.size(), lg.data());
+           })
+      .def("decode_greedy",
+           [](ModelRunner& r, size_t token, size_t steps) {
+             py::gil_scoped_release rel;
+             return r.decode_greedy(token, steps);
+           });
+
+  py::class_<HipLlamaRunner, ModelRunner>(m, "HipLlamaRunner")
       .def(py::init([](const LlamaConfig& conf, std::shared_ptr<Weights> w, std::shared_ptr<HipTensorDevice> dev,
                        size_t seq_len, bool use_f16_kv_cache, bool use_graph, bool prefetch, int tp_size, int tp_rank,
                        std::shared_ptr<TpComm> comm, bool norm_epilogue, int extra_flags, size_t attn_long_from,
@@ -406,15 +439,6 @@ PYBIND11_MODULE(_host, m) {
            py::arg("use_graph") = true, py::arg("prefetch") = true, py::arg("tp_size") = 1, py::arg("tp_rank") = 0,
            py::arg("comm") = std::shared_ptr<TpComm>(), py::arg("norm_epilogue") = true,
            py::arg("extra_flags") = 0, py::arg("attn_long_from") = 0, py::arg("prefill_chunk") = 0)
-      .def("prefill",
-           [](HipLlamaRunner& r, const std::vector<uint32_t>& tokens) {
-             std::vector<float> lg;
-             {
-               py::gil_scoped_release rel;
-               lg = r.prefill(tokens);
-             }
-             return py::array_t<float>(lg.size(), lg.data());
-           })
       .def_static("tp_sim_forward",
                   [](const std::vector<HipLlamaRunner*>& ranks, size_t token, size_t pos) {
                     std::vector<float> lg;
@@ -424,27 +448,47 @@ PYBIND11_MODULE(_host, m) {
                     }
                     return py::array_t<float>(lg.size(), lg.data());
                   })
-      .def("kv_cache_len", &HipLlamaRunner::kv_cache_len)
-      .def("reset", &HipLlamaRunner::reset)
-      .def("forward",
-           [](HipLlamaRunner& r, size_t token, size_t pos) {
-             std::vector<float> lg;
-             {
-               py::gil_scoped_release rel;
-               lg = r.forward(token, pos);
-             }
-             return py::array_t<float>(lg.size(), lg.data());
-           })
       .def("forward_async", &HipLlamaRunner::forward_async)
-      .def("decode_greedy",
-           [](HipLlamaRunner& r, size_t token, size_t steps) {
-             py::gil_scoped_release rel;
-             return r.decode_greedy(token, steps);
-           })
       .def("debug_kv", [](HipLlamaRunner& r, size_t layer, bool v, bool f16) {
         std::vector<uint8_t> b = r.debug_kv(layer, v, f16);
         return py::array_t<uint8_t>(b.size(), b.data());
       });
+
+  py::class_<HipHybridRunner, ModelRunner>(m, "HipHybridRunner")
+      .def("open", &HipHybridRunner::open)
+      .def("close", &HipHybridRunner::close)
+      .def("length", &HipHybridRunner::length)
+      .def("slab_bytes", &HipHybridRunner::slab_bytes)
+      // entries: (sequence, tokens, wanted places); returns the wanted logits [wanted, vocab]
+      .def("step",
+           [](HipHybridRunner& r, const std::vector<std::tuple<size_t, std::vector<uint32_t>, std::vector<uint32_t>>>& entries) {
+             std::vector<StepEntry> e;
+             for (const auto& t : entries) e.push_back(StepEntry{std::get<0>(t), std::get<1>(t), std::get<2>(t)});
+             std::vector<float> lg;
+             {
+               py::gil_scoped_release rel;
+               lg = r.step(e);
+             }
+             const py::ssize_t v = (py::ssize_t)r.vocab_size();
+             return py::array_t<float>({(py::ssize_t)lg.size() / v, v}, lg.data());
+           })
+      .def("decode_batch", &HipHybridRunner::decode_batch, py::call_guard<py::gil_scoped_release>())
+      .def("generate", &HipHybridRunner::generate, py::arg("prompts"), py::arg("steps"), py::call_guard<py::gil_scoped_release>());
+
+  // ---- model registry (model_registry.hpp)
+  m.def("known_architectures", &known_architectures);
+  m.def("model_architecture", &model_architecture, py::arg("path"));
+  m.def("load_model",
+        [](const std::string& path, std::shared_ptr<HipTensorDevice> dev, size_t seq_len, bool f32, bool use_graph, size_t pass_rows) {
+          LoadOptions o;
+          o.seq_len = seq_len;
+          o.f32 = f32;
+          o.use_graph = use_graph;
+          o.pass_rows = pass_rows;
+          py::gil_scoped_release rel;
+          return load_model(path, dev, o);
+        },
+        py::arg("path"), py::arg("device"), py::arg("seq_len") = 0, py::arg("f32") = false, py::arg("use_graph") = true, py::arg("pass_rows") = 0);
 
   py::class_<Runner>(m, "Llama2Runner")
       .def(py::init([](const LlamaConfig& conf, std::shared_ptr<Weights> w, std::shared_ptr<HipTensorDevice> dev,

@@ -1,0 +1,947 @@
+// hybrid.hip -- the hybrid decoder (crabml_hip_hybrid_*): host side.  Context, weight packing, the sequences' state slabs, the decode
+// step as a captured graph, the prompt pass, the C entry points.  Kernels: hybrid_step.hpp, hybrid_rows.hpp, gemv_bf16.hpp, gemm_bf16.hip.
+#include <cmath>
+#include <memory>
+
+#include "dequant.hpp"
+#include "hybrid_rows.hpp"
+#include "hybrid_step.hpp"
+#include "lazy.hpp"
+
+using namespace crabml_hip;
+
+namespace {
+
+struct Layer {
+  AttnGeom at;
+  LinGeom li;
+  int n_in = 0, ldc = 0, lin_off = 0, ff = 0, ldu = 0, splits = 0, head_blocks = 0;
+  ActRanges act;
+  unsigned short *w_in = nullptr, *w_o = nullptr, *w_up = nullptr, *w_down = nullptr;
+  float *norm1 = nullptr, *norm2 = nullptr, *xielu = nullptr;
+};
+struct Run {  // one execution of a layer: in a loop, every time is a run of its own
+  int layer = 0;
+  RunState rs;
+  bool add_emb = false;            // what is added to x in front of it
+  const float* add_vec = nullptr;
+};
+struct Seq {
+  bool open = false;
+  char* slab = nullptr;
+  size_t cap = 0;
+  size_t len = 0;
+};
+// profiling stages (crabml_hip_prof_*): decode 11 .. 16, prompt pass 21 .. 27
+enum { ST_IN = 1, ST_MIX = 2, ST_OUT = 3, ST_UP = 4, ST_DOWN = 5, ST_HEAD = 6, ST_LIN = 7, ST_ROWS = 8, ST_STEP = 10, ST_PASS = 20 };
+
+constexpr size_t LOGIT_ROWS = 256;  // rows of logits a pass keeps on the device at a time
+constexpr int META_SLOTS = 4;
+
+}  // namespace
+
+struct crabml_hip_hybrid {
+  crabml_hip_device* dev = nullptr;
+  crabml_hip_hybrid_config_t cfg{};
+  bool f32 = false;
+  int planes = 1;
+  int width = 0, vocab = 0, ldx = 0, n_sq = 0;
+  std::vector<Layer> layers;
+  std::vector<Run> runs;
+  std::vector<Seq> seqs;
+  size_t slab_bytes = 0;
+  unsigned short *embed = nullptr, *head = nullptr;
+  float *loop_step = nullptr, *final_norm = nullptr;
+  double* freq = nullptr;
+  bool keep_emb = false;
+  // decode step
+  StepSeq* st_seq = nullptr;
+  int* st_count = nullptr;
+  float *st_x = nullptr, *st_emb = nullptr, *st_proj = nullptr, *st_cat = nullptr, *st_u = nullptr, *st_ss = nullptr, *st_part = nullptr, *st_logits = nullptr;
+  unsigned* st_tick = nullptr;
+  unsigned* st_out = nullptr;
+  size_t st_out_cap = 0;
+  float* am_val = nullptr;
+  int* am_idx = nullptr;
+  int ld_proj = 0, ld_cat = 0, ld_u = 0;
+  StepSeq* h_seq = nullptr;  // pinned ring of META_SLOTS * HYB_STEP_ROWS
+  int h_seq_next = 0;
+  std::map<int, std::pair<hipGraph_t, hipGraphExec_t>> graphs;  // key: rows * 2 + sampler
+  // prompt pass (allocated on first use)
+  size_t rows_cap = 0, meta_bytes = 0;
+  char *meta = nullptr, *h_meta = nullptr;
+  int h_meta_next = 0;
+  float *pf_x = nullptr, *pf_emb = nullptr, *pf_lin = nullptr, *pf_sq = nullptr, *pf_gsq = nullptr, *pf_logits = nullptr;
+  unsigned short *pf_xp = nullptr, *pf_cat = nullptr, *pf_u = nullptr, *pf_gp = nullptr;
+  void* pf_proj = nullptr;
+  std::vector<std::pair<void*, size_t>> allocs;
+};
+
+namespace {
+
+typedef crabml_hip_hybrid Ctx;
+
+int dalloc(Ctx* c, size_t bytes, void** out, bool clear = true) {
+  size_t cap = 0;
+  if (bytes < 16) bytes = 16;
+  CH_TRY(pool_alloc(c->dev, bytes, out, &cap));
+  c->allocs.push_back({*out, cap});
+  if (clear) CH_HIP(c->dev, hipMemsetAsync(*out, 0, bytes, c->dev->stream));
+  return 0;
+}
+template <typename T>
+int dalloc_n(Ctx* c, size_t n, T** out) {
+  return dalloc(c, n * sizeof(T), (void**)out);
+}
+int up(size_t v, size_t a) { return (int)align_up(v, a); }
+
+// ---- weight packing -----------------------------------------------------------------------------------------------------------------
+// source row r -> row0 + r with every group of rg rows widened to rgp; columns the same (head widths padded; the gaps stay zero)
+__global__ __launch_bounds__(256) void k_pack_matrix(const unsigned short* __restrict__ src, int m, int k, unsigned short* __restrict__ dst, size_t ldd,
+                                                     int row0, int rg, int rgp, int col0, int cg, int cgp) {
+  const int r = blockIdx.y;
+  unsigned short* d = dst + (size_t)(row0 + r / rg * rgp + r % rg) * ldd + col0;
+  for (int c = blockIdx.x * 256 + threadIdx.x; c < k; c += gridDim.x * 256) d[c / cg * cgp + c % cg] = src[(size_t)r * k + c];
+}
+__global__ __launch_bounds__(256) void k_pack_vector(const char* __restrict__ src, int dtype, size_t off_scale, int n, float* __restrict__ dst, int g, int gp) {
+  const int i = blockIdx.x * 256 + threadIdx.x;
+  if (i < n) dst[i / g * gp + i % g] = dequant_elem(src, dtype, off_scale, i);
+}
+__global__ void k_xielu_consts(const float* __restrict__ raw, float* __restrict__ out) {
+  auto softplus = [](float z) { return log1pf(expf(-fabsf(z))) + fmaxf(z, 0.f); };
+  out[0] = softplus(raw[0]);
+  out[1] = 0.5f + softplus(raw[1]);
+}
+
+int pack_matrix(Ctx* c, const crabml_hip_buf* b, const char* what, size_t m, size_t k, unsigned short* dst, size_t ldd, size_t row0, size_t rg, size_t rgp,
+                size_t col0 = 0, size_t cg = 0, size_t cgp = 0) {
+  if (!b || b->dtype != CRABML_HIP_BF16 || b->n_elems != m * k || b->dev != c->dev)
+    CH_BAIL(c->dev, CRABML_HIP_BAD_INPUT, "hybrid: %s must be a bfloat16 matrix of %zu x %zu", what, m, k);
+  k_pack_matrix<<<dim3((unsigned)std::min<size_t>((k + 255) / 256, 64), (unsigned)m), 256, 0, c->dev->stream>>>(
+      (const unsigned short*)b->ptr, (int)m, (int)k, dst, ldd, (int)row0, (int)rg, (int)rgp, (int)col0, (int)(cg ? cg : k), (int)(cg ? cgp : k));
+  CH_HIP(c->dev, hipGetLastError());
+  return 0;
+}
+int pack_vector(Ctx* c, const crabml_hip_buf* b, const char* what, size_t n, float** out, size_t g = 0, size_t gp = 0) {
+  if (!b || b->n_elems != n || b->dev != c->dev) CH_BAIL(c->dev, CRABML_HIP_BAD_INPUT, "hybrid: %s must hold %zu numbers", what, n);
+  if (g == 0) g = gp = n;
+  CH_TRY(dalloc_n(c, n / g * gp, out));
+  k_pack_vector<<<(unsigned)((n + 255) / 256), 256, 0, c->dev->stream>>>((const char*)b->ptr, (int)b->dtype, b->wl.off_scale, (int)n, *out, (int)g, (int)gp);
+  CH_HIP(c->dev, hipGetLastError());
+  return 0;
+}
+// rows of a weight matrix: padded to 256 so that any tile of the GEMM reads inside it
+int alloc_matrix(Ctx* c, size_t rows, size_t ld, unsigned short** out) { return dalloc_n(c, align_up(rows, 256) * ld, out); }
+
+int build_layer(Ctx* c, const crabml_hip_hybrid_layer_t& s, Layer& L) {
+  crabml_hip_device* dev = c->dev;
+  const size_t W = (size_t)c->width, H = s.attn_heads, G = s.attn_kv_heads, Hl = s.lin_heads;
+  if (!H && !Hl) CH_BAIL(dev, CRABML_HIP_BAD_INPUT, "hybrid: a layer needs a mixer");
+  if (H && (!G || H % G || !s.attn_dim || !s.attn_vdim || s.attn_dim > 256 || s.attn_vdim > 256))
+    CH_BAIL(dev, H && G && H % G == 0 ? CRABML_HIP_NOT_IMPLEMENTED : CRABML_HIP_BAD_INPUT, "hybrid: attention of %zu / %zu heads of %zu / %zu (at most 256 wide)", H, G,
+            s.attn_dim, s.attn_vdim);
+  if (Hl && (!s.lin_dim || !s.lin_vdim || s.lin_dim > 256 || !s.lin_decay))
+    CH_BAIL(dev, CRABML_HIP_NOT_IMPLEMENTED, "hybrid: linear attention of %zu heads of %zu / %zu (keys at most 256 wide, decay given)", Hl, s.lin_dim, s.lin_vdim);
+  const size_t D = align_up(s.attn_dim, 8), V = align_up(s.attn_vdim, 8), Dl = align_up(s.lin_dim, 8), Vl = align_up(s.lin_vdim, 8);
+  size_t col = 0;
+  auto take = [&](size_t n) {
+    const size_t at = col;
+    col += n;
+    return (int)at;
+  };
+  AttnGeom& a = L.at;
+  LinGeom& l = L.li;
+  // columns of the projected row: raw q k v | sigmoid gate | silu q k v | sigmoid gate
+  if (H) {
+    a.H = (int)H;
+    a.G = (int)G;
+    a.D = (int)D;
+    a.V = (int)V;
+    const size_t chunk = s.attn_chunk && s.attn_chunk < ((size_t)1 << 30) ? s.attn_chunk : (size_t)1 << 30;
+    a.chunk = (int)chunk;
+    a.rows = (int)std::min(chunk, c->cfg.seq_len);
+    a.scale = s.attn_score_scale;
+    a.out_scale = s.attn_out_scale;
+    a.cq = take(H * D);
+    a.ck = take(G * D);
+    a.cv = take(G * V);
+  }
+  L.act.end[0] = (int)col;
+  if (H) a.cg = take(H * V);
+  L.act.end[1] = (int)col;
+  L.act.kind[1] = ACT_SIGMOID;
+  if (Hl) {
+    l.H = (int)Hl;
+    l.D = (int)Dl;
+    l.V = (int)Vl;
+    l.v_true = (int)s.lin_vdim;
+    l.out_scale = s.lin_out_scale;
+    l.slices = (int)((Vl + LIN_SLICE - 1) / LIN_SLICE);
+    l.cq = take(Hl * Dl);
+    l.ck = take(Hl * Dl);
+    l.cv = take(Hl * Vl);
+  }
+  L.act.end[2] = (int)col;
+  L.act.kind[2] = ACT_SILU;
+  if (Hl) l.cg = take(Hl * Vl);
+  L.act.end[3] = (int)col;
+  L.act.kind[3] = ACT_SIGMOID;
+  L.n_in = (int)col;
+  L.lin_off = up(H * V, 64);
+  L.ldc = L.lin_off + up(Hl * Vl, 64);
+  L.ff = (int)s.ff;
+  L.ldu = up(s.ff, 64);
+  L.splits = H ? (a.rows + MIX_KEYS - 1) / MIX_KEYS : 0;
+  L.head_blocks = H ? (int)((H / G + MIX_HEADS - 1) / MIX_HEADS) : 0;
+  const size_t ldw = (size_t)c->ldx;
+  CH_TRY(alloc_matrix(c, col, ldw, &L.w_in));
+  CH_TRY(alloc_matrix(c, W, (size_t)L.ldc, &L.w_o));
+  if (H) {
+    CH_TRY(pack_matrix(c, s.attn_q, "attn_q", H * s.attn_dim, W, L.w_in, ldw, a.cq, s.attn_dim, D));
+    CH_TRY(pack_matrix(c, s.attn_k, "attn_k", G * s.attn_dim, W, L.w_in, ldw, a.ck, s.attn_dim, D));
+    CH_TRY(pack_matrix(c, s.attn_v, "attn_v", G * s.attn_vdim, W, L.w_in, ldw, a.cv, s.attn_vdim, V));
+    CH_TRY(pack_matrix(c, s.attn_gate, "attn_gate", H * s.attn_vdim, W, L.w_in, ldw, a.cg, s.attn_vdim, V));
+    CH_TRY(pack_matrix(c, s.attn_o, "attn_o", W, H * s.attn_vdim, L.w_o, (size_t)L.ldc, 0, W, W, 0, s.attn_vdim, V));
+    if (!s.attn_bias_amp != !s.attn_bias_rate) CH_BAIL(dev, CRABML_HIP_BAD_INPUT, "hybrid: attn_bias_amp and attn_bias_rate come together");
+    float* p = nullptr;
+    if (s.attn_bias_amp) {
+      CH_TRY(pack_vector(c, s.attn_bias_amp, "attn_bias_amp", H, &p));
+      a.amp = p;
+      CH_TRY(pack_vector(c, s.attn_bias_rate, "attn_bias_rate", H, &p));
+      a.rate = p;
+    }
+    if (s.attn_sink) {
+      CH_TRY(pack_vector(c, s.attn_sink, "attn_sink", H, &p));
+      a.sink = p;
+    }
+  }
+  if (Hl) {
+    CH_TRY(pack_matrix(c, s.lin_q, "lin_q", Hl * s.lin_dim, W, L.w_in, ldw, l.cq, s.lin_dim, Dl));
+    CH_TRY(pack_matrix(c, s.lin_k, "lin_k", Hl * s.lin_dim, W, L.w_in, ldw, l.ck, s.lin_dim, Dl));
+    CH_TRY(pack_matrix(c, s.lin_v, "lin_v", Hl * s.lin_vdim, W, L.w_in, ldw, l.cv, s.lin_vdim, Vl));
+    CH_TRY(pack_matrix(c, s.lin_gate, "lin_gate", Hl * s.lin_vdim, W, L.w_in, ldw, l.cg, s.lin_vdim, Vl));
+    CH_TRY(pack_matrix(c, s.lin_o, "lin_o", W, Hl * s.lin_vdim, L.w_o, (size_t)L.ldc, 0, W, W, L.lin_off, s.lin_vdim, Vl));
+    float* p = nullptr;
+    CH_TRY(pack_vector(c, s.lin_norm, "lin_norm", Hl * s.lin_vdim, &p, s.lin_vdim, Vl));
+    l.norm = p;
+    std::vector<float> pw(Hl * LIN_POW);
+    for (size_t h = 0; h < Hl; h++)
+      for (int n = 0; n < LIN_POW; n++) pw[h * LIN_POW + n] = (float)pow(s.lin_decay[h], (double)n);
+    CH_TRY(dalloc_n(c, pw.size(), &p));
+    CH_HIP(dev, hipMemcpyAsync(p, pw.data(), pw.size() * 4, hipMemcpyHostToDevice, dev->stream));
+    CH_HIP(dev, hipStreamSynchronize(dev->stream));  // pw goes out of scope
+    l.decay = p;
+  }
+  CH_TRY(pack_vector(c, s.norm1, "norm1", 1, &L.norm1));
+  if (s.ff) {
+    CH_TRY(pack_vector(c, s.norm2, "norm2", 1, &L.norm2));
+    CH_TRY(alloc_matrix(c, s.ff, ldw, &L.w_up));
+    CH_TRY(alloc_matrix(c, W, (size_t)L.ldu, &L.w_down));
+    CH_TRY(pack_matrix(c, s.ff_up, "ff_up", s.ff, W, L.w_up, ldw, 0, s.ff, s.ff));
+    CH_TRY(pack_matrix(c, s.ff_down, "ff_down", W, s.ff, L.w_down, (size_t)L.ldu, 0, W, W));
+    float* raw = nullptr;
+    CH_TRY(pack_vector(c, s.ff_act, "ff_act", 2, &raw));
+    CH_TRY(dalloc_n(c, 2, &L.xielu));
+    k_xielu_consts<<<1, 1, 0, dev->stream>>>(raw, L.xielu);
+    CH_HIP(dev, hipGetLastError());
+  }
+  return 0;
+}
+
+// ---- launches with the measurement hook's event pair ---------------------------------------------------------------------------------
+struct Prof {
+  crabml_hip_device* dev;
+  crabml_hip_device::ProfRec r{};
+  bool on;
+  Prof(crabml_hip_device* d, bool enabled, int stage, double bytes) : dev(d), on(enabled && d->prof_on) {
+    if (on) on = prof_begin(d, &r, CRABML_HIP_BF16, (uint32_t)stage, bytes) == 0;
+  }
+  ~Prof() {
+    if (on) prof_end(dev, &r);
+  }
+  crabml_hip_device::ProfRec* rec() { return on ? &r : nullptr; }
+};
+
+MixStep mix_step(const Ctx* c, const Run& run, int B) {
+  const Layer& L = c->layers[run.layer];
+  MixStep m;
+  m.at = L.at;
+  m.li = L.li;
+  m.rs = run.rs;
+  m.seq = c->st_seq;
+  m.proj = c->st_proj;
+  m.cat = c->st_cat;
+  m.ss = c->st_ss;
+  m.part = c->st_part;
+  m.tick = c->st_tick;
+  m.B = B;
+  m.ldp = L.n_in;
+  m.ldc = L.ldc;
+  m.lin_off = L.lin_off;
+  m.splits = L.splits;
+  m.head_blocks = L.head_blocks;
+  return m;
+}
+
+// what is added to x behind the last linear of run r: what belongs in front of run r + 1
+void next_adds(const Ctx* c, size_t r, const float* emb, const float** rows, const float** vec) {
+  *rows = *vec = nullptr;
+  if (r + 1 < c->runs.size()) {
+    *rows = c->runs[r + 1].add_emb ? emb : nullptr;
+    *vec = c->runs[r + 1].add_vec;
+  }
+}
+
+// the classifier on f32 rows
+void head_rows(Ctx* c, const float* x, int B, bool prof) {
+  GemvBf16 g;
+  g.w = c->head;
+  g.x = x;
+  g.out = c->st_logits;
+  g.N = g.ldo = c->vocab;
+  g.K = g.ldw = g.ldx = c->ldx;
+  g.nb = B;
+  g.mean_n = c->width;
+  g.eps = c->cfg.norm_eps;
+  g.gain = c->final_norm;
+  g.cap = c->cfg.logit_softcap;
+  Prof p(c->dev, prof, ST_STEP + ST_HEAD, (double)c->vocab * c->ldx * 2);
+  launch_gemv_bf16<GEMV_IN_RMS, GEMV_OUT_SOFTCAP>(c->dev->stream, p.rec(), g);
+}
+
+int enqueue_step(Ctx* c, int B, bool sample, bool prof) {
+  crabml_hip_device* dev = c->dev;
+  hipStream_t st = dev->stream;
+  const float eps = c->cfg.norm_eps;
+  k_embed_step<<<dim3((c->width + 255) / 256, B), 256, 0, st>>>(c->embed, c->st_seq, c->width, c->ldx, c->cfg.embed_scale, c->freq, c->st_x,
+                                                               c->keep_emb ? c->st_emb : nullptr, c->runs[0].add_vec);
+  for (size_t r = 0; r < c->runs.size(); r++) {
+    const Run& run = c->runs[r];
+    const Layer& L = c->layers[run.layer];
+    const float *add_rows, *add_vec;
+    next_adds(c, r, c->st_emb, &add_rows, &add_vec);
+    {
+      GemvBf16 g;
+      g.w = L.w_in;
+      g.x = c->st_x;
+      g.out = c->st_proj;
+      g.N = g.ldo = L.n_in;
+      g.K = g.ldw = g.ldx = c->ldx;
+      g.nb = B;
+      g.mean_n = c->width;
+      g.eps = eps;
+      g.gain = L.norm1;
+      g.act = L.act;
+      Prof p(dev, prof, ST_STEP + ST_IN, (double)L.n_in * c->ldx * 2);
+      launch_gemv_bf16<GEMV_IN_RMS, GEMV_OUT_ACT>(st, p.rec(), g);
+    }
+    {
+      const MixStep m = mix_step(c, run, B);
+      const unsigned grid = (unsigned)(B * (L.at.H ? L.at.G * L.head_blocks * L.splits : 0) + B * (L.li.H ? L.li.H * L.li.slices : 0));
+      Prof p(dev, prof, ST_STEP + ST_MIX, 0.0);
+      if (c->f32)
+        launch_k(st, p.rec(), k_mix_step<float>, dim3(grid), dim3(256), mix_step_lds(m), m);
+      else
+        launch_k(st, p.rec(), k_mix_step<unsigned short>, dim3(grid), dim3(256), mix_step_lds(m), m);
+    }
+    {
+      GemvBf16 g;
+      g.w = L.w_o;
+      g.x = c->st_cat;
+      g.out = c->st_x;
+      g.N = c->width;
+      g.ldo = g.ld_add = c->ldx;
+      g.K = g.ldw = g.ldx = L.ldc;
+      g.nb = B;
+      g.mean_n = L.li.H ? L.li.H * L.li.v_true : 1;
+      g.eps = eps;
+      g.k_split = L.lin_off;
+      g.n_ss = L.li.H * L.li.slices;
+      g.ss = c->st_ss;
+      if (!L.ff) {
+        g.add_rows = add_rows;
+        g.add_vec = add_vec;
+      }
+      Prof p(dev, prof, ST_STEP + ST_OUT, (double)c->width * L.ldc * 2);
+      launch_gemv_bf16<GEMV_IN_SPLIT, GEMV_OUT_RESIDUAL>(st, p.rec(), g);
+    }
+    if (!L.ff) continue;
+    {
+      GemvBf16 g;
+      g.w = L.w_up;
+      g.x = c->st_x;
+      g.out = c->st_u;
+      g.N = L.ff;
+      g.ldo = L.ldu;
+      g.K = g.ldw = g.ldx = c->ldx;
+      g.nb = B;
+      g.mean_n = c->width;
+      g.eps = eps;
+      g.gain = L.norm2;
+      g.xielu = L.xielu;
+      Prof p(dev, prof, ST_STEP + ST_UP, (double)L.ff * c->ldx * 2);
+      launch_gemv_bf16<GEMV_IN_RMS, GEMV_OUT_XIELU>(st, p.rec(), g);
+    }
+    {
+      GemvBf16 g;
+      g.w = L.w_down;
+      g.x = c->st_u;
+      g.out = c->st_x;
+      g.N = c->width;
+      g.ldo = g.ld_add = c->ldx;
+      g.K = g.ldw = g.ldx = L.ldu;
+      g.nb = B;
+      g.add_rows = add_rows;
+      g.add_vec = add_vec;
+      Prof p(dev, prof, ST_STEP + ST_DOWN, (double)c->width * L.ldu * 2);
+      launch_gemv_bf16<GEMV_IN_PLAIN, GEMV_OUT_RESIDUAL>(st, p.rec(), g);
+    }
+  }
+  head_rows(c, c->st_x, B, prof);
+  if (sample) {
+    k_argmax_partial<<<dim3(ARGMAX_BLOCKS, B), 256, 0, st>>>(c->st_logits, c->vocab, c->am_val, c->am_idx, 0, c->vocab);
+    k_argmax_rows_step<<<B, 64, 0, st>>>(c->am_val, c->am_idx, ARGMAX_BLOCKS, c->st_seq, c->st_count, c->st_out, (int)c->st_out_cap);
+    k_step_advance<<<1, 1, 0, st>>>(c->st_count);
+  }
+  CH_HIP(dev, hipGetLastError());
+  return 0;
+}
+
+// one decode step of B rows from its graph (captured when that batch size first comes up), or eagerly
+int run_step(Ctx* c, int B, bool sample) {
+  crabml_hip_device* dev = c->dev;
+  if ((c->cfg.flags & CRABML_HIP_HYBRID_NO_GRAPH) || dev->prof_on) return enqueue_step(c, B, sample, true);
+  auto& slot = c->graphs[B * 2 + (sample ? 1 : 0)];
+  if (!slot.second) {
+    CH_HIP(dev, hipStreamBeginCapture(dev->stream, hipStreamCaptureModeThreadLocal));
+    const int rc = enqueue_step(c, B, sample, false);
+    hipGraph_t graph = nullptr;
+    const hipError_t e = hipStreamEndCapture(dev->stream, &graph);
+    hipGraphExec_t exec = nullptr;
+    if (rc != 0 || e != hipSuccess || !graph || hipGraphInstantiate(&exec, graph, nullptr, nullptr, 0) != hipSuccess) {
+      if (graph) (void)hipGraphDestroy(graph);
+      (void)hipGetLastError();
+      CH_BAIL(dev, CRABML_HIP_UNEXPECTED, "hybrid: hipGraph capture / instantiate of the decode step failed");
+    }
+    slot = {graph, exec};
+  }
+  CH_HIP(dev, hipGraphLaunch(slot.second, dev->stream));
+  return 0;
+}
+
+int step_begin(Ctx* c, size_t n, const size_t* seqs, const uint32_t* tokens) {
+  crabml_hip_device* dev = c->dev;
+  if (c->h_seq_next == META_SLOTS) {  // every slot may still be waiting for its copy
+    CH_HIP(dev, hipStreamSynchronize(dev->stream));
+    c->h_seq_next = 0;
+  }
+  StepSeq* h = c->h_seq + (size_t)HYB_STEP_ROWS * c->h_seq_next++;
+  for (size_t i = 0; i < n; i++) {
+    h[i].token = (int)tokens[i];
+    h[i].pos = (int)c->seqs[seqs[i]].len;
+    h[i].slab = c->seqs[seqs[i]].slab;
+  }
+  CH_HIP(dev, hipMemcpyAsync(c->st_seq, h, n * sizeof(StepSeq), hipMemcpyHostToDevice, dev->stream));
+  return 0;
+}
+
+// ---- prompt pass -------------------------------------------------------------------------------------------------------------------
+int pass_alloc(Ctx* c) {
+  if (c->rows_cap) return 0;
+  crabml_hip_device* dev = c->dev;
+  const size_t R = align_up(c->cfg.pass_rows ? c->cfg.pass_rows : 2048, 128), P = (size_t)c->planes;
+  size_t lin = 0;
+  for (const Layer& L : c->layers) lin = std::max(lin, (size_t)L.li.H * L.li.V);
+  CH_TRY(dalloc_n(c, R * c->ldx, &c->pf_x));
+  if (c->keep_emb) CH_TRY(dalloc_n(c, R * c->ldx, &c->pf_emb));
+  CH_TRY(dalloc_n(c, P * R * c->ldx, &c->pf_xp));
+  CH_TRY(dalloc(c, R * c->ld_proj * (c->f32 ? 4 : 2), &c->pf_proj));
+  CH_TRY(dalloc_n(c, P * R * c->ld_cat, &c->pf_cat));
+  CH_TRY(dalloc_n(c, R * lin, &c->pf_lin));
+  CH_TRY(dalloc_n(c, P * R * c->ld_u, &c->pf_u));
+  CH_TRY(dalloc_n(c, R * c->n_sq, &c->pf_sq));
+  CH_TRY(dalloc_n(c, P * LOGIT_ROWS * c->ldx, &c->pf_gp));
+  CH_TRY(dalloc_n(c, LOGIT_ROWS * c->n_sq, &c->pf_gsq));
+  CH_TRY(dalloc_n(c, LOGIT_ROWS * c->vocab, &c->pf_logits));
+  // seqs | tiles (a tile is at least one row) | rows | tokens | wanted rows
+  c->meta_bytes = R * (sizeof(PassSeq) + sizeof(PassTile) + sizeof(PassRow) + 2 * sizeof(int));
+  CH_TRY(dalloc(c, c->meta_bytes, (void**)&c->meta));
+  CH_HIP(dev, hipHostMalloc((void**)&c->h_meta, c->meta_bytes * META_SLOTS, hipHostMallocDefault));
+  c->rows_cap = R;
+  return 0;
+}
+
+struct Part {  // rows of one sequence in one pass
+  size_t seq, n;
+  const uint32_t* tokens;
+  std::vector<int> want;  // places among these rows
+};
+
+template <typename T, int CLS>
+void launch_attn_cls(Ctx* c, crabml_hip_device::ProfRec* rec, const MixRows<T>& m) {
+  launch_k(c->dev->stream, rec, k_attn_rows<T, CLS, sizeof(T) == 2 ? 1 : 3>, dim3(m.n_tiles, m.at.H), dim3(256), 0, m);
+}
+template <typename T, int CLS>
+int launch_linear_cls(Ctx* c, crabml_hip_device::ProfRec* rec, const MixRows<T>& m, size_t n_seq) {
+  const size_t lds = LinTile<T, CLS>::LDS;
+  CH_HIP(c->dev, raise_dyn_lds(c->dev, (const void*)k_linear_rows<T, CLS>, (int)lds));
+  launch_k(c->dev->stream, rec, k_linear_rows<T, CLS>, dim3(m.li.H * m.li.slices, (unsigned)n_seq), dim3(256), lds, m);
+  return 0;
+}
+
+template <typename T>
+int mix_rows(Ctx* c, const Run& run, const PassSeq* seqs, size_t n_seq, const PassTile* tiles, size_t n_tiles, const PassRow* rows, size_t n_rows) {
+  constexpr int P = sizeof(T) == 2 ? 1 : 3;
+  const Layer& L = c->layers[run.layer];
+  MixRows<T> m;
+  m.at = L.at;
+  m.li = L.li;
+  m.rs = run.rs;
+  m.seqs = seqs;
+  m.tiles = tiles;
+  m.rows = rows;
+  m.proj = (const T*)c->pf_proj;
+  m.cat = c->pf_cat;
+  m.cat_plane = c->rows_cap * (size_t)c->ld_cat;
+  m.lin = c->pf_lin;
+  m.n_tiles = (int)n_tiles;
+  m.ldp = L.n_in;
+  m.ldc = L.ldc;
+  m.lin_off = L.lin_off;
+  if (L.at.H) {
+    Prof p(c->dev, true, ST_PASS + ST_MIX, 0.0);
+    const int w = std::max(L.at.D, L.at.V);
+    if (w <= 64)
+      launch_attn_cls<T, 64>(c, p.rec(), m);
+    else if (w <= 128)
+      launch_attn_cls<T, 128>(c, p.rec(), m);
+    else
+      launch_attn_cls<T, 256>(c, p.rec(), m);
+  }
+  if (L.li.H) {
+    Prof p(c->dev, true, ST_PASS + ST_LIN, 0.0);
+    if (L.li.D <= 64)
+      CH_TRY((launch_linear_cls<T, 64>(c, p.rec(), m, n_seq)));
+    else if (L.li.D <= 128)
+      CH_TRY((launch_linear_cls<T, 128>(c, p.rec(), m, n_seq)));
+    else
+      CH_TRY((launch_linear_cls<T, 256>(c, p.rec(), m, n_seq)));
+  }
+  Prof p(c->dev, true, ST_PASS + ST_ROWS, 0.0);
+  launch_k(c->dev->stream, p.rec(), k_mix_rows<T, P>, dim3((unsigned)n_rows), dim3(256), 0, m, c->cfg.norm_eps);
+  return 0;
+}
+
+// one pass over the rows of `parts`; logits of the wanted rows go to *logits, which advances
+int run_pass(Ctx* c, const std::vector<Part>& parts, float** logits) {
+  crabml_hip_device* dev = c->dev;
+  hipStream_t st = dev->stream;
+  CH_TRY(pass_alloc(c));
+  if (c->h_meta_next == META_SLOTS) {
+    CH_HIP(dev, hipStreamSynchronize(st));
+    c->h_meta_next = 0;
+  }
+  const size_t R = c->rows_cap;
+  char* hm = c->h_meta + c->meta_bytes * c->h_meta_next++;
+  const size_t o_tile = R * sizeof(PassSeq), o_row = o_tile + R * sizeof(PassTile), o_tok = o_row + R * sizeof(PassRow), o_want = o_tok + R * sizeof(int);
+  PassSeq* hs = (PassSeq*)hm;
+  PassTile* ht = (PassTile*)(hm + o_tile);
+  PassRow* hr = (PassRow*)(hm + o_row);
+  int *hk = (int*)(hm + o_tok), *hw = (int*)(hm + o_want);
+  size_t n_tiles = 0, M = 0, nw = 0;
+  for (size_t i = 0; i < parts.size(); i++) {
+    const Part& p = parts[i];
+    const Seq& s = c->seqs[p.seq];
+    hs[i] = PassSeq{(int)M, (int)p.n, (int)s.len, 0, s.slab};
+    for (size_t r = 0; r < p.n; r += 64) ht[n_tiles++] = PassTile{(int)i, (int)(M + r), (int)(s.len + r), (int)std::min<size_t>(64, p.n - r)};
+    for (int w : p.want) hw[nw++] = (int)M + w;
+    for (size_t r = 0; r < p.n; r++) {
+      hr[M + r] = PassRow{(int)i, (int)(s.len + r)};
+      hk[M + r] = (int)p.tokens[r];
+    }
+    M += p.n;
+  }
+  CH_HIP(dev, hipMemcpyAsync(c->meta, hm, c->meta_bytes, hipMemcpyHostToDevice, st));
+  const PassSeq* ds = (const PassSeq*)c->meta;
+  const PassTile* dt = (const PassTile*)(c->meta + o_tile);
+  const PassRow* dr = (const PassRow*)(c->meta + o_row);
+  const int *dk = (const int*)(c->meta + o_tok), *dw = (const int*)(c->meta + o_want);
+  const size_t xp = R * (size_t)c->ldx;
+  const float eps = c->cfg.norm_eps;
+  float* emb = c->keep_emb ? c->pf_emb : nullptr;
+  if (c->f32)
+    k_embed_rows<3><<<(unsigned)M, 256, 0, st>>>(c->embed, dk, dr, c->width, c->ldx, c->cfg.embed_scale, c->freq, c->pf_x, emb, c->runs[0].add_vec, c->pf_xp, xp,
+                                                c->pf_sq, c->n_sq);
+  else
+    k_embed_rows<1><<<(unsigned)M, 256, 0, st>>>(c->embed, dk, dr, c->width, c->ldx, c->cfg.embed_scale, c->freq, c->pf_x, emb, c->runs[0].add_vec, c->pf_xp, xp,
+                                                c->pf_sq, c->n_sq);
+  auto normed = [&](const unsigned short* w, int n, const float* gain) {
+    GemmBf16 g;
+    g.a = c->pf_xp;
+    g.a_plane = xp;
+    g.w = w;
+    g.M = (int)M;
+    g.N = n;
+    g.K = c->ldx;
+    g.sq_in = c->pf_sq;
+    g.n_sq = c->n_sq;
+    g.mean_n = c->width;
+    g.eps = eps;
+    g.gain = gain;
+    return g;
+  };
+  auto residual = [&](const unsigned short* a, size_t a_plane, const unsigned short* w, int k) {
+    GemmBf16 g;
+    g.a = a;
+    g.a_plane = a_plane;
+    g.w = w;
+    g.M = (int)M;
+    g.N = c->width;
+    g.K = k;
+    g.x = c->pf_x;
+    g.ldx = c->ldx;
+    g.planes = c->pf_xp;
+    g.p_plane = xp;
+    g.ldp = c->ldx;
+    g.sq_out = c->pf_sq;
+    g.n_sq_out = c->n_sq;
+    return g;
+  };
+  for (size_t r = 0; r < c->runs.size(); r++) {
+    const Run& run = c->runs[r];
+    const Layer& L = c->layers[run.layer];
+    const float *add_rows, *add_vec;
+    next_adds(c, r, c->pf_emb, &add_rows, &add_vec);
+    {
+      GemmBf16 g = normed(L.w_in, L.n_in, L.norm1);
+      g.out = c->pf_proj;
+      g.ldo = L.n_in;
+      g.act = L.act;
+      Prof p(dev, true, ST_PASS + ST_IN, 0.0);
+      launch_gemm_bf16(dev, p.rec(), c->planes, c->f32 ? GEMM_OUT_ACT_F32 : GEMM_OUT_ACT_BF16, g);
+    }
+    if (c->f32)
+      CH_TRY(mix_rows<float>(c, run, ds, parts.size(), dt, n_tiles, dr, M));
+    else
+      CH_TRY(mix_rows<unsigned short>(c, run, ds, parts.size(), dt, n_tiles, dr, M));
+    {
+      GemmBf16 g = residual(c->pf_cat, R * (size_t)c->ld_cat, L.w_o, L.ldc);
+      if (!L.ff) {
+        g.add_rows = add_rows;
+        g.add_vec = add_vec;
+      }
+      Prof p(dev, true, ST_PASS + ST_OUT, 0.0);
+      launch_gemm_bf16(dev, p.rec(), c->planes, GEMM_OUT_RESIDUAL, g);
+    }
+    if (!L.ff) continue;
+    {
+      GemmBf16 g = normed(L.w_up, L.ff, L.norm2);
+      g.planes = c->pf_u;
+      g.p_plane = R * (size_t)c->ld_u;
+      g.ldp = L.ldu;
+      g.xielu = L.xielu;
+      Prof p(dev, true, ST_PASS + ST_UP, 0.0);
+      launch_gemm_bf16(dev, p.rec(), c->planes, GEMM_OUT_XIELU, g);
+    }
+    {
+      GemmBf16 g = residual(c->pf_u, R * (size_t)c->ld_u, L.w_down, L.ldu);
+      g.add_rows = add_rows;
+      g.add_vec = add_vec;
+      Prof p(dev, true, ST_PASS + ST_DOWN, 0.0);
+      launch_gemm_bf16(dev, p.rec(), c->planes, GEMM_OUT_RESIDUAL, g);
+    }
+  }
+  for (size_t w0 = 0; w0 < nw; w0 += LOGIT_ROWS) {
+    const size_t n = std::min(LOGIT_ROWS, nw - w0);
+    const float* src = c->pf_logits;
+    if (n <= 8) {  // the decode step's classifier
+      k_gather_rows<0><<<(unsigned)n, 256, 0, st>>>(c->pf_x, c->ldx, c->width, dw + w0, c->st_x, nullptr, 0, nullptr, 0);
+      head_rows(c, c->st_x, (int)n, true);
+      src = c->st_logits;
+    } else {
+      const size_t gp = LOGIT_ROWS * (size_t)c->ldx;
+      if (c->f32)
+        k_gather_rows<3><<<(unsigned)n, 256, 0, st>>>(c->pf_x, c->ldx, c->width, dw + w0, nullptr, c->pf_gp, gp, c->pf_gsq, c->n_sq);
+      else
+        k_gather_rows<1><<<(unsigned)n, 256, 0, st>>>(c->pf_x, c->ldx, c->width, dw + w0, nullptr, c->pf_gp, gp, c->pf_gsq, c->n_sq);
+      GemmBf16 g = normed(c->head, c->vocab, c->final_norm);
+      g.a = c->pf_gp;
+      g.a_plane = gp;
+      g.sq_in = c->pf_gsq;
+      g.M = (int)n;
+      g.out = c->pf_logits;
+      g.ldo = c->vocab;
+      g.cap = c->cfg.logit_softcap;
+      Prof p(dev, true, ST_PASS + ST_HEAD, 0.0);
+      launch_gemm_bf16(dev, p.rec(), c->planes, GEMM_OUT_SOFTCAP, g);
+    }
+    CH_HIP(dev, hipMemcpyAsync(*logits, src, n * c->vocab * sizeof(float), hipMemcpyDeviceToHost, st));
+    CH_HIP(dev, hipStreamSynchronize(st));
+    *logits += n * c->vocab;
+  }
+  CH_HIP(dev, hipGetLastError());
+  for (const Part& p : parts) c->seqs[p.seq].len += p.n;
+  return 0;
+}
+
+int check_seq(const Ctx* c, size_t seq) {
+  if (seq >= c->seqs.size() || !c->seqs[seq].open) CH_BAIL(c->dev, CRABML_HIP_BAD_INPUT, "hybrid: sequence %zu is not open", seq);
+  return 0;
+}
+
+int create_impl(Ctx* c, const crabml_hip_hybrid_layer_t* layers, const crabml_hip_hybrid_weights_t& w) {
+  crabml_hip_device* dev = c->dev;
+  const auto& g = c->cfg;
+  const size_t W = g.width;
+  c->f32 = g.compute == CRABML_HIP_F32;
+  c->planes = c->f32 ? 3 : 1;
+  c->width = (int)W;
+  c->vocab = (int)g.vocab_size;
+  c->ldx = up(W, 64);
+  c->n_sq = c->ldx / 64;
+  c->keep_emb = g.loop_times > 1;
+  CH_TRY(alloc_matrix(c, g.vocab_size, (size_t)c->ldx, &c->head));
+  CH_TRY(dalloc_n(c, g.vocab_size * W, &c->embed));
+  CH_TRY(pack_matrix(c, w.embed, "embed", g.vocab_size, W, c->embed, W, 0, g.vocab_size, g.vocab_size));
+  CH_TRY(pack_matrix(c, w.head, "head", g.vocab_size, W, c->head, (size_t)c->ldx, 0, g.vocab_size, g.vocab_size));
+  CH_TRY(pack_vector(c, w.final_norm, "final_norm", 1, &c->final_norm));
+  if (g.loop_times) CH_TRY(pack_vector(c, w.loop_step, "loop_step", g.loop_times * W, &c->loop_step));
+  c->layers.resize(g.n_layers);
+  size_t part = 0, tick = 0, ss = 0;
+  for (size_t i = 0; i < g.n_layers; i++) {
+    Layer& L = c->layers[i];
+    CH_TRY(build_layer(c, layers[i], L));
+    c->ld_proj = std::max(c->ld_proj, L.n_in);
+    c->ld_cat = std::max(c->ld_cat, L.ldc);
+    c->ld_u = std::max(c->ld_u, L.ldu);
+    if (L.at.H) {
+      const size_t slots = (size_t)HYB_STEP_ROWS * L.at.G * L.head_blocks;
+      part = std::max(part, slots * L.splits * mix_part_floats(L.at.V));
+      tick = std::max(tick, slots);
+    }
+    ss = std::max(ss, (size_t)HYB_STEP_ROWS * L.li.H * L.li.slices);
+    if (mix_step_lds(mix_step(c, Run{(int)i, RunState{}, false, nullptr}, 1)) > 60 * 1024)
+      CH_BAIL(dev, CRABML_HIP_NOT_IMPLEMENTED, "hybrid: layer %zu keeps %d cache rows, too many for the decode step's merge", i, L.at.rows);
+  }
+  // the order of layer runs, and each run's place in a sequence's slab
+  auto add_run = [&](size_t layer, bool first, size_t t) {
+    Run r;
+    r.layer = (int)layer;
+    const Layer& L = c->layers[layer];
+    const size_t e = c->f32 ? 4 : 2;
+    auto take = [&](size_t bytes) {
+      const size_t at = c->slab_bytes;
+      c->slab_bytes += align_up(bytes, 256);
+      return at;
+    };
+    if (L.at.H) {
+      r.rs.k = take((size_t)L.at.G * L.at.rows * L.at.D * e);
+      r.rs.v = take((size_t)L.at.G * L.at.rows * L.at.V * e);
+    }
+    if (L.li.H) r.rs.s = take((size_t)L.li.H * L.li.D * L.li.V * 4);
+    if (first) {
+      r.add_emb = t > 0;
+      r.add_vec = c->loop_step + t * W;
+    }
+    c->runs.push_back(r);
+  };
+  const size_t lo = g.loop_times ? g.loop_start : g.n_layers, hi = g.loop_times ? g.loop_stop : g.n_layers;
+  for (size_t i = 0; i < lo; i++) add_run(i, false, 0);
+  for (size_t t = 0; t < g.loop_times; t++)
+    for (size_t i = lo; i < hi; i++) add_run(i, i == lo, t);
+  for (size_t i = hi; i < g.n_layers; i++) add_run(i, false, 0);
+  {
+    std::vector<double> f((W + 1) / 2);
+    for (size_t i = 0; i < f.size(); i++) f[i] = pow(10000.0, -2.0 * (double)i / (double)W);
+    CH_TRY(dalloc_n(c, f.size(), &c->freq));
+    CH_HIP(dev, hipMemcpyAsync(c->freq, f.data(), f.size() * sizeof(double), hipMemcpyHostToDevice, dev->stream));
+    CH_HIP(dev, hipStreamSynchronize(dev->stream));
+  }
+  const size_t B = HYB_STEP_ROWS;
+  CH_TRY(dalloc_n(c, B, &c->st_seq));
+  CH_TRY(dalloc_n(c, 1, &c->st_count));
+  CH_TRY(dalloc_n(c, B * c->ldx, &c->st_x));
+  CH_TRY(dalloc_n(c, B * c->ldx, &c->st_emb));
+  CH_TRY(dalloc_n(c, B * c->ld_proj, &c->st_proj));
+  CH_TRY(dalloc_n(c, B * c->ld_cat, &c->st_cat));
+  CH_TRY(dalloc_n(c, B * c->ld_u, &c->st_u));
+  CH_TRY(dalloc_n(c, ss, &c->st_ss));
+  CH_TRY(dalloc_n(c, part, &c->st_part));
+  CH_TRY(dalloc_n(c, tick, &c->st_tick));
+  CH_TRY(dalloc_n(c, B * c->vocab, &c->st_logits));
+  c->st_out_cap = B * g.seq_len;
+  CH_TRY(dalloc_n(c, c->st_out_cap, &c->st_out));
+  CH_TRY(dalloc_n(c, B * ARGMAX_BLOCKS, &c->am_val));
+  CH_TRY(dalloc_n(c, B * ARGMAX_BLOCKS, &c->am_idx));
+  CH_HIP(dev, hipHostMalloc((void**)&c->h_seq, META_SLOTS * B * sizeof(StepSeq), hipHostMallocDefault));
+  CH_HIP(dev, hipStreamSynchronize(dev->stream));
+  return 0;
+}
+
+}  // namespace
+
+extern "C" {
+
+int crabml_hip_hybrid_create(crabml_hip_device_t* dev, const crabml_hip_hybrid_config_t* cfg, const crabml_hip_hybrid_layer_t* layers,
+                             const crabml_hip_hybrid_weights_t* w, crabml_hip_hybrid_t** out) {
+  if (!dev || !cfg || !layers || !w || !out) return CRABML_HIP_BAD_INPUT;
+  *out = nullptr;
+  CH_LIVE(dev);
+  CH_USE(dev);
+  CH_FLUSH(dev);
+  if (!cfg->width || !cfg->vocab_size || !cfg->n_layers || !cfg->seq_len || cfg->width > 65536 || cfg->vocab_size > (1u << 24) || cfg->seq_len > (1u << 24))
+    CH_BAIL(dev, CRABML_HIP_BAD_INPUT, "hybrid: width %zu, vocab %zu, %zu layers, %zu positions", cfg->width, cfg->vocab_size, cfg->n_layers, cfg->seq_len);
+  if (cfg->compute != CRABML_HIP_BF16 && cfg->compute != CRABML_HIP_F32) CH_BAIL(dev, CRABML_HIP_BAD_INPUT, "hybrid: compute is BF16 or F32, not %u", cfg->compute);
+  if (cfg->loop_times && (cfg->loop_start >= cfg->loop_stop || cfg->loop_stop > cfg->n_layers))
+    CH_BAIL(dev, CRABML_HIP_BAD_INPUT, "hybrid: loop over layers [%zu, %zu) of %zu", cfg->loop_start, cfg->loop_stop, cfg->n_layers);
+  Ctx* c = new Ctx();
+  c->dev = dev;
+  c->cfg = *cfg;
+  const int rc = create_impl(c, layers, *w);
+  if (rc != 0) {
+    crabml_hip_hybrid_destroy(c);
+    return rc;
+  }
+  *out = c;
+  return 0;
+}
+
+int crabml_hip_hybrid_destroy(crabml_hip_hybrid_t* c) {
+  if (!c) return 0;
+  (void)hipSetDevice(c->dev->ordinal);
+  (void)hipStreamSynchronize(c->dev->stream);
+  for (auto& g : c->graphs) {
+    if (g.second.second) (void)hipGraphExecDestroy(g.second.second);
+    if (g.second.first) (void)hipGraphDestroy(g.second.first);
+  }
+  for (auto& s : c->seqs)
+    if (s.open) pool_free(c->dev, s.slab, s.cap);
+  for (auto& a : c->allocs) pool_free(c->dev, a.first, a.second);
+  if (c->h_seq) (void)hipHostFree(c->h_seq);
+  if (c->h_meta) (void)hipHostFree(c->h_meta);
+  delete c;
+  return 0;
+}
+
+int crabml_hip_hybrid_open(crabml_hip_hybrid_t* c, size_t* seq) {
+  if (!c || !seq) return CRABML_HIP_BAD_INPUT;
+  CH_USE(c->dev);
+  size_t i = 0;
+  while (i < c->seqs.size() && c->seqs[i].open) i++;
+  if (i == c->seqs.size()) c->seqs.emplace_back();
+  Seq s;
+  CH_TRY(pool_alloc(c->dev, c->slab_bytes, (void**)&s.slab, &s.cap));
+  s.open = true;
+  c->seqs[i] = s;
+  *seq = i;
+  return 0;
+}
+
+int crabml_hip_hybrid_close(crabml_hip_hybrid_t* c, size_t seq) {
+  if (!c) return CRABML_HIP_BAD_INPUT;
+  CH_TRY(check_seq(c, seq));
+  pool_free(c->dev, c->seqs[seq].slab, c->seqs[seq].cap);  // (one stream: whoever gets it next is ordered behind us)
+  c->seqs[seq] = Seq();
+  return 0;
+}
+
+size_t crabml_hip_hybrid_len(const crabml_hip_hybrid_t* c, size_t seq) { return c && seq < c->seqs.size() ? c->seqs[seq].len : 0; }
+size_t crabml_hip_hybrid_slab_bytes(const crabml_hip_hybrid_t* c) { return c ? c->slab_bytes : 0; }
+
+int crabml_hip_hybrid_step(crabml_hip_hybrid_t* c, size_t n, const size_t* seqs, const size_t* counts, const uint32_t* tokens, const size_t* want_counts,
+                           const uint32_t* want, float* logits) {
+  if (!c || (n && (!seqs || !counts || !tokens))) return CRABML_HIP_BAD_INPUT;
+  crabml_hip_device* dev = c->dev;
+  CH_LIVE(dev);
+  CH_USE(dev);
+  CH_FLUSH(dev);
+  // everything is checked before anything runs
+  bool single = n <= HYB_STEP_ROWS;
+  size_t n_tok = 0, n_want = 0;
+  std::vector<char> seen(c->seqs.size(), 0);
+  for (size_t i = 0; i < n; i++) {
+    CH_TRY(check_seq(c, seqs[i]));
+    if (seen[seqs[i]]) CH_BAIL(dev, CRABML_HIP_BAD_INPUT, "hybrid: sequence %zu twice in one step", seqs[i]);
+    seen[seqs[i]] = 1;
+    if (!counts[i]) CH_BAIL(dev, CRABML_HIP_BAD_INPUT, "hybrid: sequence %zu gets no tokens", seqs[i]);
+    if (counts[i] > c->cfg.seq_len || c->seqs[seqs[i]].len + counts[i] > c->cfg.seq_len)
+      CH_BAIL(dev, CRABML_HIP_TENSOR_ERROR, "hybrid: %zu more tokens do not fit sequence %zu (%zu of %zu used)", counts[i], seqs[i], c->seqs[seqs[i]].len, c->cfg.seq_len);
+    for (size_t t = 0; t < counts[i]; t++)
+      if (tokens[n_tok + t] >= c->cfg.vocab_size) CH_BAIL(dev, CRABML_HIP_BAD_INPUT, "hybrid: token %u out of range", tokens[n_tok + t]);
+    for (size_t k = 0; want_counts && k < want_counts[i]; k++)
+      if (!want || want[n_want + k] >= counts[i] || (k && want[n_want + k] <= want[n_want + k - 1]))
+        CH_BAIL(dev, CRABML_HIP_BAD_INPUT, "hybrid: wanted places must ascend inside the new tokens");
+    n_tok += counts[i];
+    n_want += want_counts ? want_counts[i] : 0;
+    single = single && counts[i] == 1;
+  }
+  if (n_want && !logits) return CRABML_HIP_BAD_INPUT;
+  if (n == 0) return 0;
+  if (single) {
+    CH_TRY(step_begin(c, n, seqs, tokens));
+    CH_TRY(run_step(c, (int)n, false));
+    for (size_t i = 0; i < n; i++) c->seqs[seqs[i]].len++;
+    if (n_want) {
+      for (size_t i = 0; i < n; i++)
+        if (want_counts[i]) {
+          CH_HIP(dev, hipMemcpyAsync(logits, c->st_logits + i * c->vocab, c->vocab * sizeof(float), hipMemcpyDeviceToHost, dev->stream));
+          logits += c->vocab;
+        }
+      CH_HIP(dev, hipStreamSynchronize(dev->stream));
+    }
+    return 0;
+  }
+  const size_t cap = c->cfg.pass_rows ? c->cfg.pass_rows : 2048;
+  std::vector<Part> parts;
+  size_t used = 0, tok = 0, wat = 0;
+  for (size_t i = 0; i < n; i++) {
+    size_t done = 0, k = 0;
+    const size_t nw = want_counts ? want_counts[i] : 0;
+    while (done < counts[i]) {
+      if (used == cap) {
+        CH_TRY(run_pass(c, parts, &logits));
+        parts.clear();
+        used = 0;
+      }
+      Part p;
+      p.seq = seqs[i];
+      p.n = std::min(counts[i] - done, cap - used);
+      p.tokens = tokens + tok + done;
+      for (; k < nw && want[wat + k] < done + p.n; k++) p.want.push_back((int)(want[wat + k] - done));
+      done += p.n;
+      used += p.n;
+      parts.push_back(std::move(p));
+    }
+    tok += counts[i];
+    wat += nw;
+  }
+  return run_pass(c, parts, &logits);
+}
+
+int crabml_hip_hybrid_decode_greedy(crabml_hip_hybrid_t* c, size_t n, const size_t* seqs, const uint32_t* tokens, size_t n_steps, uint32_t* out_tokens) {
+  if (!c || !seqs || !tokens || (!out_tokens && n_steps)) return CRABML_HIP_BAD_INPUT;
+  crabml_hip_device* dev = c->dev;
+  CH_LIVE(dev);
+  CH_USE(dev);
+  CH_FLUSH(dev);
+  if (n == 0 || n > HYB_STEP_ROWS) CH_BAIL(dev, CRABML_HIP_BAD_INPUT, "hybrid: greedy decoding takes 1 to %d sequences, not %zu", HYB_STEP_ROWS, n);
+  std::vector<char> seen(c->seqs.size(), 0);
+  for (size_t i = 0; i < n; i++) {
+    CH_TRY(check_seq(c, seqs[i]));
+    if (seen[seqs[i]]) CH_BAIL(dev, CRABML_HIP_BAD_INPUT, "hybrid: sequence %zu twice in one step", seqs[i]);
+    seen[seqs[i]] = 1;
+    if (tokens[i] >= c->cfg.vocab_size) CH_BAIL(dev, CRABML_HIP_BAD_INPUT, "hybrid: token %u out of range", tokens[i]);
+    if (n_steps > c->cfg.seq_len || c->seqs[seqs[i]].len + n_steps > c->cfg.seq_len)
+      CH_BAIL(dev, CRABML_HIP_TENSOR_ERROR, "hybrid: %zu steps do not fit sequence %zu (%zu of %zu used)", n_steps, seqs[i], c->seqs[seqs[i]].len, c->cfg.seq_len);
+  }
+  if (n_steps == 0) return 0;
+  CH_TRY(step_begin(c, n, seqs, tokens));
+  CH_HIP(dev, hipMemsetAsync(c->st_count, 0, sizeof(int), dev->stream));
+  for (size_t s = 0; s < n_steps; s++) CH_TRY(run_step(c, (int)n, true));
+  for (size_t i = 0; i < n; i++) c->seqs[seqs[i]].len += n_steps;
+  CH_HIP(dev, hipMemcpyAsync(out_tokens, c->st_out, n_steps * n * sizeof(uint32_t), hipMemcpyDeviceToHost, dev->stream));
+  CH_HIP(dev, hipStreamSynchronize(dev->stream));
+  return 0;
+}
+
+}  // extern "C"

@@ -1,0 +1,73 @@
+// hybrid_common.hpp -- what the prompt pass (hybrid_rows.hpp) and the decode step (hybrid_step.hpp) of the hybrid decoder share:
+// the per-sequence state's layout, a layer's geometry, the embedding.
+//
+// Two mixers are built here, each usable with or without the other:
+//   softmax attention inside chunks: grouped queries, a log-distance penalty per head, a sink logit per head, an output gate
+//   linear attention with decay: S <- d S + k v^T, o = S^T q, one f32 state per head
+#pragma once
+#include "gemm_bf16.hpp"
+
+namespace crabml_hip {
+
+// KV cache element: f32, or bf16 rounded to nearest even
+template <typename T>
+__device__ __forceinline__ T kv_from(float f);
+template <>
+__device__ __forceinline__ float kv_from<float>(float f) { return f; }
+template <>
+__device__ __forceinline__ unsigned short kv_from<unsigned short>(float f) { return f2bf(f); }
+__device__ __forceinline__ float kv_to(float v) { return v; }
+__device__ __forceinline__ float kv_to(unsigned short v) { return bf2f(v); }
+// eight consecutive elements (16-byte aligned rows)
+__device__ __forceinline__ void kv_load8(const float* p, float (&o)[8]) {
+  const f32x4 a = *(const f32x4*)p, b = *(const f32x4*)(p + 4);
+#pragma unroll
+  for (int e = 0; e < 4; e++) {
+    o[e] = a[e];
+    o[e + 4] = b[e];
+  }
+}
+__device__ __forceinline__ void kv_load8(const unsigned short* p, float (&o)[8]) {
+  const i32x4 a = *(const i32x4*)p;
+#pragma unroll
+  for (int e = 0; e < 4; e++) {
+    o[2 * e] = __builtin_bit_cast(float, (unsigned)a[e] << 16);
+    o[2 * e + 1] = __builtin_bit_cast(float, (unsigned)a[e] & 0xffff0000u);
+  }
+}
+
+// One layer's mixers.  Head widths are padded to multiples of 8 (zero weight rows make the padding zero), so every head starts on a
+// 16-byte boundary of its row; D / V / ... below are the padded widths.
+struct AttnGeom {
+  int H = 0, G = 0, D = 0, V = 0;
+  int chunk = 0;  // positions per chunk
+  int rows = 0;   // cache rows per sequence: position p lives in row p % chunk, so min(chunk, longest sequence) of them
+  float scale = 0.f, out_scale = 1.f;
+  int cq = 0, ck = 0, cv = 0, cg = 0;  // columns of the projected row
+  const float *amp = nullptr, *rate = nullptr, *sink = nullptr;  // per head (nullable): penalty amp ln(1 + rate d), sink logit
+};
+struct LinGeom {
+  int H = 0, D = 0, V = 0;
+  int v_true = 0;  // unpadded value width: what the norm averages over is H * v_true
+  float out_scale = 1.f;
+  int cq = 0, ck = 0, cv = 0, cg = 0;
+  int slices = 0;                // value columns are independent: slices of 32 per workgroup
+  const float* decay = nullptr;  // [H][LIN_POW] decay^n
+  const float* norm = nullptr;   // [H * V]
+};
+#define LIN_POW 65
+#define LIN_SLICE 32
+// where a layer run keeps its share of a sequence's state (byte offsets into the sequence's slab)
+struct RunState {
+  size_t k = 0, v = 0, s = 0;
+};
+
+// ---- embedding: row * scale + interleaved sin / cos of the position ------------------------------------------------------------
+// freq[c / 2] in f64: the angle is formed and reduced in f64, its sine taken in f32
+__device__ __forceinline__ float position_entry(int pos, int c, const double* __restrict__ freq) {
+  const double turns = (double)pos * freq[c >> 1] * 0.15915494309189533577;
+  const float r = (float)((turns - rint(turns)) * 6.28318530717958647692);
+  return (c & 1) ? cosf(r) : sinf(r);
+}
+
+}  // namespace crabml_hip

@@ -1,0 +1,502 @@
+// hybrid_rows.hpp -- the hybrid decoder's prompt pass: any number of tokens of any number of sequences as one batch of rows
+//   k_gemm_bf16<ACT>       norm 1 + every projection of both mixers + their activations
+//   k_attn_rows            softmax attention, 64 query rows of one head per workgroup, on the matrix cores
+//   k_linear_rows          linear attention in blocks of rows: inside a block as a masked product, across blocks through the state
+//   k_mix_rows             the linear branch's norm and gate, the cache append
+//   k_gemm_bf16<RESIDUAL>, k_gemm_bf16<XIELU>, k_gemm_bf16<RESIDUAL>
+// Keys of this pass are read from its own projected rows, earlier ones of the first chunk from the cache; the cache is appended only
+// after the attention launch, with the rows of the chunk that the pass ends in.
+//
+// T = unsigned short: bf16 operands.  T = float: every operand f32 (v_mfma_f32_16x16x4_f32), activations in three exact planes.
+#pragma once
+#include "hybrid_common.hpp"
+
+namespace crabml_hip {
+
+struct PassSeq {
+  int row0, n, pos0, pad;  // rows row0 .. row0 + n - 1 of the pass are the sequence's positions pos0 ..
+  char* slab;
+};
+struct PassRow {
+  int seq, pos;
+};
+struct PassTile {  // up to 64 consecutive rows of one sequence
+  int seq, row, pos, n;
+};
+
+// ---- operand fragments of 16x16 matrix products out of LDS rows with k contiguous ------------------------------------------------
+// lane: row lane % 16 of the operand, k group lane / 16
+__device__ __forceinline__ void split3(const float (&v)[8], bf16x8& hi, bf16x8& mid, bf16x8& lo) {
+  unsigned short h[8], m[8], l[8];
+#pragma unroll
+  for (int e = 0; e < 8; e++) {
+    const float a = __builtin_bit_cast(float, __builtin_bit_cast(unsigned, v[e]) & 0xffff0000u), r = v[e] - a;
+    const float b = __builtin_bit_cast(float, __builtin_bit_cast(unsigned, r) & 0xffff0000u);
+    h[e] = (unsigned short)(__builtin_bit_cast(unsigned, a) >> 16);
+    m[e] = (unsigned short)(__builtin_bit_cast(unsigned, b) >> 16);
+    l[e] = f2bf(r - b);
+  }
+  __builtin_memcpy(&hi, h, 16);
+  __builtin_memcpy(&mid, m, 16);
+  __builtin_memcpy(&lo, l, 16);
+}
+__device__ __forceinline__ f32x4 mfma_bf16(bf16x8 a, bf16x8 b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0); }
+
+// acc += A B^T over k < K; a / b: this lane's rows.  K is a multiple of 32.
+__device__ __forceinline__ f32x4 mma_rows(const unsigned short* a, const unsigned short* b, int K, f32x4 acc) {
+  const int o = (threadIdx.x >> 4 & 3) * 8;
+  for (int k = 0; k < K; k += 32) acc = mfma_bf16(*(const bf16x8*)(a + k + o), *(const bf16x8*)(b + k + o), acc);
+  return acc;
+}
+// one side f32: three exact bf16 pieces of it.  w (nullable, LDS): a factor per k
+__device__ __forceinline__ f32x4 mma_rows(const float* a, const unsigned short* b, int K, f32x4 acc) {
+  const int o = (threadIdx.x >> 4 & 3) * 8;
+  for (int k = 0; k < K; k += 32) {
+    float v[8];
+    kv_load8(a + k + o, v);
+    bf16x8 h, m, l;
+    split3(v, h, m, l);
+    const bf16x8 fb = *(const bf16x8*)(b + k + o);
+    acc = mfma_bf16(h, fb, mfma_bf16(m, fb, mfma_bf16(l, fb, acc)));
+  }
+  return acc;
+}
+__device__ __forceinline__ f32x4 mma_rows(const unsigned short* a, const float* b, int K, f32x4 acc) {
+  const int o = (threadIdx.x >> 4 & 3) * 8;
+  for (int k = 0; k < K; k += 32) {
+    float v[8];
+    kv_load8(b + k + o, v);
+    bf16x8 h, m, l;
+    split3(v, h, m, l);
+    const bf16x8 fa = *(const bf16x8*)(a + k + o);
+    acc = mfma_bf16(fa, h, mfma_bf16(fa, m, mfma_bf16(fa, l, acc)));
+  }
+  return acc;
+}
+__device__ __forceinline__ f32x4 mma_rows(const float* a, const float* b, int K, f32x4 acc) {
+  const int o = threadIdx.x >> 4 & 3;
+#pragma unroll 8
+  for (int k = 0; k < K; k += 4) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a[k + o], b[k + o], acc, 0, 0, 0);
+  return acc;
+}
+// the same with a factor w[k] (LDS) on A's elements
+__device__ __forceinline__ f32x4 mma_rows_w(const unsigned short* a, const float* w, const unsigned short* b, int K, f32x4 acc) {
+  const int o = (threadIdx.x >> 4 & 3) * 8;
+  for (int k = 0; k < K; k += 32) {
+    float v[8], f[8];
+    kv_load8(a + k + o, v);
+    kv_load8(w + k + o, f);
+#pragma unroll
+    for (int e = 0; e < 8; e++) v[e] *= f[e];
+    bf16x8 h, m, l;
+    split3(v, h, m, l);
+    const bf16x8 fb = *(const bf16x8*)(b + k + o);
+    acc = mfma_bf16(h, fb, mfma_bf16(m, fb, mfma_bf16(l, fb, acc)));
+  }
+  return acc;
+}
+__device__ __forceinline__ f32x4 mma_rows_w(const float* a, const float* w, const float* b, int K, f32x4 acc) {
+  const int o = threadIdx.x >> 4 & 3;
+#pragma unroll 8
+  for (int k = 0; k < K; k += 4) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a[k + o] * w[k + o], b[k + o], acc, 0, 0, 0);
+  return acc;
+}
+
+template <typename T>
+struct Oct {  // eight elements on their way from memory to LDS
+  i32x4 d[sizeof(T) / 2];
+};
+template <typename T>
+__device__ __forceinline__ Oct<T> oct_zero() {
+  Oct<T> o;
+#pragma unroll
+  for (unsigned i = 0; i < sizeof(T) / 2; i++) o.d[i] = i32x4{0, 0, 0, 0};
+  return o;
+}
+template <typename T>
+__device__ __forceinline__ Oct<T> oct_load(const T* p) {
+  Oct<T> o;
+#pragma unroll
+  for (unsigned i = 0; i < sizeof(T) / 2; i++) o.d[i] = ((const i32x4*)p)[i];
+  return o;
+}
+template <typename T>
+__device__ __forceinline__ void oct_store(T* p, const Oct<T>& o) {
+#pragma unroll
+  for (unsigned i = 0; i < sizeof(T) / 2; i++) ((i32x4*)p)[i] = o.d[i];
+}
+template <typename T>
+__device__ __forceinline__ void oct_scatter(T* p, int stride, const Oct<T>& o) {  // element e -> p[e * stride]
+  T v[8];
+  __builtin_memcpy(v, &o, sizeof v);
+#pragma unroll
+  for (int e = 0; e < 8; e++) p[e * stride] = v[e];
+}
+
+// ---- embedding of the pass's rows: x, its planes, its square sum (piece 0; the others are cleared) --------------------------------
+template <int P>
+__global__ __launch_bounds__(256) void k_embed_rows(const unsigned short* __restrict__ table, const int* __restrict__ tokens,
+                                                    const PassRow* __restrict__ rows, int width, int ldx, float scale,
+                                                    const double* __restrict__ freq, float* __restrict__ x, float* __restrict__ emb,
+                                                    const float* __restrict__ add_vec, unsigned short* __restrict__ planes, size_t p_plane,
+                                                    float* __restrict__ sq_out, int n_sq) {
+  __shared__ float red[4];
+  const int r = blockIdx.x, tok = tokens[r], pos = rows[r].pos;
+  float s = 0.f;
+  for (int c = threadIdx.x; c < width; c += 256) {
+    float v = __builtin_fmaf(bf2f(table[(size_t)tok * width + c]), scale, position_entry(pos, c, freq));
+    if (emb) emb[(size_t)r * ldx + c] = v;
+    if (add_vec) v += add_vec[c];
+    x[(size_t)r * ldx + c] = v;
+    split_store<P>(v, planes + (size_t)r * ldx + c, p_plane);
+    s = __builtin_fmaf(v, v, s);
+  }
+  s = wave_sum_f32(s);
+  if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = s;
+  __syncthreads();
+  for (int i = threadIdx.x; i < n_sq; i += 256) sq_out[(size_t)r * n_sq + i] = i ? 0.f : (red[0] + red[1]) + (red[2] + red[3]);
+}
+
+// rows[i] of x -> dense rows of f32 (P = 0) or planes, with their square sums in piece 0
+template <int P>
+__global__ __launch_bounds__(256) void k_gather_rows(const float* __restrict__ x, int ldx, int width, const int* __restrict__ which,
+                                                     float* __restrict__ dst, unsigned short* __restrict__ planes, size_t p_plane,
+                                                     float* __restrict__ sq_out, int n_sq) {
+  __shared__ float red[4];
+  const int r = blockIdx.x;
+  const float* src = x + (size_t)which[r] * ldx;
+  float s = 0.f;
+  for (int c = threadIdx.x; c < width; c += 256) {
+    const float v = src[c];
+    if constexpr (P == 0) {
+      dst[(size_t)r * ldx + c] = v;
+    } else {
+      split_store<P>(v, planes + (size_t)r * ldx + c, p_plane);
+      s = __builtin_fmaf(v, v, s);
+    }
+  }
+  if constexpr (P != 0) {
+    s = wave_sum_f32(s);
+    if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = s;
+    __syncthreads();
+    for (int i = threadIdx.x; i < n_sq; i += 256) sq_out[(size_t)r * n_sq + i] = i ? 0.f : (red[0] + red[1]) + (red[2] + red[3]);
+  }
+}
+
+// ---- softmax attention ------------------------------------------------------------------------------------------------------------
+template <typename T>
+struct MixRows {
+  AttnGeom at;
+  LinGeom li;
+  RunState rs;
+  const PassSeq* seqs = nullptr;
+  const PassTile* tiles = nullptr;
+  const PassRow* rows = nullptr;
+  const T* proj = nullptr;  // [rows][ldp]
+  unsigned short* cat = nullptr;
+  size_t cat_plane = 0;
+  float* lin = nullptr;  // [rows][H * V] raw outputs of the linear branch
+  int n_tiles = 0, ldp = 0, ldc = 0, lin_off = 0;
+};
+
+template <typename T>
+struct AttnTile {
+  static constexpr int PAD = 16 / sizeof(T);
+  template <int CLS>
+  static constexpr int keys() {
+    return (sizeof(T) == 2 ? 64 : 32) / (CLS > 128 ? 2 : 1);
+  }
+};
+
+// CLS: head widths up to this many elements.  Four waves of 16 query rows; keys in tiles of KT through LDS (K as rows, V transposed).
+template <typename T, int CLS, int P>
+__global__ __launch_bounds__(256) void k_attn_rows(const MixRows<T> a) {
+  constexpr int KT = AttnTile<T>::template keys<CLS>(), PAD = AttnTile<T>::PAD, LK = CLS + PAD, LV = KT + PAD, VT = CLS / 16, ST = KT / 16;
+  __shared__ __attribute__((aligned(16))) T ks[KT * LK];
+  __shared__ __attribute__((aligned(16))) T vs[CLS * LV];
+  __shared__ __attribute__((aligned(16))) T ps[4 * 16 * LV];
+  const AttnGeom& g = a.at;
+  const int tid = threadIdx.x, lane = tid & 63, wave = wave_in_wg(), fr = lane & 15, fk = lane >> 4;
+  const PassTile t = a.tiles[blockIdx.x];
+  const PassSeq sq = a.seqs[t.seq];
+  const int h = blockIdx.y, kvh = h / (g.H / g.G);
+  const int DK = (g.D + 31) & ~31;
+  const T* kc = (const T*)(sq.slab + a.rs.k) + (size_t)kvh * g.rows * g.D;
+  const T* vc = (const T*)(sq.slab + a.rs.v) + (size_t)kvh * g.rows * g.V;
+  const T* proj_seq = a.proj + (size_t)sq.row0 * a.ldp;  // row of position p: + (p - pos0) * ldp
+  // this lane's query row (A operand) and its four output rows
+  const int qrow = wave * 16 + fr;
+  const T* qp = a.proj + (size_t)(t.row + (qrow < t.n ? qrow : t.n - 1)) * a.ldp + g.cq + h * g.D;
+  bf16x8 q16[sizeof(T) == 2 ? CLS / 32 : 1];
+  float q32[sizeof(T) == 4 ? CLS / 4 : 1];
+  if constexpr (sizeof(T) == 2) {
+#pragma unroll
+    for (int i = 0; i < CLS / 32; i++) {
+      const int k = i * 32 + fk * 8;
+      const Oct<T> o = k < g.D ? oct_load(qp + k) : oct_zero<T>();
+      __builtin_memcpy(&q16[i], &o, 16);
+    }
+  } else {
+#pragma unroll
+    for (int i = 0; i < CLS / 4; i++) q32[i] = i * 4 + fk < g.D ? (float)qp[i * 4 + fk] : 0.f;
+  }
+  int pos[4], first[4];
+#pragma unroll
+  for (int e = 0; e < 4; e++) {
+    pos[e] = t.pos + wave * 16 + fk * 4 + e;
+    first[e] = pos[e] - pos[e] % g.chunk;
+  }
+  float m[4], l[4];
+  f32x4 o[VT];
+#pragma unroll
+  for (int e = 0; e < 4; e++) {
+    m[e] = -INFINITY;
+    l[e] = 0.f;
+  }
+#pragma unroll
+  for (int j = 0; j < VT; j++) o[j] = f32x4{0.f, 0.f, 0.f, 0.f};
+  const float amp = g.amp ? g.amp[h] : 0.f, rate = g.amp ? g.rate[h] : 0.f;
+  const int lo = t.pos - t.pos % g.chunk, hi = t.pos + t.n;  // keys [lo, hi)
+  for (int j0 = lo; j0 < hi; j0 += KT) {
+    __syncthreads();
+    for (int i = tid; i < KT * (DK / 8); i += 256) {  // K rows
+      const int c = i % (DK / 8) * 8, key = i / (DK / 8), p = j0 + key;
+      Oct<T> v = oct_zero<T>();
+      if (p < hi && c < g.D)
+        v = oct_load(p >= sq.pos0 ? proj_seq + (size_t)(p - sq.pos0) * a.ldp + g.ck + kvh * g.D + c : kc + (size_t)(p % g.chunk) * g.D + c);
+      oct_store(ks + key * LK + c, v);
+    }
+    for (int i = tid; i < KT * (CLS / 8); i += 256) {  // V columns
+      const int key = i % KT, c = i / KT * 8, p = j0 + key;
+      if (c >= g.V) continue;
+      Oct<T> v = oct_zero<T>();
+      if (p < hi)
+        v = oct_load(p >= sq.pos0 ? proj_seq + (size_t)(p - sq.pos0) * a.ldp + g.cv + kvh * g.V + c : vc + (size_t)(p % g.chunk) * g.V + c);
+      oct_scatter(vs + c * LV + key, LV, v);
+    }
+    __syncthreads();
+    f32x4 s[ST];
+#pragma unroll
+    for (int j = 0; j < ST; j++) {
+      s[j] = f32x4{0.f, 0.f, 0.f, 0.f};
+      const T* kr = ks + (j * 16 + fr) * LK;
+      if constexpr (sizeof(T) == 2) {
+#pragma unroll
+        for (int i = 0; i < CLS / 32; i++)
+          if (i * 32 < DK) s[j] = mfma_bf16(q16[i], *(const bf16x8*)(kr + i * 32 + fk * 8), s[j]);
+      } else {
+#pragma unroll
+        for (int i = 0; i < CLS / 4; i++)
+          if (i * 4 < DK) s[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(q32[i], kr[i * 4 + fk], s[j], 0, 0, 0);
+      }
+    }
+    T* pw = ps + wave * 16 * LV;
+#pragma unroll
+    for (int e = 0; e < 4; e++) {
+      float mx = -INFINITY;
+#pragma unroll
+      for (int j = 0; j < ST; j++) {
+        const int p = j0 + j * 16 + fr;
+        float v = s[j][e] * g.scale;
+        const int d = pos[e] - p;
+        if (g.amp) v -= amp * __logf(__builtin_fmaf(rate, (float)(d > 0 ? d : 0), 1.0f));
+        v = d >= 0 && p >= first[e] ? v : -INFINITY;
+        s[j][e] = v;
+        mx = fmaxf(mx, v);
+      }
+      mx = fmaxf(m[e], row16_max_f32(mx));
+      const float ref = mx == -INFINITY ? 0.f : mx, w = __expf(m[e] - ref);
+      float sum = 0.f;
+#pragma unroll
+      for (int j = 0; j < ST; j++) {
+        const float pv = __expf(s[j][e] - ref);
+        sum += pv;
+        pw[(fk * 4 + e) * LV + j * 16 + fr] = kv_from<T>(pv);
+      }
+      l[e] = __builtin_fmaf(l[e], w, row16_sum_f32(sum));
+      m[e] = mx;
+#pragma unroll
+      for (int j = 0; j < VT; j++) o[j][e] *= w;
+    }
+    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+    __builtin_amdgcn_wave_barrier();  // (a wave's LDS operations complete in order: its rows of P are there when it reads them)
+#pragma unroll
+    for (int j = 0; j < VT; j++)
+      if (j * 16 < g.V) o[j] = mma_rows(pw + fr * LV, vs + (j * 16 + fr) * LV, KT, o[j]);
+  }
+#pragma unroll
+  for (int e = 0; e < 4; e++) {
+    const int r = wave * 16 + fk * 4 + e;
+    if (r >= t.n) continue;
+    float w = 1.f, den = l[e];
+    if (g.sink) {
+      const float top = fmaxf(m[e], g.sink[h]);
+      w = __expf(m[e] - top);
+      den = __builtin_fmaf(den, w, __expf(g.sink[h] - top));
+    }
+    w *= g.out_scale / den;
+    const size_t row = (size_t)(t.row + r);
+#pragma unroll
+    for (int j = 0; j < VT; j++) {
+      const int c = j * 16 + fr;
+      if (c < g.V) {
+        const int col = h * g.V + c;
+        split_store<P>(o[j][e] * (w * kv_to(a.proj[row * a.ldp + g.cg + col])), a.cat + row * a.ldc + col, a.cat_plane);
+      }
+    }
+  }
+}
+
+// ---- linear attention with decay --------------------------------------------------------------------------------------------------
+// One workgroup: one head of one sequence, LIN_SLICE value columns, blocks of C rows in order.  With i, j inside a block of n rows:
+//   o_i = d^(i+1) S^T q_i + sum_{j <= i} d^(i-j) (q_i . k_j) v_j          S <- d^n S + sum_j d^(n-1-j) k_j v_j^T
+// The state lives in the accumulators (transposed: value columns are matrix rows) and passes through LDS once per block for the first
+// term.  Decay powers, products with the state and the masked weights are f32 (mma_rows on an f32 side).
+template <typename T, int CLS>
+struct LinTile {
+  static constexpr int C = sizeof(T) == 2 ? 64 : 32, PAD = 16 / sizeof(T);
+  static constexpr int LD = CLS + PAD, LC = C + PAD, LP = C + 4, LS = CLS + 4;
+  static constexpr size_t T_ELEMS = (size_t)2 * C * LD + (size_t)CLS * LC + LIN_SLICE * LC;
+  static constexpr size_t F_ELEMS = (size_t)C * LP + LIN_SLICE * LS + C + LIN_POW + 7;
+  static constexpr size_t LDS = T_ELEMS * sizeof(T) + F_ELEMS * sizeof(float);
+};
+template <typename T, int CLS>
+__global__ __launch_bounds__(256) void k_linear_rows(const MixRows<T> a) {
+  typedef LinTile<T, CLS> L;
+  constexpr int C = L::C, LD = L::LD, LC = L::LC, LP = L::LP, LS = L::LS, MT = C / 16, NG = 4 / MT, ND = CLS / 64;
+  constexpr int NQ = C * CLS / 8 / 256;  // octets of Q (and of K) per thread
+  extern __shared__ __attribute__((aligned(16))) char lin_lds[];
+  T* qs = (T*)lin_lds;          // [C][LD]
+  T* ks = qs + C * LD;          // [C][LD]
+  T* kt = ks + C * LD;          // [CLS][LC]
+  T* vt = kt + CLS * LC;        // [LIN_SLICE][LC]
+  float* p = (float*)(vt + LIN_SLICE * LC);  // [C][LP]
+  float* st = p + C * LP;                    // [LIN_SLICE][LS]
+  float* wj = st + LIN_SLICE * LS;           // [C] d^(n-1-j)
+  float* pow = wj + C;                       // [LIN_POW]
+  const LinGeom& g = a.li;
+  const int tid = threadIdx.x, lane = tid & 63, wave = wave_in_wg(), fr = lane & 15, fk = lane >> 4;
+  const int slice = blockIdx.x % g.slices, h = blockIdx.x / g.slices;
+  const PassSeq sq = a.seqs[blockIdx.y];
+  const int c0 = slice * LIN_SLICE;
+  float* S = (float*)(sq.slab + a.rs.s) + (size_t)h * g.D * g.V;
+  const T* base = a.proj + (size_t)sq.row0 * a.ldp;
+  for (int i = tid; i < LIN_POW; i += 256) pow[i] = g.decay[h * LIN_POW + i];
+  // state tile (value columns c0 + 16 i + 4 fk .., key column 16 (wave + 4 n) + fr)
+  f32x4 s[2][ND];
+#pragma unroll
+  for (int i = 0; i < 2; i++)
+#pragma unroll
+    for (int n = 0; n < ND; n++) {
+      const int c = c0 + i * 16 + fk * 4, d = (wave + 4 * n) * 16 + fr;
+      s[i][n] = sq.pos0 > 0 && c < g.V && d < g.D ? *(const f32x4*)(S + (size_t)d * g.V + c) : f32x4{0.f, 0.f, 0.f, 0.f};
+    }
+  Oct<T> rq[NQ], rk[NQ], rv;
+  auto request = [&](int r0) {
+#pragma unroll
+    for (int u = 0; u < NQ; u++) {
+      const int i = u * 256 + tid, r = r0 + i % C, c = i / C * 8;
+      const bool in = r < sq.n && c < g.D;
+      const T* row = base + (size_t)r * a.ldp + h * g.D + c;
+      rq[u] = in ? oct_load(row + g.cq) : oct_zero<T>();
+      rk[u] = in ? oct_load(row + g.ck) : oct_zero<T>();
+    }
+    const int r = r0 + tid % C, c = c0 + tid / C * 8;
+    rv = tid < C * (LIN_SLICE / 8) && r < sq.n && c < g.V ? oct_load(base + (size_t)r * a.ldp + g.cv + h * g.V + c) : oct_zero<T>();
+  };
+  request(0);
+  for (int r0 = 0; r0 < sq.n; r0 += C) {
+    const int n = sq.n - r0 < C ? sq.n - r0 : C;
+    __syncthreads();  // the previous block's products are done with LDS (and pow is there)
+#pragma unroll
+    for (int u = 0; u < NQ; u++) {
+      const int i = u * 256 + tid, r = i % C, c = i / C * 8;
+      oct_store(qs + r * LD + c, rq[u]);
+      oct_store(ks + r * LD + c, rk[u]);
+      oct_scatter(kt + c * LC + r, LC, rk[u]);
+    }
+    if (tid < C * (LIN_SLICE / 8)) oct_scatter(vt + (tid / C * 8) * LC + tid % C, LC, rv);
+    if (tid < C) wj[tid] = tid < n ? pow[n - 1 - tid] : 0.f;
+#pragma unroll
+    for (int i = 0; i < 2; i++)
+#pragma unroll
+      for (int nn = 0; nn < ND; nn++)
+#pragma unroll
+        for (int e = 0; e < 4; e++) st[(i * 16 + fk * 4 + e) * LS + (wave + 4 * nn) * 16 + fr] = s[i][nn][e];
+    __syncthreads();
+    if (r0 + C < sq.n) request(r0 + C);
+    const int mt = wave % MT;
+    // masked, decayed products of the block's rows
+    for (int j = wave / MT; j < MT; j += NG) {
+      f32x4 v = {0.f, 0.f, 0.f, 0.f};
+      if (j <= mt) v = mma_rows(qs + (mt * 16 + fr) * LD, ks + (j * 16 + fr) * LD, CLS, v);
+#pragma unroll
+      for (int e = 0; e < 4; e++) {
+        const int i = mt * 16 + fk * 4 + e, d = i - (j * 16 + fr);
+        p[i * LP + j * 16 + fr] = d >= 0 ? v[e] * pow[d] : 0.f;
+      }
+    }
+    __syncthreads();
+    for (int j = wave / MT; j < 2; j += NG) {
+      f32x4 v = mma_rows(qs + (mt * 16 + fr) * LD, st + (j * 16 + fr) * LS, CLS, f32x4{0.f, 0.f, 0.f, 0.f});
+#pragma unroll
+      for (int e = 0; e < 4; e++) v[e] *= pow[mt * 16 + fk * 4 + e + 1];
+      v = mma_rows(p + (mt * 16 + fr) * LP, vt + (j * 16 + fr) * LC, C, v);
+      const int c = c0 + j * 16 + fr;
+#pragma unroll
+      for (int e = 0; e < 4; e++) {
+        const int i = mt * 16 + fk * 4 + e;
+        if (i < n && c < g.V) a.lin[(size_t)(sq.row0 + r0 + i) * (g.H * g.V) + h * g.V + c] = v[e];
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < 2; i++)
+#pragma unroll
+      for (int nn = 0; nn < ND; nn++) {
+        s[i][nn] *= pow[n];
+        s[i][nn] = mma_rows_w(vt + (i * 16 + fr) * LC, wj, kt + ((wave + 4 * nn) * 16 + fr) * LC, C, s[i][nn]);
+      }
+  }
+#pragma unroll
+  for (int i = 0; i < 2; i++)
+#pragma unroll
+    for (int nn = 0; nn < ND; nn++) {
+      const int c = c0 + i * 16 + fk * 4, d = (wave + 4 * nn) * 16 + fr;
+      if (c < g.V && d < g.D) *(f32x4*)(S + (size_t)d * g.V + c) = s[i][nn];
+    }
+}
+
+// ---- behind both: the linear branch's norm and gate; the cache rows of the chunk each sequence's part of the pass ends in ----------
+template <typename T, int P>
+__global__ __launch_bounds__(256) void k_mix_rows(const MixRows<T> a, float eps) {
+  __shared__ float red[4];
+  const int r = blockIdx.x, tid = threadIdx.x;
+  const PassRow rw = a.rows[r];
+  const T* pr = a.proj + (size_t)r * a.ldp;
+  if (a.li.H) {
+    const LinGeom& g = a.li;
+    const int n = g.H * g.V;
+    const float* o = a.lin + (size_t)r * n;
+    float s = 0.f;
+    for (int i = tid; i < n; i += 256) s = __builtin_fmaf(o[i], o[i], s);
+    s = wave_sum_f32(s);
+    if ((tid & 63) == 0) red[tid >> 6] = s;
+    __syncthreads();
+    const float f = g.out_scale / sqrtf(((red[0] + red[1]) + (red[2] + red[3])) / (float)(g.H * g.v_true) + eps);
+    for (int i = tid; i < n; i += 256)
+      split_store<P>(o[i] * (f * g.norm[i] * kv_to(pr[g.cg + i])), a.cat + (size_t)r * a.ldc + a.lin_off + i, a.cat_plane);
+  }
+  if (a.at.H) {
+    const AttnGeom& g = a.at;
+    const PassSeq sq = a.seqs[rw.seq];
+    const int last = sq.pos0 + sq.n - 1;
+    if (rw.pos / g.chunk != last / g.chunk) return;
+    T* kc = (T*)(sq.slab + a.rs.k);
+    T* vc = (T*)(sq.slab + a.rs.v);
+    const size_t at = (size_t)(rw.pos % g.chunk);
+    for (int i = tid; i < g.G * g.D; i += 256) kc[((size_t)(i / g.D) * g.rows + at) * g.D + i % g.D] = pr[g.ck + i];
+    for (int i = tid; i < g.G * g.V; i += 256) vc[((size_t)(i / g.V) * g.rows + at) * g.V + i % g.V] = pr[g.cv + i];
+  }
+}
+
+}  // namespace crabml_hip

@@ -15,6 +15,21 @@ inline void launch_k(hipStream_t st, crabml_hip_device::ProfRec* rec, K kernel, 
     hipLaunchKernelGGL(kernel, grid, block, (uint32_t)lds, st, args...);
 }
 
+// hipFuncAttributeMaxDynamicSharedMemorySize is a property of the kernel in this PROCESS, not of a context: a second context
+// with a shorter sequence must not lower the limit an earlier context's launches (and captured graphs) were sized for.
+// Only ever raise it, per device.
+inline hipError_t raise_dyn_lds(const crabml_hip_device* dev, const void* fn, int bytes) {
+  static std::mutex mu;
+  static std::map<std::pair<int, const void*>, int> have;
+  if (dev->dry) return hipErrorNoDevice;  // record-only test device
+  std::lock_guard<std::mutex> g(mu);
+  int& cur = have[{dev->ordinal, fn}];
+  if (bytes <= cur) return hipSuccess;
+  const hipError_t e = hipFuncSetAttribute(fn, hipFuncAttributeMaxDynamicSharedMemorySize, bytes);
+  if (e == hipSuccess) cur = bytes;
+  return e;
+}
+
 // ---- quantize.hip: activation quantizers (buf_q8_0.rs:87-134, buf_q8_1.rs:90-129, buf_q8_k.rs:84-131)
 void launch_quantize_act(hipStream_t st, uint32_t qtype, const float* x, size_t n, void* planes);
 void launch_quantize_act_rows(hipStream_t st, uint32_t qtype, const float* x, size_t rows, size_t n, void* planes, void* xh = nullptr,

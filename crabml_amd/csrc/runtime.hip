@@ -41,7 +41,7 @@ WeightLayout weight_layout(uint32_t dtype, size_t n_elems) {
   size_t n = wl.n_blocks;
   switch (dtype) {
     case CRABML_HIP_F32: wl.off_scale = 0; wl.total = n_elems * 4; break;
-    case CRABML_HIP_F16: wl.off_scale = 0; wl.total = n_elems * 2; break;
+    case CRABML_HIP_F16: case CRABML_HIP_BF16: wl.off_scale = 0; wl.total = n_elems * 2; break;
     case CRABML_HIP_Q4_0: wl.off_scale = align_up(n * 16, 256); wl.total = wl.off_scale + n * 2; break;
     case CRABML_HIP_Q8_0: wl.off_scale = align_up(n * 32, 256); wl.total = wl.off_scale + n * 2; break;
     case CRABML_HIP_Q4_1: wl.off_scale = align_up(n * 16, 256); wl.total = wl.off_scale + n * 4; break;
@@ -380,7 +380,7 @@ int crabml_hip_buf_from_cpu(crabml_hip_device_t* dev, const void* bytes, size_t 
   const uint8_t* src = (const uint8_t*)bytes;
   const size_t nblk = wl.n_blocks;
   hipError_t e = hipSuccess;
-  if (t == CRABML_HIP_F32 || t == CRABML_HIP_F16) {
+  if (be == 1) {
     e = hipMemcpyAsync(b->ptr, src, wl.total, hipMemcpyHostToDevice, dev->stream);
     if (e == hipSuccess) e = hipStreamSynchronize(dev->stream);
   } else {

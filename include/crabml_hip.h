@@ -70,7 +70,8 @@ typedef enum crabml_hip_ggml_type {
   CRABML_HIP_Q5_K = 13, /* weights only (rhs: Q8_K), in the REFERENCE's field order qs | qh | scales | d | dmin
                          * (crabml-core/src/cpu/buf/buf_q5_k.rs:13-21) -- not ggml's */
   CRABML_HIP_Q6_K = 14, /* weights only (rhs: Q8_K), crabml-core/src/cpu/buf/buf_q6_k.rs */
-  CRABML_HIP_Q8_K = 15
+  CRABML_HIP_Q8_K = 15,
+  CRABML_HIP_BF16 = 30 /* weights only (rhs: F32 rows as they are); GGML's id of bfloat16 -- the reference has no such type */
 } crabml_hip_ggml_type;
 
 /* crabml-core/src/tensor/api.rs:5-9 */
@@ -276,6 +277,86 @@ int crabml_hip_llama_decode_greedy(crabml_hip_llama_t* ctx, size_t token, size_t
 int crabml_hip_llama_prefill(crabml_hip_llama_t* ctx, const uint32_t* tokens, size_t n, float* logits);
 size_t crabml_hip_llama_kv_len(const crabml_hip_llama_t* ctx);
 int crabml_hip_llama_reset(crabml_hip_llama_t* ctx); /* empties the KV caches */
+/* ---- hybrid decoder: layers that mix softmax attention inside chunks with decaying linear attention ---------------------------
+ * A second step function beside the llama one, for models whose layers are described by what they contain instead of by one fixed
+ * op sequence (the Nilivik design).  bfloat16 weights; norms are RMS norms with a single gain; per layer
+ *   x += attn_out_scale * attention(norm1 x) + lin_out_scale * linear(norm1 x);  x += ff_down xielu(ff_up norm2 x)
+ * where either branch and the feed-forward may be absent.
+ *   attention  grouped queries, score = attn_score_scale q.k - bias_amp ln(1 + bias_rate distance), visible inside chunks of
+ *              attn_chunk positions counted from the sequence's start, a sink logit per head in the softmax's denominator, the
+ *              heads gated by sigmoid(attn_gate norm1 x) before attn_o
+ *   linear     q, k, v through silu; S <- decay S + k v^T, o = S^T q per head; the heads RMS-normed together (lin_norm), gated by
+ *              sigmoid(lin_gate norm1 x) before lin_o
+ * Layers [loop_start, loop_stop) run loop_times times in a row (own state each time); before every pass loop_step[t] is added to x,
+ * before every pass but the first also the embedding output.  Logits are soft-capped.
+ * Any number of sequences is open at a time; each owns one slab of state: min(attn_chunk, seq_len) cache rows and the f32 linear
+ * states of every layer run.  A step takes the next tokens of several sequences as one batch: one token each runs as the decode
+ * step (five launches per layer from a hipGraph), anything else as passes of up to pass_rows rows.
+ * compute = CRABML_HIP_BF16: matrix products of bf16 activations with f32 accumulation, bf16 cache (norms, scores, softmax, the
+ * linear states and the residual are f32 all the same); CRABML_HIP_F32: every activation, product and cache entry f32. */
+typedef struct crabml_hip_hybrid crabml_hip_hybrid_t;
+#define CRABML_HIP_HYBRID_NO_GRAPH 1 /* launch decode steps eagerly */
+typedef struct crabml_hip_hybrid_config {
+  size_t width, vocab_size, n_layers;
+  size_t loop_start, loop_stop, loop_times; /* loop_times == 0: no loop */
+  size_t seq_len;   /* longest sequence */
+  size_t pass_rows; /* rows per prompt pass (0 = default: 2048) */
+  float embed_scale, norm_eps;
+  float logit_softcap; /* 0 = none */
+  uint32_t compute;    /* CRABML_HIP_BF16 or CRABML_HIP_F32 */
+  int32_t flags;
+} crabml_hip_hybrid_config_t;
+typedef struct crabml_hip_hybrid_layer { /* heads == 0: the branch is absent; ff == 0: no feed-forward */
+  size_t attn_heads, attn_kv_heads, attn_dim, attn_vdim;
+  size_t attn_chunk; /* 0 = unlimited */
+  size_t lin_heads, lin_dim, lin_vdim;
+  size_t ff;
+  float attn_score_scale, attn_out_scale, lin_out_scale;
+  const double* lin_decay; /* host memory, lin_heads */
+  const crabml_hip_buf_t* norm1; /* 1 */
+  const crabml_hip_buf_t* attn_q;
+  const crabml_hip_buf_t* attn_k;
+  const crabml_hip_buf_t* attn_v;
+  const crabml_hip_buf_t* attn_gate;
+  const crabml_hip_buf_t* attn_o;
+  const crabml_hip_buf_t* attn_bias_amp;  /* attn_heads; NULL (both) = no distance bias */
+  const crabml_hip_buf_t* attn_bias_rate;
+  const crabml_hip_buf_t* attn_sink; /* attn_heads; NULL = no sink */
+  const crabml_hip_buf_t* lin_q;
+  const crabml_hip_buf_t* lin_k;
+  const crabml_hip_buf_t* lin_v;
+  const crabml_hip_buf_t* lin_gate;
+  const crabml_hip_buf_t* lin_o;
+  const crabml_hip_buf_t* lin_norm; /* lin_heads * lin_vdim */
+  const crabml_hip_buf_t* norm2;    /* 1 */
+  const crabml_hip_buf_t* ff_up;
+  const crabml_hip_buf_t* ff_down;
+  const crabml_hip_buf_t* ff_act; /* 2: the raw numbers of xIELU, before their softplus */
+} crabml_hip_hybrid_layer_t;
+typedef struct crabml_hip_hybrid_weights {
+  const crabml_hip_buf_t* embed;      /* (vocab_size, width) */
+  const crabml_hip_buf_t* loop_step;  /* (loop_times, width) */
+  const crabml_hip_buf_t* final_norm; /* 1 */
+  const crabml_hip_buf_t* head;       /* (vocab_size, width) */
+} crabml_hip_hybrid_weights_t;
+/* Matrices are copied into the layout the kernels read (branches' projections as one matrix, head widths padded): the caller may
+ * release its buffers afterwards. */
+int crabml_hip_hybrid_create(crabml_hip_device_t* dev, const crabml_hip_hybrid_config_t* cfg, const crabml_hip_hybrid_layer_t* layers,
+                             const crabml_hip_hybrid_weights_t* w, crabml_hip_hybrid_t** out);
+int crabml_hip_hybrid_destroy(crabml_hip_hybrid_t* ctx);
+/* sequences: opened empty, closed (their slab goes to the next one opened), asked for their length in tokens */
+int crabml_hip_hybrid_open(crabml_hip_hybrid_t* ctx, size_t* seq);
+int crabml_hip_hybrid_close(crabml_hip_hybrid_t* ctx, size_t seq);
+size_t crabml_hip_hybrid_len(const crabml_hip_hybrid_t* ctx, size_t seq);
+size_t crabml_hip_hybrid_slab_bytes(const crabml_hip_hybrid_t* ctx);
+/* the next counts[i] >= 1 tokens of seqs[i], concatenated in tokens; want: for each sequence want_counts[i] places among its new
+ * tokens, ascending, whose logits are written one row of vocab_size after the other.  BLOCKS if anything is wanted. */
+int crabml_hip_hybrid_step(crabml_hip_hybrid_t* ctx, size_t n, const size_t* seqs, const size_t* counts, const uint32_t* tokens,
+                           const size_t* want_counts, const uint32_t* want, float* logits);
+/* n_steps greedy steps (last maximum) of n <= 16 sequences, tokens[i] being the next token of seqs[i]; out_tokens: n_steps rows of n.
+ * BLOCKS once, at the end. */
+int crabml_hip_hybrid_decode_greedy(crabml_hip_hybrid_t* ctx, size_t n, const size_t* seqs, const uint32_t* tokens, size_t n_steps,
+                                    uint32_t* out_tokens);
 /* ---- tensor-parallel group over RCCL / xGMI (one process per GPU) ----
  * crabml_hip_tp_get_unique_id fills a 128-byte ncclUniqueId on rank 0; the host broadcasts it (any side channel)
  * and every rank calls crabml_hip_tp_comm_create.  librccl is bound with dlopen on first use. */

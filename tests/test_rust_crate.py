@@ -113,7 +113,8 @@ def test_ffi_declares_exactly_the_functions_of_the_header():
 def test_repr_c_structs_match_the_header():
     _, hs = parse_header()
     _, fs = parse_ffi()
-    for name in ("crabml_hip_device_options_t", "crabml_hip_llama_config_t", "crabml_hip_llama_weights_t"):
+    for name in ("crabml_hip_device_options_t", "crabml_hip_llama_config_t", "crabml_hip_llama_weights_t", "crabml_hip_hybrid_config_t",
+                 "crabml_hip_hybrid_layer_t", "crabml_hip_hybrid_weights_t"):
         assert name in hs and name in fs, name
         assert [f[0] for f in hs[name]] == [f[0] for f in fs[name]], name
         for (hn, ht), (fn, ft) in zip(hs[name], fs[name]):
@@ -172,7 +173,7 @@ def test_hip_tensor_implements_every_method_of_the_tensor_trait():
     assert "type DeviceRef = HipTensorDeviceRef;" in body
     # no elided bodies: every method ends in real code
     assert "/* ..." not in rs and "todo!" not in rs and "unimplemented!" not in rs
-    for f in ("Cargo.toml", "build.rs", "src/lib.rs", "src/ffi.rs", "src/hip_device.rs", "src/hip_tensor.rs", "src/hip_llama.rs"):
+    for f in ("Cargo.toml", "build.rs", "src/lib.rs", "src/ffi.rs", "src/hip_device.rs", "src/hip_tensor.rs", "src/hip_llama.rs", "src/hip_hybrid.rs"):
         assert os.path.getsize(os.path.join(CRATE, f)) > 200, f
 
 
