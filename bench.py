@@ -59,6 +59,14 @@ def _pmc_traffic():
         return None
 
 
+# --hybrid: layer sizes of real models; the llama beside it has the same width, heads, feed-forward, vocabulary and layer count
+HYBRID_SIZES = {
+    "2k": dict(width=2048, heads=16, kv_heads=4, dim=128, lin_heads=16, lin_dim=64, lin_vdim=128, ff=8192, vocab=32000, layers=8),
+    "4k": dict(width=4096, heads=32, kv_heads=8, dim=128, lin_heads=16, lin_dim=128, lin_vdim=128, ff=14336, vocab=128256, layers=4),
+}
+MFMA_PEAK_TFLOPS = 2500.0  # dense bf16 / f16
+
+
 def parse():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -105,6 +113,9 @@ def parse():
                     help="skip the 128-step run over positions 0..127 (rocprofv3 --kernel-trace segfaults inside the tracer on 128 "
                          "back-to-back graph launches; tools/gpu_profile.sh passes this)")
     ap.add_argument("--no-gemv-points", action="store_true", help="skip the single-kernel GEMV points (SURVEY.md 8d)")
+    ap.add_argument("--hybrid", nargs="?", const="all", default=None, choices=["all"] + sorted(HYBRID_SIZES),
+                    help="instead of the BASELINE workload: prompt and decode throughput and per-kernel roofline fractions of the hybrid "
+                         "decoder (Nilivik design, random weights) at layer sizes of real models, beside a llama of the same widths")
     ap.add_argument("--selftest-dist", action="store_true", help="CPU/gloo self test of the rank aggregation")
     return ap.parse_args()
 
@@ -451,6 +462,146 @@ def tp_dry_run(args, ca, synth, local):
     }))
 
 
+def hybrid_bench(args, ca, synth, local):
+    """Prompt and decode throughput of the hybrid decoder at HYBRID_SIZES, per-kernel times (dispatch-timestamp events) against their
+    rooflines (weight bytes / HBM peak for the decode linears, flops / MFMA peak for the prompt linears), and the llama of the same
+    widths on its own fused step and prompt pass (Q4_0) and on 16-bit weights (F16)."""
+    import shutil
+    import tempfile
+
+    from crabml_amd import synth_hybrid as sh
+
+    dev = ca.HipTensorDevice(device_ordinal=local)
+    names = {1: "in", 2: "mix", 3: "out", 4: "up", 5: "down", 6: "head", 7: "linear", 8: "rows"}
+    ctx, chunk, prompt = 1024, 2048, 2048
+
+    def timed(fn, reps=3):
+        best = 1e9
+        for _ in range(reps):
+            dev.sync()
+            t0 = time.perf_counter()
+            fn()
+            dev.sync()
+            best = min(best, time.perf_counter() - t0)
+        return best
+
+    result = {}
+    for size in sorted(HYBRID_SIZES) if args.hybrid == "all" else [args.hybrid]:
+        z = HYBRID_SIZES[size]
+        W, V, L, ff = z["width"], z["vocab"], z["layers"], z["ff"]
+        conf = sh.config(W, V, [sh.layer(z["heads"], z["kv_heads"], z["dim"], z["dim"], chunk, z["lin_heads"], z["lin_dim"], z["lin_vdim"], ff)] * L)
+        folder = tempfile.mkdtemp(prefix="hybrid-")
+        try:
+            sh.write_model(conf, sh.random_tensors(conf, 8, pool=1 << 22), folder)
+            r = ca.load_model(folder, dev, seq_len=4096)
+        finally:
+            shutil.rmtree(folder)
+        print("# hybrid %s loaded" % size, file=sys.stderr, flush=True)
+        n_in = z["dim"] * 2 * (z["heads"] + z["kv_heads"]) + 2 * z["lin_heads"] * (z["lin_dim"] + z["lin_vdim"])
+        k_o = z["heads"] * z["dim"] + z["lin_heads"] * z["lin_vdim"]
+        weights = {"in": n_in * W, "out": W * k_o, "up": ff * W, "down": ff * W, "head": V * W}
+        toks = [int(t) for t in (7 * np_arange(prompt + 1) + 3) % V]
+
+        def prefill(n_seq, n):
+            seqs = [r.open() for _ in range(n_seq)]
+            r.step([(s, toks[:n], [n - 1] if s == seqs[-1] else []) for s in seqs])
+            for s in seqs:
+                r.close(s)
+
+        out = {"layers": L, "layer_params": sum(v for k, v in weights.items() if k != "head"), "prompt": {}, "decode": {}}
+        for n_seq, n in ((1, 512), (1, prompt), (4, 512)):
+            prefill(n_seq, n)
+            t = timed(lambda: prefill(n_seq, n))
+            flops = 2.0 * n_seq * n * (L * out["layer_params"]) + 2.0 * V * W
+            out["prompt"]["%dx%d" % (n_seq, n)] = {"ms": round(t * 1e3, 3), "tokens_per_s": round(n_seq * n / t), "linear_tflops": round(flops / t / 1e12, 1)}
+        for B in (1, 4, 8, 16):
+            seqs = [r.open() for _ in range(B)]
+            for s in seqs:
+                r.step([(s, toks[:ctx], [])])
+            r.decode_batch(seqs, [1] * B, 4)
+            t = timed(lambda: r.decode_batch(seqs, [1] * B, args.steps)) / args.steps
+            byts = 2.0 * (L * out["layer_params"] + V * W)
+            out["decode"]["b%d" % B] = {"us_per_step": round(t * 1e6, 1), "tokens_per_s": round(B / t, 1), "weight_frac_of_hbm": round(byts / t / 1e9 / HBM_PEAK_GBS, 3)}
+            for s in seqs:
+                r.close(s)
+        # per kernel
+        dev.prof_enable(True)
+        s = r.open()
+        r.step([(s, toks[:ctx], [])])
+        dev.prof_read()
+        r.decode_batch([s], [1], 8)
+        kern = {}
+        for x in dev.prof_read():
+            us, nm = x["kernel_ms"] * 1e3 / x["launches"], names[x["stage"] % 10]
+            kern["decode_" + nm] = {"us": round(us, 2)}
+            if x["algo_bytes"]:
+                kern["decode_" + nm]["frac_of_hbm"] = round(x["algo_bytes"] / x["launches"] / us / 1e3 / HBM_PEAK_GBS, 3)
+        r.close(s)
+        s = r.open()
+        r.step([(s, toks[:prompt], [])])
+        for x in dev.prof_read():
+            us, nm = x["kernel_ms"] * 1e3 / x["launches"], names[x["stage"] % 10]
+            kern["prompt_" + nm] = {"us": round(us, 2)}
+            if nm in weights:
+                kern["prompt_" + nm]["frac_of_mfma"] = round(2.0 * prompt * weights[nm] / us / 1e6 / MFMA_PEAK_TFLOPS, 3)
+            elif nm == "mix":  # causal halves of q k and p v
+                kern["prompt_mix"]["frac_of_mfma"] = round(2.0 * prompt * (prompt / 2) * 2 * z["dim"] * z["heads"] / us / 1e6 / MFMA_PEAK_TFLOPS, 3)
+        r.close(s)
+        dev.prof_enable(False)
+        out["kernels"] = kern
+        del r
+        # the llama of the same widths
+        shape = synth.ModelShape("llama-" + size, W, ff, L, z["heads"], z["kv_heads"], V, 4096, 1e-5, None)
+        for fmt in ("Q4_0", "F16"):
+            m = synth.build_model(shape, synth.TYPE_BY_NAME[fmt], seed=8)
+            lconf, lw = synth.to_hip(m, dev)
+            byts = sum(t.data.nbytes for name, t in m.tensors.items() if not name.endswith("_norm.weight") and name != "token_embd.weight")
+            params = sum(int(t.shape[0]) * int(t.shape[1]) for name, t in m.tensors.items() if name.startswith("blk.") and len(t.shape) == 2)
+            lr = ca.HipLlamaRunner(lconf, lw, dev, 4096, True)
+            lo = {}
+            for n in (512, prompt):
+                if fmt == "F16" and n > 512:
+                    continue
+
+                def pf():
+                    lr.reset()
+                    lr.prefill(toks[:n])
+
+                pf()
+                t = timed(pf)
+                lo["prompt_1x%d" % n] = {"ms": round(t * 1e3, 3), "tokens_per_s": round(n / t), "linear_tflops": round((2.0 * n * params + 2.0 * V * W) / t / 1e12, 1)}
+            lr.reset()
+            lr.prefill(toks[:min(ctx, 512 if fmt == "F16" else ctx)])
+            lr.decode_greedy(1, 4)
+            t = timed(lambda: lr.decode_greedy(1, args.steps)) / args.steps
+            lo["decode_b1"] = {"us_per_step": round(t * 1e6, 1), "tokens_per_s": round(1 / t, 1), "weight_frac_of_hbm": round(byts / t / 1e9 / HBM_PEAK_GBS, 3)}
+            le = ca.HipLlamaRunner(lconf, lw, dev, 4096, True, use_graph=False)
+            le.prefill(toks[:64])
+            dev.prof_enable(True)
+            le.decode_greedy(1, 8)
+            stage = {1: "qkv", 2: "wo", 3: "gate|up", 4: "ffn_down", 5: "classifier", 7: "attention"}
+            lo["kernels"] = {}
+            for x in dev.prof_read():
+                us = x["kernel_ms"] * 1e3 / x["launches"]
+                k = {"us": round(us, 2)}
+                if x["algo_bytes"]:
+                    k["frac_of_hbm"] = round(x["algo_bytes"] / x["launches"] / us / 1e3 / HBM_PEAK_GBS, 3)
+                lo["kernels"][stage.get(x["stage"], str(x["stage"]))] = k
+            dev.prof_enable(False)
+            out["llama_" + fmt] = lo
+            del lr, le, lw
+            print("# llama %s %s done" % (size, fmt), file=sys.stderr, flush=True)
+        result[size] = out
+    print(json.dumps({"metric": "hybrid decoder throughput (not the BASELINE workload)", "dtype": "bf16", "data": "synthetic", "chunk": chunk,
+                      "decode_position": ctx, "steps": args.steps, "sizes": result}))
+
+
+def np_arange(n):
+    import numpy as np
+
+    return np.arange(n, dtype=np.int64)
+
+
 def tp_group_run(args, ca, synth, dist, rank, world, local):
     """--tp under torchrun: one tensor-parallel group over all ranks.  Every rank
     builds the LOCAL shard shapes with the same seed (identical bytes on every rank: a consistent model whose shards
@@ -613,6 +764,8 @@ def main():
 
     if args.tp_dry > 1:
         return tp_dry_run(args, ca, synth, local)
+    if args.hybrid:
+        return hybrid_bench(args, ca, synth, local)
     if args.tp and world > 1:
         rc = tp_group_run(args, ca, synth, dist, rank, world, local)
         if rc:
