@@ -47,6 +47,16 @@ __device__ __forceinline__ void split_store(float v, unsigned short* p, size_t p
   }
 }
 
+// four neighbouring columns at once (p: 8-byte aligned)
+template <int P>
+__device__ __forceinline__ void split_store4(const float (&v)[4], unsigned short* p, size_t plane_stride) {
+  unsigned short t[P][4];
+#pragma unroll
+  for (int e = 0; e < 4; e++) split_store<P>(v[e], &t[0][e], 4);
+#pragma unroll
+  for (int i = 0; i < P; i++) __builtin_memcpy(p + i * plane_stride, t[i], 8);
+}
+
 struct GemmBf16 {
   const unsigned short* a = nullptr;  // [planes][rows padded][k]
   size_t a_plane = 0;                 // elements between planes

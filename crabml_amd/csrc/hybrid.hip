@@ -337,12 +337,11 @@ int enqueue_step(Ctx* c, int B, bool sample, bool prof) {
     }
     {
       const MixStep m = mix_step(c, run, B);
-      const unsigned grid = (unsigned)(B * (L.at.H ? L.at.G * L.head_blocks * L.splits : 0) + B * (L.li.H ? L.li.H * L.li.slices : 0));
       Prof p(dev, prof, ST_STEP + ST_MIX, 0.0);
       if (c->f32)
-        launch_k(st, p.rec(), k_mix_step<float>, dim3(grid), dim3(256), mix_step_lds(m), m);
+        launch_mix_step<float>(st, p.rec(), m);
       else
-        launch_k(st, p.rec(), k_mix_step<unsigned short>, dim3(grid), dim3(256), mix_step_lds(m), m);
+        launch_mix_step<unsigned short>(st, p.rec(), m);
     }
     {
       GemvBf16 g;
@@ -463,14 +462,18 @@ int pass_alloc(Ctx* c) {
   CH_TRY(dalloc_n(c, P * LOGIT_ROWS * c->ldx, &c->pf_gp));
   CH_TRY(dalloc_n(c, LOGIT_ROWS * c->n_sq, &c->pf_gsq));
   CH_TRY(dalloc_n(c, LOGIT_ROWS * c->vocab, &c->pf_logits));
-  // seqs | tiles (a tile is at least one row) | rows | tokens | wanted rows
-  c->meta_bytes = R * (sizeof(PassSeq) + sizeof(PassTile) + sizeof(PassRow) + 2 * sizeof(int));
+  // seqs | tiles, small and big (a tile is at least one row) | rows | tokens | wanted rows
+  c->meta_bytes = R * (sizeof(PassSeq) + 2 * sizeof(PassTile) + sizeof(PassRow) + 2 * sizeof(int));
   CH_TRY(dalloc(c, c->meta_bytes, (void**)&c->meta));
   CH_HIP(dev, hipHostMalloc((void**)&c->h_meta, c->meta_bytes * META_SLOTS, hipHostMallocDefault));
   c->rows_cap = R;
   return 0;
 }
 
+struct PassTiles {  // query tiles of 64 and of 128 rows
+  const PassTile* list[2];
+  size_t n[2];
+};
 struct Part {  // rows of one sequence in one pass
   size_t seq, n;
   const uint32_t* tokens;
@@ -478,7 +481,10 @@ struct Part {  // rows of one sequence in one pass
 };
 
 template <typename T, int CLS>
-void launch_attn_cls(Ctx* c, crabml_hip_device::ProfRec* rec, const MixRows<T>& m) {
+void launch_attn_cls(Ctx* c, crabml_hip_device::ProfRec* rec, MixRows<T> m, const PassTiles& tiles) {
+  constexpr int big = AttnTile<T, CLS>::RT - 1;
+  m.tiles = tiles.list[big];
+  m.n_tiles = (int)tiles.n[big];
   launch_k(c->dev->stream, rec, k_attn_rows<T, CLS, sizeof(T) == 2 ? 1 : 3>, dim3(m.n_tiles, m.at.H), dim3(256), 0, m);
 }
 template <typename T, int CLS>
@@ -490,7 +496,7 @@ int launch_linear_cls(Ctx* c, crabml_hip_device::ProfRec* rec, const MixRows<T>&
 }
 
 template <typename T>
-int mix_rows(Ctx* c, const Run& run, const PassSeq* seqs, size_t n_seq, const PassTile* tiles, size_t n_tiles, const PassRow* rows, size_t n_rows) {
+int mix_rows(Ctx* c, const Run& run, const PassSeq* seqs, size_t n_seq, const PassTiles& tiles, const PassRow* rows, size_t n_rows) {
   constexpr int P = sizeof(T) == 2 ? 1 : 3;
   const Layer& L = c->layers[run.layer];
   MixRows<T> m;
@@ -498,13 +504,11 @@ int mix_rows(Ctx* c, const Run& run, const PassSeq* seqs, size_t n_seq, const Pa
   m.li = L.li;
   m.rs = run.rs;
   m.seqs = seqs;
-  m.tiles = tiles;
   m.rows = rows;
   m.proj = (const T*)c->pf_proj;
   m.cat = c->pf_cat;
   m.cat_plane = c->rows_cap * (size_t)c->ld_cat;
   m.lin = c->pf_lin;
-  m.n_tiles = (int)n_tiles;
   m.ldp = L.n_in;
   m.ldc = L.ldc;
   m.lin_off = L.lin_off;
@@ -512,11 +516,11 @@ int mix_rows(Ctx* c, const Run& run, const PassSeq* seqs, size_t n_seq, const Pa
     Prof p(c->dev, true, ST_PASS + ST_MIX, 0.0);
     const int w = std::max(L.at.D, L.at.V);
     if (w <= 64)
-      launch_attn_cls<T, 64>(c, p.rec(), m);
+      launch_attn_cls<T, 64>(c, p.rec(), m, tiles);
     else if (w <= 128)
-      launch_attn_cls<T, 128>(c, p.rec(), m);
+      launch_attn_cls<T, 128>(c, p.rec(), m, tiles);
     else
-      launch_attn_cls<T, 256>(c, p.rec(), m);
+      launch_attn_cls<T, 256>(c, p.rec(), m, tiles);
   }
   if (L.li.H) {
     Prof p(c->dev, true, ST_PASS + ST_LIN, 0.0);
@@ -543,17 +547,19 @@ int run_pass(Ctx* c, const std::vector<Part>& parts, float** logits) {
   }
   const size_t R = c->rows_cap;
   char* hm = c->h_meta + c->meta_bytes * c->h_meta_next++;
-  const size_t o_tile = R * sizeof(PassSeq), o_row = o_tile + R * sizeof(PassTile), o_tok = o_row + R * sizeof(PassRow), o_want = o_tok + R * sizeof(int);
+  const size_t o_tile = R * sizeof(PassSeq), o_row = o_tile + 2 * R * sizeof(PassTile), o_tok = o_row + R * sizeof(PassRow), o_want = o_tok + R * sizeof(int);
   PassSeq* hs = (PassSeq*)hm;
-  PassTile* ht = (PassTile*)(hm + o_tile);
+  PassTile* ht[2] = {(PassTile*)(hm + o_tile), (PassTile*)(hm + o_tile) + R};
   PassRow* hr = (PassRow*)(hm + o_row);
   int *hk = (int*)(hm + o_tok), *hw = (int*)(hm + o_want);
-  size_t n_tiles = 0, M = 0, nw = 0;
+  size_t n_tiles[2] = {0, 0}, M = 0, nw = 0;
   for (size_t i = 0; i < parts.size(); i++) {
     const Part& p = parts[i];
     const Seq& s = c->seqs[p.seq];
     hs[i] = PassSeq{(int)M, (int)p.n, (int)s.len, 0, s.slab};
-    for (size_t r = 0; r < p.n; r += 64) ht[n_tiles++] = PassTile{(int)i, (int)(M + r), (int)(s.len + r), (int)std::min<size_t>(64, p.n - r)};
+    for (size_t b = 0; b < 2; b++)
+      for (size_t r = 0; r < p.n; r += 64 << b)
+        ht[b][n_tiles[b]++] = PassTile{(int)i, (int)(M + r), (int)(s.len + r), (int)std::min<size_t>(64 << b, p.n - r)};
     for (int w : p.want) hw[nw++] = (int)M + w;
     for (size_t r = 0; r < p.n; r++) {
       hr[M + r] = PassRow{(int)i, (int)(s.len + r)};
@@ -563,7 +569,7 @@ int run_pass(Ctx* c, const std::vector<Part>& parts, float** logits) {
   }
   CH_HIP(dev, hipMemcpyAsync(c->meta, hm, c->meta_bytes, hipMemcpyHostToDevice, st));
   const PassSeq* ds = (const PassSeq*)c->meta;
-  const PassTile* dt = (const PassTile*)(c->meta + o_tile);
+  const PassTiles dt = {{(const PassTile*)(c->meta + o_tile), (const PassTile*)(c->meta + o_tile) + R}, {n_tiles[0], n_tiles[1]}};
   const PassRow* dr = (const PassRow*)(c->meta + o_row);
   const int *dk = (const int*)(c->meta + o_tok), *dw = (const int*)(c->meta + o_want);
   const size_t xp = R * (size_t)c->ldx;
@@ -621,9 +627,9 @@ int run_pass(Ctx* c, const std::vector<Part>& parts, float** logits) {
       launch_gemm_bf16(dev, p.rec(), c->planes, c->f32 ? GEMM_OUT_ACT_F32 : GEMM_OUT_ACT_BF16, g);
     }
     if (c->f32)
-      CH_TRY(mix_rows<float>(c, run, ds, parts.size(), dt, n_tiles, dr, M));
+      CH_TRY(mix_rows<float>(c, run, ds, parts.size(), dt, dr, M));
     else
-      CH_TRY(mix_rows<unsigned short>(c, run, ds, parts.size(), dt, n_tiles, dr, M));
+      CH_TRY(mix_rows<unsigned short>(c, run, ds, parts.size(), dt, dr, M));
     {
       GemmBf16 g = residual(c->pf_cat, R * (size_t)c->ld_cat, L.w_o, L.ldc);
       if (!L.ff) {
@@ -720,8 +726,6 @@ int create_impl(Ctx* c, const crabml_hip_hybrid_layer_t* layers, const crabml_hi
       tick = std::max(tick, slots);
     }
     ss = std::max(ss, (size_t)HYB_STEP_ROWS * L.li.H * L.li.slices);
-    if (mix_step_lds(mix_step(c, Run{(int)i, RunState{}, false, nullptr}, 1)) > 60 * 1024)
-      CH_BAIL(dev, CRABML_HIP_NOT_IMPLEMENTED, "hybrid: layer %zu keeps %d cache rows, too many for the decode step's merge", i, L.at.rows);
   }
   // the order of layer runs, and each run's place in a sequence's slab
   auto add_run = [&](size_t layer, bool first, size_t t) {

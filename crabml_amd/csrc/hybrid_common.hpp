@@ -36,6 +36,49 @@ __device__ __forceinline__ void kv_load8(const unsigned short* p, float (&o)[8])
   }
 }
 
+template <typename T>
+struct Oct {  // eight elements on their way from memory to LDS
+  i32x4 d[sizeof(T) / 2];
+};
+template <typename T>
+__device__ __forceinline__ Oct<T> oct_zero() {
+  Oct<T> o;
+#pragma unroll
+  for (unsigned i = 0; i < sizeof(T) / 2; i++) o.d[i] = i32x4{0, 0, 0, 0};
+  return o;
+}
+template <typename T>
+__device__ __forceinline__ Oct<T> oct_load(const T* p) {
+  Oct<T> o;
+#pragma unroll
+  for (unsigned i = 0; i < sizeof(T) / 2; i++) o.d[i] = ((const i32x4*)p)[i];
+  return o;
+}
+template <typename T>
+__device__ __forceinline__ void oct_store(T* p, const Oct<T>& o) {
+#pragma unroll
+  for (unsigned i = 0; i < sizeof(T) / 2; i++) ((i32x4*)p)[i] = o.d[i];
+}
+template <typename T>
+__device__ __forceinline__ void oct_scatter(T* p, int stride, const Oct<T>& o) {  // element e -> p[e * stride]
+  T v[8];
+  __builtin_memcpy(v, &o, sizeof v);
+#pragma unroll
+  for (int e = 0; e < 8; e++) p[e * stride] = v[e];
+}
+template <typename T>
+__device__ __forceinline__ void oct_floats(const Oct<T>& o, float (&f)[8]) {
+  if constexpr (sizeof(T) == 4) {
+    __builtin_memcpy(f, &o, sizeof f);
+  } else {
+#pragma unroll
+    for (int e = 0; e < 4; e++) {
+      f[2 * e] = __builtin_bit_cast(float, (unsigned)o.d[0][e] << 16);
+      f[2 * e + 1] = __builtin_bit_cast(float, (unsigned)o.d[0][e] & 0xffff0000u);
+    }
+  }
+}
+
 // One layer's mixers.  Head widths are padded to multiples of 8 (zero weight rows make the padding zero), so every head starts on a
 // 16-byte boundary of its row; D / V / ... below are the padded widths.
 struct AttnGeom {

@@ -20,7 +20,7 @@ struct PassSeq {
 struct PassRow {
   int seq, pos;
 };
-struct PassTile {  // up to 64 consecutive rows of one sequence
+struct PassTile {  // up to 64 (times AttnTile::RT) consecutive rows of one sequence
   int seq, row, pos, n;
 };
 
@@ -102,37 +102,6 @@ __device__ __forceinline__ f32x4 mma_rows_w(const float* a, const float* w, cons
   return acc;
 }
 
-template <typename T>
-struct Oct {  // eight elements on their way from memory to LDS
-  i32x4 d[sizeof(T) / 2];
-};
-template <typename T>
-__device__ __forceinline__ Oct<T> oct_zero() {
-  Oct<T> o;
-#pragma unroll
-  for (unsigned i = 0; i < sizeof(T) / 2; i++) o.d[i] = i32x4{0, 0, 0, 0};
-  return o;
-}
-template <typename T>
-__device__ __forceinline__ Oct<T> oct_load(const T* p) {
-  Oct<T> o;
-#pragma unroll
-  for (unsigned i = 0; i < sizeof(T) / 2; i++) o.d[i] = ((const i32x4*)p)[i];
-  return o;
-}
-template <typename T>
-__device__ __forceinline__ void oct_store(T* p, const Oct<T>& o) {
-#pragma unroll
-  for (unsigned i = 0; i < sizeof(T) / 2; i++) ((i32x4*)p)[i] = o.d[i];
-}
-template <typename T>
-__device__ __forceinline__ void oct_scatter(T* p, int stride, const Oct<T>& o) {  // element e -> p[e * stride]
-  T v[8];
-  __builtin_memcpy(v, &o, sizeof v);
-#pragma unroll
-  for (int e = 0; e < 8; e++) p[e * stride] = v[e];
-}
-
 // ---- embedding of the pass's rows: x, its planes, its square sum (piece 0; the others are cleared) --------------------------------
 template <int P>
 __global__ __launch_bounds__(256) void k_embed_rows(const unsigned short* __restrict__ table, const int* __restrict__ tokens,
@@ -199,149 +168,231 @@ struct MixRows {
   int n_tiles = 0, ldp = 0, ldc = 0, lin_off = 0;
 };
 
-template <typename T>
+// Shape of the attention kernel for heads up to CLS wide: KT keys per tile; RT times 16 query rows per wave.
+template <typename T, int CLS>
 struct AttnTile {
-  static constexpr int PAD = 16 / sizeof(T);
-  template <int CLS>
-  static constexpr int keys() {
-    return (sizeof(T) == 2 ? 64 : 32) / (CLS > 128 ? 2 : 1);
-  }
+  static constexpr int PAD = 16 / sizeof(T), KT = sizeof(T) == 2 ? (CLS > 128 ? 32 : 64) : 4096 / CLS;
+  static constexpr int RT = sizeof(T) == 2 && CLS <= 128 ? 2 : 1;
 };
 
-// CLS: head widths up to this many elements.  Four waves of 16 query rows; keys in tiles of KT through LDS (K as rows, V transposed).
+// One workgroup: 64 RT query rows of one head, four waves of 16 RT.  Keys come in tiles through LDS (K as rows, V transposed), the next
+// tile's rows already on their way into registers while the current one is multiplied.
+// Everything is transposed -- S^T = K Q^T, O^T = V^T P^T -- so that a lane owns one query row (its column): the softmax statistics are
+// one number per lane, and the accumulators of S^T, exponentiated, ARE the operand of the second product: k slot (lane / 16, i) of the
+// matrix instruction stands for key 4 (lane / 16) + i of a 16-key group, and V^T is read from LDS in the same order.  Scores live in
+// the log2 domain.
 template <typename T, int CLS, int P>
-__global__ __launch_bounds__(256) void k_attn_rows(const MixRows<T> a) {
-  constexpr int KT = AttnTile<T>::template keys<CLS>(), PAD = AttnTile<T>::PAD, LK = CLS + PAD, LV = KT + PAD, VT = CLS / 16, ST = KT / 16;
+__global__ __launch_bounds__(256, sizeof(T) == 2 ? 2 : 1) void k_attn_rows(const MixRows<T> a) {
+  typedef AttnTile<T, CLS> A;
+  constexpr int KT = A::KT, RT = A::RT, LK = CLS + A::PAD, LV = KT + A::PAD, VT = CLS / 16, ST = KT / 16;
+  constexpr int NK = KT * CLS / 8 / 256;  // octets of K (and of V) per thread and tile
+  static_assert(NK >= 1 && NK % 2 == 0, "V octets are handled in pairs of keys");
   __shared__ __attribute__((aligned(16))) T ks[KT * LK];
   __shared__ __attribute__((aligned(16))) T vs[CLS * LV];
-  __shared__ __attribute__((aligned(16))) T ps[4 * 16 * LV];
   const AttnGeom& g = a.at;
   const int tid = threadIdx.x, lane = tid & 63, wave = wave_in_wg(), fr = lane & 15, fk = lane >> 4;
-  const PassTile t = a.tiles[blockIdx.x];
+  const PassTile t = a.tiles[a.n_tiles - 1 - blockIdx.x];  // (a sequence's last tiles see the most keys: first)
   const PassSeq sq = a.seqs[t.seq];
   const int h = blockIdx.y, kvh = h / (g.H / g.G);
   const int DK = (g.D + 31) & ~31;
+  const int lo = t.pos - t.pos % g.chunk, hi = t.pos + t.n;  // keys [lo, hi); those before pos0 are cache rows from `lo` on
   const T* kc = (const T*)(sq.slab + a.rs.k) + (size_t)kvh * g.rows * g.D;
   const T* vc = (const T*)(sq.slab + a.rs.v) + (size_t)kvh * g.rows * g.V;
-  const T* proj_seq = a.proj + (size_t)sq.row0 * a.ldp;  // row of position p: + (p - pos0) * ldp
-  // this lane's query row (A operand) and its four output rows
-  const int qrow = wave * 16 + fr;
-  const T* qp = a.proj + (size_t)(t.row + (qrow < t.n ? qrow : t.n - 1)) * a.ldp + g.cq + h * g.D;
-  bf16x8 q16[sizeof(T) == 2 ? CLS / 32 : 1];
-  float q32[sizeof(T) == 4 ? CLS / 4 : 1];
-  if constexpr (sizeof(T) == 2) {
+  const T* pk = a.proj + (size_t)sq.row0 * a.ldp + g.ck + kvh * g.D;
+  const T* pv = a.proj + (size_t)sq.row0 * a.ldp + g.cv + kvh * g.V;
+  // this wave's rows, and the keys any of them sees
+  const int w0 = wave * 16 * RT, wn = min(16 * RT, t.n - w0);
+  const int wfirst = t.pos + w0, wlast = wfirst + wn - 1, wlo = wfirst - wfirst % g.chunk, whi_chunk = wlast - (wlast > 0 ? wlast % g.chunk : 0);
+  bf16x8 q16[RT][sizeof(T) == 2 ? CLS / 32 : 1];
+  float q32[RT][sizeof(T) == 4 ? CLS / 4 : 1];
+  int pos[RT], first[RT];
 #pragma unroll
-    for (int i = 0; i < CLS / 32; i++) {
-      const int k = i * 32 + fk * 8;
-      const Oct<T> o = k < g.D ? oct_load(qp + k) : oct_zero<T>();
-      __builtin_memcpy(&q16[i], &o, 16);
+  for (int r = 0; r < RT; r++) {
+    const int row = w0 + r * 16 + fr;
+    const T* qp = a.proj + (size_t)(t.row + (row < t.n ? row : t.n - 1)) * a.ldp + g.cq + h * g.D;
+    pos[r] = t.pos + row;
+    first[r] = pos[r] - pos[r] % g.chunk;
+    if constexpr (sizeof(T) == 2) {
+#pragma unroll
+      for (int i = 0; i < CLS / 32; i++) {
+        const int k = i * 32 + fk * 8;
+        const Oct<T> o = k < g.D ? oct_load(qp + k) : oct_zero<T>();
+        __builtin_memcpy(&q16[r][i], &o, 16);
+      }
+    } else {
+#pragma unroll
+      for (int i = 0; i < CLS / 4; i++) q32[r][i] = i * 4 + fk < g.D ? (float)qp[i * 4 + fk] : 0.f;
     }
-  } else {
-#pragma unroll
-    for (int i = 0; i < CLS / 4; i++) q32[i] = i * 4 + fk < g.D ? (float)qp[i * 4 + fk] : 0.f;
   }
-  int pos[4], first[4];
+  float m[RT], l[RT];
+  f32x4 o[RT][VT];
 #pragma unroll
-  for (int e = 0; e < 4; e++) {
-    pos[e] = t.pos + wave * 16 + fk * 4 + e;
-    first[e] = pos[e] - pos[e] % g.chunk;
+  for (int r = 0; r < RT; r++) {
+    m[r] = -INFINITY;
+    l[r] = 0.f;
+#pragma unroll
+    for (int j = 0; j < VT; j++) o[r][j] = f32x4{0.f, 0.f, 0.f, 0.f};
   }
-  float m[4], l[4];
-  f32x4 o[VT];
+  const float amp = g.amp ? g.amp[h] : 0.f, rate = g.amp ? g.rate[h] : 0.f, scale2 = g.scale * 1.44269504f;
+  Oct<T> rk[NK], rv[NK];
+  auto request = [&](int j0) {
 #pragma unroll
-  for (int e = 0; e < 4; e++) {
-    m[e] = -INFINITY;
-    l[e] = 0.f;
-  }
+    for (int u = 0; u < NK; u++) {
+      const int i = u * 256 + tid, c = i % (CLS / 8) * 8, p = j0 + i / (CLS / 8);
+      rk[u] = oct_zero<T>();
+      if (p < hi && c < g.D) rk[u] = oct_load(p >= sq.pos0 ? pk + (size_t)(p - sq.pos0) * a.ldp + c : kc + (size_t)(p - lo) * g.D + c);
+    }
 #pragma unroll
-  for (int j = 0; j < VT; j++) o[j] = f32x4{0.f, 0.f, 0.f, 0.f};
-  const float amp = g.amp ? g.amp[h] : 0.f, rate = g.amp ? g.rate[h] : 0.f;
-  const int lo = t.pos - t.pos % g.chunk, hi = t.pos + t.n;  // keys [lo, hi)
+    for (int u = 0; u < NK; u++) {  // octets u, u + 1: the same columns of two neighbouring keys
+      const int i = (u >> 1) * 256 + tid, c = i / (KT / 2) * 8, p = j0 + i % (KT / 2) * 2 + (u & 1);
+      rv[u] = oct_zero<T>();
+      if (p < hi && c < g.V) rv[u] = oct_load(p >= sq.pos0 ? pv + (size_t)(p - sq.pos0) * a.ldp + c : vc + (size_t)(p - lo) * g.V + c);
+    }
+  };
+  request(lo);
   for (int j0 = lo; j0 < hi; j0 += KT) {
     __syncthreads();
-    for (int i = tid; i < KT * (DK / 8); i += 256) {  // K rows
-      const int c = i % (DK / 8) * 8, key = i / (DK / 8), p = j0 + key;
-      Oct<T> v = oct_zero<T>();
-      if (p < hi && c < g.D)
-        v = oct_load(p >= sq.pos0 ? proj_seq + (size_t)(p - sq.pos0) * a.ldp + g.ck + kvh * g.D + c : kc + (size_t)(p % g.chunk) * g.D + c);
-      oct_store(ks + key * LK + c, v);
+#pragma unroll
+    for (int u = 0; u < NK; u++) {
+      const int i = u * 256 + tid;
+      oct_store(ks + i / (CLS / 8) * LK + i % (CLS / 8) * 8, rk[u]);
     }
-    for (int i = tid; i < KT * (CLS / 8); i += 256) {  // V columns
-      const int key = i % KT, c = i / KT * 8, p = j0 + key;
-      if (c >= g.V) continue;
-      Oct<T> v = oct_zero<T>();
-      if (p < hi)
-        v = oct_load(p >= sq.pos0 ? proj_seq + (size_t)(p - sq.pos0) * a.ldp + g.cv + kvh * g.V + c : vc + (size_t)(p % g.chunk) * g.V + c);
-      oct_scatter(vs + c * LV + key, LV, v);
+#pragma unroll
+    for (int u = 0; u < NK; u += 2) {
+      const int i = (u >> 1) * 256 + tid, c = i / (KT / 2) * 8, key = i % (KT / 2) * 2;
+      T v0[8], v1[8];
+      __builtin_memcpy(v0, &rv[u], sizeof v0);
+      __builtin_memcpy(v1, &rv[u + 1], sizeof v1);
+#pragma unroll
+      for (int e = 0; e < 8; e++) {
+        T two[2] = {v0[e], v1[e]};
+        __builtin_memcpy(vs + (c + e) * LV + key, two, sizeof two);
+      }
     }
     __syncthreads();
-    f32x4 s[ST];
+    if (j0 + KT < hi) request(j0 + KT);
+    if (wn <= 0 || j0 > wlast || j0 + KT <= wlo) continue;  // (wave-uniform: nothing here for this wave's rows)
+    const bool edge = j0 + KT - 1 > wfirst || j0 < whi_chunk;
+    f32x4 s[RT][ST];
 #pragma unroll
     for (int j = 0; j < ST; j++) {
-      s[j] = f32x4{0.f, 0.f, 0.f, 0.f};
       const T* kr = ks + (j * 16 + fr) * LK;
+#pragma unroll
+      for (int r = 0; r < RT; r++) s[r][j] = f32x4{0.f, 0.f, 0.f, 0.f};
       if constexpr (sizeof(T) == 2) {
 #pragma unroll
         for (int i = 0; i < CLS / 32; i++)
-          if (i * 32 < DK) s[j] = mfma_bf16(q16[i], *(const bf16x8*)(kr + i * 32 + fk * 8), s[j]);
+          if (i * 32 < DK) {
+            const bf16x8 kf = *(const bf16x8*)(kr + i * 32 + fk * 8);
+#pragma unroll
+            for (int r = 0; r < RT; r++) s[r][j] = mfma_bf16(kf, q16[r][i], s[r][j]);
+          }
       } else {
 #pragma unroll
         for (int i = 0; i < CLS / 4; i++)
-          if (i * 4 < DK) s[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(q32[i], kr[i * 4 + fk], s[j], 0, 0, 0);
+          if (i * 4 < DK) {
+            const float kf = kr[i * 4 + fk];
+#pragma unroll
+            for (int r = 0; r < RT; r++) s[r][j] = __builtin_amdgcn_mfma_f32_16x16x4f32(kf, q32[r][i], s[r][j], 0, 0, 0);
+          }
       }
     }
-    T* pw = ps + wave * 16 * LV;
 #pragma unroll
-    for (int e = 0; e < 4; e++) {
+    for (int r = 0; r < RT; r++) {
+      const float d0 = (float)(pos[r] - j0 - fk * 4);  // distance to this lane's first key of the tile
       float mx = -INFINITY;
 #pragma unroll
-      for (int j = 0; j < ST; j++) {
-        const int p = j0 + j * 16 + fr;
-        float v = s[j][e] * g.scale;
-        const int d = pos[e] - p;
-        if (g.amp) v -= amp * __logf(__builtin_fmaf(rate, (float)(d > 0 ? d : 0), 1.0f));
-        v = d >= 0 && p >= first[e] ? v : -INFINITY;
-        s[j][e] = v;
-        mx = fmaxf(mx, v);
-      }
-      mx = fmaxf(m[e], row16_max_f32(mx));
-      const float ref = mx == -INFINITY ? 0.f : mx, w = __expf(m[e] - ref);
+      for (int j = 0; j < ST; j++)
+#pragma unroll
+        for (int e = 0; e < 4; e++) {
+          float v = s[r][j][e] * scale2;
+          if (g.amp) v = __builtin_fmaf(-amp, __builtin_amdgcn_logf(__builtin_fmaf(rate, d0 - (float)(j * 16 + e), 1.0f)), v);
+          if (edge) {
+            const int p = j0 + j * 16 + fk * 4 + e;
+            v = p <= pos[r] && p >= first[r] ? v : -INFINITY;
+          }
+          s[r][j][e] = v;
+          mx = fmaxf(mx, v);
+        }
+      mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+      mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+      mx = fmaxf(m[r], mx);
+      const float ref = mx == -INFINITY ? 0.f : mx, w = __builtin_amdgcn_exp2f(m[r] - ref);
+      m[r] = mx;
       float sum = 0.f;
 #pragma unroll
-      for (int j = 0; j < ST; j++) {
-        const float pv = __expf(s[j][e] - ref);
-        sum += pv;
-        pw[(fk * 4 + e) * LV + j * 16 + fr] = kv_from<T>(pv);
-      }
-      l[e] = __builtin_fmaf(l[e], w, row16_sum_f32(sum));
-      m[e] = mx;
+      for (int j = 0; j < ST; j++)
 #pragma unroll
-      for (int j = 0; j < VT; j++) o[j][e] *= w;
+        for (int e = 0; e < 4; e++) {
+          const float pe = __builtin_amdgcn_exp2f(s[r][j][e] - ref);
+          s[r][j][e] = pe;
+          sum += pe;
+        }
+      l[r] = __builtin_fmaf(l[r], w, sum);  // (this lane's keys; the four lanes of a row are added at the end)
+#pragma unroll
+      for (int j = 0; j < VT; j++) o[r][j] *= w;
     }
-    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
-    __builtin_amdgcn_wave_barrier();  // (a wave's LDS operations complete in order: its rows of P are there when it reads them)
+    if constexpr (sizeof(T) == 2) {
 #pragma unroll
-    for (int j = 0; j < VT; j++)
-      if (j * 16 < g.V) o[j] = mma_rows(pw + fr * LV, vs + (j * 16 + fr) * LV, KT, o[j]);
+      for (int jj = 0; jj < ST; jj += 2) {
+        bf16x8 pf[RT];
+#pragma unroll
+        for (int r = 0; r < RT; r++)
+#pragma unroll
+          for (int e = 0; e < 4; e++) {
+            pf[r][e] = (__bf16)s[r][jj][e];
+            pf[r][e + 4] = (__bf16)s[r][jj + 1][e];
+          }
+#pragma unroll
+        for (int j = 0; j < VT; j++)
+          if (j * 16 < g.V) {
+            const T* vr = vs + (j * 16 + fr) * LV + jj * 16 + fk * 4;
+            bf16x8 vf;
+            __builtin_memcpy(&vf, vr, 8);
+            __builtin_memcpy((char*)&vf + 8, vr + 16, 8);
+#pragma unroll
+            for (int r = 0; r < RT; r++) o[r][j] = mfma_bf16(vf, pf[r], o[r][j]);
+          }
+      }
+    } else {
+#pragma unroll
+      for (int jj = 0; jj < ST; jj++)
+#pragma unroll
+        for (int j = 0; j < VT; j++)
+          if (j * 16 < g.V) {
+            const f32x4 vf = *(const f32x4*)(vs + (j * 16 + fr) * LV + jj * 16 + fk * 4);
+#pragma unroll
+            for (int r = 0; r < RT; r++)
+#pragma unroll
+              for (int e = 0; e < 4; e++) o[r][j] = __builtin_amdgcn_mfma_f32_16x16x4f32(vf[e], s[r][jj][e], o[r][j], 0, 0, 0);
+          }
+    }
   }
 #pragma unroll
-  for (int e = 0; e < 4; e++) {
-    const int r = wave * 16 + fk * 4 + e;
-    if (r >= t.n) continue;
-    float w = 1.f, den = l[e];
+  for (int r = 0; r < RT; r++) {
+    float den = l[r];
+    den += __shfl_xor(den, 16, 64);
+    den += __shfl_xor(den, 32, 64);
+    const int row = w0 + r * 16 + fr;
+    if (row >= t.n) continue;
+    float w = 1.f;
     if (g.sink) {
-      const float top = fmaxf(m[e], g.sink[h]);
-      w = __expf(m[e] - top);
-      den = __builtin_fmaf(den, w, __expf(g.sink[h] - top));
+      const float s2 = g.sink[h] * 1.44269504f, top = fmaxf(m[r], s2);
+      w = __builtin_amdgcn_exp2f(m[r] - top);
+      den = __builtin_fmaf(den, w, __builtin_amdgcn_exp2f(s2 - top));
     }
     w *= g.out_scale / den;
-    const size_t row = (size_t)(t.row + r);
+    const size_t at = (size_t)(t.row + row);
 #pragma unroll
     for (int j = 0; j < VT; j++) {
-      const int c = j * 16 + fr;
-      if (c < g.V) {
+      const int c = j * 16 + fk * 4;
+      if (c < g.V) {  // (widths are multiples of 8: four columns at a time)
         const int col = h * g.V + c;
-        split_store<P>(o[j][e] * (w * kv_to(a.proj[row * a.ldp + g.cg + col])), a.cat + row * a.ldc + col, a.cat_plane);
+        const T* gp = a.proj + at * a.ldp + g.cg + col;
+        float v[4];
+#pragma unroll
+        for (int e = 0; e < 4; e++) v[e] = o[r][j][e] * (w * kv_to(gp[e]));
+        split_store4<P>(v, a.cat + at * a.ldc + col, a.cat_plane);
       }
     }
   }

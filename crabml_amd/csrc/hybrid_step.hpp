@@ -47,8 +47,12 @@ struct MixStep {
 // floats of one partial: per head its V sums, the running maximum and the denominator
 __host__ __device__ inline int mix_part_floats(int V) { return MIX_HEADS * (V + 2); }
 
-template <typename T>
+// One workgroup: up to MIX_HEADS query heads of one kv head over MIX_KEYS cached rows; heads up to CLS wide.  Everything it needs from
+// memory is requested up front; the rest is register and LDS work.  (The launch runs cold: its code is kept short.)
+template <typename T, int CLS>
 __device__ __forceinline__ void mix_attention(const MixStep& a, int blk, float* lds) {
+  constexpr int NU = CLS / 32;                             // K: four lanes per row, their octets interleaved
+  constexpr int CP = CLS / 8, GR = 256 / CP, NV = MIX_KEYS / GR;  // V: CP lanes across the columns, GR groups of rows
   const AttnGeom& g = a.at;
   const int tid = threadIdx.x, lane = tid & 63, wave = wave_in_wg();
   const int split = blk % a.splits;
@@ -57,61 +61,85 @@ __device__ __forceinline__ void mix_attention(const MixStep& a, int blk, float* 
   rest /= a.head_blocks;
   const int kvh = rest % g.G, b = rest / g.G;
   const StepSeq sq = a.seq[b];
+  const int hpg = g.H / g.G, h0 = kvh * hpg + hb * MIX_HEADS;
+  const int nh = hpg - hb * MIX_HEADS < MIX_HEADS ? hpg - hb * MIX_HEADS : MIX_HEADS;
+  const float* pr = a.proj + (size_t)b * a.ldp;
+  float* ml = lds;                          // [MIX_HEADS][2]: maximum, denominator
+  float* hp_s = ml + 2 * MIX_HEADS;         // [3][MIX_HEADS]: penalty factor, its rate, sink; padded to 4
+  T* kn_s = (T*)(hp_s + 4 * MIX_HEADS);     // [CLS], [CLS]: the new token's row as the cache holds it
+  T* vn_s = kn_s + CLS;
+  float* g_s = (float*)(vn_s + CLS);        // [MIX_HEADS][V]: gates
+  float* q_s = g_s + MIX_HEADS * g.V;       // [MIX_HEADS][D]
+  float* p_s = q_s + MIX_HEADS * g.D;       // [MIX_HEADS][MIX_KEYS]
+  float* o_s = p_s + MIX_HEADS * MIX_KEYS;  // [4 waves][MIX_HEADS][V]
+  // what does not depend on the position: on its way together with it
+  for (int i = tid; i < nh * g.D; i += 256) q_s[i] = pr[g.cq + h0 * g.D + i] * g.scale;
+  for (int i = tid; i < nh * g.V; i += 256) g_s[i] = pr[g.cg + h0 * g.V + i] * g.out_scale;
+  if (tid < g.D) kn_s[tid] = kv_from<T>(pr[g.ck + kvh * g.D + tid]);
+  if (tid < g.V) vn_s[tid] = kv_from<T>(pr[g.cv + kvh * g.V + tid]);
+  if (tid < nh) {
+    hp_s[tid] = g.amp ? g.amp[h0 + tid] : 0.f;
+    hp_s[MIX_HEADS + tid] = g.amp ? g.rate[h0 + tid] : 0.f;
+    hp_s[2 * MIX_HEADS + tid] = g.sink ? g.sink[h0 + tid] : -INFINITY;
+  }
   const int in_chunk = sq.pos % g.chunk, n_rows = in_chunk + 1;  // this chunk's rows, the new one included
   const int r0 = split * MIX_KEYS;
   if (r0 >= n_rows) return;  // (whole workgroup)
   const int active = (n_rows + MIX_KEYS - 1) / MIX_KEYS;
   const int nk = n_rows - r0 < MIX_KEYS ? n_rows - r0 : MIX_KEYS;
-  const int hpg = g.H / g.G, h0 = kvh * hpg + hb * MIX_HEADS;
-  const int nh = hpg - hb * MIX_HEADS < MIX_HEADS ? hpg - hb * MIX_HEADS : MIX_HEADS;
   T* kc = (T*)(sq.slab + a.rs.k) + (size_t)kvh * g.rows * g.D;
   T* vc = (T*)(sq.slab + a.rs.v) + (size_t)kvh * g.rows * g.V;
-  const float* pr = a.proj + (size_t)b * a.ldp;
-  const bool own_new = in_chunk >= r0 && in_chunk < r0 + MIX_KEYS;
-  float* ml = lds;                          // [MIX_HEADS][2]: maximum, denominator
-  float* q_s = ml + 2 * MIX_HEADS;          // [MIX_HEADS][D]
-  float* p_s = q_s + MIX_HEADS * g.D;       // [MIX_HEADS][MIX_KEYS]
-  float* o_s = p_s + MIX_HEADS * MIX_KEYS;  // [MIX_HEADS][256]: column sums by row group
-  for (int i = tid; i < nh * g.D; i += 256) q_s[i] = pr[g.cq + h0 * g.D + i] * g.scale;
-  if (own_new && hb == 0) {  // cache append (read back below by this workgroup only through pr, never through memory)
-    for (int i = tid; i < g.D; i += 256) kc[(size_t)in_chunk * g.D + i] = kv_from<T>(pr[g.ck + kvh * g.D + i]);
-    for (int i = tid; i < g.V; i += 256) vc[(size_t)in_chunk * g.V + i] = kv_from<T>(pr[g.cv + kvh * g.V + i]);
+  const bool own_new = in_chunk < r0 + MIX_KEYS;
+  const int key = tid >> 2, part = tid & 3, vcol = tid % CP * 8, vgrp = tid / CP;
+  Oct<T> kr[NU], vr[NV];
+#pragma unroll
+  for (int u = 0; u < NU; u++) {
+    const int c = part * 8 + u * 32;
+    kr[u] = oct_zero<T>();
+    if (c < g.D && key < nk && r0 + key != in_chunk) kr[u] = oct_load(kc + (size_t)(r0 + key) * g.D + c);
+  }
+#pragma unroll
+  for (int u = 0; u < NV; u++) {
+    const int k = vgrp + u * GR;
+    vr[u] = oct_zero<T>();
+    if (k < nk && vcol < g.V && r0 + k != in_chunk) vr[u] = oct_load(vc + (size_t)(r0 + k) * g.V + vcol);
   }
   __syncthreads();
-  {  // scores: four lanes per row, their 8-element pieces interleaved
-    const int key = tid >> 2, part = tid & 3, row = r0 + key;
-    float s[MIX_HEADS];
-#pragma unroll
-    for (int h = 0; h < MIX_HEADS; h++) s[h] = 0.f;
-    if (key < nk) {
-      for (int c = part * 8; c < g.D; c += 32) {
-        float kk[8];
-        if (row == in_chunk) {
-#pragma unroll
-          for (int e = 0; e < 8; e++) kk[e] = kv_to(kv_from<T>(pr[g.ck + kvh * g.D + c + e]));
-        } else {
-          kv_load8(kc + (size_t)row * g.D + c, kk);
-        }
-#pragma unroll
-        for (int h = 0; h < MIX_HEADS; h++) {
-          if (h < nh) {
-            const f32x4 q0 = *(const f32x4*)(q_s + h * g.D + c), q1 = *(const f32x4*)(q_s + h * g.D + c + 4);
-#pragma unroll
-            for (int e = 0; e < 4; e++) s[h] = __builtin_fmaf(q0[e], kk[e], __builtin_fmaf(q1[e], kk[e + 4], s[h]));
-          }
-        }
-      }
+  if (own_new) {  // the new row: appended to the cache by one head block, taken from LDS by all
+    if (hb == 0) {
+      if (tid < g.D) kc[(size_t)in_chunk * g.D + tid] = kn_s[tid];
+      if (tid < g.V) vc[(size_t)in_chunk * g.V + tid] = vn_s[tid];
     }
-    const float dist = (float)(in_chunk - row);
+    if (r0 + key == in_chunk) {
 #pragma unroll
-    for (int h = 0; h < MIX_HEADS; h++) {
-      float v = s[h];
-      v += dpp_f<0xB1>(v);
-      v += dpp_f<0x4E>(v);
-      if (part == 0 && h < nh) {
-        if (g.amp) v -= g.amp[h0 + h] * __logf(__builtin_fmaf(g.rate[h0 + h], dist, 1.0f));
-        p_s[h * MIX_KEYS + key] = key < nk ? v : -INFINITY;
+      for (int u = 0; u < NU; u++)
+        if (part * 8 + u * 32 < g.D) kr[u] = oct_load(kn_s + part * 8 + u * 32);
+    }
+#pragma unroll
+    for (int u = 0; u < NV; u++)
+      if (r0 + vgrp + u * GR == in_chunk && vcol < g.V) vr[u] = oct_load(vn_s + vcol);
+  }
+  {
+    const float dist = (float)(in_chunk - (r0 + key));
+    float kk[NU][8];
+#pragma unroll
+    for (int u = 0; u < NU; u++) oct_floats(kr[u], kk[u]);
+#pragma unroll 2
+    for (int h = 0; h < nh; h++) {
+      const float* q = q_s + h * g.D + part * 8;
+      float s = 0.f;
+#pragma unroll
+      for (int u = 0; u < NU; u++) {
+        if (part * 8 + u * 32 < g.D) {
+          const f32x4 q0 = *(const f32x4*)(q + u * 32), q1 = *(const f32x4*)(q + u * 32 + 4);
+#pragma unroll
+          for (int e = 0; e < 4; e++) s = __builtin_fmaf(q0[e], kk[u][e], __builtin_fmaf(q1[e], kk[u][e + 4], s));
+        }
       }
+      s += dpp_f<0xB1>(s);
+      s += dpp_f<0x4E>(s);
+      s -= hp_s[h] * __logf(__builtin_fmaf(hp_s[MIX_HEADS + h], dist > 0.f ? dist : 0.f, 1.0f));
+      if (part == 0) p_s[h * MIX_KEYS + key] = key < nk ? s : -INFINITY;
     }
   }
   __syncthreads();
@@ -127,91 +155,79 @@ __device__ __forceinline__ void mix_attention(const MixStep& a, int blk, float* 
     }
   }
   __syncthreads();
-  // weighted value rows: a thread owns one column of one of KG row groups
-  const int vp = g.V <= 32 ? 32 : g.V <= 64 ? 64 : g.V <= 128 ? 128 : 256, kg = 256 / vp;
-  {
-    const int col = tid % vp, grp = tid / vp;
-    float o[MIX_HEADS];
+  {  // weighted value rows, added over the wave's row groups by lane exchange, over the waves through LDS
+    float vv[NV][8];
 #pragma unroll
-    for (int h = 0; h < MIX_HEADS; h++) o[h] = 0.f;
-    if (col < g.V) {
-#pragma unroll 4
-      for (int key = grp; key < nk; key += kg) {
-        const int row = r0 + key;
-        const float v = row == in_chunk ? kv_to(kv_from<T>(pr[g.cv + kvh * g.V + col])) : kv_to(vc[(size_t)row * g.V + col]);
+    for (int u = 0; u < NV; u++) oct_floats(vr[u], vv[u]);
+#pragma unroll 2
+    for (int h = 0; h < nh; h++) {
+      float o[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int h = 0; h < MIX_HEADS; h++) o[h] = __builtin_fmaf(p_s[h * MIX_KEYS + key], v, o[h]);  // (heads past nh: unused)
+      for (int u = 0; u < NV; u++) {
+        const float w = p_s[h * MIX_KEYS + vgrp + u * GR];
+#pragma unroll
+        for (int e = 0; e < 8; e++) o[e] = __builtin_fmaf(w, vv[u][e], o[e]);
+      }
+#pragma unroll
+      for (int x = CP; x < 64; x <<= 1)
+#pragma unroll
+        for (int e = 0; e < 8; e++) o[e] += __shfl_xor(o[e], x, 64);
+      if (lane < CP && vcol < g.V) {
+        float* d = o_s + (wave * MIX_HEADS + h) * g.V + vcol;
+        *(f32x4*)d = f32x4{o[0], o[1], o[2], o[3]};
+        *(f32x4*)(d + 4) = f32x4{o[4], o[5], o[6], o[7]};
       }
     }
-#pragma unroll
-    for (int h = 0; h < MIX_HEADS; h++) o_s[h * 256 + tid] = o[h];
   }
   __syncthreads();
   const int slot = (b * g.G + kvh) * a.head_blocks + hb;
-  auto sum_groups = [&](int h, int c) {
-    float s = 0.f;
-    for (int k = 0; k < kg; k++) s += o_s[h * 256 + k * vp + c];
-    return s;
-  };
-  auto finish = [&](int h, int c, float o, float l) {
-    const int col = (h0 + h) * g.V + c;
-    a.cat[(size_t)b * a.ldc + col] = o / l * (g.out_scale * pr[g.cg + col]);
-  };
-  if (active == 1) {
-    for (int i = tid; i < nh * g.V; i += 256) {
-      const int h = i / g.V, c = i % g.V;
-      float m = ml[2 * h], l = ml[2 * h + 1], o = sum_groups(h, c);
-      if (g.sink) {
-        const float t = fmaxf(m, g.sink[h0 + h]), w = __expf(m - t);
-        l = __builtin_fmaf(l, w, __expf(g.sink[h0 + h] - t));
-        o *= w;
-      }
-      finish(h, c, o, l);
-    }
-    return;
-  }
-  // partials through write-through stores; whoever arrives last merges them in row order
-  const int pf = mix_part_floats(g.V);
-  float* mine = a.part + ((size_t)slot * a.splits + split) * pf;
-  for (int i = tid; i < nh * g.V; i += 256)
-    __hip_atomic_store(mine + i, sum_groups(i / g.V, i % g.V), __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-  for (int i = tid; i < 2 * nh; i += 256) __hip_atomic_store(mine + MIX_HEADS * g.V + i, ml[i], __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-  asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // this thread's write-through stores have been acknowledged
+  const int wstr = MIX_HEADS * g.V, pf = mix_part_floats(g.V), n_out = nh * g.V;
+  float* base = a.part + (size_t)slot * a.splits * pf;
   __shared__ unsigned s_last;
-  __syncthreads();
-  if (tid == 0) s_last = __hip_atomic_fetch_add(a.tick + slot, 1u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) == (unsigned)(active - 1);
-  __syncthreads();
-  if (!s_last) return;
-  if (tid == 0) __hip_atomic_store(a.tick + slot, 0u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-  const float* base = a.part + (size_t)slot * a.splits * pf;
-  // weights e^(m_s - m) / l per head and split, in LDS over the queries and scores
-  float* w_s = q_s;  // [MIX_HEADS][active]
-  __syncthreads();
-  for (int h = wave; h < nh; h += 4) {
-    float m = -INFINITY;
-    for (int s = lane; s < active; s += 64)
-      m = fmaxf(m, __hip_atomic_load(base + (size_t)s * pf + MIX_HEADS * g.V + 2 * h, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT));
-    m = wave_max_f32(m);
-    if (g.sink) m = fmaxf(m, g.sink[h0 + h]);
-    float l = 0.f;
-    for (int s = lane; s < active; s += 64) {
-      const float* p = base + (size_t)s * pf + MIX_HEADS * g.V + 2 * h;
-      const float w = __expf(__hip_atomic_load(p, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) - m);
-      w_s[h * active + s] = w;
-      l = __builtin_fmaf(__hip_atomic_load(p + 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT), w, l);
-    }
-    l = wave_sum_f32(l);
-    if (g.sink) l += __expf(g.sink[h0 + h] - m);
-    if (lane == 0) ml[2 * h + 1] = l;
+  if (active > 1) {  // partials through write-through stores; whoever arrives last merges them in row order
+    float* mine = base + (size_t)split * pf;
+    for (int i = tid; i < n_out; i += 256)
+      __hip_atomic_store(mine + i, (o_s[i] + o_s[wstr + i]) + (o_s[2 * wstr + i] + o_s[3 * wstr + i]), __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    if (tid < 2 * nh) __hip_atomic_store(mine + wstr + tid, ml[tid], __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // this thread's write-through stores have been acknowledged
+    __syncthreads();
+    if (tid == 0) s_last = __hip_atomic_fetch_add(a.tick + slot, 1u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) == (unsigned)(active - 1);
+    __syncthreads();
+    if (!s_last) return;
+    if (tid == 0) __hip_atomic_store(a.tick + slot, 0u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
   }
-  __syncthreads();
-  for (int i = tid; i < nh * g.V; i += 256) {
-    const int h = i / g.V, c = i % g.V;
-    float o = 0.f;
-#pragma unroll 4
-    for (int s = 0; s < active; s++)
-      o = __builtin_fmaf(__hip_atomic_load(base + (size_t)s * pf + i, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT), w_s[h * active + s], o);
-    finish(h, c, o, ml[2 * h + 1]);
+  for (int i = tid; i < n_out; i += 256) {
+    const int h = i / g.V;
+    float m = hp_s[2 * MIX_HEADS + h], l = m == -INFINITY ? 0.f : 1.f, o = 0.f;  // the sink: a key without a value (or none)
+    if (active == 1) {
+      const float mx = fmaxf(m, ml[2 * h]), w = __expf(ml[2 * h] - mx);
+      l = __builtin_fmaf(l, __expf(m - mx), ml[2 * h + 1] * w);
+      o = ((o_s[i] + o_s[wstr + i]) + (o_s[2 * wstr + i] + o_s[3 * wstr + i])) * w;
+    } else {
+      for (int s0 = 0; s0 < active; s0 += 16) {
+        float ps[16], ms[16], ls[16], mx = m;
+#pragma unroll
+        for (int s = 0; s < 16; s++) {
+          const float* p = base + (size_t)(s0 + s < active ? s0 + s : s0) * pf;
+          ps[s] = __hip_atomic_load(p + i, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+          ms[s] = __hip_atomic_load(p + wstr + 2 * h, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+          ls[s] = __hip_atomic_load(p + wstr + 2 * h + 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+        }
+#pragma unroll
+        for (int s = 0; s < 16; s++) mx = fmaxf(mx, ms[s]);
+        const float w0 = __expf(m - mx);
+        m = mx;
+        l *= w0;
+        o *= w0;
+#pragma unroll
+        for (int s = 0; s < 16; s++) {
+          const float w = s0 + s < active ? __expf(ms[s] - mx) : 0.f;
+          l = __builtin_fmaf(ls[s], w, l);
+          o = __builtin_fmaf(ps[s], w, o);
+        }
+      }
+    }
+    a.cat[(size_t)b * a.ldc + h0 * g.V + i] = o / l * g_s[i];
   }
 }
 
@@ -226,62 +242,80 @@ __device__ __forceinline__ void mix_linear(const MixStep& a, int blk, float* lds
   float* k_s = lds;        // [D]
   float* q_s = k_s + g.D;  // [D]
   float* o_s = q_s + g.D;  // [32][32 + 4]
-  for (int i = tid; i < g.D; i += 256) {
-    k_s[i] = pr[g.ck + h * g.D + i];
-    q_s[i] = pr[g.cq + h * g.D + i];
-  }
   const int c = slice * LIN_SLICE + (tid & 7) * 4, grp = tid >> 3;
   const bool live = c < g.V;
+  const bool fresh = sq.pos == 0;  // a sequence's first token: whatever the slab holds, the state is zero
+  f32x4 s[8];  // (at most 256 key rows)
+#pragma unroll
+  for (int u = 0; u < 8; u++) {
+    const int d = grp + u * 32;
+    s[u] = live && !fresh && d < g.D ? *(const f32x4*)(S + (size_t)d * g.V + c) : f32x4{0.f, 0.f, 0.f, 0.f};
+  }
+  if (tid < g.D) {
+    k_s[tid] = pr[g.ck + h * g.D + tid];
+    q_s[tid] = pr[g.cq + h * g.D + tid];
+  }
   const f32x4 v = live ? *(const f32x4*)(pr + g.cv + h * g.V + c) : f32x4{0.f, 0.f, 0.f, 0.f};
   const float dec = g.decay[h * LIN_POW + 1];
-  const bool fresh = sq.pos == 0;  // a sequence's first token: whatever the slab holds, the state is zero
+  // (the output side's factors, for the half-wave that will need them)
+  const int oc = slice * LIN_SLICE + lane, occ = h * g.V + (oc < g.V ? oc : 0);
+  float factor = 0.f;
+  if (wave == 0 && lane < LIN_SLICE && oc < g.V) factor = g.norm[occ] * (g.out_scale * pr[g.cg + occ]);
   f32x4 o = {0.f, 0.f, 0.f, 0.f};
   __syncthreads();
-  if (live) {
-#pragma unroll 4
-    for (int d = grp; d < g.D; d += 32) {
-      f32x4* p = (f32x4*)(S + (size_t)d * g.V + c);
-      f32x4 s = fresh ? f32x4{0.f, 0.f, 0.f, 0.f} : *p;
+#pragma unroll
+  for (int u = 0; u < 8; u++) {
+    const int d = grp + u * 32;
+    if (live && d < g.D) {
       const float k = k_s[d], q = q_s[d];
 #pragma unroll
       for (int e = 0; e < 4; e++) {
-        s[e] = __builtin_fmaf(dec, s[e], k * v[e]);
-        o[e] = __builtin_fmaf(s[e], q, o[e]);
+        s[u][e] = __builtin_fmaf(dec, s[u][e], k * v[e]);
+        o[e] = __builtin_fmaf(s[u][e], q, o[e]);
       }
-      *p = s;
+      *(f32x4*)(S + (size_t)d * g.V + c) = s[u];
     }
   }
   *(f32x4*)(o_s + grp * 36 + (tid & 7) * 4) = o;
   __syncthreads();
   if (wave == 0) {  // 32 columns; the upper half-wave adds nothing to the square sum
-    const int col = slice * LIN_SLICE + lane;
     float r = 0.f;
-    if (lane < LIN_SLICE)
+    if (lane < LIN_SLICE) {
+#pragma unroll
       for (int i = 0; i < 32; i++) r += o_s[i * 36 + lane];
-    const bool in = lane < LIN_SLICE && col < g.V;
+    }
+    const bool in = lane < LIN_SLICE && oc < g.V;
     const float ss = wave_sum_f32(in ? r * r : 0.f);
     if (lane == 0) a.ss[(size_t)b * g.H * g.slices + h * g.slices + slice] = ss;
-    if (in) {
-      const int cc = h * g.V + col;
-      a.cat[(size_t)b * a.ldc + a.lin_off + cc] = r * (g.norm[cc] * (g.out_scale * pr[g.cg + cc]));
-    }
+    if (in) a.cat[(size_t)b * a.ldc + a.lin_off + occ] = r * factor;
   }
 }
 
-template <typename T>
+template <typename T, int CLS>
 __global__ __launch_bounds__(256) void k_mix_step(const MixStep a) {
   extern __shared__ __attribute__((aligned(16))) float mix_lds[];
   const int n_attn = a.at.H ? a.B * a.at.G * a.head_blocks * a.splits : 0;
   if ((int)blockIdx.x < n_attn)
-    mix_attention<T>(a, blockIdx.x, mix_lds);
+    mix_attention<T, CLS>(a, blockIdx.x, mix_lds);
   else
     mix_linear(a, blockIdx.x - n_attn, mix_lds);
 }
-inline size_t mix_step_lds(const MixStep& a) {
-  const size_t work = (size_t)(MIX_HEADS * a.at.D + MIX_HEADS * MIX_KEYS + 256 * MIX_HEADS), merge = (size_t)MIX_HEADS * a.splits;
-  const size_t at = a.at.H ? 2 * MIX_HEADS + (work > merge ? work : merge) : 0;
+template <typename T, int CLS>
+inline void launch_mix_step_t(hipStream_t st, crabml_hip_device::ProfRec* rec, const MixStep& a) {
+  const size_t at = a.at.H ? 6 * MIX_HEADS + 2 * CLS * sizeof(T) / 4 + (size_t)MIX_HEADS * (a.at.D + MIX_KEYS + 5 * a.at.V) : 0;
   const size_t li = a.li.H ? (size_t)(2 * a.li.D + 32 * 36) : 0;
-  return (at > li ? at : li) * sizeof(float);
+  const unsigned grid = (unsigned)(a.B * ((a.at.H ? a.at.G * a.head_blocks * a.splits : 0) + a.li.H * a.li.slices));
+  launch_k(st, rec, k_mix_step<T, CLS>, dim3(grid), dim3(256), (at > li ? at : li) * sizeof(float), a);  // (at most 57 KiB)
+}
+template <typename T>
+inline void launch_mix_step(hipStream_t st, crabml_hip_device::ProfRec* rec, const MixStep& a) {
+  const int w = a.at.D > a.at.V ? a.at.D : a.at.V;
+  if (w <= 64)
+    launch_mix_step_t<T, 64>(st, rec, a);
+  else if (w <= 128)
+    launch_mix_step_t<T, 128>(st, rec, a);
+  else
+    launch_mix_step_t<T, 256>(st, rec, a);
 }
 
 // ---- greedy sampler over the rows of a batch (last maximum, as k_argmax_step) ---------------------------------------------------
