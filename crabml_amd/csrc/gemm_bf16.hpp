@@ -21,7 +21,6 @@
 
 namespace crabml_hip {
 
-typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
 typedef unsigned short u16x4 __attribute__((ext_vector_type(4)));
 
 enum {

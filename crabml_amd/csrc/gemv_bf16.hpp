@@ -81,6 +81,21 @@ __device__ __forceinline__ float xielu_apply(float z, float right, float left) {
 }
 __device__ __forceinline__ float soft_cap(float z, float cap) { return cap > 0.0f ? cap * tanhf(z / cap) : z; }
 
+template <int OUT>
+__device__ __forceinline__ void gemv_out(const GemvBf16& a, int row, int b, float v) {
+  float* o = a.out + (size_t)b * a.ldo + row;
+  if constexpr (OUT == GEMV_OUT_STORE) *o = v;
+  if constexpr (OUT == GEMV_OUT_ACT) *o = act_ranges(v, row, a.act);
+  if constexpr (OUT == GEMV_OUT_RESIDUAL) {
+    float s = *o + v;
+    if (a.add_rows) s += a.add_rows[(size_t)b * a.ld_add + row];
+    if (a.add_vec) s += a.add_vec[row];
+    *o = s;
+  }
+  if constexpr (OUT == GEMV_OUT_XIELU) *o = xielu_apply(v, a.xielu[0], a.xielu[1]);
+  if constexpr (OUT == GEMV_OUT_SOFTCAP) *o = soft_cap(v, a.cap);
+}
+
 #define GEMV_BF16_LDS_FLOATS 8192  // rhs elements staged at a time, all rows together: a cut segment is a multiple of the steps in flight
 
 template <int NB, int R, int IN, int OUT>
@@ -213,19 +228,145 @@ __global__ __launch_bounds__(256) void k_gemv_bf16(const GemvBf16 a) {
       const float v = wave_sum_f32(acc[r][b]) * scale[b];
       const int row = row0 + r, bb = b0 + b;
       if (lane == ((r * NB + b) & 63) && row < a.N && bb < a.nb) {
-        float* o = a.out + (size_t)bb * a.ldo + row;
-        if constexpr (OUT == GEMV_OUT_STORE) *o = v;
-        if constexpr (OUT == GEMV_OUT_ACT) *o = act_ranges(v, row, a.act);
-        if constexpr (OUT == GEMV_OUT_RESIDUAL) {
-          float s = *o + v;
-          if (a.add_rows) s += a.add_rows[(size_t)bb * a.ld_add + row];
-          if (a.add_vec) s += a.add_vec[row];
-          *o = s;
-        }
-        if constexpr (OUT == GEMV_OUT_XIELU) *o = xielu_apply(v, a.xielu[0], a.xielu[1]);
-        if constexpr (OUT == GEMV_OUT_SOFTCAP) *o = soft_cap(v, a.cap);
+        gemv_out<OUT>(a, row, bb, v);
       }
     }
+}
+
+// ---- the same linear for 3 .. 16 rhs rows: one pass over the weights on the matrix cores ---------------------------------------------
+// A 512-thread workgroup owns 16 RT weight rows; its eight waves take the 64-element pieces of k in turn and their tiles are added
+// through LDS at the end.  Both operands come straight from memory in fragment order (16 rows x 64 bytes per request; the rhs, a few
+// hundred KB, lives in L2), the next piece's requests out before the current one is multiplied.  The rhs becomes bf16 on the way:
+// rounded (SPL = 1), or as three exact pieces (SPL = 3; see split_store in gemm_bf16.hpp).  K is a multiple of 64.
+typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+// f32 -> its upper, middle and lower eight significand bits as bf16: their sum is exact
+__device__ __forceinline__ void split3(const float (&v)[8], bf16x8& hi, bf16x8& mid, bf16x8& lo) {
+  unsigned short h[8], m[8], l[8];
+#pragma unroll
+  for (int e = 0; e < 8; e++) {
+    const float a = __builtin_bit_cast(float, __builtin_bit_cast(unsigned, v[e]) & 0xffff0000u), r = v[e] - a;
+    const float b = __builtin_bit_cast(float, __builtin_bit_cast(unsigned, r) & 0xffff0000u);
+    h[e] = (unsigned short)(__builtin_bit_cast(unsigned, a) >> 16);
+    m[e] = (unsigned short)(__builtin_bit_cast(unsigned, b) >> 16);
+    l[e] = f2bf(r - b);
+  }
+  __builtin_memcpy(&hi, h, 16);
+  __builtin_memcpy(&mid, m, 16);
+  __builtin_memcpy(&lo, l, 16);
+}
+__device__ __forceinline__ f32x4 mfma_bf16(bf16x8 a, bf16x8 b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0); }
+
+template <int RT, int SPL, int IN, int OUT>
+__global__ __launch_bounds__(512) void k_gemv16_bf16(const GemvBf16 a) {
+  constexpr int W = 8, LD = 20;
+  __shared__ __attribute__((aligned(16))) float tile[W][RT][16 * LD];
+  __shared__ float sums[W][16], scale[16];
+  const int tid = threadIdx.x, lane = tid & 63, wave = wave_in_wg(), fr = lane & 15, fk = lane >> 4;
+  const int row0 = blockIdx.x * 16 * RT;
+  const unsigned short* wr[RT];
+#pragma unroll
+  for (int t = 0; t < RT; t++) {
+    const int row = row0 + t * 16 + fr;
+    wr[t] = a.w + (size_t)(row < a.N ? row : a.N - 1) * a.ldw + fk * 8;
+  }
+  const float* xr = a.x + (size_t)(fr < a.nb ? fr : a.nb - 1) * a.ldx + fk * 8;
+  bf16x8 wv[2][RT];
+  f32x4 xv[2][2];
+  auto request = [&](int k) {
+#pragma unroll
+    for (int u = 0; u < 2; u++) {
+#pragma unroll
+      for (int t = 0; t < RT; t++) wv[u][t] = *(const bf16x8*)(wr[t] + k + u * 32);
+      xv[u][0] = *(const f32x4*)(xr + k + u * 32);
+      xv[u][1] = *(const f32x4*)(xr + k + u * 32 + 4);
+    }
+  };
+  const int n = a.K / 64;
+  if (wave < n) request(wave * 64);
+  float tail = 1.f, sq = 0.f;
+  if constexpr (IN == GEMV_IN_SPLIT) {
+    float s = 0.f;
+    for (int i = fk; i < a.n_ss; i += 4) s += a.ss[(size_t)(fr < a.nb ? fr : a.nb - 1) * a.n_ss + i];
+    s += __shfl_xor(s, 16, 64);
+    s += __shfl_xor(s, 32, 64);
+    tail = 1.0f / sqrtf(s / (float)a.mean_n + a.eps);
+  }
+  f32x4 acc[RT];
+#pragma unroll
+  for (int t = 0; t < RT; t++) acc[t] = f32x4{0.f, 0.f, 0.f, 0.f};
+  for (int i = wave; i < n; i += W) {
+    bf16x8 wc[2][RT];
+    f32x4 xc[2][2];
+#pragma unroll
+    for (int u = 0; u < 2; u++) {
+#pragma unroll
+      for (int t = 0; t < RT; t++) wc[u][t] = wv[u][t];
+      xc[u][0] = xv[u][0];
+      xc[u][1] = xv[u][1];
+    }
+    if (i + W < n) request((i + W) * 64);
+#pragma unroll
+    for (int u = 0; u < 2; u++) {
+      float v[8] = {xc[u][0][0], xc[u][0][1], xc[u][0][2], xc[u][0][3], xc[u][1][0], xc[u][1][1], xc[u][1][2], xc[u][1][3]};
+      if constexpr (IN == GEMV_IN_RMS) {
+#pragma unroll
+        for (int e = 0; e < 8; e++) sq = __builtin_fmaf(v[e], v[e], sq);
+      }
+      if constexpr (IN == GEMV_IN_SPLIT) {
+        const float f = i * 64 >= a.k_split ? tail : 1.f;  // (k_split is a multiple of 64)
+#pragma unroll
+        for (int e = 0; e < 8; e++) v[e] *= f;
+      }
+      if constexpr (SPL == 1) {
+        bf16x8 b;
+#pragma unroll
+        for (int e = 0; e < 8; e++) b[e] = (__bf16)v[e];
+#pragma unroll
+        for (int t = 0; t < RT; t++) acc[t] = mfma_bf16(wc[u][t], b, acc[t]);
+      } else {
+        bf16x8 h, m, l;
+        split3(v, h, m, l);
+#pragma unroll
+        for (int t = 0; t < RT; t++) acc[t] = mfma_bf16(wc[u][t], h, mfma_bf16(wc[u][t], m, mfma_bf16(wc[u][t], l, acc[t])));
+      }
+    }
+  }
+  // lane: weight rows 4 fk .. of rhs row fr
+#pragma unroll
+  for (int t = 0; t < RT; t++) *(f32x4*)&tile[wave][t][fr * LD + fk * 4] = acc[t];
+  if constexpr (IN == GEMV_IN_RMS) {
+    sq += __shfl_xor(sq, 16, 64);
+    sq += __shfl_xor(sq, 32, 64);
+    if (fk == 0) sums[wave][fr] = sq;
+  }
+  __syncthreads();
+  if constexpr (IN == GEMV_IN_RMS) {
+    if (tid < 16) {
+      float s = 0.f;
+#pragma unroll
+      for (int w = 0; w < W; w++) s += sums[w][tid];
+      scale[tid] = *a.gain / sqrtf(s / (float)a.mean_n + a.eps);
+    }
+    __syncthreads();
+  }
+  for (int i = tid; i < RT * 256; i += 512) {
+    const int t = i >> 8, b = (i >> 4) & 15, r = i & 15, row = row0 + t * 16 + r;
+    float v = 0.f;
+#pragma unroll
+    for (int w = 0; w < W; w++) v += tile[w][t][b * LD + r];
+    if constexpr (IN == GEMV_IN_RMS) v *= scale[b];
+    if (b < a.nb && row < a.N) gemv_out<OUT>(a, row, b, v);
+  }
+}
+
+template <int IN, int OUT>
+inline void launch_gemv16_bf16(hipStream_t st, crabml_hip_device::ProfRec* rec, const GemvBf16& a, bool exact) {
+  const bool two = a.N >= 16384;
+  const dim3 grid((a.N + (two ? 31 : 15)) / (two ? 32 : 16));
+  if (exact)
+    launch_k(st, rec, two ? k_gemv16_bf16<2, 3, IN, OUT> : k_gemv16_bf16<1, 3, IN, OUT>, grid, dim3(512), 0, a);
+  else
+    launch_k(st, rec, two ? k_gemv16_bf16<2, 1, IN, OUT> : k_gemv16_bf16<1, 1, IN, OUT>, grid, dim3(512), 0, a);
 }
 
 template <int NB, int R, int IN, int OUT>

@@ -262,6 +262,15 @@ struct Prof {
   crabml_hip_device::ProfRec* rec() { return on ? &r : nullptr; }
 };
 
+// a decode linear: up to two rows on the vector kernel, more on the matrix cores
+template <int IN, int OUT>
+void step_linear(Ctx* c, crabml_hip_device::ProfRec* rec, const GemvBf16& g) {
+  if (g.nb <= 2)
+    launch_gemv_bf16<IN, OUT>(c->dev->stream, rec, g);
+  else
+    launch_gemv16_bf16<IN, OUT>(c->dev->stream, rec, g, c->f32);
+}
+
 MixStep mix_step(const Ctx* c, const Run& run, int B) {
   const Layer& L = c->layers[run.layer];
   MixStep m;
@@ -306,7 +315,7 @@ void head_rows(Ctx* c, const float* x, int B, bool prof) {
   g.gain = c->final_norm;
   g.cap = c->cfg.logit_softcap;
   Prof p(c->dev, prof, ST_STEP + ST_HEAD, (double)c->vocab * c->ldx * 2);
-  launch_gemv_bf16<GEMV_IN_RMS, GEMV_OUT_SOFTCAP>(c->dev->stream, p.rec(), g);
+  step_linear<GEMV_IN_RMS, GEMV_OUT_SOFTCAP>(c, p.rec(), g);
 }
 
 int enqueue_step(Ctx* c, int B, bool sample, bool prof) {
@@ -333,7 +342,7 @@ int enqueue_step(Ctx* c, int B, bool sample, bool prof) {
       g.gain = L.norm1;
       g.act = L.act;
       Prof p(dev, prof, ST_STEP + ST_IN, (double)L.n_in * c->ldx * 2);
-      launch_gemv_bf16<GEMV_IN_RMS, GEMV_OUT_ACT>(st, p.rec(), g);
+      step_linear<GEMV_IN_RMS, GEMV_OUT_ACT>(c, p.rec(), g);
     }
     {
       const MixStep m = mix_step(c, run, B);
@@ -362,7 +371,7 @@ int enqueue_step(Ctx* c, int B, bool sample, bool prof) {
         g.add_vec = add_vec;
       }
       Prof p(dev, prof, ST_STEP + ST_OUT, (double)c->width * L.ldc * 2);
-      launch_gemv_bf16<GEMV_IN_SPLIT, GEMV_OUT_RESIDUAL>(st, p.rec(), g);
+      step_linear<GEMV_IN_SPLIT, GEMV_OUT_RESIDUAL>(c, p.rec(), g);
     }
     if (!L.ff) continue;
     {
@@ -379,7 +388,7 @@ int enqueue_step(Ctx* c, int B, bool sample, bool prof) {
       g.gain = L.norm2;
       g.xielu = L.xielu;
       Prof p(dev, prof, ST_STEP + ST_UP, (double)L.ff * c->ldx * 2);
-      launch_gemv_bf16<GEMV_IN_RMS, GEMV_OUT_XIELU>(st, p.rec(), g);
+      step_linear<GEMV_IN_RMS, GEMV_OUT_XIELU>(c, p.rec(), g);
     }
     {
       GemvBf16 g;
@@ -393,7 +402,7 @@ int enqueue_step(Ctx* c, int B, bool sample, bool prof) {
       g.add_rows = add_rows;
       g.add_vec = add_vec;
       Prof p(dev, prof, ST_STEP + ST_DOWN, (double)c->width * L.ldu * 2);
-      launch_gemv_bf16<GEMV_IN_PLAIN, GEMV_OUT_RESIDUAL>(st, p.rec(), g);
+      step_linear<GEMV_IN_PLAIN, GEMV_OUT_RESIDUAL>(c, p.rec(), g);
     }
   }
   head_rows(c, c->st_x, B, prof);

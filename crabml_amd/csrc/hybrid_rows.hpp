@@ -26,22 +26,6 @@ struct PassTile {  // up to 64 (times AttnTile::RT) consecutive rows of one sequ
 
 // ---- operand fragments of 16x16 matrix products out of LDS rows with k contiguous ------------------------------------------------
 // lane: row lane % 16 of the operand, k group lane / 16
-__device__ __forceinline__ void split3(const float (&v)[8], bf16x8& hi, bf16x8& mid, bf16x8& lo) {
-  unsigned short h[8], m[8], l[8];
-#pragma unroll
-  for (int e = 0; e < 8; e++) {
-    const float a = __builtin_bit_cast(float, __builtin_bit_cast(unsigned, v[e]) & 0xffff0000u), r = v[e] - a;
-    const float b = __builtin_bit_cast(float, __builtin_bit_cast(unsigned, r) & 0xffff0000u);
-    h[e] = (unsigned short)(__builtin_bit_cast(unsigned, a) >> 16);
-    m[e] = (unsigned short)(__builtin_bit_cast(unsigned, b) >> 16);
-    l[e] = f2bf(r - b);
-  }
-  __builtin_memcpy(&hi, h, 16);
-  __builtin_memcpy(&mid, m, 16);
-  __builtin_memcpy(&lo, l, 16);
-}
-__device__ __forceinline__ f32x4 mfma_bf16(bf16x8 a, bf16x8 b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0); }
-
 // acc += A B^T over k < K; a / b: this lane's rows.  K is a multiple of 32.
 __device__ __forceinline__ f32x4 mma_rows(const unsigned short* a, const unsigned short* b, int K, f32x4 acc) {
   const int o = (threadIdx.x >> 4 & 3) * 8;

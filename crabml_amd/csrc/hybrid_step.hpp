@@ -124,7 +124,6 @@ __device__ __forceinline__ void mix_attention(const MixStep& a, int blk, float* 
     float kk[NU][8];
 #pragma unroll
     for (int u = 0; u < NU; u++) oct_floats(kr[u], kk[u]);
-#pragma unroll 2
     for (int h = 0; h < nh; h++) {
       const float* q = q_s + h * g.D + part * 8;
       float s = 0.f;
@@ -159,7 +158,6 @@ __device__ __forceinline__ void mix_attention(const MixStep& a, int blk, float* 
     float vv[NV][8];
 #pragma unroll
     for (int u = 0; u < NV; u++) oct_floats(vr[u], vv[u]);
-#pragma unroll 2
     for (int h = 0; h < nh; h++) {
       float o[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
 #pragma unroll
