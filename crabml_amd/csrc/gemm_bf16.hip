@@ -1,4 +1,6 @@
 // gemm_bf16.hip -- the kernel behind gemm_bf16.hpp
+#include <cmath>
+
 #include "gemm_bf16.hpp"
 
 namespace crabml_hip {
@@ -7,26 +9,35 @@ __device__ __forceinline__ void lds_dma16(const void* g, void* l) {
   __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)g, (__attribute__((address_space(3))) void*)l, 16, 0, 0);
 }
 
+// four values as f32 / as bf16 planes (16- and 8-byte stores)
+__device__ __forceinline__ void store4(float* p, const float (&v)[4]) { *(f32x4*)p = f32x4{v[0], v[1], v[2], v[3]}; }
+
+// S > 1: k is cut into S pieces, one workgroup each.  A workgroup leaves its accumulators in ws (write-through) and counts itself in; the
+// one that comes last adds the others' pieces to its own, in piece order, and goes on to the epilogue.  The counter is left at zero.
 template <int BM, int BN, int WGM, int WGN, int P, int OUT>
-__global__ __launch_bounds__(256) void k_gemm_bf16(const GemmBf16 g) {
+__global__ __launch_bounds__(256) void k_gemm_bf16(const GemmBf16 g, int S, float* __restrict__ ws, unsigned* __restrict__ tick) {
   constexpr int WM = BM / WGM, WN = BN / WGN, TM = WM / 16, TN = WN / 16;
-  static_assert(WGM * WGN == 4 && WN == 64, "a wave's columns are one square-sum piece");
+  constexpr int HR = BM < 64 ? BM : 64, LC = BN + 4;  // the epilogue's slab of rows in LDS
+  static_assert(WGM * WGN == 4 && WN == 64 && HR % WM == 0, "a wave's columns are one square-sum piece; its rows lie in one slab");
   __shared__ __attribute__((aligned(16))) unsigned short lds[2][(BM + BN) * 64];
+  static_assert(sizeof(lds) >= (HR * LC + BM) * sizeof(float), "the epilogue reuses the tiles' LDS");
   const int tid = threadIdx.x, lane = tid & 63, wave = wave_in_wg();
   const int wm = wave / WGN, wn = wave % WGN;
-  const int mt = (g.M + BM - 1) / BM, nt = (g.N + BN - 1) / BN, total = mt * nt;
+  const int mt = (g.M + BM - 1) / BM, nt = (g.N + BN - 1) / BN, total = mt * nt * S;
   int id = blockIdx.x;
   {  // XCD x (= id % 8) takes a contiguous run of tiles
     const int x = id & 7, i = id >> 3, q = total >> 3, r = total & 7;
     id = x * q + (x < r ? x : r) + i;
   }
-  const int row0 = (id % mt) * BM, col0 = (id / mt) * BN;
+  const int piece = id / mt % S, tile = id / mt / S * mt + id % mt;  // row tiles fastest, then pieces: a weight tile's readers are neighbours
+  const int row0 = (tile % mt) * BM, col0 = (tile / mt) * BN;
   f32x4 acc[TM][TN];
 #pragma unroll
   for (int i = 0; i < TM; i++)
 #pragma unroll
     for (int j = 0; j < TN; j++) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
-  const int steps = g.K / 64;
+  const int steps = g.K / 64, all = steps * P;
+  const int s_lo = (int)((long long)all * piece / S), s_hi = (int)((long long)all * (piece + 1) / S);
   auto fetch = [&](int s, int buf) {
     const int p = P == 1 ? 0 : s / steps, k0 = (P == 1 ? s : s - p * steps) * 64;
     const unsigned short* ap = g.a + (P == 1 ? 0 : (size_t)(P - 1 - p) * g.a_plane) + k0;  // (the smallest plane first)
@@ -41,14 +52,22 @@ __global__ __launch_bounds__(256) void k_gemm_bf16(const GemmBf16 g) {
       lds_dma16(g.w + (size_t)(col0 + r) * g.K + k0 + c * 8, &lds[buf][BM * 64 + (it * 256 + wave * 64) * 8]);
     }
   };
-  fetch(0, 0);
-  const int n_steps = steps * P;
+  fetch(s_lo, 0);
+  float factor = 1.f;  // of row tid, waiting for the epilogue
+  if (g.sq_in != nullptr && tid < BM) {
+    const float* q = g.sq_in + (size_t)(row0 + tid < g.M ? row0 + tid : g.M - 1) * g.n_sq;
+    float s = 0.f;
+#pragma unroll 8
+    for (int i = 0; i < g.n_sq; i++) s += q[i];
+    factor = *g.gain / sqrtf(s / (float)g.mean_n + g.eps);
+  }
   const int fr = lane & 15, fk = lane >> 4;
-  for (int s = 0; s < n_steps; s++) {
+  for (int s = s_lo; s < s_hi; s++) {
     asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // this wave's part of step s has landed ...
     __syncthreads();                                  // ... and everybody's; and step s - 1 has been read by every wave
-    if (s + 1 < n_steps) fetch(s + 1, (s + 1) & 1);
-    const unsigned short* la = &lds[s & 1][0];
+    const int buf = (s - s_lo) & 1;
+    if (s + 1 < s_hi) fetch(s + 1, buf ^ 1);
+    const unsigned short* la = &lds[buf][0];
     const unsigned short* lb = la + BM * 64;
 #pragma unroll
     for (int kk = 0; kk < 2; kk++) {
@@ -66,91 +85,215 @@ __global__ __launch_bounds__(256) void k_gemm_bf16(const GemmBf16 g) {
 #pragma unroll
       for (int i = 0; i < TM; i++)
 #pragma unroll
-        for (int j = 0; j < TN; j++) acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fa[i], fb[j], acc[i][j], 0, 0, 0);
+        for (int j = 0; j < TN; j++) acc[i][j] = mfma_bf16(fa[i], fb[j], acc[i][j]);
     }
   }
-  // C layout: lane holds rows 4 (lane / 16) .. + 3 of column lane % 16
+  if (S > 1) {
+    constexpr int FRAG = TM * TN * 2;  // 8-byte halves of a lane's accumulators
+    unsigned long long* base = (unsigned long long*)ws + (size_t)tile * S * 256 * FRAG + tid;
+    unsigned long long* mine = base + (size_t)piece * 256 * FRAG;
+#pragma unroll
+    for (int i = 0; i < TM; i++)
+#pragma unroll
+      for (int j = 0; j < TN; j++)
+#pragma unroll
+        for (int e = 0; e < 2; e++) {
+          const f32x2 v = {acc[i][j][2 * e], acc[i][j][2 * e + 1]};
+          __hip_atomic_store(mine + ((i * TN + j) * 2 + e) * 256, __builtin_bit_cast(unsigned long long, v), __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+        }
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // this thread's write-through stores have been acknowledged
+    __shared__ unsigned s_last;
+    __syncthreads();
+    if (tid == 0) s_last = __hip_atomic_fetch_add(tick + tile, 1u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) == (unsigned)(S - 1);
+    __syncthreads();
+    if (!s_last) return;
+    if (tid == 0) __hip_atomic_store(tick + tile, 0u, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+#pragma unroll
+    for (int i = 0; i < TM; i++)
+#pragma unroll
+      for (int j = 0; j < TN; j++) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
+    for (int q = 0; q < S; q++) {  // (its own piece from memory as well: one order of addition, whoever is last)
+      const unsigned long long* p = base + (size_t)q * 256 * FRAG;
+#pragma unroll
+      for (int i = 0; i < TM; i++)
+#pragma unroll
+        for (int j = 0; j < TN; j++)
+#pragma unroll
+          for (int e = 0; e < 2; e++) {
+            const f32x2 v = __builtin_bit_cast(f32x2, __hip_atomic_load(p + ((i * TN + j) * 2 + e) * 256, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT));
+            acc[i][j][2 * e] += v[0];
+            acc[i][j][2 * e + 1] += v[1];
+          }
+    }
+  }
+  // epilogue: the tile goes through LDS in slabs of HR rows, so that a thread has eight neighbouring columns of a row
+  float* lc = (float*)lds;            // [HR][LC]
+  float* lf = lc + HR * LC;           // [BM] row factors
   float xr = 0.f, xl = 0.f;
   if constexpr (OUT == GEMM_OUT_XIELU) {
     xr = g.xielu[0];
     xl = g.xielu[1];
   }
+  for (int h = 0; h < BM / HR; h++) {
+    __syncthreads();
+    if (h == 0 && tid < BM) lf[tid] = factor;
+    if (wm * WM / HR == h) {
 #pragma unroll
-  for (int i = 0; i < TM; i++) {
+      for (int i = 0; i < TM; i++)
 #pragma unroll
-    for (int e = 0; e < 4; e++) {
-      const int row = row0 + wm * WM + i * 16 + fk * 4 + e;
-      const bool live = row < g.M;
-      const int rr = live ? row : g.M - 1;
-      float f = 1.f;
-      if (g.sq_in != nullptr) {
-        float s = 0.f;
-        for (int q = fr; q < g.n_sq; q += 16) s += g.sq_in[(size_t)rr * g.n_sq + q];
-        f = *g.gain / sqrtf(row16_sum_f32(s) / (float)g.mean_n + g.eps);
+        for (int j = 0; j < TN; j++)
+#pragma unroll
+          for (int e = 0; e < 4; e++) lc[(wm * WM % HR + i * 16 + fk * 4 + e) * LC + wn * WN + j * 16 + fr] = acc[i][j][e];
+    }
+    __syncthreads();
+    constexpr int UNITS = HR * BN / 8 / 256;
+    int row[UNITS], col[UNITS];
+    bool in[UNITS];
+    float v[UNITS][8], x[UNITS][8];
+#pragma unroll
+    for (int u = 0; u < UNITS; u++) {
+      const int unit = u * 256 + tid, r = unit / (BN / 8), c = unit % (BN / 8) * 8;
+      row[u] = row0 + h * HR + r;
+      col[u] = col0 + c;
+      in[u] = row[u] < g.M && col[u] < g.N;
+      if constexpr (OUT == GEMM_OUT_RESIDUAL) {  // (rows are padded past N: eight columns from any col < N lie inside)
+#pragma unroll
+        for (int e = 0; e < 8; e++) x[u][e] = 0.f;
+        if (in[u]) read8(g.x + (size_t)row[u] * g.ldx + col[u], x[u]);
       }
-      float sq = 0.f;
+      const f32x4 a = *(const f32x4*)(lc + r * LC + c), b = *(const f32x4*)(lc + r * LC + c + 4);
+      const float f = lf[h * HR + r];
 #pragma unroll
-      for (int j = 0; j < TN; j++) {
-        const int col = col0 + wn * WN + j * 16 + fr;
-        const bool in = live && col < g.N;
-        const float v = acc[i][j][e] * f;
-        if constexpr (OUT == GEMM_OUT_ACT_BF16) {
-          if (in) ((unsigned short*)g.out)[(size_t)row * g.ldo + col] = f2bf(act_ranges(v, col, g.act));
-        } else if constexpr (OUT == GEMM_OUT_ACT_F32) {
-          if (in) ((float*)g.out)[(size_t)row * g.ldo + col] = act_ranges(v, col, g.act);
-        } else if constexpr (OUT == GEMM_OUT_SOFTCAP) {
-          if (in) ((float*)g.out)[(size_t)row * g.ldo + col] = soft_cap(v, g.cap);
-        } else if constexpr (OUT == GEMM_OUT_XIELU) {
-          if (in) split_store<P>(xielu_apply(v, xr, xl), g.planes + (size_t)row * g.ldp + col, g.p_plane);
-        } else {
-          if (in) {
-            float* px = g.x + (size_t)row * g.ldx + col;
-            float s = *px + v;
-            if (g.add_rows) s += g.add_rows[(size_t)row * g.ldx + col];
-            if (g.add_vec) s += g.add_vec[col];
-            *px = s;
-            split_store<P>(s, g.planes + (size_t)row * g.ldp + col, g.p_plane);
-            sq = __builtin_fmaf(s, s, sq);
+      for (int e = 0; e < 4; e++) {
+        v[u][e] = a[e] * f;
+        v[u][e + 4] = b[e] * f;
+      }
+    }
+    if constexpr (OUT == GEMM_OUT_RESIDUAL) {
+      if (g.add_rows) {
+#pragma unroll
+        for (int u = 0; u < UNITS; u++) {
+          float t[8];
+          if (in[u]) {
+            read8(g.add_rows + (size_t)row[u] * g.ldx + col[u], t);
+#pragma unroll
+            for (int e = 0; e < 8; e++) x[u][e] += t[e];
           }
         }
       }
-      if constexpr (OUT == GEMM_OUT_RESIDUAL) {
-        sq = row16_sum_f32(sq);
-        const int piece = (col0 + wn * WN) / 64;
-        if (fr == 0 && live && piece < g.n_sq_out) g.sq_out[(size_t)row * g.n_sq_out + piece] = sq;
+      if (g.add_vec) {
+#pragma unroll
+        for (int u = 0; u < UNITS; u++)
+#pragma unroll
+          for (int e = 0; e < 8; e++)
+            if (in[u] && col[u] + e < g.N) x[u][e] += g.add_vec[col[u] + e];
+      }
+    }
+#pragma unroll
+    for (int u = 0; u < UNITS; u++) {
+      float sq = 0.f;
+      if constexpr (OUT == GEMM_OUT_SOFTCAP) {
+        if (in[u]) {
+#pragma unroll
+          for (int e = 0; e < 8; e++)
+            if (col[u] + e < g.N) ((float*)g.out)[(size_t)row[u] * g.ldo + col[u] + e] = soft_cap(v[u][e], g.cap);
+        }
+        continue;
+      }
+#pragma unroll
+      for (int e = 0; e < 8; e++) {
+        if constexpr (OUT == GEMM_OUT_ACT_BF16 || OUT == GEMM_OUT_ACT_F32) v[u][e] = act_ranges(v[u][e], col[u], g.act);  // (ranges end on multiples of 8)
+        if constexpr (OUT == GEMM_OUT_XIELU) v[u][e] = xielu_apply(v[u][e], xr, xl);
+        if constexpr (OUT == GEMM_OUT_RESIDUAL) {
+          v[u][e] += x[u][e];
+          sq = __builtin_fmaf(v[u][e], v[u][e], sq);
+        }
+      }
+      float lo[4], hi[4];
+#pragma unroll
+      for (int e = 0; e < 4; e++) {
+        lo[e] = v[u][e];
+        hi[e] = v[u][e + 4];
+      }
+      if constexpr (OUT == GEMM_OUT_RESIDUAL) {  // eight lanes hold a row's 64 columns
+        sq = in[u] ? sq : 0.f;
+        sq += dpp_f<0xB1>(sq);
+        sq += dpp_f<0x4E>(sq);
+        sq += dpp_f<0x141>(sq);
+        if (in[u] && (tid & 7) == 0) g.sq_out[(size_t)row[u] * g.n_sq_out + col[u] / 64] = sq;
+      }
+      if (!in[u]) continue;
+      if constexpr (OUT == GEMM_OUT_ACT_F32) {
+        store4((float*)g.out + (size_t)row[u] * g.ldo + col[u], lo);
+        store4((float*)g.out + (size_t)row[u] * g.ldo + col[u] + 4, hi);
+      } else if constexpr (OUT == GEMM_OUT_ACT_BF16) {
+        split_store8<1>(v[u], (unsigned short*)g.out + (size_t)row[u] * g.ldo + col[u], 0);
+      } else {
+        if constexpr (OUT == GEMM_OUT_RESIDUAL) {
+          store4(g.x + (size_t)row[u] * g.ldx + col[u], lo);
+          store4(g.x + (size_t)row[u] * g.ldx + col[u] + 4, hi);
+        }
+        split_store8<P>(v[u], g.planes + (size_t)row[u] * g.ldp + col[u], g.p_plane);
       }
     }
   }
 }
 
-// the tile that covers the chip: 128 x 128 when that makes enough workgroups, smaller row tiles below
-template <int P, int OUT>
-static void launch_t(hipStream_t st, crabml_hip_device::ProfRec* rec, const GemmBf16& g, int n_cu) {
-  auto tiles = [&](int bm, int bn) { return ((g.M + bm - 1) / bm) * ((g.N + bn - 1) / bn); };
-  if (g.M > 64 && tiles(128, 128) >= n_cu)
-    launch_k(st, rec, k_gemm_bf16<128, 128, 2, 2, P, OUT>, dim3(tiles(128, 128)), dim3(256), 0, g);
-  else if (g.M > 32 && (tiles(64, 128) >= n_cu || g.M > 512))
-    launch_k(st, rec, k_gemm_bf16<64, 128, 2, 2, P, OUT>, dim3(tiles(64, 128)), dim3(256), 0, g);
-  else
-    launch_k(st, rec, k_gemm_bf16<32, 128, 2, 2, P, OUT>, dim3(tiles(32, 128)), dim3(256), 0, g);
+// Tile and k pieces: 128-row tiles unless there are fewer rows, k cut so that the launch fills the chip.  The estimate counts steps of
+// 64: what the busiest CU multiplies, against the latency of a workgroup's own chain; a cut costs the hand-over of the pieces.
+struct GemmPlan {
+  int bm, S;
+};
+static GemmPlan plan(const GemmBf16& g, int planes, int n_cu, size_t ws_floats) {
+  GemmPlan best{128, 1};
+  double best_cost = 1e30;
+  const int steps = g.K / 64 * planes;
+  for (int bm : {128, 64, 32}) {
+    if (bm > 32 && g.M <= bm / 2) continue;
+    const int tiles = ((g.M + bm - 1) / bm) * ((g.N + 127) / 128), resident = bm == 128 ? 2 : 3;
+    for (int S : {1, 2, 3, 4, 6, 8}) {
+      if (S > 1 && (steps / S < 6 || (size_t)tiles * S * bm * 128 > ws_floats || tiles > GEMM_TICKS)) break;
+      const double per = (double)steps / S, wgs = (double)tiles * S;
+      const double busy = ceil(wgs / n_cu) * (per * 0.36 * (bm == 128 ? 1.0 : bm == 64 ? 0.6 : 0.45) + 1.5);
+      const double chain = ceil(wgs / (n_cu * resident)) * (per * 0.55 + 3.0);
+      const double cost = (busy > chain ? busy : chain) + (S > 1 ? 4.0 + 0.8 * S * bm / 128 : 0.0);
+      if (cost < best_cost) {
+        best_cost = cost;
+        best = {bm, S};
+      }
+    }
+  }
+  return best;
 }
 
-void launch_gemm_bf16(crabml_hip_device* dev, crabml_hip_device::ProfRec* rec, int planes, int out, const GemmBf16& g) {
+template <int P, int OUT>
+static void launch_t(hipStream_t st, crabml_hip_device::ProfRec* rec, const GemmBf16& g, int n_cu, const GemmScratch& w) {
+  const GemmPlan p = plan(g, P, n_cu, w.floats);
+  const dim3 grid(((g.M + p.bm - 1) / p.bm) * ((g.N + 127) / 128) * p.S);
+  if (p.bm == 128)
+    launch_k(st, rec, k_gemm_bf16<128, 128, 2, 2, P, OUT>, grid, dim3(256), 0, g, p.S, w.partials, w.ticks);
+  else if (p.bm == 64)
+    launch_k(st, rec, k_gemm_bf16<64, 128, 2, 2, P, OUT>, grid, dim3(256), 0, g, p.S, w.partials, w.ticks);
+  else
+    launch_k(st, rec, k_gemm_bf16<32, 128, 2, 2, P, OUT>, grid, dim3(256), 0, g, p.S, w.partials, w.ticks);
+}
+
+void launch_gemm_bf16(crabml_hip_device* dev, crabml_hip_device::ProfRec* rec, int planes, int out, const GemmBf16& g, const GemmScratch& w) {
   const int n = dev->n_cu;
   hipStream_t st = dev->stream;
   if (planes == 1) {
     switch (out) {
-      case GEMM_OUT_ACT_BF16: launch_t<1, GEMM_OUT_ACT_BF16>(st, rec, g, n); break;
-      case GEMM_OUT_RESIDUAL: launch_t<1, GEMM_OUT_RESIDUAL>(st, rec, g, n); break;
-      case GEMM_OUT_XIELU: launch_t<1, GEMM_OUT_XIELU>(st, rec, g, n); break;
-      default: launch_t<1, GEMM_OUT_SOFTCAP>(st, rec, g, n); break;
+      case GEMM_OUT_ACT_BF16: launch_t<1, GEMM_OUT_ACT_BF16>(st, rec, g, n, w); break;
+      case GEMM_OUT_RESIDUAL: launch_t<1, GEMM_OUT_RESIDUAL>(st, rec, g, n, w); break;
+      case GEMM_OUT_XIELU: launch_t<1, GEMM_OUT_XIELU>(st, rec, g, n, w); break;
+      default: launch_t<1, GEMM_OUT_SOFTCAP>(st, rec, g, n, w); break;
     }
   } else {
     switch (out) {
-      case GEMM_OUT_ACT_F32: launch_t<3, GEMM_OUT_ACT_F32>(st, rec, g, n); break;
-      case GEMM_OUT_RESIDUAL: launch_t<3, GEMM_OUT_RESIDUAL>(st, rec, g, n); break;
-      case GEMM_OUT_XIELU: launch_t<3, GEMM_OUT_XIELU>(st, rec, g, n); break;
-      default: launch_t<3, GEMM_OUT_SOFTCAP>(st, rec, g, n); break;
+      case GEMM_OUT_ACT_F32: launch_t<3, GEMM_OUT_ACT_F32>(st, rec, g, n, w); break;
+      case GEMM_OUT_RESIDUAL: launch_t<3, GEMM_OUT_RESIDUAL>(st, rec, g, n, w); break;
+      case GEMM_OUT_XIELU: launch_t<3, GEMM_OUT_XIELU>(st, rec, g, n, w); break;
+      default: launch_t<3, GEMM_OUT_SOFTCAP>(st, rec, g, n, w); break;
     }
   }
 }

@@ -10,7 +10,8 @@
 // (global_load_lds, 16 bytes per lane), double-buffered: the next step's requests are out before the current one is multiplied.  LDS
 // holds rows of 128 bytes whose 16-byte chunks are permuted by (row / 2) % 8 -- on the SOURCE side, the LDS side of the instruction
 // being linear -- so that the 16 rows a fragment read touches spread over all 64 banks.  Operands are padded by their owners (k to 64,
-// weight rows to 256, activation rows to 128), so the loop has no bounds checks; stores have.  Workgroups are dealt to the eight XCDs
+// weight rows to 256, activation rows to 128), so the loop has no bounds checks; stores have.  Short launches cut k into pieces (the
+// last workgroup of a tile adds them).  Workgroups are dealt to the eight XCDs
 // in contiguous runs of the tile order, row tiles fastest: an XCD's L2 keeps the weight tile that its row tiles share.
 //
 // The row operations around a linear are folded into it.  In: an RMS norm with a single gain is a factor per row, applied to the
@@ -56,6 +57,28 @@ __device__ __forceinline__ void split_store4(const float (&v)[4], unsigned short
   for (int i = 0; i < P; i++) __builtin_memcpy(p + i * plane_stride, t[i], 8);
 }
 
+// eight of them (p: 16-byte aligned)
+template <int P>
+__device__ __forceinline__ void split_store8(const float (&v)[8], unsigned short* p, size_t plane_stride) {
+  unsigned short t[P][8];
+#pragma unroll
+  for (int e = 0; e < 8; e++) split_store<P>(v[e], &t[0][e], 8);
+#pragma unroll
+  for (int i = 0; i < P; i++) {
+    i32x4 w;
+    __builtin_memcpy(&w, t[i], 16);
+    *(i32x4*)(p + i * plane_stride) = w;
+  }
+}
+__device__ __forceinline__ void read8(const float* p, float (&o)[8]) {
+  const f32x4 a = *(const f32x4*)p, b = *(const f32x4*)(p + 4);
+#pragma unroll
+  for (int e = 0; e < 4; e++) {
+    o[e] = a[e];
+    o[e + 4] = b[e];
+  }
+}
+
 struct GemmBf16 {
   const unsigned short* a = nullptr;  // [planes][rows padded][k]
   size_t a_plane = 0;                 // elements between planes
@@ -82,7 +105,14 @@ struct GemmBf16 {
   int n_sq_out = 0;
 };
 
+// room for k pieces: partial tiles, and a zeroed counter per tile
+#define GEMM_TICKS 4096
+struct GemmScratch {
+  float* partials = nullptr;
+  size_t floats = 0;
+  unsigned* ticks = nullptr;
+};
 // planes: 1 or 3 (GEMM_OUT_ACT_BF16 goes with one, GEMM_OUT_ACT_F32 with three)
-void launch_gemm_bf16(crabml_hip_device* dev, crabml_hip_device::ProfRec* rec, int planes, int out, const GemmBf16& g);
+void launch_gemm_bf16(crabml_hip_device* dev, crabml_hip_device::ProfRec* rec, int planes, int out, const GemmBf16& g, const GemmScratch& w);
 
 }  // namespace crabml_hip

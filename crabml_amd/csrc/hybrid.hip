@@ -74,6 +74,7 @@ struct crabml_hip_hybrid {
   float *pf_x = nullptr, *pf_emb = nullptr, *pf_lin = nullptr, *pf_sq = nullptr, *pf_gsq = nullptr, *pf_logits = nullptr;
   unsigned short *pf_xp = nullptr, *pf_cat = nullptr, *pf_u = nullptr, *pf_gp = nullptr;
   void* pf_proj = nullptr;
+  GemmScratch pf_scratch;
   std::vector<std::pair<void*, size_t>> allocs;
 };
 
@@ -468,6 +469,9 @@ int pass_alloc(Ctx* c) {
   CH_TRY(dalloc_n(c, R * lin, &c->pf_lin));
   CH_TRY(dalloc_n(c, P * R * c->ld_u, &c->pf_u));
   CH_TRY(dalloc_n(c, R * c->n_sq, &c->pf_sq));
+  c->pf_scratch.floats = (size_t)16 << 20;
+  CH_TRY(dalloc(c, c->pf_scratch.floats * sizeof(float), (void**)&c->pf_scratch.partials, false));
+  CH_TRY(dalloc_n(c, GEMM_TICKS, &c->pf_scratch.ticks));
   CH_TRY(dalloc_n(c, P * LOGIT_ROWS * c->ldx, &c->pf_gp));
   CH_TRY(dalloc_n(c, LOGIT_ROWS * c->n_sq, &c->pf_gsq));
   CH_TRY(dalloc_n(c, LOGIT_ROWS * c->vocab, &c->pf_logits));
@@ -633,7 +637,7 @@ int run_pass(Ctx* c, const std::vector<Part>& parts, float** logits) {
       g.ldo = L.n_in;
       g.act = L.act;
       Prof p(dev, true, ST_PASS + ST_IN, 0.0);
-      launch_gemm_bf16(dev, p.rec(), c->planes, c->f32 ? GEMM_OUT_ACT_F32 : GEMM_OUT_ACT_BF16, g);
+      launch_gemm_bf16(dev, p.rec(), c->planes, c->f32 ? GEMM_OUT_ACT_F32 : GEMM_OUT_ACT_BF16, g, c->pf_scratch);
     }
     if (c->f32)
       CH_TRY(mix_rows<float>(c, run, ds, parts.size(), dt, dr, M));
@@ -646,7 +650,7 @@ int run_pass(Ctx* c, const std::vector<Part>& parts, float** logits) {
         g.add_vec = add_vec;
       }
       Prof p(dev, true, ST_PASS + ST_OUT, 0.0);
-      launch_gemm_bf16(dev, p.rec(), c->planes, GEMM_OUT_RESIDUAL, g);
+      launch_gemm_bf16(dev, p.rec(), c->planes, GEMM_OUT_RESIDUAL, g, c->pf_scratch);
     }
     if (!L.ff) continue;
     {
@@ -656,14 +660,14 @@ int run_pass(Ctx* c, const std::vector<Part>& parts, float** logits) {
       g.ldp = L.ldu;
       g.xielu = L.xielu;
       Prof p(dev, true, ST_PASS + ST_UP, 0.0);
-      launch_gemm_bf16(dev, p.rec(), c->planes, GEMM_OUT_XIELU, g);
+      launch_gemm_bf16(dev, p.rec(), c->planes, GEMM_OUT_XIELU, g, c->pf_scratch);
     }
     {
       GemmBf16 g = residual(c->pf_u, R * (size_t)c->ld_u, L.w_down, L.ldu);
       g.add_rows = add_rows;
       g.add_vec = add_vec;
       Prof p(dev, true, ST_PASS + ST_DOWN, 0.0);
-      launch_gemm_bf16(dev, p.rec(), c->planes, GEMM_OUT_RESIDUAL, g);
+      launch_gemm_bf16(dev, p.rec(), c->planes, GEMM_OUT_RESIDUAL, g, c->pf_scratch);
     }
   }
   for (size_t w0 = 0; w0 < nw; w0 += LOGIT_ROWS) {
@@ -688,7 +692,7 @@ int run_pass(Ctx* c, const std::vector<Part>& parts, float** logits) {
       g.ldo = c->vocab;
       g.cap = c->cfg.logit_softcap;
       Prof p(dev, true, ST_PASS + ST_HEAD, 0.0);
-      launch_gemm_bf16(dev, p.rec(), c->planes, GEMM_OUT_SOFTCAP, g);
+      launch_gemm_bf16(dev, p.rec(), c->planes, GEMM_OUT_SOFTCAP, g, c->pf_scratch);
     }
     CH_HIP(dev, hipMemcpyAsync(*logits, src, n * c->vocab * sizeof(float), hipMemcpyDeviceToHost, st));
     CH_HIP(dev, hipStreamSynchronize(st));

@@ -19,14 +19,7 @@ __device__ __forceinline__ unsigned short kv_from<unsigned short>(float f) { ret
 __device__ __forceinline__ float kv_to(float v) { return v; }
 __device__ __forceinline__ float kv_to(unsigned short v) { return bf2f(v); }
 // eight consecutive elements (16-byte aligned rows)
-__device__ __forceinline__ void kv_load8(const float* p, float (&o)[8]) {
-  const f32x4 a = *(const f32x4*)p, b = *(const f32x4*)(p + 4);
-#pragma unroll
-  for (int e = 0; e < 4; e++) {
-    o[e] = a[e];
-    o[e + 4] = b[e];
-  }
-}
+__device__ __forceinline__ void kv_load8(const float* p, float (&o)[8]) { read8(p, o); }
 __device__ __forceinline__ void kv_load8(const unsigned short* p, float (&o)[8]) {
   const i32x4 a = *(const i32x4*)p;
 #pragma unroll
