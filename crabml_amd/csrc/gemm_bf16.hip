@@ -1,25 +1,36 @@
 // gemm_bf16.hip -- the kernel behind gemm_bf16.hpp
 #include <cmath>
+#include <cstdlib>
 
 #include "gemm_bf16.hpp"
 
 namespace crabml_hip {
 
-__device__ __forceinline__ void lds_dma16(const void* g, void* l) {
-  __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)g, (__attribute__((address_space(3))) void*)l, 16, 0, 0);
+// 16 bytes per lane from memory into LDS at l + 16 lane (l: wave-uniform).  As assembly, because the compiler would wait for ALL of them
+// in front of the next LDS read (it cannot tell the buffers apart); who waits for what is landed_barrier's business.
+// (m0, the LDS address of such a load, needs one wait state behind its write; nothing else here uses it.)
+__device__ __forceinline__ void lds_dma16(const void* g, const void* l) {
+  const unsigned at = (unsigned)__builtin_amdgcn_readfirstlane((int)(unsigned)(size_t)(const __attribute__((address_space(3))) void*)l);
+  asm volatile("s_mov_b32 m0, %1\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %0, off" ::"v"(g), "s"(at) : "memory");
 }
-
 // four values as f32 / as bf16 planes (16- and 8-byte stores)
 __device__ __forceinline__ void store4(float* p, const float (&v)[4]) { *(f32x4*)p = f32x4{v[0], v[1], v[2], v[3]}; }
 
 // S > 1: k is cut into S pieces, one workgroup each.  A workgroup leaves its accumulators in ws (write-through) and counts itself in; the
 // one that comes last adds the others' pieces to its own, in piece order, and goes on to the epilogue.  The counter is left at zero.
-template <int BM, int BN, int WGM, int WGN, int P, int OUT>
-__global__ __launch_bounds__(256) void k_gemm_bf16(const GemmBf16 g, int S, float* __restrict__ ws, unsigned* __restrict__ tick) {
+// waits until at most N of this wave's memory requests are outstanding, then for the workgroup.  (__syncthreads would drain them all.)
+template <int N>
+__device__ __forceinline__ void landed_barrier() {
+  asm volatile("s_waitcnt vmcnt(%0) lgkmcnt(0)\n\ts_barrier" ::"n"(N) : "memory");
+}
+
+template <int BM, int BN, int WGM, int WGN, int ST, int P, int OUT>
+__global__ __launch_bounds__(64 * WGM * WGN) void k_gemm_bf16(const GemmBf16 g, int S, float* __restrict__ ws, unsigned* __restrict__ tick) {
   constexpr int WM = BM / WGM, WN = BN / WGN, TM = WM / 16, TN = WN / 16;
   constexpr int HR = BM < 64 ? BM : 64, LC = BN + 4;  // the epilogue's slab of rows in LDS
-  static_assert(WGM * WGN == 4 && WN == 64 && HR % WM == 0, "a wave's columns are one square-sum piece; its rows lie in one slab");
-  __shared__ __attribute__((aligned(16))) unsigned short lds[2][(BM + BN) * 64];
+  constexpr int NT = 64 * WGM * WGN, FA = BM * 8 / NT, FB = BN * 8 / NT;  // threads; a step's requests per thread
+  static_assert(WN == 64 && HR % WM == 0 && BM * 8 % NT == 0 && BN * 8 % NT == 0, "a wave's columns are one square-sum piece; its rows lie in one slab");
+  __shared__ __attribute__((aligned(16))) unsigned short lds[ST][(BM + BN) * 64];
   static_assert(sizeof(lds) >= (HR * LC + BM) * sizeof(float), "the epilogue reuses the tiles' LDS");
   const int tid = threadIdx.x, lane = tid & 63, wave = wave_in_wg();
   const int wm = wave / WGN, wn = wave % WGN;
@@ -42,17 +53,16 @@ __global__ __launch_bounds__(256) void k_gemm_bf16(const GemmBf16 g, int S, floa
     const int p = P == 1 ? 0 : s / steps, k0 = (P == 1 ? s : s - p * steps) * 64;
     const unsigned short* ap = g.a + (P == 1 ? 0 : (size_t)(P - 1 - p) * g.a_plane) + k0;  // (the smallest plane first)
 #pragma unroll
-    for (int it = 0; it < BM / 32; it++) {
-      const int slot = it * 256 + tid, r = slot >> 3, c = (slot & 7) ^ ((r >> 1) & 7);
-      lds_dma16(ap + (size_t)(row0 + r) * g.K + c * 8, &lds[buf][(it * 256 + wave * 64) * 8]);
+    for (int it = 0; it < FA; it++) {
+      const int slot = it * NT + tid, r = slot >> 3, c = (slot & 7) ^ ((r >> 1) & 7);
+      lds_dma16(ap + (size_t)(row0 + r) * g.K + c * 8, &lds[buf][(it * NT + wave * 64) * 8]);
     }
 #pragma unroll
-    for (int it = 0; it < BN / 32; it++) {
-      const int slot = it * 256 + tid, r = slot >> 3, c = (slot & 7) ^ ((r >> 1) & 7);
-      lds_dma16(g.w + (size_t)(col0 + r) * g.K + k0 + c * 8, &lds[buf][BM * 64 + (it * 256 + wave * 64) * 8]);
+    for (int it = 0; it < FB; it++) {
+      const int slot = it * NT + tid, r = slot >> 3, c = (slot & 7) ^ ((r >> 1) & 7);
+      lds_dma16(g.w + (size_t)(col0 + r) * g.K + k0 + c * 8, &lds[buf][BM * 64 + (it * NT + wave * 64) * 8]);
     }
   };
-  fetch(s_lo, 0);
   float factor = 1.f;  // of row tid, waiting for the epilogue
   if (g.sq_in != nullptr && tid < BM) {
     const float* q = g.sq_in + (size_t)(row0 + tid < g.M ? row0 + tid : g.M - 1) * g.n_sq;
@@ -62,11 +72,17 @@ __global__ __launch_bounds__(256) void k_gemm_bf16(const GemmBf16 g, int S, floa
     factor = *g.gain / sqrtf(s / (float)g.mean_n + g.eps);
   }
   const int fr = lane & 15, fk = lane >> 4;
+#pragma unroll
+  for (int i = 0; i < ST - 1; i++)
+    if (s_lo + i < s_hi) fetch(s_lo + i, i);
+  int buf = 0;
   for (int s = s_lo; s < s_hi; s++) {
-    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // this wave's part of step s has landed ...
-    __syncthreads();                                  // ... and everybody's; and step s - 1 has been read by every wave
-    const int buf = (s - s_lo) & 1;
-    if (s + 1 < s_hi) fetch(s + 1, buf ^ 1);
+    // step s has landed -- this wave's part (later steps' requests stay out), then everybody's -- and step s - 1 has been read by all
+    if (s + ST - 2 < s_hi)
+      landed_barrier<(ST - 2) * (FA + FB)>();
+    else
+      landed_barrier<0>();
+    if (s + ST - 1 < s_hi) fetch(s + ST - 1, buf == 0 ? ST - 1 : buf - 1);
     const unsigned short* la = &lds[buf][0];
     const unsigned short* lb = la + BM * 64;
 #pragma unroll
@@ -87,11 +103,12 @@ __global__ __launch_bounds__(256) void k_gemm_bf16(const GemmBf16 g, int S, floa
 #pragma unroll
         for (int j = 0; j < TN; j++) acc[i][j] = mfma_bf16(fa[i], fb[j], acc[i][j]);
     }
+    buf = buf + 1 == ST ? 0 : buf + 1;
   }
   if (S > 1) {
     constexpr int FRAG = TM * TN * 2;  // 8-byte halves of a lane's accumulators
-    unsigned long long* base = (unsigned long long*)ws + (size_t)tile * S * 256 * FRAG + tid;
-    unsigned long long* mine = base + (size_t)piece * 256 * FRAG;
+    unsigned long long* base = (unsigned long long*)ws + (size_t)tile * S * NT * FRAG + tid;
+    unsigned long long* mine = base + (size_t)piece * NT * FRAG;
 #pragma unroll
     for (int i = 0; i < TM; i++)
 #pragma unroll
@@ -99,7 +116,7 @@ __global__ __launch_bounds__(256) void k_gemm_bf16(const GemmBf16 g, int S, floa
 #pragma unroll
         for (int e = 0; e < 2; e++) {
           const f32x2 v = {acc[i][j][2 * e], acc[i][j][2 * e + 1]};
-          __hip_atomic_store(mine + ((i * TN + j) * 2 + e) * 256, __builtin_bit_cast(unsigned long long, v), __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+          __hip_atomic_store(mine + ((i * TN + j) * 2 + e) * NT, __builtin_bit_cast(unsigned long long, v), __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
         }
     asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // this thread's write-through stores have been acknowledged
     __shared__ unsigned s_last;
@@ -113,14 +130,14 @@ __global__ __launch_bounds__(256) void k_gemm_bf16(const GemmBf16 g, int S, floa
 #pragma unroll
       for (int j = 0; j < TN; j++) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
     for (int q = 0; q < S; q++) {  // (its own piece from memory as well: one order of addition, whoever is last)
-      const unsigned long long* p = base + (size_t)q * 256 * FRAG;
+      const unsigned long long* p = base + (size_t)q * NT * FRAG;
 #pragma unroll
       for (int i = 0; i < TM; i++)
 #pragma unroll
         for (int j = 0; j < TN; j++)
 #pragma unroll
           for (int e = 0; e < 2; e++) {
-            const f32x2 v = __builtin_bit_cast(f32x2, __hip_atomic_load(p + ((i * TN + j) * 2 + e) * 256, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT));
+            const f32x2 v = __builtin_bit_cast(f32x2, __hip_atomic_load(p + ((i * TN + j) * 2 + e) * NT, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT));
             acc[i][j][2 * e] += v[0];
             acc[i][j][2 * e + 1] += v[1];
           }
@@ -146,13 +163,13 @@ __global__ __launch_bounds__(256) void k_gemm_bf16(const GemmBf16 g, int S, floa
           for (int e = 0; e < 4; e++) lc[(wm * WM % HR + i * 16 + fk * 4 + e) * LC + wn * WN + j * 16 + fr] = acc[i][j][e];
     }
     __syncthreads();
-    constexpr int UNITS = HR * BN / 8 / 256;
+    constexpr int UNITS = HR * BN / 8 / NT;
     int row[UNITS], col[UNITS];
     bool in[UNITS];
     float v[UNITS][8], x[UNITS][8];
 #pragma unroll
     for (int u = 0; u < UNITS; u++) {
-      const int unit = u * 256 + tid, r = unit / (BN / 8), c = unit % (BN / 8) * 8;
+      const int unit = u * NT + tid, r = unit / (BN / 8), c = unit % (BN / 8) * 8;
       row[u] = row0 + h * HR + r;
       col[u] = col0 + c;
       in[u] = row[u] < g.M && col[u] < g.N;
@@ -239,29 +256,42 @@ __global__ __launch_bounds__(256) void k_gemm_bf16(const GemmBf16 g, int S, floa
   }
 }
 
-// Tile and k pieces: 128-row tiles unless there are fewer rows, k cut so that the launch fills the chip.  The estimate counts steps of
-// 64: what the busiest CU multiplies, against the latency of a workgroup's own chain; a cut costs the hand-over of the pieces.
+// Tile and k pieces.  A CU's time for a step of 64 (tile by tile, one workgroup after the other or side by side) and a workgroup's own
+// chain of steps are what was measured; a cut of k costs the hand-over of the pieces.
 struct GemmPlan {
   int bm, S;
 };
+struct TileCost {
+  int bm, resident;     // workgroups of this tile a CU holds
+  double step, chain;  // us per step of 64: the CU's share of the work; one workgroup's latency
+};
 static GemmPlan plan(const GemmBf16& g, int planes, int n_cu, size_t ws_floats) {
+  static const TileCost costs[] = {{256, 1, 0.95, 0.95}, {128, 1, 0.62, 0.62}, {64, 2, 0.40, 0.55}, {32, 2, 0.28, 0.45}};
   GemmPlan best{128, 1};
   double best_cost = 1e30;
   const int steps = g.K / 64 * planes;
-  for (int bm : {128, 64, 32}) {
-    if (bm > 32 && g.M <= bm / 2) continue;
-    const int tiles = ((g.M + bm - 1) / bm) * ((g.N + 127) / 128), resident = bm == 128 ? 2 : 3;
+  for (const TileCost& t : costs) {
+    if (t.bm > 32 && g.M <= t.bm / 2) continue;
+    const int tiles = ((g.M + t.bm - 1) / t.bm) * ((g.N + 127) / 128);
     for (int S : {1, 2, 3, 4, 6, 8}) {
-      if (S > 1 && (steps / S < 6 || (size_t)tiles * S * bm * 128 > ws_floats || tiles > GEMM_TICKS)) break;
+      if (S > 1 && (steps / S < 6 || (size_t)tiles * S * t.bm * 128 > ws_floats || tiles > GEMM_TICKS)) break;
       const double per = (double)steps / S, wgs = (double)tiles * S;
-      const double busy = ceil(wgs / n_cu) * (per * 0.36 * (bm == 128 ? 1.0 : bm == 64 ? 0.6 : 0.45) + 1.5);
-      const double chain = ceil(wgs / (n_cu * resident)) * (per * 0.55 + 3.0);
-      const double cost = (busy > chain ? busy : chain) + (S > 1 ? 4.0 + 0.8 * S * bm / 128 : 0.0);
+      const double busy = ceil(wgs / n_cu) * (per * t.step + 2.0), chain = ceil(wgs / (n_cu * t.resident)) * (per * t.chain + 4.0);
+      const double cost = (busy > chain ? busy : chain) + (S > 1 ? 4.0 + 1.2 * S * t.bm / 128 : 0.0);
       if (cost < best_cost) {
         best_cost = cost;
-        best = {bm, S};
+        best = {t.bm, S};
       }
     }
+  }
+  static const int force = [] {  // lab hook (CRABML_HIP_TEST_HOOKS=1 CRABML_HIP_GEMM_BF16_PLAN=rows*100+pieces)
+    const char* h = getenv("CRABML_HIP_TEST_HOOKS");
+    const char* e = getenv("CRABML_HIP_GEMM_BF16_PLAN");
+    return h && h[0] == '1' && e ? atoi(e) : 0;
+  }();
+  if (force) {
+    const int bm = force / 100, S = force % 100, tiles = ((g.M + bm - 1) / bm) * ((g.N + 127) / 128);
+    if ((bm == 256 || bm == 128 || bm == 64 || bm == 32) && S >= 1 && S <= steps && (S == 1 || ((size_t)tiles * S * bm * 128 <= ws_floats && tiles <= GEMM_TICKS))) return {bm, S};
   }
   return best;
 }
@@ -270,12 +300,14 @@ template <int P, int OUT>
 static void launch_t(hipStream_t st, crabml_hip_device::ProfRec* rec, const GemmBf16& g, int n_cu, const GemmScratch& w) {
   const GemmPlan p = plan(g, P, n_cu, w.floats);
   const dim3 grid(((g.M + p.bm - 1) / p.bm) * ((g.N + 127) / 128) * p.S);
-  if (p.bm == 128)
-    launch_k(st, rec, k_gemm_bf16<128, 128, 2, 2, P, OUT>, grid, dim3(256), 0, g, p.S, w.partials, w.ticks);
+  if (p.bm == 256)
+    launch_k(st, rec, k_gemm_bf16<256, 128, 4, 2, 3, P, OUT>, grid, dim3(512), 0, g, p.S, w.partials, w.ticks);
+  else if (p.bm == 128)
+    launch_k(st, rec, k_gemm_bf16<128, 128, 2, 2, 4, P, OUT>, grid, dim3(256), 0, g, p.S, w.partials, w.ticks);
   else if (p.bm == 64)
-    launch_k(st, rec, k_gemm_bf16<64, 128, 2, 2, P, OUT>, grid, dim3(256), 0, g, p.S, w.partials, w.ticks);
+    launch_k(st, rec, k_gemm_bf16<64, 128, 2, 2, 3, P, OUT>, grid, dim3(256), 0, g, p.S, w.partials, w.ticks);
   else
-    launch_k(st, rec, k_gemm_bf16<32, 128, 2, 2, P, OUT>, grid, dim3(256), 0, g, p.S, w.partials, w.ticks);
+    launch_k(st, rec, k_gemm_bf16<32, 128, 2, 2, 4, P, OUT>, grid, dim3(256), 0, g, p.S, w.partials, w.ticks);
 }
 
 void launch_gemm_bf16(crabml_hip_device* dev, crabml_hip_device::ProfRec* rec, int planes, int out, const GemmBf16& g, const GemmScratch& w) {

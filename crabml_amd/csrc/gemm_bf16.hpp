@@ -6,11 +6,11 @@
 // bits (split3): every f32 is the exact sum of its planes and every plane times a bf16 weight is exact in f32, so three planes give
 // true f32 products with f32 sums -- the weights ARE bf16 numbers -- at a fifth of the time the f32 matrix instruction would take.
 //
-// Mapping: BM x BN output tile per 256-thread workgroup, k in steps of 64.  A step's tiles go from memory straight into LDS
-// (global_load_lds, 16 bytes per lane), double-buffered: the next step's requests are out before the current one is multiplied.  LDS
-// holds rows of 128 bytes whose 16-byte chunks are permuted by (row / 2) % 8 -- on the SOURCE side, the LDS side of the instruction
+// Mapping: BM x 128 output tile per workgroup (BM = 256: eight waves; else four), k in steps of 64.  A step's tiles go from memory
+// straight into LDS (global_load_lds, 16 bytes per lane); three or four steps are in LDS or on their way, and a wave waits for the oldest
+// only (s_waitcnt vmcnt(n)).  LDS holds rows of 128 bytes whose 16-byte chunks are permuted by (row / 2) % 8 -- on the SOURCE side, the LDS side of the instruction
 // being linear -- so that the 16 rows a fragment read touches spread over all 64 banks.  Operands are padded by their owners (k to 64,
-// weight rows to 256, activation rows to 128), so the loop has no bounds checks; stores have.  Short launches cut k into pieces (the
+// weight rows to 256, activation rows to 256), so the loop has no bounds checks; stores have.  Short launches cut k into pieces (the
 // last workgroup of a tile adds them).  Workgroups are dealt to the eight XCDs
 // in contiguous runs of the tile order, row tiles fastest: an XCD's L2 keeps the weight tile that its row tiles share.
 //

@@ -458,7 +458,7 @@ int step_begin(Ctx* c, size_t n, const size_t* seqs, const uint32_t* tokens) {
 int pass_alloc(Ctx* c) {
   if (c->rows_cap) return 0;
   crabml_hip_device* dev = c->dev;
-  const size_t R = align_up(c->cfg.pass_rows ? c->cfg.pass_rows : 2048, 128), P = (size_t)c->planes;
+  const size_t R = align_up(c->cfg.pass_rows ? c->cfg.pass_rows : 2048, 256), P = (size_t)c->planes;
   size_t lin = 0;
   for (const Layer& L : c->layers) lin = std::max(lin, (size_t)L.li.H * L.li.V);
   CH_TRY(dalloc_n(c, R * c->ldx, &c->pf_x));
