@@ -263,10 +263,10 @@ struct GemmPlan {
 };
 struct TileCost {
   int bm, resident;     // workgroups of this tile a CU holds
-  double step, chain;  // us per step of 64: the CU's share of the work; one workgroup's latency
+  double step, chain;   // us per step of 64: a workgroup's share of a busy CU; the latency of one alone
 };
 static GemmPlan plan(const GemmBf16& g, int planes, int n_cu, size_t ws_floats) {
-  static const TileCost costs[] = {{256, 1, 0.95, 0.95}, {128, 1, 0.62, 0.62}, {64, 2, 0.40, 0.55}, {32, 2, 0.28, 0.45}};
+  static const TileCost costs[] = {{256, 1, 1.03, 1.03}, {128, 1, 0.68, 0.68}, {64, 2, 0.42, 0.51}, {32, 2, 0.41, 0.41}};
   GemmPlan best{128, 1};
   double best_cost = 1e30;
   const int steps = g.K / 64 * planes;
@@ -275,9 +275,9 @@ static GemmPlan plan(const GemmBf16& g, int planes, int n_cu, size_t ws_floats) 
     const int tiles = ((g.M + t.bm - 1) / t.bm) * ((g.N + 127) / 128);
     for (int S : {1, 2, 3, 4, 6, 8}) {
       if (S > 1 && (steps / S < 6 || (size_t)tiles * S * t.bm * 128 > ws_floats || tiles > GEMM_TICKS)) break;
-      const double per = (double)steps / S, wgs = (double)tiles * S;
-      const double busy = ceil(wgs / n_cu) * (per * t.step + 2.0), chain = ceil(wgs / (n_cu * t.resident)) * (per * t.chain + 4.0);
-      const double cost = (busy > chain ? busy : chain) + (S > 1 ? 4.0 + 1.2 * S * t.bm / 128 : 0.0);
+      const double per = (double)steps / S, wgs = (double)tiles * S, rounds = ceil(wgs / (n_cu * t.resident));
+      const double busy = ceil(wgs / n_cu) * per * t.step, chain = rounds * per * t.chain;
+      const double cost = (busy > chain ? busy : chain) + 6.0 * rounds + (S > 1 ? 8.0 + 1.3 * S * t.bm / 128 : 0.0);
       if (cost < best_cost) {
         best_cost = cost;
         best = {t.bm, S};

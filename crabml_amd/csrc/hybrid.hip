@@ -75,6 +75,8 @@ struct crabml_hip_hybrid {
   unsigned short *pf_xp = nullptr, *pf_cat = nullptr, *pf_u = nullptr, *pf_gp = nullptr;
   void* pf_proj = nullptr;
   GemmScratch pf_scratch;
+  hipStream_t side = nullptr;  // the linear branch of a long pass, beside the softmax branch
+  hipEvent_t fork = nullptr, join = nullptr;
   std::vector<std::pair<void*, size_t>> allocs;
 };
 
@@ -479,6 +481,9 @@ int pass_alloc(Ctx* c) {
   c->meta_bytes = R * (sizeof(PassSeq) + 2 * sizeof(PassTile) + sizeof(PassRow) + 2 * sizeof(int));
   CH_TRY(dalloc(c, c->meta_bytes, (void**)&c->meta));
   CH_HIP(dev, hipHostMalloc((void**)&c->h_meta, c->meta_bytes * META_SLOTS, hipHostMallocDefault));
+  CH_HIP(dev, hipStreamCreateWithFlags(&c->side, hipStreamNonBlocking));
+  CH_HIP(dev, hipEventCreateWithFlags(&c->fork, hipEventDisableTiming));
+  CH_HIP(dev, hipEventCreateWithFlags(&c->join, hipEventDisableTiming));
   c->rows_cap = R;
   return 0;
 }
@@ -501,10 +506,10 @@ void launch_attn_cls(Ctx* c, crabml_hip_device::ProfRec* rec, MixRows<T> m, cons
   launch_k(c->dev->stream, rec, k_attn_rows<T, CLS, sizeof(T) == 2 ? 1 : 3>, dim3(m.n_tiles, m.at.H), dim3(256), 0, m);
 }
 template <typename T, int CLS>
-int launch_linear_cls(Ctx* c, crabml_hip_device::ProfRec* rec, const MixRows<T>& m, size_t n_seq) {
+int launch_linear_cls(Ctx* c, hipStream_t st, crabml_hip_device::ProfRec* rec, const MixRows<T>& m, size_t n_seq) {
   const size_t lds = LinTile<T, CLS>::LDS;
   CH_HIP(c->dev, raise_dyn_lds(c->dev, (const void*)k_linear_rows<T, CLS>, (int)lds));
-  launch_k(c->dev->stream, rec, k_linear_rows<T, CLS>, dim3(m.li.H * m.li.slices, (unsigned)n_seq), dim3(256), lds, m);
+  launch_k(st, rec, k_linear_rows<T, CLS>, dim3(m.li.H * m.li.slices, (unsigned)n_seq), dim3(256), lds, m);
   return 0;
 }
 
@@ -525,6 +530,23 @@ int mix_rows(Ctx* c, const Run& run, const PassSeq* seqs, size_t n_seq, const Pa
   m.ldp = L.n_in;
   m.ldc = L.ldc;
   m.lin_off = L.lin_off;
+  // the linear branch is a chain of blocks on few CUs: beside the softmax branch, when both are long enough to hide a fork
+  hipStream_t st = c->dev->stream, lin_st = st;
+  if (L.at.H && L.li.H && n_rows >= 192 && !c->dev->prof_on) {
+    lin_st = c->side;
+    CH_HIP(c->dev, hipEventRecord(c->fork, st));
+    CH_HIP(c->dev, hipStreamWaitEvent(lin_st, c->fork, 0));
+  }
+  if (L.li.H) {
+    Prof p(c->dev, true, ST_PASS + ST_LIN, 0.0);
+    if (L.li.D <= 64)
+      CH_TRY((launch_linear_cls<T, 64>(c, lin_st, p.rec(), m, n_seq)));
+    else if (L.li.D <= 128)
+      CH_TRY((launch_linear_cls<T, 128>(c, lin_st, p.rec(), m, n_seq)));
+    else
+      CH_TRY((launch_linear_cls<T, 256>(c, lin_st, p.rec(), m, n_seq)));
+  }
+  if (lin_st != st) CH_HIP(c->dev, hipEventRecord(c->join, lin_st));
   if (L.at.H) {
     Prof p(c->dev, true, ST_PASS + ST_MIX, 0.0);
     const int w = std::max(L.at.D, L.at.V);
@@ -535,15 +557,7 @@ int mix_rows(Ctx* c, const Run& run, const PassSeq* seqs, size_t n_seq, const Pa
     else
       launch_attn_cls<T, 256>(c, p.rec(), m, tiles);
   }
-  if (L.li.H) {
-    Prof p(c->dev, true, ST_PASS + ST_LIN, 0.0);
-    if (L.li.D <= 64)
-      CH_TRY((launch_linear_cls<T, 64>(c, p.rec(), m, n_seq)));
-    else if (L.li.D <= 128)
-      CH_TRY((launch_linear_cls<T, 128>(c, p.rec(), m, n_seq)));
-    else
-      CH_TRY((launch_linear_cls<T, 256>(c, p.rec(), m, n_seq)));
-  }
+  if (lin_st != st) CH_HIP(c->dev, hipStreamWaitEvent(st, c->join, 0));
   Prof p(c->dev, true, ST_PASS + ST_ROWS, 0.0);
   launch_k(c->dev->stream, p.rec(), k_mix_rows<T, P>, dim3((unsigned)n_rows), dim3(256), 0, m, c->cfg.norm_eps);
   return 0;
@@ -834,6 +848,12 @@ int crabml_hip_hybrid_destroy(crabml_hip_hybrid_t* c) {
   for (auto& s : c->seqs)
     if (s.open) pool_free(c->dev, s.slab, s.cap);
   for (auto& a : c->allocs) pool_free(c->dev, a.first, a.second);
+  if (c->side) {
+    (void)hipStreamSynchronize(c->side);
+    (void)hipStreamDestroy(c->side);
+  }
+  if (c->fork) (void)hipEventDestroy(c->fork);
+  if (c->join) (void)hipEventDestroy(c->join);
   if (c->h_seq) (void)hipHostFree(c->h_seq);
   if (c->h_meta) (void)hipHostFree(c->h_meta);
   delete c;
