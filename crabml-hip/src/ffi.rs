@@ -30,6 +30,9 @@ pub const CRABML_HIP_LLAMA_TP_SPLIT_VOCAB: i32 = 1048576;
 
 /// the hybrid decoder: launch decode steps eagerly
 pub const CRABML_HIP_HYBRID_NO_GRAPH: i32 = 1;
+/// ... norm gains per element, and stored around zero
+pub const CRABML_HIP_HYBRID_NORM_VECTOR: i32 = 2;
+pub const CRABML_HIP_HYBRID_NORM_ONE_PLUS: i32 = 4;
 /// GGML's id of bfloat16 (weights only; crabml's own GGMLType has no such entry)
 pub const CRABML_HIP_BF16: u32 = 30;
 
@@ -115,6 +118,8 @@ pub struct crabml_hip_hybrid_config_t {
     pub logit_softcap: f32,
     pub compute: u32,
     pub flags: i32,
+    pub streams: usize,
+    pub position_base: f64,
 }
 
 #[repr(C)]
@@ -151,6 +156,28 @@ pub struct crabml_hip_hybrid_layer_t {
     pub ff_up: *const crabml_hip_buf_t,
     pub ff_down: *const crabml_hip_buf_t,
     pub ff_act: *const crabml_hip_buf_t,
+    pub attn_window: usize,
+    pub attn_latent: usize,
+    pub attn_rot: usize,
+    pub attn_rot_base: f64,
+    pub attn_q_bias: *const crabml_hip_buf_t,
+    pub attn_k_bias: *const crabml_hip_buf_t,
+    pub attn_v_bias: *const crabml_hip_buf_t,
+    pub attn_o_bias: *const crabml_hip_buf_t,
+    pub attn_q_norm: *const crabml_hip_buf_t,
+    pub attn_k_norm: *const crabml_hip_buf_t,
+    pub attn_vmix: *const crabml_hip_buf_t,
+    pub attn_latent_down: *const crabml_hip_buf_t,
+    pub attn_latent_norm: *const crabml_hip_buf_t,
+    pub attn_key_up: *const crabml_hip_buf_t,
+    pub attn_value_up: *const crabml_hip_buf_t,
+    pub ff_gate: *const crabml_hip_buf_t,
+    pub hc1_in: *const crabml_hip_buf_t,
+    pub hc1_out: *const crabml_hip_buf_t,
+    pub hc1_mix: *const crabml_hip_buf_t,
+    pub hc2_in: *const crabml_hip_buf_t,
+    pub hc2_out: *const crabml_hip_buf_t,
+    pub hc2_mix: *const crabml_hip_buf_t,
 }
 
 #[repr(C)]

@@ -1,5 +1,6 @@
 //! `HipHybridRunner`: sequences and batched steps of the hybrid decoder (`crabml_hip_hybrid_*`) -- models whose layers mix
-//! chunked softmax attention with decaying linear attention, which crabml's `Tensor` trait has no op sequence for.  The caller
+//! softmax attention (in chunks, in a window, on latents) with decaying linear attention, gated units and residual streams,
+//! which crabml's `Tensor` trait has no op sequence for.  The caller
 //! fills `crabml_hip_hybrid_config_t` / `_layer_t` / `_weights_t` from its model files; matrices are copied at creation, so the
 //! tensors behind the handles may be dropped afterwards.
 

@@ -69,7 +69,7 @@ __global__ __launch_bounds__(64 * WGM * WGN) void k_gemm_bf16(const GemmBf16 g, 
     float s = 0.f;
 #pragma unroll 8
     for (int i = 0; i < g.n_sq; i++) s += q[i];
-    factor = *g.gain / sqrtf(s / (float)g.mean_n + g.eps);
+    factor = (g.gain ? *g.gain : 1.0f) / sqrtf(s / (float)g.mean_n + g.eps);
   }
   const int fr = lane & 15, fk = lane >> 4;
 #pragma unroll
@@ -164,6 +164,35 @@ __global__ __launch_bounds__(64 * WGM * WGN) void k_gemm_bf16(const GemmBf16 g, 
     }
     __syncthreads();
     constexpr int UNITS = HR * BN / 8 / NT;
+    if constexpr (OUT == GEMM_OUT_STREAMS) {  // four columns of all streams in registers at a time
+#pragma unroll 1
+      for (int unit = tid; unit < HR * BN / 8; unit += NT) {
+        const int r = unit / (BN / 8), c = unit % (BN / 8) * 8, row = row0 + h * HR + r, col = col0 + c;
+        const bool in = row < g.M && col < g.N;
+        float sq = 0.f;
+        if (in) {
+          const float f = lf[h * HR + r];
+          float v[8];
+#pragma unroll
+          for (int k = 0; k < 8; k += 4) {
+            f32x4 y = *(const f32x4*)(lc + r * LC + c + k) * f;
+            if (g.bias) y += *(const f32x4*)(g.bias + col + k);
+            const f32x4 n = stream_mix(g.sm, g.x + (size_t)row * g.ldx + col + k, y), gain = *(const f32x4*)(g.gain_next + col + k);
+#pragma unroll
+            for (int e = 0; e < 4; e++) {
+              sq = __builtin_fmaf(n[e], n[e], sq);
+              v[k + e] = n[e] * gain[e];
+            }
+          }
+          split_store8<P>(v, g.planes + (size_t)row * g.ldp + col, g.p_plane);
+        }
+        sq += dpp_f<0xB1>(sq);  // eight lanes hold a row's 64 columns
+        sq += dpp_f<0x4E>(sq);
+        sq += dpp_f<0x141>(sq);
+        if (in && (tid & 7) == 0) g.sq_out[(size_t)row * g.n_sq_out + col / 64] = sq;
+      }
+      continue;
+    }
     int row[UNITS], col[UNITS];
     bool in[UNITS];
     float v[UNITS][8], x[UNITS][8];
@@ -215,6 +244,22 @@ __global__ __launch_bounds__(64 * WGM * WGN) void k_gemm_bf16(const GemmBf16 g, 
           for (int e = 0; e < 8; e++)
             if (col[u] + e < g.N) ((float*)g.out)[(size_t)row[u] * g.ldo + col[u] + e] = soft_cap(v[u][e], g.cap);
         }
+        continue;
+      }
+      if constexpr (OUT == GEMM_OUT_ACT_BF16 || OUT == GEMM_OUT_ACT_F32) {
+        if (g.bias && in[u]) {
+          float t[8];
+          read8(g.bias + col[u], t);
+#pragma unroll
+          for (int e = 0; e < 8; e++) v[u][e] += t[e];
+        }
+      }
+      if constexpr (OUT == GEMM_OUT_GLU) {
+        if (!in[u]) continue;
+        float t[4];
+#pragma unroll
+        for (int e = 0; e < 4; e++) t[e] = gelu_tanh(v[u][2 * e]) * v[u][2 * e + 1];
+        split_store4<P>(t, g.planes + (size_t)row[u] * g.ldp + col[u] / 2, g.p_plane);
         continue;
       }
 #pragma unroll
@@ -318,6 +363,8 @@ void launch_gemm_bf16(crabml_hip_device* dev, crabml_hip_device::ProfRec* rec, i
       case GEMM_OUT_ACT_BF16: launch_t<1, GEMM_OUT_ACT_BF16>(st, rec, g, n, w); break;
       case GEMM_OUT_RESIDUAL: launch_t<1, GEMM_OUT_RESIDUAL>(st, rec, g, n, w); break;
       case GEMM_OUT_XIELU: launch_t<1, GEMM_OUT_XIELU>(st, rec, g, n, w); break;
+      case GEMM_OUT_STREAMS: launch_t<1, GEMM_OUT_STREAMS>(st, rec, g, n, w); break;
+      case GEMM_OUT_GLU: launch_t<1, GEMM_OUT_GLU>(st, rec, g, n, w); break;
       default: launch_t<1, GEMM_OUT_SOFTCAP>(st, rec, g, n, w); break;
     }
   } else {
@@ -325,6 +372,8 @@ void launch_gemm_bf16(crabml_hip_device* dev, crabml_hip_device::ProfRec* rec, i
       case GEMM_OUT_ACT_F32: launch_t<3, GEMM_OUT_ACT_F32>(st, rec, g, n, w); break;
       case GEMM_OUT_RESIDUAL: launch_t<3, GEMM_OUT_RESIDUAL>(st, rec, g, n, w); break;
       case GEMM_OUT_XIELU: launch_t<3, GEMM_OUT_XIELU>(st, rec, g, n, w); break;
+      case GEMM_OUT_STREAMS: launch_t<3, GEMM_OUT_STREAMS>(st, rec, g, n, w); break;
+      case GEMM_OUT_GLU: launch_t<3, GEMM_OUT_GLU>(st, rec, g, n, w); break;
       default: launch_t<3, GEMM_OUT_SOFTCAP>(st, rec, g, n, w); break;
     }
   }

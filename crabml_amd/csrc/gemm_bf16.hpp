@@ -15,8 +15,9 @@
 // in contiguous runs of the tile order, row tiles fastest: an XCD's L2 keeps the weight tile that its row tiles share.
 //
 // The row operations around a linear are folded into it.  In: an RMS norm with a single gain is a factor per row, applied to the
-// accumulators (the producers leave each row's sum of squares in 64-column pieces).  Out: activations by column range, xIELU, soft
-// cap, or the residual add, which also leaves the new row's bf16 planes and square sums for the next linear.
+// accumulators (the producers leave each row's sum of squares in 64-column pieces); a gain per column is in the planes already.  Out:
+// activations by column range, xIELU, a gated unit, soft cap, or the residual add (of one stream or of several that mix), which also
+// leaves the new row's bf16 planes and square sums for the next linear.
 #pragma once
 #include "gemv_bf16.hpp"
 
@@ -30,6 +31,8 @@ enum {
   GEMM_OUT_RESIDUAL = 2,   // x += acc (+ add_rows + add_vec); planes of x; square sums
   GEMM_OUT_XIELU = 3,      // planes of xielu(acc)
   GEMM_OUT_SOFTCAP = 4,    // f32 rows
+  GEMM_OUT_STREAMS = 5,    // the residual streams take acc (+ bias); planes of gain_next * what the next linear reads; its square sums
+  GEMM_OUT_GLU = 6,        // weight rows 2 j, 2 j + 1 are gate j and up j: planes of gelu(gate) * up
 };
 
 // an f32 as bf16 planes: 1 plane = rounded to nearest even; 3 planes = upper / middle / lower bits, their sum exact
@@ -84,7 +87,7 @@ struct GemmBf16 {
   size_t a_plane = 0;                 // elements between planes
   const unsigned short* w = nullptr;  // [N padded][k]
   int M = 0, N = 0, K = 0;            // K % 64 == 0
-  // row factor (nullable sq): gain / sqrt(sum_i sq[row][i] / mean_n + eps)
+  // row factor (nullable sq): gain (nullable: 1) / sqrt(sum_i sq[row][i] / mean_n + eps)
   const float* sq_in = nullptr;
   int n_sq = 0, mean_n = 1;
   float eps = 0.f;
@@ -95,10 +98,13 @@ struct GemmBf16 {
   ActRanges act;
   const float* xielu = nullptr;
   float cap = 0.f;
-  float* x = nullptr;  // RESIDUAL
+  const float* bias = nullptr;  // [N padded to 8], nullable (ACT, STREAMS)
+  float* x = nullptr;           // RESIDUAL; STREAMS: stream 0
+  StreamMix sm;
+  const float* gain_next = nullptr;  // STREAMS: a gain per column of the next RMS norm
   int ldx = 0;
   const float *add_rows = nullptr, *add_vec = nullptr;
-  unsigned short* planes = nullptr;  // RESIDUAL / XIELU: [planes][rows padded][ldp]
+  unsigned short* planes = nullptr;  // RESIDUAL / STREAMS / XIELU / GLU: [planes][rows padded][ldp]
   size_t p_plane = 0;
   int ldp = 0;
   float* sq_out = nullptr;  // [row][n_sq_out]: square sums by 64 columns

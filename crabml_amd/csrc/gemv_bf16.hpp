@@ -18,20 +18,60 @@ enum {
   GEMV_IN_RMS = 1,    // the row is RMS-normalized with a single gain.  The row factor is taken from the staged row itself and
                       // applied to the finished dots: W (s x) = s (W x)
   GEMV_IN_SPLIT = 2,  // elements from k_split on still want their RMS normalization; their sum of squares arrives in pieces (ss)
+  GEMV_IN_RMSV = 3,   // GEMV_IN_RMS with a gain per element (gain: K numbers), applied while the row is staged
 };
 // what happens to a dot product on the way out
 enum {
   GEMV_OUT_STORE = 0,
-  GEMV_OUT_ACT = 1,      // column ranges with their own activation (ActRanges)
+  GEMV_OUT_ACT = 1,      // (+ bias) column ranges with their own activation (ActRanges)
   GEMV_OUT_RESIDUAL = 2, // out += dot (+ add_rows[b] + add_vec)
   GEMV_OUT_XIELU = 3,    // xielu(dot)
   GEMV_OUT_SOFTCAP = 4,  // cap * tanh(dot / cap)
+  GEMV_OUT_STREAMS = 5,  // (+ bias) into the residual streams; what the next linear reads goes to u
+  GEMV_OUT_GLU = 6,      // weight rows 2 j, 2 j + 1 are gate j and up j: out[j] = gelu(gate) * up
 };
 enum { ACT_NONE = 0, ACT_SIGMOID = 1, ACT_SILU = 2 };
 struct ActRanges {  // columns [end[i-1], end[i]) take activation kind[i]
   int end[4] = {0, 0, 0, 0};
   int kind[4] = {0, 0, 0, 0};
 };
+
+// Residual streams: a sublayer's result y turns the n streams x_s into x_t = sum_s mix[s][t] x_s + out[t] y, and the next linear reads
+// u = sum_t in[t] x_t.  All of it is local to an element, so it is the epilogue of the sublayer's last linear.
+#define HC_MAX 8
+#define HC_ROW (HC_MAX + 1)
+struct StreamMix {
+  int n = 0;
+  size_t stride = 0;            // floats between the streams
+  const float* coef = nullptr;  // [n][HC_ROW]: row t = mix[0 .. HC_MAX)[t] (zeros from n on), out[t]
+  const float* in = nullptr;    // [n]: of the sublayer that comes next
+};
+template <typename V>
+__device__ __forceinline__ V stream_mix(const StreamMix& m, float* x, V y) {  // x: this element (or vector of neighbours) of stream 0
+  V old[HC_MAX], u = V{};
+  // (four at a time without a branch each -- past the last stream the first one again, with a zero coefficient)
+#pragma unroll
+  for (int s = 0; s < 4; s++) old[s] = *(const V*)(x + (s < m.n ? s : 0) * m.stride);
+#pragma unroll
+  for (int s = 4; s < HC_MAX; s++) old[s] = V{};
+  if (m.n > 4) {
+#pragma unroll
+    for (int s = 4; s < HC_MAX; s++) old[s] = *(const V*)(x + (s < m.n ? s : 0) * m.stride);
+  }
+  // (constant address space: scalar loads, which the stores below cannot be taken to change)
+  typedef const float __attribute__((address_space(4))) constant;
+  constant *coef = (constant*)(size_t)m.coef, *in = (constant*)(size_t)m.in;
+#pragma unroll 1
+  for (int t = 0; t < m.n; t++) {
+    constant* c = coef + t * HC_ROW;
+    V v = c[HC_MAX] * y;
+#pragma unroll
+    for (int s = 0; s < HC_MAX; s++) v += c[s] * old[s];
+    *(V*)(x + t * m.stride) = v;
+    u += in[t] * v;
+  }
+  return u;
+}
 
 struct GemvBf16 {
   const unsigned short* w = nullptr;  // [N][ldw]
@@ -49,6 +89,9 @@ struct GemvBf16 {
   const float *add_rows = nullptr, *add_vec = nullptr;
   int ld_add = 0;
   float cap = 0.f;
+  const float* bias = nullptr;  // [N], nullable (ACT, STREAMS)
+  StreamMix sm;                 // STREAMS: out = stream 0, u[b][ldo] = what the next linear reads
+  float* u = nullptr;
 };
 
 __device__ __forceinline__ float act_sigmoid(float z) { return 1.0f / (1.0f + __expf(-z)); }
@@ -79,13 +122,20 @@ __device__ __forceinline__ float xielu_apply(float z, float right, float left) {
   const float curved = z > 0.0f ? right * z * z : left * exp_minus_line(z);
   return __builtin_fmaf(0.5f, z, curved);
 }
+// z / 2 (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3))), the bracket's half being a logistic function of twice the argument
+__device__ __forceinline__ float gelu_tanh(float z) {
+  const float t = 1.5957691216057308f * __builtin_fmaf(0.044715f * z, z * z, z);
+  return z / (1.0f + __expf(-t));
+}
 __device__ __forceinline__ float soft_cap(float z, float cap) { return cap > 0.0f ? cap * tanhf(z / cap) : z; }
 
 template <int OUT>
 __device__ __forceinline__ void gemv_out(const GemvBf16& a, int row, int b, float v) {
   float* o = a.out + (size_t)b * a.ldo + row;
   if constexpr (OUT == GEMV_OUT_STORE) *o = v;
+  if constexpr (OUT == GEMV_OUT_ACT || OUT == GEMV_OUT_STREAMS) v += a.bias ? a.bias[row] : 0.f;
   if constexpr (OUT == GEMV_OUT_ACT) *o = act_ranges(v, row, a.act);
+  if constexpr (OUT == GEMV_OUT_STREAMS) a.u[(size_t)b * a.ldo + row] = stream_mix(a.sm, o, v);
   if constexpr (OUT == GEMV_OUT_RESIDUAL) {
     float s = *o + v;
     if (a.add_rows) s += a.add_rows[(size_t)b * a.ld_add + row];
@@ -155,9 +205,13 @@ __global__ __launch_bounds__(256) void k_gemv_bf16(const GemvBf16 a) {
       float* lo = gemv_lds + b * 2 * half;
       for (int q = tid; q < n / 8; q += 256) {
         f32x4 v0 = *(const f32x4*)(xr + q * 8), v1 = *(const f32x4*)(xr + q * 8 + 4);
-        if constexpr (IN == GEMV_IN_RMS) {
+        if constexpr (IN == GEMV_IN_RMS || IN == GEMV_IN_RMSV) {
 #pragma unroll
           for (int e = 0; e < 4; e++) sq[b] = __builtin_fmaf(v0[e], v0[e], __builtin_fmaf(v1[e], v1[e], sq[b]));
+        }
+        if constexpr (IN == GEMV_IN_RMSV) {
+          v0 *= *(const f32x4*)(a.gain + s0 + q * 8);
+          v1 *= *(const f32x4*)(a.gain + s0 + q * 8 + 4);
         }
         if constexpr (IN == GEMV_IN_SPLIT) {
           if (s0 + q * 8 >= a.k_split) {
@@ -169,7 +223,7 @@ __global__ __launch_bounds__(256) void k_gemv_bf16(const GemvBf16 a) {
         *(f32x4*)(lo + half + q * 4) = v1;
       }
     }
-    if constexpr (IN == GEMV_IN_RMS) {
+    if constexpr (IN == GEMV_IN_RMS || IN == GEMV_IN_RMSV) {
       if (s0 + seg >= a.K) {
 #pragma unroll
         for (int b = 0; b < NB; b++) {
@@ -216,10 +270,22 @@ __global__ __launch_bounds__(256) void k_gemv_bf16(const GemvBf16 a) {
 #pragma unroll
   for (int b = 0; b < NB; b++) {
     scale[b] = 1.f;
-    if constexpr (IN == GEMV_IN_RMS) {
+    if constexpr (IN == GEMV_IN_RMS || IN == GEMV_IN_RMSV) {
       const float s = (red[0][b] + red[1][b]) + (red[2][b] + red[3][b]);
-      scale[b] = *a.gain / sqrtf(s / (float)a.mean_n + a.eps);
+      scale[b] = (IN == GEMV_IN_RMS ? *a.gain : 1.0f) / sqrtf(s / (float)a.mean_n + a.eps);
     }
+  }
+  if constexpr (OUT == GEMV_OUT_GLU) {
+    static_assert(R % 2 == 0, "a wave holds both rows of a pair");
+#pragma unroll
+    for (int r = 0; r < R; r += 2)
+#pragma unroll
+      for (int b = 0; b < NB; b++) {
+        const float gate = wave_sum_f32(acc[r][b]) * scale[b], up = wave_sum_f32(acc[r + 1][b]) * scale[b];
+        const int row = row0 + r, bb = b0 + b;
+        if (lane == ((r / 2 * NB + b) & 63) && row < a.N && bb < a.nb) a.out[(size_t)bb * a.ldo + row / 2] = gelu_tanh(gate) * up;
+      }
+    return;
   }
 #pragma unroll
   for (int r = 0; r < R; r++)
@@ -271,7 +337,7 @@ __global__ __launch_bounds__(512) void k_gemv16_bf16(const GemvBf16 a) {
   }
   const float* xr = a.x + (size_t)(fr < a.nb ? fr : a.nb - 1) * a.ldx + fk * 8;
   bf16x8 wv[2][RT];
-  f32x4 xv[2][2];
+  f32x4 xv[2][2], gv[2][2];
   auto request = [&](int k) {
 #pragma unroll
     for (int u = 0; u < 2; u++) {
@@ -279,6 +345,10 @@ __global__ __launch_bounds__(512) void k_gemv16_bf16(const GemvBf16 a) {
       for (int t = 0; t < RT; t++) wv[u][t] = *(const bf16x8*)(wr[t] + k + u * 32);
       xv[u][0] = *(const f32x4*)(xr + k + u * 32);
       xv[u][1] = *(const f32x4*)(xr + k + u * 32 + 4);
+      if constexpr (IN == GEMV_IN_RMSV) {
+        gv[u][0] = *(const f32x4*)(a.gain + k + u * 32 + fk * 8);
+        gv[u][1] = *(const f32x4*)(a.gain + k + u * 32 + fk * 8 + 4);
+      }
     }
   };
   const int n = a.K / 64;
@@ -296,21 +366,29 @@ __global__ __launch_bounds__(512) void k_gemv16_bf16(const GemvBf16 a) {
   for (int t = 0; t < RT; t++) acc[t] = f32x4{0.f, 0.f, 0.f, 0.f};
   for (int i = wave; i < n; i += W) {
     bf16x8 wc[2][RT];
-    f32x4 xc[2][2];
+    f32x4 xc[2][2], gc[2][2];
 #pragma unroll
     for (int u = 0; u < 2; u++) {
 #pragma unroll
       for (int t = 0; t < RT; t++) wc[u][t] = wv[u][t];
       xc[u][0] = xv[u][0];
       xc[u][1] = xv[u][1];
+      if constexpr (IN == GEMV_IN_RMSV) {
+        gc[u][0] = gv[u][0];
+        gc[u][1] = gv[u][1];
+      }
     }
     if (i + W < n) request((i + W) * 64);
 #pragma unroll
     for (int u = 0; u < 2; u++) {
       float v[8] = {xc[u][0][0], xc[u][0][1], xc[u][0][2], xc[u][0][3], xc[u][1][0], xc[u][1][1], xc[u][1][2], xc[u][1][3]};
-      if constexpr (IN == GEMV_IN_RMS) {
+      if constexpr (IN == GEMV_IN_RMS || IN == GEMV_IN_RMSV) {
 #pragma unroll
         for (int e = 0; e < 8; e++) sq = __builtin_fmaf(v[e], v[e], sq);
+      }
+      if constexpr (IN == GEMV_IN_RMSV) {
+#pragma unroll
+        for (int e = 0; e < 8; e++) v[e] *= gc[u][e >> 2][e & 3];
       }
       if constexpr (IN == GEMV_IN_SPLIT) {
         const float f = i * 64 >= a.k_split ? tail : 1.f;  // (k_split is a multiple of 64)
@@ -334,27 +412,44 @@ __global__ __launch_bounds__(512) void k_gemv16_bf16(const GemvBf16 a) {
   // lane: weight rows 4 fk .. of rhs row fr
 #pragma unroll
   for (int t = 0; t < RT; t++) *(f32x4*)&tile[wave][t][fr * LD + fk * 4] = acc[t];
-  if constexpr (IN == GEMV_IN_RMS) {
+  if constexpr (IN == GEMV_IN_RMS || IN == GEMV_IN_RMSV) {
     sq += __shfl_xor(sq, 16, 64);
     sq += __shfl_xor(sq, 32, 64);
     if (fk == 0) sums[wave][fr] = sq;
   }
   __syncthreads();
-  if constexpr (IN == GEMV_IN_RMS) {
+  if constexpr (IN == GEMV_IN_RMS || IN == GEMV_IN_RMSV) {
     if (tid < 16) {
       float s = 0.f;
 #pragma unroll
       for (int w = 0; w < W; w++) s += sums[w][tid];
-      scale[tid] = *a.gain / sqrtf(s / (float)a.mean_n + a.eps);
+      scale[tid] = (IN == GEMV_IN_RMS ? *a.gain : 1.0f) / sqrtf(s / (float)a.mean_n + a.eps);
     }
     __syncthreads();
+  }
+  if constexpr (OUT == GEMV_OUT_GLU) {
+    for (int i = tid; i < RT * 128; i += 512) {
+      const int t = i >> 7, b = (i >> 3) & 15, r = (i & 7) * 2, row = row0 + t * 16 + r;
+      float gate = 0.f, up = 0.f;
+#pragma unroll
+      for (int w = 0; w < W; w++) {
+        gate += tile[w][t][b * LD + r];
+        up += tile[w][t][b * LD + r + 1];
+      }
+      if constexpr (IN == GEMV_IN_RMS || IN == GEMV_IN_RMSV) {
+        gate *= scale[b];
+        up *= scale[b];
+      }
+      if (b < a.nb && row < a.N) a.out[(size_t)b * a.ldo + row / 2] = gelu_tanh(gate) * up;
+    }
+    return;
   }
   for (int i = tid; i < RT * 256; i += 512) {
     const int t = i >> 8, b = (i >> 4) & 15, r = i & 15, row = row0 + t * 16 + r;
     float v = 0.f;
 #pragma unroll
     for (int w = 0; w < W; w++) v += tile[w][t][b * LD + r];
-    if constexpr (IN == GEMV_IN_RMS) v *= scale[b];
+    if constexpr (IN == GEMV_IN_RMS || IN == GEMV_IN_RMSV) v *= scale[b];
     if (b < a.nb && row < a.N) gemv_out<OUT>(a, row, b, v);
   }
 }
@@ -382,9 +477,9 @@ inline void launch_gemv_bf16(hipStream_t st, crabml_hip_device::ProfRec* rec, co
   if (a.nb <= 1) {
     if (wide)
       launch_gemv_bf16_t<1, 4, IN, OUT>(st, rec, a);
-    else if (a.N >= 2048)
+    else if (a.N >= 2048 || OUT == GEMV_OUT_GLU)
       launch_gemv_bf16_t<1, 2, IN, OUT>(st, rec, a);
-    else
+    else if constexpr (OUT != GEMV_OUT_GLU)
       launch_gemv_bf16_t<1, 1, IN, OUT>(st, rec, a);
   } else if (a.nb <= 2) {
     launch_gemv_bf16_t<2, 2, IN, OUT>(st, rec, a);

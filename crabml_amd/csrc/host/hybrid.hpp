@@ -1,5 +1,5 @@
 // hybrid.hpp -- models on the hybrid decoder (crabml_hip_hybrid_*): configuration (config.json), weights (safetensors), and the
-// runner: sequences, batched steps, greedy generation of many prompts.  The Nilivik design is the one model class built on it.
+// runner: sequences, batched steps, greedy generation of many prompts.  The Nilivik and Bifazen designs are model classes built on it.
 #pragma once
 #include <algorithm>
 #include <deque>
@@ -13,8 +13,10 @@ namespace crabml_host {
 
 struct HybridLayerConfig {
   struct Attention {
-    size_t heads = 0, kv_heads = 0, dim = 0, vdim = 0, chunk = 0;
-    double scale = 0, out_scale = 1;
+    size_t heads = 0, kv_heads = 0, dim = 0, vdim = 0, chunk = 0, window = 0;
+    size_t latent = 0, rot = 0;  // latent attention: rank of the latent, rotated key part
+    double scale = 0, out_scale = 1, rot_base = 0;
+    bool v_mix = false;
   } attn;
   struct Linear {
     size_t heads = 0, dim = 0, vdim = 0;
@@ -23,18 +25,26 @@ struct HybridLayerConfig {
   } lin;
   size_t ff = 0;
 };
+enum class NormGain { Single, Vector, VectorAroundZero };
+
 struct HybridConfig {
   std::string architecture;
   size_t width = 0, vocab_size = 0;
   double embed_scale = 1, norm_eps = 0, logit_softcap = 0;
   size_t loop_start = 0, loop_stop = 0, loop_times = 0;
+  size_t streams = 0;        // residual streams; 0: a plain residual sum
+  double position_base = 0;  // of the position vectors added to the embedding; 0: none
+  NormGain gain = NormGain::Single;
   std::vector<HybridLayerConfig> layers;
 };
 
 // the tensors of a layer as the C ABI takes them; absent ones stay empty
 struct HybridLayerWeights {
   HipTensor norm1, norm2, attn_q, attn_k, attn_v, attn_gate, attn_o, attn_bias_amp, attn_bias_rate, attn_sink;
-  HipTensor lin_q, lin_k, lin_v, lin_gate, lin_o, lin_norm, ff_up, ff_down, ff_act;
+  HipTensor lin_q, lin_k, lin_v, lin_gate, lin_o, lin_norm, ff_up, ff_down, ff_act, ff_gate;
+  HipTensor attn_q_bias, attn_k_bias, attn_v_bias, attn_o_bias, attn_q_norm, attn_k_norm, attn_vmix;
+  HipTensor attn_latent_down, attn_latent_norm, attn_key_up, attn_value_up;
+  HipTensor hc1_in, hc1_out, hc1_mix, hc2_in, hc2_out, hc2_mix;
 };
 struct HybridWeights {
   HipTensor embed, loop_step, final_norm, head;
@@ -48,6 +58,7 @@ inline HybridConfig nilivik_config(const Json& j) {
   c.width = j.at("width").size();
   c.vocab_size = j.at("vocab").size();
   c.embed_scale = j.at("embedding").at("scale").number();
+  c.position_base = 10000.0;
   c.norm_eps = j.at("norm").at("eps").number();
   if (!j["logit_softcap"].is_null()) c.logit_softcap = j["logit_softcap"].number();
   if (!j["loop"].is_null()) {
@@ -120,6 +131,98 @@ inline HybridWeights nilivik_weights(const SafeTensorsFile& f, const HybridConfi
   return w;
 }
 
+// ---- Bifazen: config.json and tensor names -----------------------------------------------------------------------------------------
+inline HybridConfig bifazen_config(const Json& j) {
+  HybridConfig c;
+  c.architecture = j.at("architecture").str();
+  c.width = j.at("width").size();
+  c.vocab_size = j.at("vocab").size();
+  c.norm_eps = j.at("norm").at("eps").number();
+  c.gain = NormGain::VectorAroundZero;
+  c.streams = j.at("streams").size();
+  if (!c.streams) throw Error(ErrorKind::ModelError, "`streams` must be at least 1");
+  for (const Json& l : j.at("layers").items()) {
+    const std::string& type = l.at("type").str();
+    const Json& m = l.at("mixer");
+    HybridLayerConfig L;
+    HybridLayerConfig::Attention& a = L.attn;
+    a.heads = m.at("heads").size();
+    a.dim = m.at("dim").size();
+    a.vdim = m.at("vdim").size();
+    a.window = m.at("mask").at("size").size();
+    a.scale = m.at("scale").number();
+    if (type == "latent_attention") {
+      a.latent = m.at("kv_rank").size();
+      a.rot = m.at("rot_dim").size();
+      a.rot_base = m.at("rot").at("base").number();
+      if (m.at("rot").at("dims").size() != a.rot) throw Error(ErrorKind::ModelError, "`rot.dims` must be `rot_dim`: the shared key part is rotated whole");
+      if (!a.latent || a.rot % 2) throw Error(ErrorKind::ModelError, "a `latent_attention` mixer needs a latent, and pairs of rotated dimensions");
+    } else if (type == "attention") {
+      a.kv_heads = m.at("kv_heads").size();
+      a.v_mix = !m["v_mix"].is_null() && m["v_mix"].truth();
+      if (!a.kv_heads) throw Error(ErrorKind::ModelError, "an `attention` mixer needs key/value heads");
+    } else {
+      throw Error(ErrorKind::NotImplemented, "unknown mixer `" + type + "`");
+    }
+    if (!a.heads || !a.window) throw Error(ErrorKind::ModelError, "a mixer needs heads and a window size");
+    if (!l["mlp"].is_null()) {
+      if (l["mlp"].at("kind").str() != "dense") throw Error(ErrorKind::NotImplemented, "unknown feed-forward `" + l["mlp"].at("kind").str() + "`");
+      L.ff = l["mlp"].at("ff").size();
+    }
+    c.layers.push_back(std::move(L));
+  }
+  return c;
+}
+
+inline HybridWeights bifazen_weights(const SafeTensorsFile& f, const HybridConfig& c, const HipTensorDeviceRef& dev) {
+  HybridWeights w;
+  const size_t W = c.width, S = c.streams;
+  w.embed = f.load("embed", {c.vocab_size, W}, dev);
+  w.final_norm = f.load("final.norm", {W}, dev);
+  for (size_t i = 0; i < c.layers.size(); i++) {
+    const HybridLayerConfig& L = c.layers[i];
+    const HybridLayerConfig::Attention& a = L.attn;
+    const std::string p = "l" + std::to_string(i) + ".", x = p + "mix.", m = p + "mlp.";
+    const size_t H = a.heads, G = a.kv_heads;
+    HybridLayerWeights o;
+    o.norm1 = f.load(p + "norm1", {W}, dev);
+    o.hc1_in = f.load(p + "hc1.in", {S}, dev);
+    o.hc1_out = f.load(p + "hc1.out", {S}, dev);
+    o.hc1_mix = f.load(p + "hc1.mix", {S, S}, dev);
+    o.attn_o = f.load(x + "o", {W, H * a.vdim}, dev);
+    if (a.latent) {
+      o.attn_q = f.load(x + "q", {H * (a.dim + a.rot), W}, dev);
+      o.attn_latent_down = f.load(x + "dkv", {a.latent + a.rot, W}, dev);
+      o.attn_latent_norm = f.load(x + "dkv.norm", {a.latent}, dev);
+      o.attn_key_up = f.load(x + "uk", {H * a.dim, a.latent}, dev);
+      o.attn_value_up = f.load(x + "uv", {H * a.vdim, a.latent}, dev);
+    } else {
+      o.attn_q = f.load(x + "q", {H * a.dim, W}, dev);
+      o.attn_k = f.load(x + "k", {G * a.dim, W}, dev);
+      o.attn_v = f.load(x + "v", {G * a.vdim, W}, dev);
+      o.attn_q_bias = f.load(x + "q.b", {H * a.dim}, dev);
+      o.attn_k_bias = f.load(x + "k.b", {G * a.dim}, dev);
+      o.attn_v_bias = f.load(x + "v.b", {G * a.vdim}, dev);
+      o.attn_o_bias = f.load(x + "o.b", {W}, dev);
+      o.attn_q_norm = f.load(x + "q.norm", {H * a.dim}, dev);
+      o.attn_k_norm = f.load(x + "k.norm", {G * a.dim}, dev);
+      o.attn_gate = f.load(x + "g", {H, W}, dev);
+      if (a.v_mix) o.attn_vmix = f.load(x + "vmix", {}, dev);
+    }
+    if (L.ff) {
+      o.norm2 = f.load(p + "norm2", {W}, dev);
+      o.hc2_in = f.load(p + "hc2.in", {S}, dev);
+      o.hc2_out = f.load(p + "hc2.out", {S}, dev);
+      o.hc2_mix = f.load(p + "hc2.mix", {S, S}, dev);
+      o.ff_gate = f.load(m + "gate", {L.ff, W}, dev);
+      o.ff_up = f.load(m + "up", {L.ff, W}, dev);
+      o.ff_down = f.load(m + "down", {W, L.ff}, dev);
+    }
+    w.layers.push_back(std::move(o));
+  }
+  return w;
+}
+
 // one sequence's part of a step
 struct StepEntry {
   size_t seq = 0;
@@ -146,7 +249,10 @@ class HipHybridRunner : public ModelRunner {
     c.norm_eps = (float)conf_.norm_eps;
     c.logit_softcap = (float)conf_.logit_softcap;
     c.compute = f32 ? CRABML_HIP_F32 : CRABML_HIP_BF16;
-    c.flags = use_graph ? 0 : CRABML_HIP_HYBRID_NO_GRAPH;
+    c.flags = (use_graph ? 0 : CRABML_HIP_HYBRID_NO_GRAPH) | (conf_.gain != NormGain::Single ? CRABML_HIP_HYBRID_NORM_VECTOR : 0) |
+              (conf_.gain == NormGain::VectorAroundZero ? CRABML_HIP_HYBRID_NORM_ONE_PLUS : 0);
+    c.streams = conf_.streams;
+    c.position_base = conf_.position_base;
     if (w.layers.size() != conf_.layers.size()) throw Error(ErrorKind::ModelError, "weights do not have n_layers entries");
     std::vector<crabml_hip_hybrid_layer_t> ls(conf_.layers.size());
     for (size_t i = 0; i < ls.size(); i++) {
@@ -185,6 +291,28 @@ class HipHybridRunner : public ModelRunner {
       o.ff_up = x.ff_up.raw();
       o.ff_down = x.ff_down.raw();
       o.ff_act = x.ff_act.raw();
+      o.attn_window = L.attn.window;
+      o.attn_latent = L.attn.latent;
+      o.attn_rot = L.attn.rot;
+      o.attn_rot_base = L.attn.rot_base;
+      o.attn_q_bias = x.attn_q_bias.raw();
+      o.attn_k_bias = x.attn_k_bias.raw();
+      o.attn_v_bias = x.attn_v_bias.raw();
+      o.attn_o_bias = x.attn_o_bias.raw();
+      o.attn_q_norm = x.attn_q_norm.raw();
+      o.attn_k_norm = x.attn_k_norm.raw();
+      o.attn_vmix = x.attn_vmix.raw();
+      o.attn_latent_down = x.attn_latent_down.raw();
+      o.attn_latent_norm = x.attn_latent_norm.raw();
+      o.attn_key_up = x.attn_key_up.raw();
+      o.attn_value_up = x.attn_value_up.raw();
+      o.ff_gate = x.ff_gate.raw();
+      o.hc1_in = x.hc1_in.raw();
+      o.hc1_out = x.hc1_out.raw();
+      o.hc1_mix = x.hc1_mix.raw();
+      o.hc2_in = x.hc2_in.raw();
+      o.hc2_out = x.hc2_out.raw();
+      o.hc2_mix = x.hc2_mix.raw();
     }
     crabml_hip_hybrid_weights_t cw{};
     cw.embed = w.embed.raw();

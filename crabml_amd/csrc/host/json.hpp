@@ -60,6 +60,10 @@ class Json {
     if (v < 0 || v != std::floor(v) || v > 9007199254740992.0) throw Error(ErrorKind::ModelError, "expected a whole number");
     return (size_t)v;
   }
+  bool truth() const {
+    need(Kind::Bool, "true or false");
+    return num_ != 0;
+  }
   const std::string& str() const {
     need(Kind::String, "a string");
     return str_;

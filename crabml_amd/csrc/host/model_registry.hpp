@@ -39,14 +39,18 @@ struct ModelFolder {
 typedef std::function<std::unique_ptr<ModelRunner>(const ModelFolder&, const HipTensorDeviceRef&, const LoadOptions&)> FolderLoader;
 typedef std::function<std::unique_ptr<ModelRunner>(const GGUFFile&, const HipTensorDeviceRef&, const LoadOptions&)> GgufLoader;
 
+// a model class on the hybrid decoder: what reads its config.json, what finds its tensors
+inline FolderLoader hybrid_model(HybridConfig (*config)(const Json&), HybridWeights (*weights)(const SafeTensorsFile&, const HybridConfig&, const HipTensorDeviceRef&)) {
+  return [config, weights](const ModelFolder& f, const HipTensorDeviceRef& dev, const LoadOptions& o) -> std::unique_ptr<ModelRunner> {
+    const HybridConfig c = config(f.config);
+    const SafeTensorsFile st(f.path + "/model.safetensors");
+    return std::make_unique<HipHybridRunner>(c, weights(st, c, dev), dev, o.seq_len ? o.seq_len : 8192, o.f32, o.use_graph, o.pass_rows);
+  };
+}
 inline const std::map<std::string, FolderLoader>& folder_models() {
   static const std::map<std::string, FolderLoader> m = {
-      {"Nilivik",
-       [](const ModelFolder& f, const HipTensorDeviceRef& dev, const LoadOptions& o) -> std::unique_ptr<ModelRunner> {
-         const HybridConfig c = nilivik_config(f.config);
-         const SafeTensorsFile st(f.path + "/model.safetensors");
-         return std::make_unique<HipHybridRunner>(c, nilivik_weights(st, c, dev), dev, o.seq_len ? o.seq_len : 8192, o.f32, o.use_graph, o.pass_rows);
-       }},
+      {"Bifazen", hybrid_model(bifazen_config, bifazen_weights)},
+      {"Nilivik", hybrid_model(nilivik_config, nilivik_weights)},
   };
   return m;
 }

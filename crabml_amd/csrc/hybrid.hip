@@ -1,9 +1,11 @@
 // hybrid.hip -- the hybrid decoder (crabml_hip_hybrid_*): host side.  Context, weight packing, the sequences' state slabs, the decode
-// step as a captured graph, the prompt pass, the C entry points.  Kernels: hybrid_step.hpp, hybrid_rows.hpp, gemv_bf16.hpp, gemm_bf16.hip.
+// step as a captured graph, the prompt pass, the C entry points.  Kernels: hybrid_step.hpp, hybrid_rows.hpp, hybrid_latent.hpp, gemv_bf16.hpp,
+// gemm_bf16.hip.
 #include <cmath>
 #include <memory>
 
 #include "dequant.hpp"
+#include "hybrid_latent.hpp"
 #include "hybrid_rows.hpp"
 #include "hybrid_step.hpp"
 #include "lazy.hpp"
@@ -12,9 +14,16 @@ using namespace crabml_hip;
 
 namespace {
 
+struct Connection {  // a sublayer between the residual streams
+  float *coef = nullptr, *in = nullptr;
+};
 struct Layer {
   AttnGeom at;
+  LatGeom la;
   LinGeom li;
+  Connection hc[2];  // mixer, feed-forward
+  bool glu = false;
+  float *bias_in = nullptr, *bias_o = nullptr;
   int n_in = 0, ldc = 0, lin_off = 0, ff = 0, ldu = 0, splits = 0, head_blocks = 0;
   ActRanges act;
   unsigned short *w_in = nullptr, *w_o = nullptr, *w_up = nullptr, *w_down = nullptr;
@@ -32,8 +41,9 @@ struct Seq {
   size_t cap = 0;
   size_t len = 0;
 };
-// profiling stages (crabml_hip_prof_*): decode 11 .. 16, prompt pass 21 .. 27
-enum { ST_IN = 1, ST_MIX = 2, ST_OUT = 3, ST_UP = 4, ST_DOWN = 5, ST_HEAD = 6, ST_LIN = 7, ST_ROWS = 8, ST_STEP = 10, ST_PASS = 20 };
+// profiling stages (crabml_hip_prof_*): decode 11 .., prompt pass 21 ..
+// (ROWS: row kernels around a mixer, in a decode step the latent values; LAT: latent queries, in a pass the keys and values)
+enum { ST_IN = 1, ST_MIX = 2, ST_OUT = 3, ST_UP = 4, ST_DOWN = 5, ST_HEAD = 6, ST_LIN = 7, ST_ROWS = 8, ST_LAT = 9, ST_STEP = 10, ST_PASS = 20 };
 
 constexpr size_t LOGIT_ROWS = 256;  // rows of logits a pass keeps on the device at a time
 constexpr int META_SLOTS = 4;
@@ -51,13 +61,17 @@ struct crabml_hip_hybrid {
   std::vector<Seq> seqs;
   size_t slab_bytes = 0;
   unsigned short *embed = nullptr, *head = nullptr;
-  float *loop_step = nullptr, *final_norm = nullptr;
+  float *loop_step = nullptr, *final_norm = nullptr, *ones = nullptr;
+  int streams = 0;  // 0: one residual row, norms with a single gain; else gains per element
   double* freq = nullptr;
   bool keep_emb = false;
   // decode step
   StepSeq* st_seq = nullptr;
   int* st_count = nullptr;
   float *st_x = nullptr, *st_emb = nullptr, *st_proj = nullptr, *st_cat = nullptr, *st_u = nullptr, *st_ss = nullptr, *st_part = nullptr, *st_logits = nullptr;
+  float *st_in = nullptr, *st_vk = nullptr, *st_q = nullptr, *st_lpart = nullptr;  // streams: what the next linear reads; kept values; latent queries, partials
+  int ld_vk = 0, ld_kv = 0, ld_lat = 0, ld_rot = 0;
+  size_t hist = 0;  // earlier positions a latent layer can see
   unsigned* st_tick = nullptr;
   unsigned* st_out = nullptr;
   size_t st_out_cap = 0;
@@ -68,12 +82,13 @@ struct crabml_hip_hybrid {
   int h_seq_next = 0;
   std::map<int, std::pair<hipGraph_t, hipGraphExec_t>> graphs;  // key: rows * 2 + sampler
   // prompt pass (allocated on first use)
-  size_t rows_cap = 0, meta_bytes = 0;
+  size_t rows_cap = 0, hist_cap = 0, meta_bytes = 0;
   char *meta = nullptr, *h_meta = nullptr;
   int h_meta_next = 0;
   float *pf_x = nullptr, *pf_emb = nullptr, *pf_lin = nullptr, *pf_sq = nullptr, *pf_gsq = nullptr, *pf_logits = nullptr;
   unsigned short *pf_xp = nullptr, *pf_cat = nullptr, *pf_u = nullptr, *pf_gp = nullptr;
-  void* pf_proj = nullptr;
+  void *pf_proj = nullptr, *pf_vk = nullptr, *pf_rot = nullptr, *pf_kv = nullptr;
+  unsigned short* pf_lat = nullptr;
   GemmScratch pf_scratch;
   hipStream_t side = nullptr;  // the linear branch of a long pass, beside the softmax branch
   hipEvent_t fork = nullptr, join = nullptr;
@@ -99,16 +114,32 @@ int dalloc_n(Ctx* c, size_t n, T** out) {
 int up(size_t v, size_t a) { return (int)align_up(v, a); }
 
 // ---- weight packing -----------------------------------------------------------------------------------------------------------------
-// source row r -> row0 + r with every group of rg rows widened to rgp; columns the same (head widths padded; the gaps stay zero)
+// row r -> row0 + r with every group of rg rows widened to rgp; columns the same (head widths padded; the gaps stay zero).  The rows are
+// the `rg` from `so` on of every group of sg source rows.
 __global__ __launch_bounds__(256) void k_pack_matrix(const unsigned short* __restrict__ src, int m, int k, unsigned short* __restrict__ dst, size_t ldd,
-                                                     int row0, int rg, int rgp, int col0, int cg, int cgp) {
+                                                     int row0, int rg, int rgp, int col0, int cg, int cgp, int sg, int so) {
   const int r = blockIdx.y;
+  const unsigned short* x = src + (size_t)(r / rg * sg + so + r % rg) * k;
   unsigned short* d = dst + (size_t)(row0 + r / rg * rgp + r % rg) * ldd + col0;
-  for (int c = blockIdx.x * 256 + threadIdx.x; c < k; c += gridDim.x * 256) d[c / cg * cgp + c % cg] = src[(size_t)r * k + c];
+  for (int c = blockIdx.x * 256 + threadIdx.x; c < k; c += gridDim.x * 256) d[c / cg * cgp + c % cg] = x[c];
 }
-__global__ __launch_bounds__(256) void k_pack_vector(const char* __restrict__ src, int dtype, size_t off_scale, int n, float* __restrict__ dst, int g, int gp) {
+// [heads][dim][k] -> [heads][kp][dimp]
+__global__ __launch_bounds__(256) void k_pack_transposed(const unsigned short* __restrict__ src, int dim, int k, unsigned short* __restrict__ dst, int kp, int dimp) {
+  const int h = blockIdx.z, d = blockIdx.y;
+  const unsigned short* x = src + ((size_t)h * dim + d) * k;
+  for (int c = blockIdx.x * 256 + threadIdx.x; c < k; c += gridDim.x * 256) dst[((size_t)h * kp + c) * dimp + d] = x[c];
+}
+__global__ __launch_bounds__(256) void k_pack_vector(const char* __restrict__ src, int dtype, size_t off_scale, int n, float* __restrict__ dst, int g, int gp,
+                                                     float plus, int wrap) {
   const int i = blockIdx.x * 256 + threadIdx.x;
-  if (i < n) dst[i / g * gp + i % g] = dequant_elem(src, dtype, off_scale, i);
+  if (i < n) dst[i / g * gp + i % g] = dequant_elem(src, dtype, off_scale, i % wrap) + plus;
+}
+// a connection's raw numbers -> rows of StreamMix::coef
+__global__ void k_pack_connection(const float* __restrict__ mix, const float* __restrict__ out, int n, float* __restrict__ coef) {
+  for (int t = 0; t < n; t++) {
+    for (int s = 0; s < HC_MAX; s++) coef[t * HC_ROW + s] = s < n ? mix[s * n + t] : 0.f;
+    coef[t * HC_ROW + HC_MAX] = out[t];
+  }
 }
 __global__ void k_xielu_consts(const float* __restrict__ raw, float* __restrict__ out) {
   auto softplus = [](float z) { return log1pf(expf(-fabsf(z))) + fmaxf(z, 0.f); };
@@ -117,19 +148,52 @@ __global__ void k_xielu_consts(const float* __restrict__ raw, float* __restrict_
 }
 
 int pack_matrix(Ctx* c, const crabml_hip_buf* b, const char* what, size_t m, size_t k, unsigned short* dst, size_t ldd, size_t row0, size_t rg, size_t rgp,
-                size_t col0 = 0, size_t cg = 0, size_t cgp = 0) {
-  if (!b || b->dtype != CRABML_HIP_BF16 || b->n_elems != m * k || b->dev != c->dev)
-    CH_BAIL(c->dev, CRABML_HIP_BAD_INPUT, "hybrid: %s must be a bfloat16 matrix of %zu x %zu", what, m, k);
+                size_t col0 = 0, size_t cg = 0, size_t cgp = 0, size_t sg = 0, size_t so = 0) {
+  if (sg == 0) sg = rg;
+  const size_t rows = rg ? m / rg * sg : m;  // (m: the rows that are taken)
+  if (!b || b->dtype != CRABML_HIP_BF16 || b->n_elems != rows * k || b->dev != c->dev)
+    CH_BAIL(c->dev, CRABML_HIP_BAD_INPUT, "hybrid: %s must be a bfloat16 matrix of %zu x %zu", what, rows, k);
   k_pack_matrix<<<dim3((unsigned)std::min<size_t>((k + 255) / 256, 64), (unsigned)m), 256, 0, c->dev->stream>>>(
-      (const unsigned short*)b->ptr, (int)m, (int)k, dst, ldd, (int)row0, (int)rg, (int)rgp, (int)col0, (int)(cg ? cg : k), (int)(cg ? cgp : k));
+      (const unsigned short*)b->ptr, (int)m, (int)k, dst, ldd, (int)row0, (int)rg, (int)rgp, (int)col0, (int)(cg ? cg : k), (int)(cg ? cgp : k), (int)sg, (int)so);
+  CH_HIP(c->dev, hipGetLastError());
+  return 0;
+}
+// n numbers into dst, every group of g widened to gp
+int pack_into(Ctx* c, const crabml_hip_buf* b, const char* what, size_t n, float* dst, size_t g = 0, size_t gp = 0, float plus = 0.f) {
+  if (!b || b->n_elems != n || b->dev != c->dev) CH_BAIL(c->dev, CRABML_HIP_BAD_INPUT, "hybrid: %s must hold %zu numbers", what, n);
+  if (g == 0) g = gp = n;
+  k_pack_vector<<<(unsigned)((n + 255) / 256), 256, 0, c->dev->stream>>>((const char*)b->ptr, (int)b->dtype, b->wl.off_scale, (int)n, dst, (int)g, (int)gp, plus, (int)n);
   CH_HIP(c->dev, hipGetLastError());
   return 0;
 }
 int pack_vector(Ctx* c, const crabml_hip_buf* b, const char* what, size_t n, float** out, size_t g = 0, size_t gp = 0) {
-  if (!b || b->n_elems != n || b->dev != c->dev) CH_BAIL(c->dev, CRABML_HIP_BAD_INPUT, "hybrid: %s must hold %zu numbers", what, n);
   if (g == 0) g = gp = n;
   CH_TRY(dalloc_n(c, n / g * gp, out));
-  k_pack_vector<<<(unsigned)((n + 255) / 256), 256, 0, c->dev->stream>>>((const char*)b->ptr, (int)b->dtype, b->wl.off_scale, (int)n, *out, (int)g, (int)gp);
+  return pack_into(c, b, what, n, *out, g, gp);
+}
+// an RMS norm's gain: one number, or (streams) one per element of a padded row, wherever the design has a single one
+int pack_norm(Ctx* c, const crabml_hip_buf* b, const char* what, float** out) {
+  const float plus = c->cfg.flags & CRABML_HIP_HYBRID_NORM_ONE_PLUS ? 1.f : 0.f;
+  const size_t n = c->cfg.flags & CRABML_HIP_HYBRID_NORM_VECTOR ? (size_t)c->width : 1;
+  if (!b || b->n_elems != n || b->dev != c->dev) CH_BAIL(c->dev, CRABML_HIP_BAD_INPUT, "hybrid: %s must hold %zu numbers", what, n);
+  const size_t m = c->streams ? (size_t)c->width : 1;
+  CH_TRY(dalloc_n(c, c->streams ? align_up(m, 64) : m, out));
+  k_pack_vector<<<(unsigned)((m + 255) / 256), 256, 0, c->dev->stream>>>((const char*)b->ptr, (int)b->dtype, b->wl.off_scale, (int)m, *out, (int)m, (int)m, plus, (int)n);
+  CH_HIP(c->dev, hipGetLastError());
+  return 0;
+}
+int pack_connection(Ctx* c, const crabml_hip_buf* in, const crabml_hip_buf* out, const crabml_hip_buf* mix, Connection& h) {
+  const size_t n = (size_t)c->streams;
+  float *m = nullptr, *o = nullptr;
+  if (!c->cfg.streams) {  // a plain residual: one stream that keeps itself
+    h.in = o = m = c->ones;
+  } else {
+    CH_TRY(pack_vector(c, in, "a connection's input weights", n, &h.in));
+    CH_TRY(pack_vector(c, out, "a connection's output weights", n, &o));
+    CH_TRY(pack_vector(c, mix, "a connection's mixing matrix", n * n, &m));
+  }
+  CH_TRY(dalloc_n(c, n * HC_ROW, &h.coef));
+  k_pack_connection<<<1, 1, 0, c->dev->stream>>>(m, o, (int)n, h.coef);
   CH_HIP(c->dev, hipGetLastError());
   return 0;
 }
@@ -138,14 +202,22 @@ int alloc_matrix(Ctx* c, size_t rows, size_t ld, unsigned short** out) { return 
 
 int build_layer(Ctx* c, const crabml_hip_hybrid_layer_t& s, Layer& L) {
   crabml_hip_device* dev = c->dev;
-  const size_t W = (size_t)c->width, H = s.attn_heads, G = s.attn_kv_heads, Hl = s.lin_heads;
+  const size_t W = (size_t)c->width, H = s.attn_heads, Hl = s.lin_heads, rank = s.attn_latent, rot = rank ? s.attn_rot : 0;
+  const size_t G = rank ? H : s.attn_kv_heads;
   if (!H && !Hl) CH_BAIL(dev, CRABML_HIP_BAD_INPUT, "hybrid: a layer needs a mixer");
   if (H && (!G || H % G || !s.attn_dim || !s.attn_vdim || s.attn_dim > 256 || s.attn_vdim > 256))
     CH_BAIL(dev, H && G && H % G == 0 ? CRABML_HIP_NOT_IMPLEMENTED : CRABML_HIP_BAD_INPUT, "hybrid: attention of %zu / %zu heads of %zu / %zu (at most 256 wide)", H, G,
             s.attn_dim, s.attn_vdim);
+  const size_t dimp = align_up(s.attn_dim, 8), rotp = align_up(rot, 8), rankp = align_up(rank, 8);
+  if (H && rank && (rot % 2 || dimp + rotp > 256 || rankp + rotp > LAT_MAX_ROW || !(s.attn_rot_base > 0 || !rot)))
+    CH_BAIL(dev, CRABML_HIP_NOT_IMPLEMENTED, "hybrid: latent attention of rank %zu, heads of %zu + %zu rotated (rows at most %d, heads at most 256 wide, pairs rotated)", rank,
+            s.attn_dim, rot, LAT_MAX_ROW);
+  if (H && rank && (s.attn_gate || s.attn_sink || s.attn_bias_amp || s.attn_q_norm || s.attn_k_norm || s.attn_vmix || s.attn_q_bias || s.attn_k_bias || s.attn_v_bias || Hl))
+    CH_BAIL(dev, CRABML_HIP_NOT_IMPLEMENTED, "hybrid: latent attention has no gate, sink, distance bias, query or key norm, value mixing or input biases, and no branch beside it");
+  if (s.attn_chunk && s.attn_window) CH_BAIL(dev, CRABML_HIP_BAD_INPUT, "hybrid: attention inside chunks or a window, not both");
   if (Hl && (!s.lin_dim || !s.lin_vdim || s.lin_dim > 256 || !s.lin_decay))
     CH_BAIL(dev, CRABML_HIP_NOT_IMPLEMENTED, "hybrid: linear attention of %zu heads of %zu / %zu (keys at most 256 wide, decay given)", Hl, s.lin_dim, s.lin_vdim);
-  const size_t D = align_up(s.attn_dim, 8), V = align_up(s.attn_vdim, 8), Dl = align_up(s.lin_dim, 8), Vl = align_up(s.lin_vdim, 8);
+  const size_t D = dimp + rotp, V = align_up(s.attn_vdim, 8), Dl = align_up(s.lin_dim, 8), Vl = align_up(s.lin_vdim, 8);
   size_t col = 0;
   auto take = [&](size_t n) {
     const size_t at = col;
@@ -160,17 +232,28 @@ int build_layer(Ctx* c, const crabml_hip_hybrid_layer_t& s, Layer& L) {
     a.G = (int)G;
     a.D = (int)D;
     a.V = (int)V;
-    const size_t chunk = s.attn_chunk && s.attn_chunk < ((size_t)1 << 30) ? s.attn_chunk : (size_t)1 << 30;
-    a.chunk = (int)chunk;
-    a.rows = (int)std::min(chunk, c->cfg.seq_len);
+    const size_t limit = s.attn_window ? s.attn_window : s.attn_chunk;
+    const size_t span = limit && limit < ((size_t)1 << 30) ? limit : (size_t)1 << 30;
+    a.span = (int)span;
+    a.window = s.attn_window != 0;
+    a.rows = (int)std::min(span, c->cfg.seq_len);
+    a.eps = c->cfg.norm_eps;
     a.scale = s.attn_score_scale;
     a.out_scale = s.attn_out_scale;
     a.cq = take(H * D);
-    a.ck = take(G * D);
-    a.cv = take(G * V);
+    if (rank) {
+      L.la.cc = take(rankp);
+      L.la.cr = take(rotp);
+    } else {
+      a.ck = take(G * D);
+      a.cv = take(G * V);
+    }
   }
   L.act.end[0] = (int)col;
-  if (H) a.cg = take(H * V);
+  if (H && s.attn_gate) {
+    a.gate = s.attn_gate->n_elems == H * W && s.attn_vdim != 1 ? GATE_HEAD : GATE_ELEMENT;
+    a.cg = a.gate == GATE_HEAD ? take(align_up(H, 8)) : take(H * V);
+  }
   L.act.end[1] = (int)col;
   L.act.kind[1] = ACT_SIGMOID;
   if (Hl) {
@@ -194,16 +277,79 @@ int build_layer(Ctx* c, const crabml_hip_hybrid_layer_t& s, Layer& L) {
   L.ldc = L.lin_off + up(Hl * Vl, 64);
   L.ff = (int)s.ff;
   L.ldu = up(s.ff, 64);
-  L.splits = H ? (a.rows + MIX_KEYS - 1) / MIX_KEYS : 0;
-  L.head_blocks = H ? (int)((H / G + MIX_HEADS - 1) / MIX_HEADS) : 0;
+  L.splits = H && !rank ? (a.rows + MIX_KEYS - 1) / MIX_KEYS : 0;
+  L.head_blocks = H && !rank ? (int)((H / G + MIX_HEADS - 1) / MIX_HEADS) : 0;
   const size_t ldw = (size_t)c->ldx;
   CH_TRY(alloc_matrix(c, col, ldw, &L.w_in));
   CH_TRY(alloc_matrix(c, W, (size_t)L.ldc, &L.w_o));
-  if (H) {
+  if (H && (s.attn_q_bias || s.attn_k_bias || s.attn_v_bias)) {
+    CH_TRY(dalloc_n(c, col, &L.bias_in));
+    if (s.attn_q_bias) CH_TRY(pack_into(c, s.attn_q_bias, "attn_q_bias", H * s.attn_dim, L.bias_in + a.cq, s.attn_dim, D));
+    if (s.attn_k_bias) CH_TRY(pack_into(c, s.attn_k_bias, "attn_k_bias", G * s.attn_dim, L.bias_in + a.ck, s.attn_dim, D));
+    if (s.attn_v_bias) CH_TRY(pack_into(c, s.attn_v_bias, "attn_v_bias", G * s.attn_vdim, L.bias_in + a.cv, s.attn_vdim, V));
+  }
+  if (s.attn_o_bias) {
+    if (!c->streams) CH_BAIL(dev, CRABML_HIP_NOT_IMPLEMENTED, "hybrid: an output bias goes with norms of a gain per element or with residual streams");
+    CH_TRY(dalloc_n(c, align_up(W, 64), &L.bias_o));
+    CH_TRY(pack_into(c, s.attn_o_bias, "attn_o_bias", W, L.bias_o));
+  }
+  if (H && rank) {
+    LatGeom& la = L.la;
+    la.rank = (int)rankp;
+    la.dim = (int)dimp;
+    la.rot = (int)rotp;
+    la.rank_true = (int)rank;
+    la.rot_true = (int)rot;
+    la.ldl = up(rank, 64);
+    CH_TRY(pack_matrix(c, s.attn_q, "attn_q", H * s.attn_dim, W, L.w_in, ldw, a.cq, s.attn_dim, D, 0, 0, 0, s.attn_dim + rot, 0));
+    if (rot) CH_TRY(pack_matrix(c, s.attn_q, "attn_q", H * rot, W, L.w_in, ldw, a.cq + dimp, rot, D, 0, 0, 0, s.attn_dim + rot, s.attn_dim));
+    CH_TRY(pack_matrix(c, s.attn_latent_down, "attn_latent_down", rank, W, L.w_in, ldw, la.cc, rank, rankp, 0, 0, 0, rank + rot, 0));
+    if (rot) CH_TRY(pack_matrix(c, s.attn_latent_down, "attn_latent_down", rot, W, L.w_in, ldw, la.cr, rot, rotp, 0, 0, 0, rank + rot, rank));
+    unsigned short *wq = nullptr, *wkv = nullptr;
+    CH_TRY(alloc_matrix(c, H * (dimp + V), (size_t)la.ldl, &wkv));
+    CH_TRY(pack_matrix(c, s.attn_key_up, "attn_key_up", H * s.attn_dim, rank, wkv, (size_t)la.ldl, 0, s.attn_dim, dimp));
+    CH_TRY(pack_matrix(c, s.attn_value_up, "attn_value_up", H * s.attn_vdim, rank, wkv, (size_t)la.ldl, H * dimp, s.attn_vdim, V));
+    CH_TRY(dalloc_n(c, H * rankp * dimp, &wq));
+    k_pack_transposed<<<dim3((unsigned)((rank + 255) / 256), (unsigned)s.attn_dim, (unsigned)H), 256, 0, dev->stream>>>((const unsigned short*)s.attn_key_up->ptr, (int)s.attn_dim,
+                                                                                                             (int)rank, wq, la.rank, la.dim);
+    CH_HIP(dev, hipGetLastError());
+    la.w_q = wq;
+    la.w_kv = wkv;
+    CH_TRY(pack_matrix(c, s.attn_o, "attn_o", W, H * s.attn_vdim, L.w_o, (size_t)L.ldc, 0, W, W, 0, s.attn_vdim, V));
+    float* p = nullptr;
+    CH_TRY(pack_vector(c, s.attn_latent_norm, "attn_latent_norm", rank, &p, rank, rankp));
+    la.norm = p;
+    std::vector<double> f(rotp / 2 + 1, 0.0);
+    for (size_t i = 0; i < rot / 2; i++) f[i] = pow(s.attn_rot_base, -2.0 * (double)i / (double)rot);
+    double* df = nullptr;
+    CH_TRY(dalloc_n(c, f.size(), &df));
+    CH_HIP(dev, hipMemcpyAsync(df, f.data(), f.size() * sizeof(double), hipMemcpyHostToDevice, dev->stream));
+    CH_HIP(dev, hipStreamSynchronize(dev->stream));  // f goes out of scope
+    la.freq = df;
+  }
+  if (H && !rank) {
+    if (!s.attn_q_norm != !s.attn_k_norm) CH_BAIL(dev, CRABML_HIP_BAD_INPUT, "hybrid: attn_q_norm and attn_k_norm come together");
+    float* np = nullptr;
+    if (s.attn_q_norm) {
+      CH_TRY(pack_vector(c, s.attn_q_norm, "attn_q_norm", H * s.attn_dim, &np, s.attn_dim, D));
+      a.q_norm = np;
+      CH_TRY(pack_vector(c, s.attn_k_norm, "attn_k_norm", G * s.attn_dim, &np, s.attn_dim, D));
+      a.k_norm = np;
+      a.q_mean = (int)(H * s.attn_dim);
+      a.k_mean = (int)(G * s.attn_dim);
+    }
+    if (s.attn_vmix) {  // the first such layer's values are the ones the others take
+      if (c->ld_vk && c->ld_vk != (int)(G * V)) CH_BAIL(dev, CRABML_HIP_BAD_INPUT, "hybrid: layers that mix values must agree in their value heads");
+      a.vmix = c->ld_vk ? VMIX_MIX : VMIX_KEEP;
+      c->ld_vk = (int)(G * V);
+      CH_TRY(pack_vector(c, s.attn_vmix, "attn_vmix", 1, &np));
+      a.lambda = np;
+    }
     CH_TRY(pack_matrix(c, s.attn_q, "attn_q", H * s.attn_dim, W, L.w_in, ldw, a.cq, s.attn_dim, D));
     CH_TRY(pack_matrix(c, s.attn_k, "attn_k", G * s.attn_dim, W, L.w_in, ldw, a.ck, s.attn_dim, D));
     CH_TRY(pack_matrix(c, s.attn_v, "attn_v", G * s.attn_vdim, W, L.w_in, ldw, a.cv, s.attn_vdim, V));
-    CH_TRY(pack_matrix(c, s.attn_gate, "attn_gate", H * s.attn_vdim, W, L.w_in, ldw, a.cg, s.attn_vdim, V));
+    if (a.gate == GATE_HEAD) CH_TRY(pack_matrix(c, s.attn_gate, "attn_gate", H, W, L.w_in, ldw, a.cg, H, H));
+    if (a.gate == GATE_ELEMENT) CH_TRY(pack_matrix(c, s.attn_gate, "attn_gate", H * s.attn_vdim, W, L.w_in, ldw, a.cg, s.attn_vdim, V));
     CH_TRY(pack_matrix(c, s.attn_o, "attn_o", W, H * s.attn_vdim, L.w_o, (size_t)L.ldc, 0, W, W, 0, s.attn_vdim, V));
     if (!s.attn_bias_amp != !s.attn_bias_rate) CH_BAIL(dev, CRABML_HIP_BAD_INPUT, "hybrid: attn_bias_amp and attn_bias_rate come together");
     float* p = nullptr;
@@ -235,13 +381,22 @@ int build_layer(Ctx* c, const crabml_hip_hybrid_layer_t& s, Layer& L) {
     CH_HIP(dev, hipStreamSynchronize(dev->stream));  // pw goes out of scope
     l.decay = p;
   }
-  CH_TRY(pack_vector(c, s.norm1, "norm1", 1, &L.norm1));
+  CH_TRY(pack_norm(c, s.norm1, "norm1", &L.norm1));
+  if (c->streams) CH_TRY(pack_connection(c, s.hc1_in, s.hc1_out, s.hc1_mix, L.hc[0]));
   if (s.ff) {
-    CH_TRY(pack_vector(c, s.norm2, "norm2", 1, &L.norm2));
-    CH_TRY(alloc_matrix(c, s.ff, ldw, &L.w_up));
+    CH_TRY(pack_norm(c, s.norm2, "norm2", &L.norm2));
+    if (c->streams) CH_TRY(pack_connection(c, s.hc2_in, s.hc2_out, s.hc2_mix, L.hc[1]));
+    L.glu = s.ff_gate != nullptr;
+    CH_TRY(alloc_matrix(c, s.ff * (L.glu ? 2 : 1), ldw, &L.w_up));
     CH_TRY(alloc_matrix(c, W, (size_t)L.ldu, &L.w_down));
-    CH_TRY(pack_matrix(c, s.ff_up, "ff_up", s.ff, W, L.w_up, ldw, 0, s.ff, s.ff));
+    if (L.glu) {  // gate j, up j, gate j + 1, ..
+      CH_TRY(pack_matrix(c, s.ff_gate, "ff_gate", s.ff, W, L.w_up, ldw, 0, 1, 2));
+      CH_TRY(pack_matrix(c, s.ff_up, "ff_up", s.ff, W, L.w_up, ldw, 1, 1, 2));
+    } else {
+      CH_TRY(pack_matrix(c, s.ff_up, "ff_up", s.ff, W, L.w_up, ldw, 0, s.ff, s.ff));
+    }
     CH_TRY(pack_matrix(c, s.ff_down, "ff_down", W, s.ff, L.w_down, (size_t)L.ldu, 0, W, W));
+    if (L.glu) return 0;
     float* raw = nullptr;
     CH_TRY(pack_vector(c, s.ff_act, "ff_act", 2, &raw));
     CH_TRY(dalloc_n(c, 2, &L.xielu));
@@ -286,6 +441,8 @@ MixStep mix_step(const Ctx* c, const Run& run, int B) {
   m.ss = c->st_ss;
   m.part = c->st_part;
   m.tick = c->st_tick;
+  m.v_kept = c->st_vk;
+  m.ld_vk = c->ld_vk;
   m.B = B;
   m.ldp = L.n_in;
   m.ldc = L.ldc;
@@ -304,6 +461,43 @@ void next_adds(const Ctx* c, size_t r, const float* emb, const float** rows, con
   }
 }
 
+// the residual streams behind sublayer q (0: mixer, 1: feed-forward) of run r, and the gain of the norm that reads them next
+StreamMix streams_behind(const Ctx* c, size_t r, int q, size_t stride, const float** gain) {
+  const Layer& L = c->layers[c->runs[r].layer];
+  StreamMix m;
+  m.n = c->streams;
+  m.stride = stride;
+  m.coef = L.hc[q].coef;
+  if (q == 0 && L.ff) {
+    m.in = L.hc[1].in;
+    *gain = L.norm2;
+  } else if (r + 1 < c->runs.size()) {
+    const Layer& N = c->layers[c->runs[r + 1].layer];
+    m.in = N.hc[0].in;
+    *gain = N.norm1;
+  } else {
+    m.in = c->ones;
+    *gain = c->final_norm;
+  }
+  return m;
+}
+// in front of the first layer
+StreamMix streams_at_start(const Ctx* c, size_t stride) {
+  StreamMix m;
+  m.n = c->streams;
+  m.stride = stride;
+  m.in = c->streams ? c->layers[c->runs[0].layer].hc[0].in : nullptr;
+  return m;
+}
+// an RMS norm and a linear behind it
+template <int OUT>
+void normed_linear(Ctx* c, crabml_hip_device::ProfRec* rec, const GemvBf16& g) {
+  if (c->streams)
+    step_linear<GEMV_IN_RMSV, OUT>(c, rec, g);
+  else
+    step_linear<GEMV_IN_RMS, OUT>(c, rec, g);
+}
+
 // the classifier on f32 rows
 void head_rows(Ctx* c, const float* x, int B, bool prof) {
   GemvBf16 g;
@@ -318,15 +512,48 @@ void head_rows(Ctx* c, const float* x, int B, bool prof) {
   g.gain = c->final_norm;
   g.cap = c->cfg.logit_softcap;
   Prof p(c->dev, prof, ST_STEP + ST_HEAD, (double)c->vocab * c->ldx * 2);
-  step_linear<GEMV_IN_RMS, GEMV_OUT_SOFTCAP>(c, p.rec(), g);
+  normed_linear<GEMV_OUT_SOFTCAP>(c, p.rec(), g);
 }
+
+template <typename T>
+int latent_step(Ctx* c, const Run& run, int B, bool prof) {
+  const Layer& L = c->layers[run.layer];
+  LatStep m;
+  m.at = L.at;
+  m.la = L.la;
+  m.rs = run.rs;
+  m.seq = c->st_seq;
+  m.proj = c->st_proj;
+  m.q = c->st_q;
+  m.part = c->st_lpart;
+  m.cat = c->st_cat;
+  m.B = B;
+  m.ldp = L.n_in;
+  m.ldc = L.ldc;
+  hipStream_t st = c->dev->stream;
+  {
+    Prof p(c->dev, prof, ST_STEP + ST_LAT, (double)L.at.H * L.la.rank * L.la.dim * 2);
+    launch_latent_query<T>(st, p.rec(), m);
+  }
+  {
+    Prof p(c->dev, prof, ST_STEP + ST_MIX, 0.0);
+    CH_TRY(launch_latent_attn<T>(c->dev, p.rec(), m));
+  }
+  Prof p(c->dev, prof, ST_STEP + ST_ROWS, (double)L.at.H * L.la.rank * L.at.V * 2);
+  launch_latent_value<T>(st, p.rec(), m);
+  return 0;
+}
+
 
 int enqueue_step(Ctx* c, int B, bool sample, bool prof) {
   crabml_hip_device* dev = c->dev;
   hipStream_t st = dev->stream;
   const float eps = c->cfg.norm_eps;
+  const size_t stride = (size_t)HYB_STEP_ROWS * c->ldx;
+  const float* next_gain = nullptr;
+  float* x_in = c->streams ? c->st_in : c->st_x;  // what a norm reads
   k_embed_step<<<dim3((c->width + 255) / 256, B), 256, 0, st>>>(c->embed, c->st_seq, c->width, c->ldx, c->cfg.embed_scale, c->freq, c->st_x,
-                                                               c->keep_emb ? c->st_emb : nullptr, c->runs[0].add_vec);
+                                                               c->keep_emb ? c->st_emb : nullptr, c->runs[0].add_vec, streams_at_start(c, stride), c->st_in);
   for (size_t r = 0; r < c->runs.size(); r++) {
     const Run& run = c->runs[r];
     const Layer& L = c->layers[run.layer];
@@ -335,7 +562,7 @@ int enqueue_step(Ctx* c, int B, bool sample, bool prof) {
     {
       GemvBf16 g;
       g.w = L.w_in;
-      g.x = c->st_x;
+      g.x = x_in;
       g.out = c->st_proj;
       g.N = g.ldo = L.n_in;
       g.K = g.ldw = g.ldx = c->ldx;
@@ -344,10 +571,13 @@ int enqueue_step(Ctx* c, int B, bool sample, bool prof) {
       g.eps = eps;
       g.gain = L.norm1;
       g.act = L.act;
+      g.bias = L.bias_in;
       Prof p(dev, prof, ST_STEP + ST_IN, (double)L.n_in * c->ldx * 2);
-      step_linear<GEMV_IN_RMS, GEMV_OUT_ACT>(c, p.rec(), g);
+      normed_linear<GEMV_OUT_ACT>(c, p.rec(), g);
     }
-    {
+    if (L.la.rank) {
+      CH_TRY(c->f32 ? latent_step<float>(c, run, B, prof) : latent_step<unsigned short>(c, run, B, prof));
+    } else {
       const MixStep m = mix_step(c, run, B);
       Prof p(dev, prof, ST_STEP + ST_MIX, 0.0);
       if (c->f32)
@@ -374,15 +604,22 @@ int enqueue_step(Ctx* c, int B, bool sample, bool prof) {
         g.add_vec = add_vec;
       }
       Prof p(dev, prof, ST_STEP + ST_OUT, (double)c->width * L.ldc * 2);
-      step_linear<GEMV_IN_SPLIT, GEMV_OUT_RESIDUAL>(c, p.rec(), g);
+      if (c->streams) {
+        g.bias = L.bias_o;
+        g.sm = streams_behind(c, r, 0, stride, &next_gain);
+        g.u = c->st_in;
+        step_linear<GEMV_IN_SPLIT, GEMV_OUT_STREAMS>(c, p.rec(), g);
+      } else {
+        step_linear<GEMV_IN_SPLIT, GEMV_OUT_RESIDUAL>(c, p.rec(), g);
+      }
     }
     if (!L.ff) continue;
     {
       GemvBf16 g;
       g.w = L.w_up;
-      g.x = c->st_x;
+      g.x = x_in;
       g.out = c->st_u;
-      g.N = L.ff;
+      g.N = L.glu ? 2 * L.ff : L.ff;
       g.ldo = L.ldu;
       g.K = g.ldw = g.ldx = c->ldx;
       g.nb = B;
@@ -390,8 +627,11 @@ int enqueue_step(Ctx* c, int B, bool sample, bool prof) {
       g.eps = eps;
       g.gain = L.norm2;
       g.xielu = L.xielu;
-      Prof p(dev, prof, ST_STEP + ST_UP, (double)L.ff * c->ldx * 2);
-      step_linear<GEMV_IN_RMS, GEMV_OUT_XIELU>(c, p.rec(), g);
+      Prof p(dev, prof, ST_STEP + ST_UP, (double)g.N * c->ldx * 2);
+      if (L.glu)
+        normed_linear<GEMV_OUT_GLU>(c, p.rec(), g);
+      else
+        normed_linear<GEMV_OUT_XIELU>(c, p.rec(), g);
     }
     {
       GemvBf16 g;
@@ -405,10 +645,16 @@ int enqueue_step(Ctx* c, int B, bool sample, bool prof) {
       g.add_rows = add_rows;
       g.add_vec = add_vec;
       Prof p(dev, prof, ST_STEP + ST_DOWN, (double)c->width * L.ldu * 2);
-      step_linear<GEMV_IN_PLAIN, GEMV_OUT_RESIDUAL>(c, p.rec(), g);
+      if (c->streams) {
+        g.sm = streams_behind(c, r, 1, stride, &next_gain);
+        g.u = c->st_in;
+        step_linear<GEMV_IN_PLAIN, GEMV_OUT_STREAMS>(c, p.rec(), g);
+      } else {
+        step_linear<GEMV_IN_PLAIN, GEMV_OUT_RESIDUAL>(c, p.rec(), g);
+      }
     }
   }
-  head_rows(c, c->st_x, B, prof);
+  head_rows(c, x_in, B, prof);
   if (sample) {
     k_argmax_partial<<<dim3(ARGMAX_BLOCKS, B), 256, 0, st>>>(c->st_logits, c->vocab, c->am_val, c->am_idx, 0, c->vocab);
     k_argmax_rows_step<<<B, 64, 0, st>>>(c->am_val, c->am_idx, ARGMAX_BLOCKS, c->st_seq, c->st_count, c->st_out, (int)c->st_out_cap);
@@ -463,10 +709,17 @@ int pass_alloc(Ctx* c) {
   const size_t R = align_up(c->cfg.pass_rows ? c->cfg.pass_rows : 2048, 256), P = (size_t)c->planes;
   size_t lin = 0;
   for (const Layer& L : c->layers) lin = std::max(lin, (size_t)L.li.H * L.li.V);
-  CH_TRY(dalloc_n(c, R * c->ldx, &c->pf_x));
+  const size_t S = c->streams ? (size_t)c->streams : 1, e = c->f32 ? 4 : 2, Hc = c->hist ? align_up(std::max(R, c->hist), 256) : 0;
+  CH_TRY(dalloc_n(c, S * R * c->ldx, &c->pf_x));
   if (c->keep_emb) CH_TRY(dalloc_n(c, R * c->ldx, &c->pf_emb));
   CH_TRY(dalloc_n(c, P * R * c->ldx, &c->pf_xp));
-  CH_TRY(dalloc(c, R * c->ld_proj * (c->f32 ? 4 : 2), &c->pf_proj));
+  CH_TRY(dalloc(c, R * c->ld_proj * e, &c->pf_proj));
+  if (c->ld_vk) CH_TRY(dalloc(c, R * c->ld_vk * e, &c->pf_vk));
+  if (c->ld_kv) {
+    CH_TRY(dalloc_n(c, P * (R + Hc) * c->ld_lat, &c->pf_lat));
+    CH_TRY(dalloc(c, (R + Hc) * c->ld_rot * e, &c->pf_rot));
+    CH_TRY(dalloc(c, (R + Hc) * c->ld_kv * e, &c->pf_kv));
+  }
   CH_TRY(dalloc_n(c, P * R * c->ld_cat, &c->pf_cat));
   CH_TRY(dalloc_n(c, R * lin, &c->pf_lin));
   CH_TRY(dalloc_n(c, P * R * c->ld_u, &c->pf_u));
@@ -477,14 +730,15 @@ int pass_alloc(Ctx* c) {
   CH_TRY(dalloc_n(c, P * LOGIT_ROWS * c->ldx, &c->pf_gp));
   CH_TRY(dalloc_n(c, LOGIT_ROWS * c->n_sq, &c->pf_gsq));
   CH_TRY(dalloc_n(c, LOGIT_ROWS * c->vocab, &c->pf_logits));
-  // seqs | tiles, small and big (a tile is at least one row) | rows | tokens | wanted rows
-  c->meta_bytes = R * (sizeof(PassSeq) + 2 * sizeof(PassTile) + sizeof(PassRow) + 2 * sizeof(int));
+  // seqs | tiles, small and big (a tile is at least one row) | rows, earlier positions behind them | tokens | wanted rows
+  c->meta_bytes = R * (sizeof(PassSeq) + 2 * sizeof(PassTile) + 2 * sizeof(int)) + (R + Hc) * sizeof(PassRow);
   CH_TRY(dalloc(c, c->meta_bytes, (void**)&c->meta));
   CH_HIP(dev, hipHostMalloc((void**)&c->h_meta, c->meta_bytes * META_SLOTS, hipHostMallocDefault));
   CH_HIP(dev, hipStreamCreateWithFlags(&c->side, hipStreamNonBlocking));
   CH_HIP(dev, hipEventCreateWithFlags(&c->fork, hipEventDisableTiming));
   CH_HIP(dev, hipEventCreateWithFlags(&c->join, hipEventDisableTiming));
   c->rows_cap = R;
+  c->hist_cap = Hc;
   return 0;
 }
 
@@ -498,12 +752,22 @@ struct Part {  // rows of one sequence in one pass
   std::vector<int> want;  // places among these rows
 };
 
-template <typename T, int CLS>
+template <typename T, int KC, int VC, bool LAT>
 void launch_attn_cls(Ctx* c, crabml_hip_device::ProfRec* rec, MixRows<T> m, const PassTiles& tiles) {
-  constexpr int big = AttnTile<T, CLS>::RT - 1;
+  constexpr int big = AttnTile<T, KC, VC>::RT - 1;
   m.tiles = tiles.list[big];
   m.n_tiles = (int)tiles.n[big];
-  launch_k(c->dev->stream, rec, k_attn_rows<T, CLS, sizeof(T) == 2 ? 1 : 3>, dim3(m.n_tiles, m.at.H), dim3(256), 0, m);
+  launch_k(c->dev->stream, rec, k_attn_rows<T, KC, VC, sizeof(T) == 2 ? 1 : 3, LAT>, dim3(m.n_tiles, m.at.H), dim3(256), 0, m);
+}
+template <typename T, bool LAT>
+void launch_attn(Ctx* c, const MixRows<T>& m, const PassTiles& tiles) {
+  Prof p(c->dev, true, ST_PASS + ST_MIX, 0.0);
+  const int w = std::max(m.at.D, m.at.V);
+  if (w <= 64) return launch_attn_cls<T, 64, 64, LAT>(c, p.rec(), m, tiles);
+  if (w <= 128) return launch_attn_cls<T, 128, 128, LAT>(c, p.rec(), m, tiles);
+  if constexpr (LAT && sizeof(T) == 2)
+    if (w <= 192 && m.at.V <= 128) return launch_attn_cls<T, 192, 128, LAT>(c, p.rec(), m, tiles);
+  launch_attn_cls<T, 256, 256, LAT>(c, p.rec(), m, tiles);
 }
 template <typename T, int CLS>
 int launch_linear_cls(Ctx* c, hipStream_t st, crabml_hip_device::ProfRec* rec, const MixRows<T>& m, size_t n_seq) {
@@ -514,7 +778,7 @@ int launch_linear_cls(Ctx* c, hipStream_t st, crabml_hip_device::ProfRec* rec, c
 }
 
 template <typename T>
-int mix_rows(Ctx* c, const Run& run, const PassSeq* seqs, size_t n_seq, const PassTiles& tiles, const PassRow* rows, size_t n_rows) {
+int mix_rows(Ctx* c, const Run& run, const PassSeq* seqs, size_t n_seq, const PassTiles& tiles, const PassRow* rows, size_t n_rows, size_t n_hist) {
   constexpr int P = sizeof(T) == 2 ? 1 : 3;
   const Layer& L = c->layers[run.layer];
   MixRows<T> m;
@@ -523,6 +787,10 @@ int mix_rows(Ctx* c, const Run& run, const PassSeq* seqs, size_t n_seq, const Pa
   m.rs = run.rs;
   m.seqs = seqs;
   m.rows = rows;
+  m.la = L.la;
+  m.M = (int)n_rows;
+  m.v_kept = (T*)c->pf_vk;
+  m.ld_vk = c->ld_vk;
   m.proj = (const T*)c->pf_proj;
   m.cat = c->pf_cat;
   m.cat_plane = c->rows_cap * (size_t)c->ld_cat;
@@ -530,6 +798,37 @@ int mix_rows(Ctx* c, const Run& run, const PassSeq* seqs, size_t n_seq, const Pa
   m.ldp = L.n_in;
   m.ldc = L.ldc;
   m.lin_off = L.lin_off;
+  if (L.la.rank) {
+    const int all = (int)(n_rows + n_hist);
+    m.lat = c->pf_lat;
+    m.lat_plane = (c->rows_cap + c->hist_cap) * (size_t)c->ld_lat;
+    m.rot = (T*)c->pf_rot;
+    m.kv = (const T*)c->pf_kv;
+    {
+      Prof p(c->dev, true, ST_PASS + ST_ROWS, 0.0);
+      launch_k(c->dev->stream, p.rec(), k_latent_rows<T, P>, dim3(all), dim3(256), 0, m);
+    }
+    {
+      GemmBf16 g;
+      g.a = c->pf_lat;
+      g.a_plane = m.lat_plane;
+      g.w = L.la.w_kv;
+      g.M = all;
+      g.N = g.ldo = L.at.H * (L.la.dim + L.at.V);
+      g.K = L.la.ldl;
+      g.out = c->pf_kv;
+      Prof p(c->dev, true, ST_PASS + ST_LAT, 0.0);
+      launch_gemm_bf16(c->dev, p.rec(), P, sizeof(T) == 4 ? GEMM_OUT_ACT_F32 : GEMM_OUT_ACT_BF16, g, c->pf_scratch);
+    }
+    launch_attn<T, true>(c, m, tiles);
+    Prof p(c->dev, true, ST_PASS + ST_ROWS, 0.0);
+    launch_k(c->dev->stream, p.rec(), k_latent_append<T, P>, dim3((unsigned)n_rows), dim3(256), 0, m);
+    return 0;
+  }
+  if (L.at.H && (L.at.q_norm || L.at.vmix)) {
+    Prof p(c->dev, true, ST_PASS + ST_ROWS, 0.0);
+    launch_k(c->dev->stream, p.rec(), k_qkv_rows<T>, dim3((unsigned)n_rows), dim3(256), 0, m);
+  }
   // the linear branch is a chain of blocks on few CUs: beside the softmax branch, when both are long enough to hide a fork
   hipStream_t st = c->dev->stream, lin_st = st;
   if (L.at.H && L.li.H && n_rows >= 192 && !c->dev->prof_on) {
@@ -547,16 +846,7 @@ int mix_rows(Ctx* c, const Run& run, const PassSeq* seqs, size_t n_seq, const Pa
       CH_TRY((launch_linear_cls<T, 256>(c, lin_st, p.rec(), m, n_seq)));
   }
   if (lin_st != st) CH_HIP(c->dev, hipEventRecord(c->join, lin_st));
-  if (L.at.H) {
-    Prof p(c->dev, true, ST_PASS + ST_MIX, 0.0);
-    const int w = std::max(L.at.D, L.at.V);
-    if (w <= 64)
-      launch_attn_cls<T, 64>(c, p.rec(), m, tiles);
-    else if (w <= 128)
-      launch_attn_cls<T, 128>(c, p.rec(), m, tiles);
-    else
-      launch_attn_cls<T, 256>(c, p.rec(), m, tiles);
-  }
+  if (L.at.H) launch_attn<T, false>(c, m, tiles);
   if (lin_st != st) CH_HIP(c->dev, hipStreamWaitEvent(st, c->join, 0));
   Prof p(c->dev, true, ST_PASS + ST_ROWS, 0.0);
   launch_k(c->dev->stream, p.rec(), k_mix_rows<T, P>, dim3((unsigned)n_rows), dim3(256), 0, m, c->cfg.norm_eps);
@@ -574,7 +864,7 @@ int run_pass(Ctx* c, const std::vector<Part>& parts, float** logits) {
   }
   const size_t R = c->rows_cap;
   char* hm = c->h_meta + c->meta_bytes * c->h_meta_next++;
-  const size_t o_tile = R * sizeof(PassSeq), o_row = o_tile + 2 * R * sizeof(PassTile), o_tok = o_row + R * sizeof(PassRow), o_want = o_tok + R * sizeof(int);
+  const size_t o_tile = R * sizeof(PassSeq), o_row = o_tile + 2 * R * sizeof(PassTile), o_tok = o_row + (R + c->hist_cap) * sizeof(PassRow), o_want = o_tok + R * sizeof(int);
   PassSeq* hs = (PassSeq*)hm;
   PassTile* ht[2] = {(PassTile*)(hm + o_tile), (PassTile*)(hm + o_tile) + R};
   PassRow* hr = (PassRow*)(hm + o_row);
@@ -583,7 +873,7 @@ int run_pass(Ctx* c, const std::vector<Part>& parts, float** logits) {
   for (size_t i = 0; i < parts.size(); i++) {
     const Part& p = parts[i];
     const Seq& s = c->seqs[p.seq];
-    hs[i] = PassSeq{(int)M, (int)p.n, (int)s.len, 0, s.slab};
+    hs[i] = PassSeq{(int)M, (int)p.n, (int)s.len, (int)M, s.slab};
     for (size_t b = 0; b < 2; b++)
       for (size_t r = 0; r < p.n; r += 64 << b)
         ht[b][n_tiles[b]++] = PassTile{(int)i, (int)(M + r), (int)(s.len + r), (int)std::min<size_t>(64 << b, p.n - r)};
@@ -594,6 +884,12 @@ int run_pass(Ctx* c, const std::vector<Part>& parts, float** logits) {
     }
     M += p.n;
   }
+  size_t n_hist = 0;  // earlier positions that latent layers read again
+  for (size_t i = 0; i < parts.size(); i++) {
+    const int len = (int)c->seqs[parts[i].seq].len, n = (int)std::min(c->hist, (size_t)len);
+    for (int p = len - n; p < len; p++) hr[M + n_hist++] = PassRow{(int)i, p};
+    hs[i].hist_end = (int)(M + n_hist);
+  }
   CH_HIP(dev, hipMemcpyAsync(c->meta, hm, c->meta_bytes, hipMemcpyHostToDevice, st));
   const PassSeq* ds = (const PassSeq*)c->meta;
   const PassTiles dt = {{(const PassTile*)(c->meta + o_tile), (const PassTile*)(c->meta + o_tile) + R}, {n_tiles[0], n_tiles[1]}};
@@ -602,12 +898,14 @@ int run_pass(Ctx* c, const std::vector<Part>& parts, float** logits) {
   const size_t xp = R * (size_t)c->ldx;
   const float eps = c->cfg.norm_eps;
   float* emb = c->keep_emb ? c->pf_emb : nullptr;
-  if (c->f32)
-    k_embed_rows<3><<<(unsigned)M, 256, 0, st>>>(c->embed, dk, dr, c->width, c->ldx, c->cfg.embed_scale, c->freq, c->pf_x, emb, c->runs[0].add_vec, c->pf_xp, xp,
-                                                c->pf_sq, c->n_sq);
-  else
-    k_embed_rows<1><<<(unsigned)M, 256, 0, st>>>(c->embed, dk, dr, c->width, c->ldx, c->cfg.embed_scale, c->freq, c->pf_x, emb, c->runs[0].add_vec, c->pf_xp, xp,
-                                                c->pf_sq, c->n_sq);
+  const size_t stride = R * (size_t)c->ldx;
+  const float* next_gain = c->streams ? c->layers[c->runs[0].layer].norm1 : nullptr;
+  {
+    const StreamMix sm = streams_at_start(c, stride);
+    auto embed = c->f32 ? k_embed_rows<3> : k_embed_rows<1>;
+    embed<<<(unsigned)M, 256, 0, st>>>(c->embed, dk, dr, c->width, c->ldx, c->cfg.embed_scale, c->freq, c->pf_x, emb, c->runs[0].add_vec, c->pf_xp, xp, c->pf_sq, c->n_sq, sm,
+                                       next_gain);
+  }
   auto normed = [&](const unsigned short* w, int n, const float* gain) {
     GemmBf16 g;
     g.a = c->pf_xp;
@@ -620,7 +918,7 @@ int run_pass(Ctx* c, const std::vector<Part>& parts, float** logits) {
     g.n_sq = c->n_sq;
     g.mean_n = c->width;
     g.eps = eps;
-    g.gain = gain;
+    g.gain = c->streams ? nullptr : gain;  // (a gain per element is in the planes)
     return g;
   };
   auto residual = [&](const unsigned short* a, size_t a_plane, const unsigned short* w, int k) {
@@ -650,53 +948,60 @@ int run_pass(Ctx* c, const std::vector<Part>& parts, float** logits) {
       g.out = c->pf_proj;
       g.ldo = L.n_in;
       g.act = L.act;
+      g.bias = L.bias_in;
       Prof p(dev, true, ST_PASS + ST_IN, 0.0);
       launch_gemm_bf16(dev, p.rec(), c->planes, c->f32 ? GEMM_OUT_ACT_F32 : GEMM_OUT_ACT_BF16, g, c->pf_scratch);
     }
     if (c->f32)
-      CH_TRY(mix_rows<float>(c, run, ds, parts.size(), dt, dr, M));
+      CH_TRY(mix_rows<float>(c, run, ds, parts.size(), dt, dr, M, n_hist));
     else
-      CH_TRY(mix_rows<unsigned short>(c, run, ds, parts.size(), dt, dr, M));
+      CH_TRY(mix_rows<unsigned short>(c, run, ds, parts.size(), dt, dr, M, n_hist));
     {
       GemmBf16 g = residual(c->pf_cat, R * (size_t)c->ld_cat, L.w_o, L.ldc);
       if (!L.ff) {
         g.add_rows = add_rows;
         g.add_vec = add_vec;
       }
+      if (c->streams) {
+        g.bias = L.bias_o;
+        g.sm = streams_behind(c, r, 0, stride, &g.gain_next);
+      }
       Prof p(dev, true, ST_PASS + ST_OUT, 0.0);
-      launch_gemm_bf16(dev, p.rec(), c->planes, GEMM_OUT_RESIDUAL, g, c->pf_scratch);
+      launch_gemm_bf16(dev, p.rec(), c->planes, c->streams ? GEMM_OUT_STREAMS : GEMM_OUT_RESIDUAL, g, c->pf_scratch);
     }
     if (!L.ff) continue;
     {
-      GemmBf16 g = normed(L.w_up, L.ff, L.norm2);
+      GemmBf16 g = normed(L.w_up, L.glu ? 2 * L.ff : L.ff, L.norm2);
       g.planes = c->pf_u;
       g.p_plane = R * (size_t)c->ld_u;
       g.ldp = L.ldu;
       g.xielu = L.xielu;
       Prof p(dev, true, ST_PASS + ST_UP, 0.0);
-      launch_gemm_bf16(dev, p.rec(), c->planes, GEMM_OUT_XIELU, g, c->pf_scratch);
+      launch_gemm_bf16(dev, p.rec(), c->planes, L.glu ? GEMM_OUT_GLU : GEMM_OUT_XIELU, g, c->pf_scratch);
     }
     {
       GemmBf16 g = residual(c->pf_u, R * (size_t)c->ld_u, L.w_down, L.ldu);
       g.add_rows = add_rows;
       g.add_vec = add_vec;
+      if (c->streams) g.sm = streams_behind(c, r, 1, stride, &g.gain_next);
       Prof p(dev, true, ST_PASS + ST_DOWN, 0.0);
-      launch_gemm_bf16(dev, p.rec(), c->planes, GEMM_OUT_RESIDUAL, g, c->pf_scratch);
+      launch_gemm_bf16(dev, p.rec(), c->planes, c->streams ? GEMM_OUT_STREAMS : GEMM_OUT_RESIDUAL, g, c->pf_scratch);
     }
   }
   for (size_t w0 = 0; w0 < nw; w0 += LOGIT_ROWS) {
     const size_t n = std::min(LOGIT_ROWS, nw - w0);
     const float* src = c->pf_logits;
+    StreamMix sum = streams_at_start(c, stride);
+    if (c->streams) sum.in = c->ones;
     if (n <= 8) {  // the decode step's classifier
-      k_gather_rows<0><<<(unsigned)n, 256, 0, st>>>(c->pf_x, c->ldx, c->width, dw + w0, c->st_x, nullptr, 0, nullptr, 0);
-      head_rows(c, c->st_x, (int)n, true);
+      float* x = c->streams ? c->st_in : c->st_x;
+      k_gather_rows<0><<<(unsigned)n, 256, 0, st>>>(c->pf_x, c->ldx, c->width, dw + w0, x, nullptr, 0, nullptr, 0, sum, nullptr);
+      head_rows(c, x, (int)n, true);
       src = c->st_logits;
     } else {
       const size_t gp = LOGIT_ROWS * (size_t)c->ldx;
-      if (c->f32)
-        k_gather_rows<3><<<(unsigned)n, 256, 0, st>>>(c->pf_x, c->ldx, c->width, dw + w0, nullptr, c->pf_gp, gp, c->pf_gsq, c->n_sq);
-      else
-        k_gather_rows<1><<<(unsigned)n, 256, 0, st>>>(c->pf_x, c->ldx, c->width, dw + w0, nullptr, c->pf_gp, gp, c->pf_gsq, c->n_sq);
+      auto gather = c->f32 ? k_gather_rows<3> : k_gather_rows<1>;
+      gather<<<(unsigned)n, 256, 0, st>>>(c->pf_x, c->ldx, c->width, dw + w0, nullptr, c->pf_gp, gp, c->pf_gsq, c->n_sq, sum, c->streams ? c->final_norm : nullptr);
       GemmBf16 g = normed(c->head, c->vocab, c->final_norm);
       g.a = c->pf_gp;
       g.a_plane = gp;
@@ -733,21 +1038,34 @@ int create_impl(Ctx* c, const crabml_hip_hybrid_layer_t* layers, const crabml_hi
   c->ldx = up(W, 64);
   c->n_sq = c->ldx / 64;
   c->keep_emb = g.loop_times > 1;
+  c->streams = g.streams ? (int)g.streams : (g.flags & CRABML_HIP_HYBRID_NORM_VECTOR ? 1 : 0);
+  CH_TRY(dalloc_n(c, HC_MAX, &c->ones));
+  const std::vector<float> ones(HC_MAX, 1.f);
+  CH_HIP(dev, hipMemcpyAsync(c->ones, ones.data(), HC_MAX * sizeof(float), hipMemcpyHostToDevice, dev->stream));
+  CH_HIP(dev, hipStreamSynchronize(dev->stream));
   CH_TRY(alloc_matrix(c, g.vocab_size, (size_t)c->ldx, &c->head));
   CH_TRY(dalloc_n(c, g.vocab_size * W, &c->embed));
   CH_TRY(pack_matrix(c, w.embed, "embed", g.vocab_size, W, c->embed, W, 0, g.vocab_size, g.vocab_size));
-  CH_TRY(pack_matrix(c, w.head, "head", g.vocab_size, W, c->head, (size_t)c->ldx, 0, g.vocab_size, g.vocab_size));
-  CH_TRY(pack_vector(c, w.final_norm, "final_norm", 1, &c->final_norm));
+  CH_TRY(pack_matrix(c, w.head ? w.head : w.embed, "head", g.vocab_size, W, c->head, (size_t)c->ldx, 0, g.vocab_size, g.vocab_size));
+  CH_TRY(pack_norm(c, w.final_norm, "final_norm", &c->final_norm));
   if (g.loop_times) CH_TRY(pack_vector(c, w.loop_step, "loop_step", g.loop_times * W, &c->loop_step));
   c->layers.resize(g.n_layers);
-  size_t part = 0, tick = 0, ss = 0;
+  size_t part = 0, tick = 0, ss = 0, lat_q = 0, lat_part = 0;
   for (size_t i = 0; i < g.n_layers; i++) {
     Layer& L = c->layers[i];
     CH_TRY(build_layer(c, layers[i], L));
     c->ld_proj = std::max(c->ld_proj, L.n_in);
     c->ld_cat = std::max(c->ld_cat, L.ldc);
     c->ld_u = std::max(c->ld_u, L.ldu);
-    if (L.at.H) {
+    if (L.la.rank) {
+      const size_t row = (size_t)L.la.rank + L.la.rot;
+      lat_q = std::max(lat_q, (size_t)HYB_STEP_ROWS * L.at.H * row);
+      lat_part = std::max(lat_part, (size_t)HYB_STEP_ROWS * L.at.H * LAT_SPLITS * (L.la.rank + 2));
+      c->ld_kv = std::max(c->ld_kv, L.at.H * (L.la.dim + L.at.V));
+      c->ld_lat = std::max(c->ld_lat, L.la.ldl);
+      c->ld_rot = std::max(c->ld_rot, L.la.rot);
+      c->hist = std::max(c->hist, (size_t)L.at.rows - (L.at.window ? 1 : 0));
+    } else if (L.at.H) {
       const size_t slots = (size_t)HYB_STEP_ROWS * L.at.G * L.head_blocks;
       part = std::max(part, slots * L.splits * mix_part_floats(L.at.V));
       tick = std::max(tick, slots);
@@ -765,7 +1083,9 @@ int create_impl(Ctx* c, const crabml_hip_hybrid_layer_t* layers, const crabml_hi
       c->slab_bytes += align_up(bytes, 256);
       return at;
     };
-    if (L.at.H) {
+    if (L.la.rank) {
+      r.rs.k = take((size_t)L.at.rows * (L.la.rank + L.la.rot) * e);
+    } else if (L.at.H) {
       r.rs.k = take((size_t)L.at.G * L.at.rows * L.at.D * e);
       r.rs.v = take((size_t)L.at.G * L.at.rows * L.at.V * e);
     }
@@ -781,9 +1101,9 @@ int create_impl(Ctx* c, const crabml_hip_hybrid_layer_t* layers, const crabml_hi
   for (size_t t = 0; t < g.loop_times; t++)
     for (size_t i = lo; i < hi; i++) add_run(i, i == lo, t);
   for (size_t i = hi; i < g.n_layers; i++) add_run(i, false, 0);
-  {
+  if (g.position_base > 0) {
     std::vector<double> f((W + 1) / 2);
-    for (size_t i = 0; i < f.size(); i++) f[i] = pow(10000.0, -2.0 * (double)i / (double)W);
+    for (size_t i = 0; i < f.size(); i++) f[i] = pow(g.position_base, -2.0 * (double)i / (double)W);
     CH_TRY(dalloc_n(c, f.size(), &c->freq));
     CH_HIP(dev, hipMemcpyAsync(c->freq, f.data(), f.size() * sizeof(double), hipMemcpyHostToDevice, dev->stream));
     CH_HIP(dev, hipStreamSynchronize(dev->stream));
@@ -791,7 +1111,11 @@ int create_impl(Ctx* c, const crabml_hip_hybrid_layer_t* layers, const crabml_hi
   const size_t B = HYB_STEP_ROWS;
   CH_TRY(dalloc_n(c, B, &c->st_seq));
   CH_TRY(dalloc_n(c, 1, &c->st_count));
-  CH_TRY(dalloc_n(c, B * c->ldx, &c->st_x));
+  CH_TRY(dalloc_n(c, (c->streams ? c->streams : 1) * B * c->ldx, &c->st_x));
+  if (c->streams) CH_TRY(dalloc_n(c, B * c->ldx, &c->st_in));
+  if (c->ld_vk) CH_TRY(dalloc_n(c, B * c->ld_vk, &c->st_vk));
+  CH_TRY(dalloc_n(c, lat_q, &c->st_q));
+  CH_TRY(dalloc_n(c, lat_part, &c->st_lpart));
   CH_TRY(dalloc_n(c, B * c->ldx, &c->st_emb));
   CH_TRY(dalloc_n(c, B * c->ld_proj, &c->st_proj));
   CH_TRY(dalloc_n(c, B * c->ld_cat, &c->st_cat));
@@ -825,6 +1149,9 @@ int crabml_hip_hybrid_create(crabml_hip_device_t* dev, const crabml_hip_hybrid_c
   if (cfg->compute != CRABML_HIP_BF16 && cfg->compute != CRABML_HIP_F32) CH_BAIL(dev, CRABML_HIP_BAD_INPUT, "hybrid: compute is BF16 or F32, not %u", cfg->compute);
   if (cfg->loop_times && (cfg->loop_start >= cfg->loop_stop || cfg->loop_stop > cfg->n_layers))
     CH_BAIL(dev, CRABML_HIP_BAD_INPUT, "hybrid: loop over layers [%zu, %zu) of %zu", cfg->loop_start, cfg->loop_stop, cfg->n_layers);
+  if (cfg->streams > HC_MAX) CH_BAIL(dev, CRABML_HIP_NOT_IMPLEMENTED, "hybrid: %zu residual streams (at most %d)", cfg->streams, HC_MAX);
+  if (cfg->loop_times && (cfg->streams || (cfg->flags & CRABML_HIP_HYBRID_NORM_VECTOR)))
+    CH_BAIL(dev, CRABML_HIP_NOT_IMPLEMENTED, "hybrid: a loop goes with a single residual row and norms of a single gain");
   Ctx* c = new Ctx();
   c->dev = dev;
   c->cfg = *cfg;
@@ -930,15 +1257,18 @@ int crabml_hip_hybrid_step(crabml_hip_hybrid_t* c, size_t n, const size_t* seqs,
   }
   const size_t cap = c->cfg.pass_rows ? c->cfg.pass_rows : 2048;
   std::vector<Part> parts;
-  size_t used = 0, tok = 0, wat = 0;
+  CH_TRY(pass_alloc(c));
+  size_t used = 0, hist = 0, tok = 0, wat = 0;
   for (size_t i = 0; i < n; i++) {
     size_t done = 0, k = 0;
     const size_t nw = want_counts ? want_counts[i] : 0;
     while (done < counts[i]) {
-      if (used == cap) {
+      const size_t back = std::min(c->hist, c->seqs[seqs[i]].len);  // (a part that waits in `parts` is not of this sequence)
+      if (used == cap || (hist && hist + back > c->hist_cap)) {
         CH_TRY(run_pass(c, parts, &logits));
         parts.clear();
-        used = 0;
+        used = hist = 0;
+        continue;
       }
       Part p;
       p.seq = seqs[i];
@@ -947,6 +1277,7 @@ int crabml_hip_hybrid_step(crabml_hip_hybrid_t* c, size_t n, const size_t* seqs,
       for (; k < nw && want[wat + k] < done + p.n; k++) p.want.push_back((int)(want[wat + k] - done));
       done += p.n;
       used += p.n;
+      hist += back;
       parts.push_back(std::move(p));
     }
     tok += counts[i];

@@ -4,8 +4,8 @@
 //   k_linear_rows          linear attention in blocks of rows: inside a block as a masked product, across blocks through the state
 //   k_mix_rows             the linear branch's norm and gate, the cache append
 //   k_gemm_bf16<RESIDUAL>, k_gemm_bf16<XIELU>, k_gemm_bf16<RESIDUAL>
-// Keys of this pass are read from its own projected rows, earlier ones of the first chunk from the cache; the cache is appended only
-// after the attention launch, with the rows of the chunk that the pass ends in.
+// Keys of this pass are read from its own projected rows, earlier ones from the cache; the cache is appended only after the attention
+// launch, with the rows that later tokens can see.
 //
 // T = unsigned short: bf16 operands.  T = float: every operand f32 (v_mfma_f32_16x16x4_f32), activations in three exact planes.
 #pragma once
@@ -14,7 +14,8 @@
 namespace crabml_hip {
 
 struct PassSeq {
-  int row0, n, pos0, pad;  // rows row0 .. row0 + n - 1 of the pass are the sequence's positions pos0 ..
+  int row0, n, pos0;  // rows row0 .. row0 + n - 1 of the pass are the sequence's positions pos0 ..
+  int hist_end;       // earlier positions that latent layers read again, as rows: position p < pos0 is row hist_end - (pos0 - p)
   char* slab;
 };
 struct PassRow {
@@ -92,16 +93,25 @@ __global__ __launch_bounds__(256) void k_embed_rows(const unsigned short* __rest
                                                     const PassRow* __restrict__ rows, int width, int ldx, float scale,
                                                     const double* __restrict__ freq, float* __restrict__ x, float* __restrict__ emb,
                                                     const float* __restrict__ add_vec, unsigned short* __restrict__ planes, size_t p_plane,
-                                                    float* __restrict__ sq_out, int n_sq) {
+                                                    float* __restrict__ sq_out, int n_sq, const StreamMix sm, const float* __restrict__ gain) {
   __shared__ float red[4];
   const int r = blockIdx.x, tok = tokens[r], pos = rows[r].pos;
   float s = 0.f;
   for (int c = threadIdx.x; c < width; c += 256) {
     float v = __builtin_fmaf(bf2f(table[(size_t)tok * width + c]), scale, position_entry(pos, c, freq));
-    if (emb) emb[(size_t)r * ldx + c] = v;
-    if (add_vec) v += add_vec[c];
-    x[(size_t)r * ldx + c] = v;
-    split_store<P>(v, planes + (size_t)r * ldx + c, p_plane);
+    if (sm.n) {  // every stream starts as the embedding
+      float u = 0.f;
+      for (int t = 0; t < sm.n; t++) {
+        x[t * sm.stride + (size_t)r * ldx + c] = v;
+        u = __builtin_fmaf(sm.in[t], v, u);
+      }
+      v = u;
+    } else {
+      if (emb) emb[(size_t)r * ldx + c] = v;
+      if (add_vec) v += add_vec[c];
+      x[(size_t)r * ldx + c] = v;
+    }
+    split_store<P>(gain ? v * gain[c] : v, planes + (size_t)r * ldx + c, p_plane);
     s = __builtin_fmaf(v, v, s);
   }
   s = wave_sum_f32(s);
@@ -110,21 +120,25 @@ __global__ __launch_bounds__(256) void k_embed_rows(const unsigned short* __rest
   for (int i = threadIdx.x; i < n_sq; i += 256) sq_out[(size_t)r * n_sq + i] = i ? 0.f : (red[0] + red[1]) + (red[2] + red[3]);
 }
 
-// rows[i] of x -> dense rows of f32 (P = 0) or planes, with their square sums in piece 0
+// rows[i] of x (the weighted sum of its streams) -> dense rows of f32 (P = 0) or planes, with their square sums in piece 0
 template <int P>
 __global__ __launch_bounds__(256) void k_gather_rows(const float* __restrict__ x, int ldx, int width, const int* __restrict__ which,
                                                      float* __restrict__ dst, unsigned short* __restrict__ planes, size_t p_plane,
-                                                     float* __restrict__ sq_out, int n_sq) {
+                                                     float* __restrict__ sq_out, int n_sq, const StreamMix sm, const float* __restrict__ gain) {
   __shared__ float red[4];
   const int r = blockIdx.x;
   const float* src = x + (size_t)which[r] * ldx;
   float s = 0.f;
   for (int c = threadIdx.x; c < width; c += 256) {
-    const float v = src[c];
+    float v = src[c];
+    if (sm.n) {
+      v *= sm.in[0];
+      for (int t = 1; t < sm.n; t++) v = __builtin_fmaf(sm.in[t], src[t * sm.stride + c], v);
+    }
     if constexpr (P == 0) {
       dst[(size_t)r * ldx + c] = v;
     } else {
-      split_store<P>(v, planes + (size_t)r * ldx + c, p_plane);
+      split_store<P>(gain ? v * gain[c] : v, planes + (size_t)r * ldx + c, p_plane);
       s = __builtin_fmaf(v, v, s);
     }
   }
@@ -141,6 +155,7 @@ template <typename T>
 struct MixRows {
   AttnGeom at;
   LinGeom li;
+  LatGeom la;
   RunState rs;
   const PassSeq* seqs = nullptr;
   const PassTile* tiles = nullptr;
@@ -150,13 +165,21 @@ struct MixRows {
   size_t cat_plane = 0;
   float* lin = nullptr;  // [rows][H * V] raw outputs of the linear branch
   int n_tiles = 0, ldp = 0, ldc = 0, lin_off = 0;
+  T* v_kept = nullptr;  // [rows][ld_vk] values that VMIX_KEEP leaves
+  int ld_vk = 0;
+  // latent attention: rows of this pass, then the earlier ones (PassSeq::hist_end)
+  unsigned short* lat = nullptr;  // [planes][rows][la.ldl] normed latents
+  size_t lat_plane = 0;
+  T* rot = nullptr;       // [rows][la.rot] rotated key parts
+  const T* kv = nullptr;  // [rows][H * (la.dim + V)] keys of all heads, values of all heads
+  int M = 0;              // rows of this pass
 };
 
-// Shape of the attention kernel for heads up to CLS wide: KT keys per tile; RT times 16 query rows per wave.
-template <typename T, int CLS>
+// Shape of the attention kernel for keys up to KC and values up to VC wide: KT keys per tile; RT times 16 query rows per wave.
+template <typename T, int KC, int VC>
 struct AttnTile {
-  static constexpr int PAD = 16 / sizeof(T), KT = sizeof(T) == 2 ? (CLS > 128 ? 32 : 64) : 4096 / CLS;
-  static constexpr int RT = sizeof(T) == 2 && CLS <= 128 ? 2 : 1;
+  static constexpr int PAD = 16 / sizeof(T), KT = sizeof(T) == 2 ? (KC > 128 ? 32 : 64) : 4096 / KC;
+  static constexpr int RT = sizeof(T) == 2 && KC <= 192 && VC <= 128 ? 2 : 1;
 };
 
 // One workgroup: 64 RT query rows of one head, four waves of 16 RT.  Keys come in tiles through LDS (K as rows, V transposed), the next
@@ -165,47 +188,70 @@ struct AttnTile {
 // one number per lane, and the accumulators of S^T, exponentiated, ARE the operand of the second product: k slot (lane / 16, i) of the
 // matrix instruction stands for key 4 (lane / 16) + i of a 16-key group, and V^T is read from LDS in the same order.  Scores live in
 // the log2 domain.
-template <typename T, int CLS, int P>
+template <typename T, int KC, int VC, int P, bool LAT>
 __global__ __launch_bounds__(256, sizeof(T) == 2 ? 2 : 1) void k_attn_rows(const MixRows<T> a) {
-  typedef AttnTile<T, CLS> A;
-  constexpr int KT = A::KT, RT = A::RT, LK = CLS + A::PAD, LV = KT + A::PAD, VT = CLS / 16, ST = KT / 16;
-  constexpr int NK = KT * CLS / 8 / 256;  // octets of K (and of V) per thread and tile
-  static_assert(NK >= 1 && NK % 2 == 0, "V octets are handled in pairs of keys");
+  typedef AttnTile<T, KC, VC> A;
+  constexpr int KT = A::KT, RT = A::RT, LK = KC + A::PAD, LV = KT + A::PAD, VT = VC / 16, ST = KT / 16;
+  constexpr int NK = KT * KC / 8 / 256, NV = KT * VC / 8 / 256;  // octets of K and of V per thread and tile
+  static_assert(NK >= 1 && NV >= 2 && NV % 2 == 0, "V octets are handled in pairs of keys");
   __shared__ __attribute__((aligned(16))) T ks[KT * LK];
-  __shared__ __attribute__((aligned(16))) T vs[CLS * LV];
+  __shared__ __attribute__((aligned(16))) T vs[VC * LV];
   const AttnGeom& g = a.at;
   const int tid = threadIdx.x, lane = tid & 63, wave = wave_in_wg(), fr = lane & 15, fk = lane >> 4;
   const PassTile t = a.tiles[a.n_tiles - 1 - blockIdx.x];  // (a sequence's last tiles see the most keys: first)
   const PassSeq sq = a.seqs[t.seq];
   const int h = blockIdx.y, kvh = h / (g.H / g.G);
   const int DK = (g.D + 31) & ~31;
-  const int lo = t.pos - t.pos % g.chunk, hi = t.pos + t.n;  // keys [lo, hi); those before pos0 are cache rows from `lo` on
+  const int lo = attn_first(g, t.pos), hi = t.pos + t.n;  // keys [lo, hi); those before pos0 are cache rows from that of `lo` on
+  const int ring = lo % g.span;
   const T* kc = (const T*)(sq.slab + a.rs.k) + (size_t)kvh * g.rows * g.D;
   const T* vc = (const T*)(sq.slab + a.rs.v) + (size_t)kvh * g.rows * g.V;
   const T* pk = a.proj + (size_t)sq.row0 * a.ldp + g.ck + kvh * g.D;
   const T* pv = a.proj + (size_t)sq.row0 * a.ldp + g.cv + kvh * g.V;
+  const int ldkv = LAT ? g.H * (a.la.dim + g.V) : 0;
+  // position p, column c -> the octet of its key / value
+  auto k_at = [&](int p, int c) -> const T* {
+    if constexpr (LAT) {
+      const size_t row = (size_t)((p >= sq.pos0 ? sq.row0 : sq.hist_end) + (p - sq.pos0));
+      return c < a.la.dim ? a.kv + row * ldkv + h * a.la.dim + c : a.rot + row * a.la.rot + (c - a.la.dim);
+    } else {
+      if (p >= sq.pos0) return pk + (size_t)(p - sq.pos0) * a.ldp + c;
+      const int r = ring + (p - lo);
+      return kc + (size_t)(r < g.span ? r : r - g.span) * g.D + c;
+    }
+  };
+  auto v_at = [&](int p, int c) -> const T* {
+    if constexpr (LAT) {
+      const size_t row = (size_t)((p >= sq.pos0 ? sq.row0 : sq.hist_end) + (p - sq.pos0));
+      return a.kv + row * ldkv + g.H * a.la.dim + h * g.V + c;
+    } else {
+      if (p >= sq.pos0) return pv + (size_t)(p - sq.pos0) * a.ldp + c;
+      const int r = ring + (p - lo);
+      return vc + (size_t)(r < g.span ? r : r - g.span) * g.V + c;
+    }
+  };
   // this wave's rows, and the keys any of them sees
   const int w0 = wave * 16 * RT, wn = min(16 * RT, t.n - w0);
-  const int wfirst = t.pos + w0, wlast = wfirst + wn - 1, wlo = wfirst - wfirst % g.chunk, whi_chunk = wlast - (wlast > 0 ? wlast % g.chunk : 0);
-  bf16x8 q16[RT][sizeof(T) == 2 ? CLS / 32 : 1];
-  float q32[RT][sizeof(T) == 4 ? CLS / 4 : 1];
+  const int wfirst = t.pos + w0, wlast = wfirst + wn - 1, wlo = attn_first(g, wfirst), wlast_lo = attn_first(g, wlast > 0 ? wlast : 0);
+  bf16x8 q16[RT][sizeof(T) == 2 ? KC / 32 : 1];
+  float q32[RT][sizeof(T) == 4 ? KC / 4 : 1];
   int pos[RT], first[RT];
 #pragma unroll
   for (int r = 0; r < RT; r++) {
     const int row = w0 + r * 16 + fr;
     const T* qp = a.proj + (size_t)(t.row + (row < t.n ? row : t.n - 1)) * a.ldp + g.cq + h * g.D;
     pos[r] = t.pos + row;
-    first[r] = pos[r] - pos[r] % g.chunk;
+    first[r] = attn_first(g, pos[r]);
     if constexpr (sizeof(T) == 2) {
 #pragma unroll
-      for (int i = 0; i < CLS / 32; i++) {
+      for (int i = 0; i < KC / 32; i++) {
         const int k = i * 32 + fk * 8;
         const Oct<T> o = k < g.D ? oct_load(qp + k) : oct_zero<T>();
         __builtin_memcpy(&q16[r][i], &o, 16);
       }
     } else {
 #pragma unroll
-      for (int i = 0; i < CLS / 4; i++) q32[r][i] = i * 4 + fk < g.D ? (float)qp[i * 4 + fk] : 0.f;
+      for (int i = 0; i < KC / 4; i++) q32[r][i] = i * 4 + fk < g.D ? (float)qp[i * 4 + fk] : 0.f;
     }
   }
   float m[RT], l[RT];
@@ -218,19 +264,19 @@ __global__ __launch_bounds__(256, sizeof(T) == 2 ? 2 : 1) void k_attn_rows(const
     for (int j = 0; j < VT; j++) o[r][j] = f32x4{0.f, 0.f, 0.f, 0.f};
   }
   const float amp = g.amp ? g.amp[h] : 0.f, rate = g.amp ? g.rate[h] : 0.f, scale2 = g.scale * 1.44269504f;
-  Oct<T> rk[NK], rv[NK];
+  Oct<T> rk[NK], rv[NV];
   auto request = [&](int j0) {
 #pragma unroll
     for (int u = 0; u < NK; u++) {
-      const int i = u * 256 + tid, c = i % (CLS / 8) * 8, p = j0 + i / (CLS / 8);
+      const int i = u * 256 + tid, c = i % (KC / 8) * 8, p = j0 + i / (KC / 8);
       rk[u] = oct_zero<T>();
-      if (p < hi && c < g.D) rk[u] = oct_load(p >= sq.pos0 ? pk + (size_t)(p - sq.pos0) * a.ldp + c : kc + (size_t)(p - lo) * g.D + c);
+      if (p < hi && c < g.D) rk[u] = oct_load(k_at(p, c));
     }
 #pragma unroll
-    for (int u = 0; u < NK; u++) {  // octets u, u + 1: the same columns of two neighbouring keys
+    for (int u = 0; u < NV; u++) {  // octets u, u + 1: the same columns of two neighbouring keys
       const int i = (u >> 1) * 256 + tid, c = i / (KT / 2) * 8, p = j0 + i % (KT / 2) * 2 + (u & 1);
       rv[u] = oct_zero<T>();
-      if (p < hi && c < g.V) rv[u] = oct_load(p >= sq.pos0 ? pv + (size_t)(p - sq.pos0) * a.ldp + c : vc + (size_t)(p - lo) * g.V + c);
+      if (p < hi && c < g.V) rv[u] = oct_load(v_at(p, c));
     }
   };
   request(lo);
@@ -239,10 +285,10 @@ __global__ __launch_bounds__(256, sizeof(T) == 2 ? 2 : 1) void k_attn_rows(const
 #pragma unroll
     for (int u = 0; u < NK; u++) {
       const int i = u * 256 + tid;
-      oct_store(ks + i / (CLS / 8) * LK + i % (CLS / 8) * 8, rk[u]);
+      oct_store(ks + i / (KC / 8) * LK + i % (KC / 8) * 8, rk[u]);
     }
 #pragma unroll
-    for (int u = 0; u < NK; u += 2) {
+    for (int u = 0; u < NV; u += 2) {
       const int i = (u >> 1) * 256 + tid, c = i / (KT / 2) * 8, key = i % (KT / 2) * 2;
       T v0[8], v1[8];
       __builtin_memcpy(v0, &rv[u], sizeof v0);
@@ -256,7 +302,7 @@ __global__ __launch_bounds__(256, sizeof(T) == 2 ? 2 : 1) void k_attn_rows(const
     __syncthreads();
     if (j0 + KT < hi) request(j0 + KT);
     if (wn <= 0 || j0 > wlast || j0 + KT <= wlo) continue;  // (wave-uniform: nothing here for this wave's rows)
-    const bool edge = j0 + KT - 1 > wfirst || j0 < whi_chunk;
+    const bool edge = j0 + KT - 1 > wfirst || j0 < wlast_lo;
     f32x4 s[RT][ST];
 #pragma unroll
     for (int j = 0; j < ST; j++) {
@@ -265,7 +311,7 @@ __global__ __launch_bounds__(256, sizeof(T) == 2 ? 2 : 1) void k_attn_rows(const
       for (int r = 0; r < RT; r++) s[r][j] = f32x4{0.f, 0.f, 0.f, 0.f};
       if constexpr (sizeof(T) == 2) {
 #pragma unroll
-        for (int i = 0; i < CLS / 32; i++)
+        for (int i = 0; i < KC / 32; i++)
           if (i * 32 < DK) {
             const bf16x8 kf = *(const bf16x8*)(kr + i * 32 + fk * 8);
 #pragma unroll
@@ -273,7 +319,7 @@ __global__ __launch_bounds__(256, sizeof(T) == 2 ? 2 : 1) void k_attn_rows(const
           }
       } else {
 #pragma unroll
-        for (int i = 0; i < CLS / 4; i++)
+        for (int i = 0; i < KC / 4; i++)
           if (i * 4 < DK) {
             const float kf = kr[i * 4 + fk];
 #pragma unroll
@@ -372,10 +418,10 @@ __global__ __launch_bounds__(256, sizeof(T) == 2 ? 2 : 1) void k_attn_rows(const
       const int c = j * 16 + fk * 4;
       if (c < g.V) {  // (widths are multiples of 8: four columns at a time)
         const int col = h * g.V + c;
-        const T* gp = a.proj + at * a.ldp + g.cg + col;
+        const T* gp = a.proj + at * a.ldp + g.cg + (g.gate == GATE_HEAD ? h : col);
         float v[4];
 #pragma unroll
-        for (int e = 0; e < 4; e++) v[e] = o[r][j][e] * (w * kv_to(gp[e]));
+        for (int e = 0; e < 4; e++) v[e] = o[r][j][e] * (g.gate == GATE_NONE ? w : w * kv_to(gp[g.gate == GATE_HEAD ? 0 : e]));
         split_store4<P>(v, a.cat + at * a.ldc + col, a.cat_plane);
       }
     }
@@ -501,6 +547,54 @@ __global__ __launch_bounds__(256) void k_linear_rows(const MixRows<T> a) {
     }
 }
 
+// ---- in front of attention: the norms over all of a row's queries (keys), the values of an earlier layer ------------------------------
+template <typename T>
+__device__ __forceinline__ void octet_scale(T* p, float f, const float* gain) {
+  float v[8], n[8];
+  kv_load8(p, v);
+  read8(gain, n);
+#pragma unroll
+  for (int e = 0; e < 8; e++) p[e] = kv_from<T>(v[e] * (f * n[e]));
+}
+template <typename T>
+__global__ __launch_bounds__(256) void k_qkv_rows(const MixRows<T> a) {
+  __shared__ float red[8];
+  const AttnGeom& g = a.at;
+  const int r = blockIdx.x, tid = threadIdx.x, nq = g.H * g.D, nk = g.G * g.D, nv = g.G * g.V;
+  T* pr = const_cast<T*>(a.proj) + (size_t)r * a.ldp;
+  if (g.q_norm) {
+    float sq = 0.f, sk = 0.f, v[8];
+    for (int i = tid * 8; i < nq; i += 2048) {
+      kv_load8(pr + g.cq + i, v);
+#pragma unroll
+      for (int e = 0; e < 8; e++) sq = __builtin_fmaf(v[e], v[e], sq);
+    }
+    for (int i = tid * 8; i < nk; i += 2048) {
+      kv_load8(pr + g.ck + i, v);
+#pragma unroll
+      for (int e = 0; e < 8; e++) sk = __builtin_fmaf(v[e], v[e], sk);
+    }
+    sq = wave_sum_f32(sq);
+    sk = wave_sum_f32(sk);
+    if ((tid & 63) == 0) {
+      red[tid >> 6] = sq;
+      red[4 + (tid >> 6)] = sk;
+    }
+    __syncthreads();
+    const float fq = 1.0f / sqrtf(((red[0] + red[1]) + (red[2] + red[3])) / (float)g.q_mean + g.eps);
+    const float fk = 1.0f / sqrtf(((red[4] + red[5]) + (red[6] + red[7])) / (float)g.k_mean + g.eps);
+    for (int i = tid * 8; i < nq; i += 2048) octet_scale(pr + g.cq + i, fq, g.q_norm + i);
+    for (int i = tid * 8; i < nk; i += 2048) octet_scale(pr + g.ck + i, fk, g.k_norm + i);
+  }
+  T* vk = a.v_kept + (size_t)r * a.ld_vk;
+  if (g.vmix == VMIX_KEEP)
+    for (int i = tid; i < nv; i += 256) vk[i] = pr[g.cv + i];
+  if (g.vmix == VMIX_MIX) {
+    const float la = *g.lambda;
+    for (int i = tid; i < nv; i += 256) pr[g.cv + i] = kv_from<T>(__builtin_fmaf(la, kv_to(vk[i]), (1.0f - la) * kv_to(pr[g.cv + i])));
+  }
+}
+
 // ---- behind both: the linear branch's norm and gate; the cache rows of the chunk each sequence's part of the pass ends in ----------
 template <typename T, int P>
 __global__ __launch_bounds__(256) void k_mix_rows(const MixRows<T> a, float eps) {
@@ -525,10 +619,10 @@ __global__ __launch_bounds__(256) void k_mix_rows(const MixRows<T> a, float eps)
     const AttnGeom& g = a.at;
     const PassSeq sq = a.seqs[rw.seq];
     const int last = sq.pos0 + sq.n - 1;
-    if (rw.pos / g.chunk != last / g.chunk) return;
+    if (rw.pos < attn_first(g, last)) return;
     T* kc = (T*)(sq.slab + a.rs.k);
     T* vc = (T*)(sq.slab + a.rs.v);
-    const size_t at = (size_t)(rw.pos % g.chunk);
+    const size_t at = (size_t)(rw.pos % g.span);
     for (int i = tid; i < g.G * g.D; i += 256) kc[((size_t)(i / g.D) * g.rows + at) * g.D + i % g.D] = pr[g.ck + i];
     for (int i = tid; i < g.G * g.V; i += 256) vc[((size_t)(i / g.V) * g.rows + at) * g.V + i % g.V] = pr[g.cv + i];
   }

@@ -23,11 +23,20 @@ struct StepSeq {
 
 __global__ __launch_bounds__(256) void k_embed_step(const unsigned short* __restrict__ table, const StepSeq* __restrict__ seq, int width, int ldx,
                                                     float scale, const double* __restrict__ freq, float* __restrict__ x, float* __restrict__ emb,
-                                                    const float* __restrict__ add_vec) {
+                                                    const float* __restrict__ add_vec, const StreamMix sm, float* __restrict__ u) {
   const int c = blockIdx.x * 256 + threadIdx.x, b = blockIdx.y;
   if (c >= width) return;
   const StepSeq s = seq[b];
   const float v = __builtin_fmaf(bf2f(table[(size_t)s.token * width + c]), scale, position_entry(s.pos, c, freq));
+  if (sm.n) {  // every stream starts as the embedding
+    float r = 0.f;
+    for (int t = 0; t < sm.n; t++) {
+      x[t * sm.stride + (size_t)b * ldx + c] = v;
+      r = __builtin_fmaf(sm.in[t], v, r);
+    }
+    u[(size_t)b * ldx + c] = r;
+    return;
+  }
   if (emb) emb[(size_t)b * ldx + c] = v;
   x[(size_t)b * ldx + c] = add_vec ? v + add_vec[c] : v;
 }
@@ -41,6 +50,8 @@ struct MixStep {
   float* cat = nullptr;         // [B][ldc]: attention columns from 0, linear columns from lin_off
   float* ss = nullptr;          // [B][H * slices] square sums of the linear branch
   float* part = nullptr;        // attention partials
+  float* v_kept = nullptr;      // [B][ld_vk] values that VMIX_KEEP leaves
+  int ld_vk = 0;
   unsigned* tick = nullptr;     // arrivals per (sequence, kv head, head block); the last one puts it back to zero
   int B = 0, ldp = 0, ldc = 0, lin_off = 0, splits = 0, head_blocks = 0;
 };
@@ -65,31 +76,58 @@ __device__ __forceinline__ void mix_attention(const MixStep& a, int blk, float* 
   const int nh = hpg - hb * MIX_HEADS < MIX_HEADS ? hpg - hb * MIX_HEADS : MIX_HEADS;
   const float* pr = a.proj + (size_t)b * a.ldp;
   float* ml = lds;                          // [MIX_HEADS][2]: maximum, denominator
-  float* hp_s = ml + 2 * MIX_HEADS;         // [3][MIX_HEADS]: penalty factor, its rate, sink; padded to 4
-  T* kn_s = (T*)(hp_s + 4 * MIX_HEADS);     // [CLS], [CLS]: the new token's row as the cache holds it
+  float* hp_s = ml + 2 * MIX_HEADS;         // [3][MIX_HEADS]: penalty factor, its rate, sink; then the waves' square sums of q and k
+  T* kn_s = (T*)(hp_s + 5 * MIX_HEADS);     // [CLS], [CLS]: the new token's row as the cache holds it
   T* vn_s = kn_s + CLS;
   float* g_s = (float*)(vn_s + CLS);        // [MIX_HEADS][V]: gates
   float* q_s = g_s + MIX_HEADS * g.V;       // [MIX_HEADS][D]
   float* p_s = q_s + MIX_HEADS * g.D;       // [MIX_HEADS][MIX_KEYS]
   float* o_s = p_s + MIX_HEADS * MIX_KEYS;  // [4 waves][MIX_HEADS][V]
   // what does not depend on the position: on its way together with it
-  for (int i = tid; i < nh * g.D; i += 256) q_s[i] = pr[g.cq + h0 * g.D + i] * g.scale;
-  for (int i = tid; i < nh * g.V; i += 256) g_s[i] = pr[g.cg + h0 * g.V + i] * g.out_scale;
-  if (tid < g.D) kn_s[tid] = kv_from<T>(pr[g.ck + kvh * g.D + tid]);
-  if (tid < g.V) vn_s[tid] = kv_from<T>(pr[g.cv + kvh * g.V + tid]);
+  float q_f = g.scale, k_f = 1.f;
+  if (g.q_norm) {  // (the same for the whole workgroup)
+    float sq2 = 0.f, sk2 = 0.f;
+    for (int i = tid; i < g.H * g.D; i += 256) sq2 = __builtin_fmaf(pr[g.cq + i], pr[g.cq + i], sq2);
+    for (int i = tid; i < g.G * g.D; i += 256) sk2 = __builtin_fmaf(pr[g.ck + i], pr[g.ck + i], sk2);
+    sq2 = wave_sum_f32(sq2);
+    sk2 = wave_sum_f32(sk2);
+    float* red = hp_s + 3 * MIX_HEADS;
+    if (lane == 0) {
+      red[wave] = sq2;
+      red[4 + wave] = sk2;
+    }
+    __syncthreads();
+    q_f *= 1.0f / sqrtf(((red[0] + red[1]) + (red[2] + red[3])) / (float)g.q_mean + g.eps);
+    k_f = 1.0f / sqrtf(((red[4] + red[5]) + (red[6] + red[7])) / (float)g.k_mean + g.eps);
+  }
+  for (int i = tid; i < nh * g.D; i += 256) q_s[i] = pr[g.cq + h0 * g.D + i] * (g.q_norm ? q_f * g.q_norm[h0 * g.D + i] : q_f);
+  for (int i = tid; i < nh * g.V; i += 256)
+    g_s[i] = (g.gate == GATE_ELEMENT ? pr[g.cg + h0 * g.V + i] : g.gate == GATE_HEAD ? pr[g.cg + h0 + i / g.V] : 1.f) * g.out_scale;
+  if (tid < g.D) kn_s[tid] = kv_from<T>(pr[g.ck + kvh * g.D + tid] * (g.k_norm ? k_f * g.k_norm[kvh * g.D + tid] : 1.f));
+  float v_raw = 0.f;
+  if (tid < g.V) {
+    v_raw = pr[g.cv + kvh * g.V + tid];
+    float v = v_raw;
+    if (g.vmix == VMIX_MIX) {
+      const float la = *g.lambda;
+      v = __builtin_fmaf(la, a.v_kept[(size_t)b * a.ld_vk + kvh * g.V + tid], (1.0f - la) * v);
+    }
+    vn_s[tid] = kv_from<T>(v);
+  }
   if (tid < nh) {
     hp_s[tid] = g.amp ? g.amp[h0 + tid] : 0.f;
     hp_s[MIX_HEADS + tid] = g.amp ? g.rate[h0 + tid] : 0.f;
     hp_s[2 * MIX_HEADS + tid] = g.sink ? g.sink[h0 + tid] : -INFINITY;
   }
-  const int in_chunk = sq.pos % g.chunk, n_rows = in_chunk + 1;  // this chunk's rows, the new one included
+  // the new token's row, and the rows it sees: its chunk's up to itself, or the whole ring once the window has gone round
+  const int in_chunk = sq.pos % g.span, n_rows = g.window && sq.pos >= g.span ? g.span : in_chunk + 1;
   const int r0 = split * MIX_KEYS;
   if (r0 >= n_rows) return;  // (whole workgroup)
   const int active = (n_rows + MIX_KEYS - 1) / MIX_KEYS;
   const int nk = n_rows - r0 < MIX_KEYS ? n_rows - r0 : MIX_KEYS;
   T* kc = (T*)(sq.slab + a.rs.k) + (size_t)kvh * g.rows * g.D;
   T* vc = (T*)(sq.slab + a.rs.v) + (size_t)kvh * g.rows * g.V;
-  const bool own_new = in_chunk < r0 + MIX_KEYS;
+  const bool own_new = in_chunk >= r0 && in_chunk < r0 + MIX_KEYS;
   const int key = tid >> 2, part = tid & 3, vcol = tid % CP * 8, vgrp = tid / CP;
   Oct<T> kr[NU], vr[NV];
 #pragma unroll
@@ -109,6 +147,7 @@ __device__ __forceinline__ void mix_attention(const MixStep& a, int blk, float* 
     if (hb == 0) {
       if (tid < g.D) kc[(size_t)in_chunk * g.D + tid] = kn_s[tid];
       if (tid < g.V) vc[(size_t)in_chunk * g.V + tid] = vn_s[tid];
+      if (g.vmix == VMIX_KEEP && tid < g.V) a.v_kept[(size_t)b * a.ld_vk + kvh * g.V + tid] = v_raw;
     }
     if (r0 + key == in_chunk) {
 #pragma unroll
@@ -120,7 +159,8 @@ __device__ __forceinline__ void mix_attention(const MixStep& a, int blk, float* 
       if (r0 + vgrp + u * GR == in_chunk && vcol < g.V) vr[u] = oct_load(vn_s + vcol);
   }
   {
-    const float dist = (float)(in_chunk - (r0 + key));
+    const int behind = in_chunk - (r0 + key);
+    const float dist = (float)(g.window && behind < 0 ? behind + g.span : behind);
     float kk[NU][8];
 #pragma unroll
     for (int u = 0; u < NU; u++) oct_floats(kr[u], kk[u]);
@@ -300,7 +340,7 @@ __global__ __launch_bounds__(256) void k_mix_step(const MixStep a) {
 }
 template <typename T, int CLS>
 inline void launch_mix_step_t(hipStream_t st, crabml_hip_device::ProfRec* rec, const MixStep& a) {
-  const size_t at = a.at.H ? 6 * MIX_HEADS + 2 * CLS * sizeof(T) / 4 + (size_t)MIX_HEADS * (a.at.D + MIX_KEYS + 5 * a.at.V) : 0;
+  const size_t at = a.at.H ? 7 * MIX_HEADS + 2 * CLS * sizeof(T) / 4 + (size_t)MIX_HEADS * (a.at.D + MIX_KEYS + 5 * a.at.V) : 0;
   const size_t li = a.li.H ? (size_t)(2 * a.li.D + 32 * 36) : 0;
   const unsigned grid = (unsigned)(a.B * ((a.at.H ? a.at.G * a.head_blocks * a.splits : 0) + a.li.H * a.li.slices));
   launch_k(st, rec, k_mix_step<T, CLS>, dim3(grid), dim3(256), (at > li ? at : li) * sizeof(float), a);  // (at most 57 KiB)

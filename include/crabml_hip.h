@@ -277,14 +277,24 @@ int crabml_hip_llama_decode_greedy(crabml_hip_llama_t* ctx, size_t token, size_t
 int crabml_hip_llama_prefill(crabml_hip_llama_t* ctx, const uint32_t* tokens, size_t n, float* logits);
 size_t crabml_hip_llama_kv_len(const crabml_hip_llama_t* ctx);
 int crabml_hip_llama_reset(crabml_hip_llama_t* ctx); /* empties the KV caches */
-/* ---- hybrid decoder: layers that mix softmax attention inside chunks with decaying linear attention ---------------------------
+/* ---- hybrid decoder: layers described by what they contain ---------------------------------------------------------------------
  * A second step function beside the llama one, for models whose layers are described by what they contain instead of by one fixed
- * op sequence (the Nilivik design).  bfloat16 weights; norms are RMS norms with a single gain; per layer
- *   x += attn_out_scale * attention(norm1 x) + lin_out_scale * linear(norm1 x);  x += ff_down xielu(ff_up norm2 x)
+ * op sequence (the Nilivik and Bifazen designs).  bfloat16 weights; RMS norms with a single gain or one per element; per layer
+ *   x += attn_out_scale * attention(norm1 x) + lin_out_scale * linear(norm1 x);  x += ff(norm2 x)
  * where either branch and the feed-forward may be absent.
  *   attention  grouped queries, score = attn_score_scale q.k - bias_amp ln(1 + bias_rate distance), visible inside chunks of
- *              attn_chunk positions counted from the sequence's start, a sink logit per head in the softmax's denominator, the
- *              heads gated by sigmoid(attn_gate norm1 x) before attn_o
+ *              attn_chunk positions counted from the sequence's start or inside a sliding window of attn_window, a sink logit per
+ *              head in the softmax's denominator, the heads gated by sigmoid(attn_gate norm1 x), per element or per head, before
+ *              attn_o; biases; an RMS norm over all of a token's queries (keys) at once; values mixed with those of the first layer
+ *              that has attn_vmix: v <- (1 - attn_vmix) v + attn_vmix v_first
+ *   latent     attn_latent > 0: attn_latent_down gives a latent (RMS-normed, attn_latent_norm) and a key part of attn_rot elements
+ *              shared by all heads; per head the other attn_dim elements of the key are attn_key_up latent, the value attn_value_up
+ *              latent; queries are [attn_dim, attn_rot] per head; pairs (2 i, 2 i + 1) of the attn_rot elements of queries and keys
+ *              turn by position * attn_rot_base^(-2 i / attn_rot).  The cache holds latents and shared key parts only.
+ *   ff         ff_gate == NULL: ff_down xielu(ff_up h); else ff_down (gelu(ff_gate h) * (ff_up h)), the tanh form of gelu
+ *   streams    > 0: so many residual rows x_s, each the embedding at the start.  A sublayer with in, out, mix (hc1: mixer, hc2:
+ *              feed-forward) reads sum_s in[s] x_s and turns them into x_t = sum_s mix[s][t] x_s + out[t] y; the final norm reads
+ *              their sum
  *   linear     q, k, v through silu; S <- decay S + k v^T, o = S^T q per head; the heads RMS-normed together (lin_norm), gated by
  *              sigmoid(lin_gate norm1 x) before lin_o
  * Layers [loop_start, loop_stop) run loop_times times in a row (own state each time); before every pass loop_step[t] is added to x,
@@ -295,7 +305,9 @@ int crabml_hip_llama_reset(crabml_hip_llama_t* ctx); /* empties the KV caches */
  * compute = CRABML_HIP_BF16: matrix products of bf16 activations with f32 accumulation, bf16 cache (norms, scores, softmax, the
  * linear states and the residual are f32 all the same); CRABML_HIP_F32: every activation, product and cache entry f32. */
 typedef struct crabml_hip_hybrid crabml_hip_hybrid_t;
-#define CRABML_HIP_HYBRID_NO_GRAPH 1 /* launch decode steps eagerly */
+#define CRABML_HIP_HYBRID_NO_GRAPH 1      /* launch decode steps eagerly */
+#define CRABML_HIP_HYBRID_NORM_VECTOR 2   /* norm1, norm2, final_norm: a gain per element (width numbers); else one number */
+#define CRABML_HIP_HYBRID_NORM_ONE_PLUS 4 /* ... stored around zero: the gain is 1 + the stored number */
 typedef struct crabml_hip_hybrid_config {
   size_t width, vocab_size, n_layers;
   size_t loop_start, loop_stop, loop_times; /* loop_times == 0: no loop */
@@ -305,6 +317,8 @@ typedef struct crabml_hip_hybrid_config {
   float logit_softcap; /* 0 = none */
   uint32_t compute;    /* CRABML_HIP_BF16 or CRABML_HIP_F32 */
   int32_t flags;
+  size_t streams;       /* residual streams, at most 8; 0 = a plain residual sum */
+  double position_base; /* sin / cos of the position added to the embedding, frequencies falling with this base; 0 = none */
 } crabml_hip_hybrid_config_t;
 typedef struct crabml_hip_hybrid_layer { /* heads == 0: the branch is absent; ff == 0: no feed-forward */
   size_t attn_heads, attn_kv_heads, attn_dim, attn_vdim;
@@ -317,7 +331,7 @@ typedef struct crabml_hip_hybrid_layer { /* heads == 0: the branch is absent; ff
   const crabml_hip_buf_t* attn_q;
   const crabml_hip_buf_t* attn_k;
   const crabml_hip_buf_t* attn_v;
-  const crabml_hip_buf_t* attn_gate;
+  const crabml_hip_buf_t* attn_gate; /* attn_heads * attn_vdim rows, or attn_heads; NULL = none */
   const crabml_hip_buf_t* attn_o;
   const crabml_hip_buf_t* attn_bias_amp;  /* attn_heads; NULL (both) = no distance bias */
   const crabml_hip_buf_t* attn_bias_rate;
@@ -332,12 +346,34 @@ typedef struct crabml_hip_hybrid_layer { /* heads == 0: the branch is absent; ff
   const crabml_hip_buf_t* ff_up;
   const crabml_hip_buf_t* ff_down;
   const crabml_hip_buf_t* ff_act; /* 2: the raw numbers of xIELU, before their softplus */
+  size_t attn_window;             /* 0 = none */
+  size_t attn_latent;             /* > 0: latent attention (attn_kv_heads, attn_k, attn_v unused) */
+  size_t attn_rot;
+  double attn_rot_base;
+  const crabml_hip_buf_t* attn_q_bias; /* NULL = none, as are all below */
+  const crabml_hip_buf_t* attn_k_bias;
+  const crabml_hip_buf_t* attn_v_bias;
+  const crabml_hip_buf_t* attn_o_bias;
+  const crabml_hip_buf_t* attn_q_norm; /* attn_heads * attn_dim (both norms or none) */
+  const crabml_hip_buf_t* attn_k_norm; /* attn_kv_heads * attn_dim */
+  const crabml_hip_buf_t* attn_vmix;   /* 1 */
+  const crabml_hip_buf_t* attn_latent_down; /* (attn_latent + attn_rot, width) */
+  const crabml_hip_buf_t* attn_latent_norm; /* attn_latent */
+  const crabml_hip_buf_t* attn_key_up;      /* (attn_heads * attn_dim, attn_latent) */
+  const crabml_hip_buf_t* attn_value_up;    /* (attn_heads * attn_vdim, attn_latent) */
+  const crabml_hip_buf_t* ff_gate;          /* (ff, width) */
+  const crabml_hip_buf_t* hc1_in;           /* streams > 0: streams numbers; mix is [from][to] */
+  const crabml_hip_buf_t* hc1_out;
+  const crabml_hip_buf_t* hc1_mix;
+  const crabml_hip_buf_t* hc2_in;
+  const crabml_hip_buf_t* hc2_out;
+  const crabml_hip_buf_t* hc2_mix;
 } crabml_hip_hybrid_layer_t;
 typedef struct crabml_hip_hybrid_weights {
   const crabml_hip_buf_t* embed;      /* (vocab_size, width) */
   const crabml_hip_buf_t* loop_step;  /* (loop_times, width) */
   const crabml_hip_buf_t* final_norm; /* 1 */
-  const crabml_hip_buf_t* head;       /* (vocab_size, width) */
+  const crabml_hip_buf_t* head;       /* (vocab_size, width); NULL = embed */
 } crabml_hip_hybrid_weights_t;
 /* Matrices are copied into the layout the kernels read (branches' projections as one matrix, head widths padded): the caller may
  * release its buffers afterwards. */

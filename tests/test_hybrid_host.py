@@ -119,7 +119,7 @@ def changed(*path, value):
 
 
 def test_registry_knows_both_kinds_of_models(ca, tmp_path):
-    assert {"Nilivik", "llama"} <= set(ca.known_architectures())
+    assert {"Nilivik", "Bifazen", "llama"} <= set(ca.known_architectures())
     assert ca.model_architecture(write(tmp_path / "m")) == "Nilivik"
     assert ca.model_architecture(os.path.join(ROOT, "tests", "golden", "tinyllamas-stories-260k-f32.gguf")) == "llama"
     with pytest.raises(ca.CrabmlError):
