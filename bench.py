@@ -64,6 +64,8 @@ HYBRID_SIZES = {
     "2k": dict(width=2048, heads=16, kv_heads=4, dim=128, lin_heads=16, lin_dim=64, lin_vdim=128, ff=8192, vocab=32000, layers=8),
     "4k": dict(width=4096, heads=32, kv_heads=8, dim=128, lin_heads=16, lin_dim=128, lin_vdim=128, ff=14336, vocab=128256, layers=4),
 }
+# --bifazen: the same widths, heads, feed-forward and vocabulary
+BIFAZEN_SIZES = {k: dict(z, rank=512, rot=64, window=1024, streams=4) for k, z in HYBRID_SIZES.items()}
 MFMA_PEAK_TFLOPS = 2500.0  # dense bf16 / f16
 
 
@@ -116,6 +118,9 @@ def parse():
     ap.add_argument("--hybrid", nargs="?", const="all", default=None, choices=["all"] + sorted(HYBRID_SIZES),
                     help="instead of the BASELINE workload: prompt and decode throughput and per-kernel roofline fractions of the hybrid "
                          "decoder (Nilivik design, random weights) at layer sizes of real models, beside a llama of the same widths")
+    ap.add_argument("--bifazen", nargs="?", const="all", default=None, choices=["all"] + sorted(BIFAZEN_SIZES),
+                    help="instead of the BASELINE workload: prompt and decode throughput and per-kernel roofline fractions of the Bifazen design "
+                         "(random weights) beside the Nilivik design of the same widths, both on the hybrid decoder")
     ap.add_argument("--selftest-dist", action="store_true", help="CPU/gloo self test of the rank aggregation")
     return ap.parse_args()
 
@@ -596,6 +601,140 @@ def hybrid_bench(args, ca, synth, local):
                       "decode_position": ctx, "steps": args.steps, "sizes": result}))
 
 
+def decoder_points(args, dev, r, V, ctx, prompt):
+    """prompt and decode times of a runner on the hybrid decoder, and its kernels' times by profiling stage"""
+    toks = [int(t) for t in (7 * np_arange(prompt + 1) + 3) % V]
+
+    def timed(fn, reps=4):
+        best = 1e9
+        for _ in range(reps):
+            dev.sync()
+            t0 = time.perf_counter()
+            fn()
+            dev.sync()
+            best = min(best, time.perf_counter() - t0)
+        return best
+
+    def prefill(n_seq, n):
+        seqs = [r.open() for _ in range(n_seq)]
+        r.step([(s, toks[:n], [n - 1] if s == seqs[-1] else []) for s in seqs])
+        for s in seqs:
+            r.close(s)
+
+    out = {"prompt": {}, "decode": {}, "kernels": {}}
+    for n_seq, n in ((1, 512), (1, prompt), (4, 512)):
+        prefill(n_seq, n)
+        t = timed(lambda: prefill(n_seq, n))
+        out["prompt"]["%dx%d" % (n_seq, n)] = {"ms": round(t * 1e3, 3), "tokens_per_s": round(n_seq * n / t)}
+    for B in (1, 4, 8, 16):
+        seqs = [r.open() for _ in range(B)]
+        for s in seqs:
+            r.step([(s, toks[:ctx], [])])
+        r.decode_batch(seqs, [1] * B, 4)
+        t = timed(lambda: r.decode_batch(seqs, [1] * B, args.steps)) / args.steps
+        out["decode"]["b%d" % B] = {"us_per_step": round(t * 1e6, 1), "tokens_per_s": round(B / t, 1)}
+        for s in seqs:
+            r.close(s)
+    names = {1: "in", 2: "mix", 3: "out", 4: "up", 5: "down", 6: "head", 7: "linear", 8: "rows", 9: "latent"}
+    dev.prof_enable(True)
+    for B in (1, 16):
+        seqs = [r.open() for _ in range(B)]
+        for s in seqs:
+            r.step([(s, toks[:ctx], [])])
+        dev.prof_read()
+        r.decode_batch(seqs, [1] * B, 8)
+        for x in dev.prof_read():
+            out["kernels"]["decode_b%d_%s" % (B, names[x["stage"] % 10])] = {"us": round(x["kernel_ms"] * 1e3 / x["launches"], 2)}
+        for s in seqs:
+            r.close(s)
+    s = r.open()
+    r.step([(s, toks[:prompt], [])])
+    for x in dev.prof_read():
+        out["kernels"]["prompt_" + names[x["stage"] % 10]] = {"us": round(x["kernel_ms"] * 1e3 / x["launches"], 2), "launches": x["launches"]}
+    r.close(s)
+    dev.prof_enable(False)
+    return out
+
+
+def bifazen_bench(args, ca, local):
+    """The Bifazen design at BIFAZEN_SIZES beside the Nilivik design of the same widths.  Throughput on a model that alternates the two kinds
+    of layers; kernels on models of one kind each.  A kernel's roofline is the longer of its flops at the matrix cores' bf16 peak and its
+    bytes (weights, activations, residual streams, cached rows) at the HBM peak."""
+    import shutil
+    import tempfile
+
+    from crabml_amd import synth_bifazen as sb
+    from crabml_amd import synth_hybrid as sh
+
+    dev = ca.HipTensorDevice(device_ordinal=local)
+    ctx, prompt = 1024, 2048
+
+    def load(conf, tensors):
+        folder = tempfile.mkdtemp(prefix="bifazen-")
+        try:
+            sh.write_model(conf, tensors(conf, 8, pool=1 << 22), folder)
+            return ca.load_model(folder, dev, seq_len=4096)
+        finally:
+            shutil.rmtree(folder)
+
+    result = {}
+    for size in sorted(BIFAZEN_SIZES) if args.bifazen == "all" else [args.bifazen]:
+        z = BIFAZEN_SIZES[size]
+        W, V, L, ff, H, G, D, R, rot, win, S = (z[k] for k in ("width", "vocab", "layers", "ff", "heads", "kv_heads", "dim", "rank", "rot", "window", "streams"))
+        lat, att = sb.latent(H, D, rot, D, R, win, ff), sb.attention(H, G, D, D, win, ff)
+        nil = sh.layer(H, G, D, D, 2 * win, z["lin_heads"], z["lin_dim"], z["lin_vdim"], ff)
+        pairs_win = win * win / 2 + (prompt - win) * win  # (query, key) pairs of the prompt
+        pairs_chunk = prompt * prompt / 2
+        ns = z["lin_heads"] * z["lin_vdim"]
+        models = {
+            "bifazen": (sb.config(W, V, [lat, att] * (L // 2), S), sb.random_tensors, None),
+            "bifazen_latent": (sb.config(W, V, [lat] * L, S), sb.random_tensors,
+                               dict(n_in=H * (D + rot) + R + rot, k_o=H * D, up=2 * ff, S=S, pairs=pairs_win, width=2 * D + rot, cache=2 * win * (R + rot), lat=(R, 2 * H * D))),
+            "bifazen_attention": (sb.config(W, V, [att] * L, S), sb.random_tensors,
+                                  dict(n_in=D * (H + 2 * G) + H, k_o=H * D, up=2 * ff, S=S, pairs=pairs_win, width=2 * D, cache=2 * win * 2 * G * D, lat=None)),
+            "nilivik": (sh.config(W, V, [nil] * L), sh.random_tensors,
+                        dict(n_in=D * 2 * (H + G) + 2 * z["lin_heads"] * (z["lin_dim"] + z["lin_vdim"]), k_o=H * D + ns, up=ff, S=1, pairs=pairs_chunk, width=2 * D,
+                             cache=2 * ctx * 2 * G * D + 8 * ns * z["lin_dim"], lat=None)),
+        }
+        out = {}
+        for name, (conf, tensors, k) in models.items():
+            r = load(conf, tensors)
+            o = decoder_points(args, dev, r, V, ctx, prompt)
+            del r
+            print("# %s %s done" % (name, size), file=sys.stderr, flush=True)
+            if k is None:
+                del o["kernels"]
+            else:
+                n_up = k["up"]
+                u_out = ff  # width of the hidden row
+                weights = {"in": k["n_in"] * W, "out": W * k["k_o"], "up": n_up * W, "down": ff * W, "head": V * W}
+                for key, v in o["kernels"].items():
+                    leg, stage = key.rsplit("_", 1)
+                    M = prompt if leg == "prompt" else int(leg[8:])
+                    flops = byts = 0.0
+                    if stage in weights:
+                        rows = 1 if stage == "head" and leg == "prompt" else M
+                        flops = 2.0 * rows * weights[stage]
+                        act = {"in": W + k["n_in"], "out": k["k_o"] + W, "up": W + u_out, "down": u_out + W, "head": W + V}[stage]
+                        byts = 2.0 * weights[stage] + rows * 2.0 * act + (8.0 * k["S"] * W * rows if stage in ("out", "down") else 0)
+                    elif stage == "mix" and leg == "prompt":
+                        flops = 2.0 * k["pairs"] * k["width"] * H
+                    elif stage == "mix":
+                        byts = float(k["cache"]) * M
+                    elif stage == "latent" and leg == "prompt":
+                        flops = 2.0 * M * k["lat"][0] * k["lat"][1]
+                        byts = 2.0 * (k["lat"][0] * k["lat"][1] + M * (k["lat"][0] + k["lat"][1]))
+                    elif stage in ("latent", "rows") and k["lat"] and leg != "prompt":
+                        byts = 2.0 * R * D * H
+                    if flops or byts:
+                        roof = max(flops / MFMA_PEAK_TFLOPS / 1e6, byts / HBM_PEAK_GBS / 1e3)
+                        v["frac_of_roofline"] = round(roof / v["us"], 3)
+            out[name] = o
+        result[size] = out
+    print(json.dumps({"metric": "Bifazen design throughput (not the BASELINE workload)", "dtype": "bf16", "data": "synthetic", "decode_position": ctx,
+                      "steps": args.steps, "sizes": result}))
+
+
 def np_arange(n):
     import numpy as np
 
@@ -766,6 +905,8 @@ def main():
         return tp_dry_run(args, ca, synth, local)
     if args.hybrid:
         return hybrid_bench(args, ca, synth, local)
+    if args.bifazen:
+        return bifazen_bench(args, ca, local)
     if args.tp and world > 1:
         rc = tp_group_run(args, ca, synth, dist, rank, world, local)
         if rc:

@@ -116,4 +116,4 @@ def test_wrong_configurations_are_named(tmp_path, path, value, says):
 def test_wrong_tensor_files_are_named(tmp_path):
     for name in ("l0.hc1.mix", "l0.mix.dkv.norm", "l1.mix.q.b", "l2.mix.vmix", "final.norm"):
         assert "failed to find tensor " + name in load_error(write(tmp_path / name, edit=lambda b: b.pop(name)))
-    assert "l1.mix.o" in load_error(write(tmp_path / "o", edit=lambda b: b.update({"l1.mix.o": b["l1.mix.o"].T.copy()})))
+    assert "l0.mix.o" in load_error(write(tmp_path / "o", edit=lambda b: b.update({"l0.mix.o": b["l0.mix.o"].T.copy()})))
