@@ -24,7 +24,8 @@ __device__ __forceinline__ void landed_barrier() {
   asm volatile("s_waitcnt vmcnt(%0) lgkmcnt(0)\n\ts_barrier" ::"n"(N) : "memory");
 }
 
-template <int BM, int BN, int WGM, int WGN, int ST, int P, int OUT>
+// (NS: GEMM_OUT_STREAMS with up to that many streams)
+template <int BM, int BN, int WGM, int WGN, int ST, int P, int OUT, int NS>
 __global__ __launch_bounds__(64 * WGM * WGN) void k_gemm_bf16(const GemmBf16 g, int S, float* __restrict__ ws, unsigned* __restrict__ tick) {
   constexpr int WM = BM / WGM, WN = BN / WGN, TM = WM / 16, TN = WN / 16;
   constexpr int HR = BM < 64 ? BM : 64, LC = BN + 4;  // the epilogue's slab of rows in LDS
@@ -150,6 +151,96 @@ __global__ __launch_bounds__(64 * WGM * WGN) void k_gemm_bf16(const GemmBf16 g, 
   if constexpr (OUT == GEMM_OUT_XIELU) {
     xr = g.xielu[0];
     xl = g.xielu[1];
+  }
+  if constexpr (OUT == GEMM_OUT_STREAMS && NS == 4) {
+    // Up to four streams: a slab's rows of all of them are requested, two units of eight columns at a time, before the accumulators take
+    // their way through LDS, so that a thread has sixteen requests out.
+    constexpr int UNITS = HR * BN / 8 / NT, UG = 2;
+    static_assert(UNITS % UG == 0, "units come in pairs");
+    typedef const float __attribute__((address_space(4))) constant;
+    constant *coef = (constant*)(size_t)g.sm.coef, *inw = (constant*)(size_t)g.sm.in;
+#pragma unroll 1
+    for (int h = 0; h < BM / HR; h++) {
+#pragma unroll
+      for (int u0 = 0; u0 < UNITS; u0 += UG) {
+        f32x4 old[UG][2][4];
+        float* xs[UG];
+        int row[UG], col[UG], lr[UG];
+        bool in[UG];
+#pragma unroll
+        for (int u = 0; u < UG; u++) {
+          const int unit = (u0 + u) * NT + tid, r = unit / (BN / 8), c = unit % (BN / 8) * 8;
+          row[u] = row0 + h * HR + r;
+          col[u] = col0 + c;
+          lr[u] = r * LC + c;
+          in[u] = row[u] < g.M && col[u] < g.N;
+          xs[u] = g.x + (size_t)row[u] * g.ldx + col[u];
+          if (in[u]) {
+#pragma unroll
+            for (int s = 0; s < 4; s++) {
+              const float* p = xs[u] + (s < g.sm.n ? s : 0) * g.sm.stride;
+              old[u][0][s] = *(const f32x4*)p;
+              old[u][1][s] = *(const f32x4*)(p + 4);
+            }
+          }
+        }
+        if (u0 == 0) {  // (LDS hand-overs that leave the requests out)
+          asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
+          if (h == 0 && tid < BM) lf[tid] = factor;
+          if (wm * WM / HR == h) {
+#pragma unroll
+            for (int i = 0; i < TM; i++)
+#pragma unroll
+              for (int j = 0; j < TN; j++)
+#pragma unroll
+                for (int e = 0; e < 4; e++) lc[(wm * WM % HR + i * 16 + fk * 4 + e) * LC + wn * WN + j * 16 + fr] = acc[i][j][e];
+          }
+          asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
+        }
+#pragma unroll
+        for (int u = 0; u < UG; u++) {
+          float sq = 0.f;
+          if (in[u]) {
+            const float f = lf[h * HR + lr[u] / LC];
+            f32x4 y[2], n[2] = {f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}};
+#pragma unroll
+            for (int k = 0; k < 2; k++) {
+              y[k] = *(const f32x4*)(lc + lr[u] + 4 * k) * f;
+              if (g.bias) y[k] += *(const f32x4*)(g.bias + col[u] + 4 * k);
+            }
+#pragma unroll
+            for (int t = 0; t < 4; t++)
+              if (t < g.sm.n) {
+                constant* c = coef + t * HC_ROW;
+#pragma unroll
+                for (int k = 0; k < 2; k++) {
+                  f32x4 v = c[HC_MAX] * y[k];
+#pragma unroll
+                  for (int s = 0; s < 4; s++) v += c[s] * old[u][k][s];
+                  *(f32x4*)(xs[u] + t * g.sm.stride + 4 * k) = v;
+                  n[k] += inw[t] * v;
+                }
+              }
+            float v[8];
+#pragma unroll
+            for (int k = 0; k < 2; k++) {
+              const f32x4 gain = *(const f32x4*)(g.gain_next + col[u] + 4 * k);
+#pragma unroll
+              for (int e = 0; e < 4; e++) {
+                sq = __builtin_fmaf(n[k][e], n[k][e], sq);
+                v[4 * k + e] = n[k][e] * gain[e];
+              }
+            }
+            split_store8<P>(v, g.planes + (size_t)row[u] * g.ldp + col[u], g.p_plane);
+          }
+          sq += dpp_f<0xB1>(sq);  // eight lanes hold a row's 64 columns
+          sq += dpp_f<0x4E>(sq);
+          sq += dpp_f<0x141>(sq);
+          if (in[u] && (tid & 7) == 0) g.sq_out[(size_t)row[u] * g.n_sq_out + col[u] / 64] = sq;
+        }
+      }
+    }
+    return;
   }
   for (int h = 0; h < BM / HR; h++) {
     __syncthreads();
@@ -341,18 +432,18 @@ static GemmPlan plan(const GemmBf16& g, int planes, int n_cu, size_t ws_floats) 
   return best;
 }
 
-template <int P, int OUT>
+template <int P, int OUT, int NS = 0>
 static void launch_t(hipStream_t st, crabml_hip_device::ProfRec* rec, const GemmBf16& g, int n_cu, const GemmScratch& w) {
   const GemmPlan p = plan(g, P, n_cu, w.floats);
   const dim3 grid(((g.M + p.bm - 1) / p.bm) * ((g.N + 127) / 128) * p.S);
   if (p.bm == 256)
-    launch_k(st, rec, k_gemm_bf16<256, 128, 4, 2, 3, P, OUT>, grid, dim3(512), 0, g, p.S, w.partials, w.ticks);
+    launch_k(st, rec, k_gemm_bf16<256, 128, 4, 2, 3, P, OUT, NS>, grid, dim3(512), 0, g, p.S, w.partials, w.ticks);
   else if (p.bm == 128)
-    launch_k(st, rec, k_gemm_bf16<128, 128, 2, 2, 4, P, OUT>, grid, dim3(256), 0, g, p.S, w.partials, w.ticks);
+    launch_k(st, rec, k_gemm_bf16<128, 128, 2, 2, 4, P, OUT, NS>, grid, dim3(256), 0, g, p.S, w.partials, w.ticks);
   else if (p.bm == 64)
-    launch_k(st, rec, k_gemm_bf16<64, 128, 2, 2, 3, P, OUT>, grid, dim3(256), 0, g, p.S, w.partials, w.ticks);
+    launch_k(st, rec, k_gemm_bf16<64, 128, 2, 2, 3, P, OUT, NS>, grid, dim3(256), 0, g, p.S, w.partials, w.ticks);
   else
-    launch_k(st, rec, k_gemm_bf16<32, 128, 2, 2, 4, P, OUT>, grid, dim3(256), 0, g, p.S, w.partials, w.ticks);
+    launch_k(st, rec, k_gemm_bf16<32, 128, 2, 2, 4, P, OUT, NS>, grid, dim3(256), 0, g, p.S, w.partials, w.ticks);
 }
 
 void launch_gemm_bf16(crabml_hip_device* dev, crabml_hip_device::ProfRec* rec, int planes, int out, const GemmBf16& g, const GemmScratch& w) {
@@ -363,7 +454,12 @@ void launch_gemm_bf16(crabml_hip_device* dev, crabml_hip_device::ProfRec* rec, i
       case GEMM_OUT_ACT_BF16: launch_t<1, GEMM_OUT_ACT_BF16>(st, rec, g, n, w); break;
       case GEMM_OUT_RESIDUAL: launch_t<1, GEMM_OUT_RESIDUAL>(st, rec, g, n, w); break;
       case GEMM_OUT_XIELU: launch_t<1, GEMM_OUT_XIELU>(st, rec, g, n, w); break;
-      case GEMM_OUT_STREAMS: launch_t<1, GEMM_OUT_STREAMS>(st, rec, g, n, w); break;
+      case GEMM_OUT_STREAMS:
+        if (g.sm.n <= 4)
+          launch_t<1, GEMM_OUT_STREAMS, 4>(st, rec, g, n, w);
+        else
+          launch_t<1, GEMM_OUT_STREAMS, HC_MAX>(st, rec, g, n, w);
+        break;
       case GEMM_OUT_GLU: launch_t<1, GEMM_OUT_GLU>(st, rec, g, n, w); break;
       default: launch_t<1, GEMM_OUT_SOFTCAP>(st, rec, g, n, w); break;
     }
@@ -372,7 +468,12 @@ void launch_gemm_bf16(crabml_hip_device* dev, crabml_hip_device::ProfRec* rec, i
       case GEMM_OUT_ACT_F32: launch_t<3, GEMM_OUT_ACT_F32>(st, rec, g, n, w); break;
       case GEMM_OUT_RESIDUAL: launch_t<3, GEMM_OUT_RESIDUAL>(st, rec, g, n, w); break;
       case GEMM_OUT_XIELU: launch_t<3, GEMM_OUT_XIELU>(st, rec, g, n, w); break;
-      case GEMM_OUT_STREAMS: launch_t<3, GEMM_OUT_STREAMS>(st, rec, g, n, w); break;
+      case GEMM_OUT_STREAMS:
+        if (g.sm.n <= 4)
+          launch_t<3, GEMM_OUT_STREAMS, 4>(st, rec, g, n, w);
+        else
+          launch_t<3, GEMM_OUT_STREAMS, HC_MAX>(st, rec, g, n, w);
+        break;
       case GEMM_OUT_GLU: launch_t<3, GEMM_OUT_GLU>(st, rec, g, n, w); break;
       default: launch_t<3, GEMM_OUT_SOFTCAP>(st, rec, g, n, w); break;
     }

@@ -309,7 +309,7 @@ int build_layer(Ctx* c, const crabml_hip_hybrid_layer_t& s, Layer& L) {
     CH_TRY(alloc_matrix(c, H * (dimp + V), (size_t)la.ldl, &wkv));
     CH_TRY(pack_matrix(c, s.attn_key_up, "attn_key_up", H * s.attn_dim, rank, wkv, (size_t)la.ldl, 0, s.attn_dim, dimp));
     CH_TRY(pack_matrix(c, s.attn_value_up, "attn_value_up", H * s.attn_vdim, rank, wkv, (size_t)la.ldl, H * dimp, s.attn_vdim, V));
-    CH_TRY(dalloc_n(c, H * rankp * dimp, &wq));
+    CH_TRY(dalloc_n(c, H * rankp * dimp + 32, &wq));
     k_pack_transposed<<<dim3((unsigned)((rank + 255) / 256), (unsigned)s.attn_dim, (unsigned)H), 256, 0, dev->stream>>>((const unsigned short*)s.attn_key_up->ptr, (int)s.attn_dim,
                                                                                                              (int)rank, wq, la.rank, la.dim);
     CH_HIP(dev, hipGetLastError());

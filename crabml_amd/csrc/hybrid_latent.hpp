@@ -125,7 +125,7 @@ __device__ __forceinline__ LatRange latent_range(const AttnGeom& g, int pos) {
 // grid: H * slices workgroups of one head's latent columns (all rows of the batch), then one per row for everything else
 template <typename T>
 __global__ __launch_bounds__(256) void k_latent_query(const LatStep a) {
-  extern __shared__ __attribute__((aligned(16))) float lat_lds[];  // [B][dim]; the last workgroups: cos, sin per pair
+  extern __shared__ __attribute__((aligned(16))) float lat_lds[];  // [16][ldq]; the last workgroups: cos, sin per pair
   __shared__ float red[4];
   const AttnGeom& g = a.at;
   const LatGeom& l = a.la;
@@ -166,36 +166,37 @@ __global__ __launch_bounds__(256) void k_latent_query(const LatStep a) {
   }
   const int h = blockIdx.x / slices, r0 = blockIdx.x % slices * LAT_SLICE;
   const int r1 = r0 + LAT_SLICE < l.rank ? r0 + LAT_SLICE : l.rank;
-  int lpr = 1;  // lanes per weight row
-  while (lpr * 8 < l.dim) lpr <<= 1;
-  const int rows = 64 / lpr, sub = lane / lpr, k = lane % lpr * 8;
-  const unsigned short* w = l.w_q + (size_t)h * l.rank * l.dim;
-  i32x4 first = {0, 0, 0, 0};  // (on its way while the queries are staged)
-  int r = r0 + wave * rows + sub;
-  if (r < r1 && k < l.dim) first = *(const i32x4*)(w + (size_t)r * l.dim + k);
-  for (int i = tid; i < a.B * l.dim; i += 256) lat_lds[i] = a.proj[(size_t)(i / l.dim) * a.ldp + g.cq + h * g.D + i % l.dim];
-  __syncthreads();
-  for (int n = 0; r0 + n < r1; n += 4 * rows) {  // (the same number of rounds for every wave: the exchange below wants whole waves)
-    r = r0 + n + wave * rows + sub;
-    const bool live = r < r1 && k < l.dim;
-    i32x4 v = first;
-    if (n > 0) {
-      v = i32x4{0, 0, 0, 0};
-      if (live) v = *(const i32x4*)(w + (size_t)r * l.dim + k);
-    }
-    for (int b = 0; b < a.B; b++) {
-      float s = 0.f;
-      if (live) {
-        const float* x = lat_lds + b * l.dim + k;
+  // a wave: 16 latent columns of every row of the batch.  (The last weight row's reads run past its end into zeros: dim is padded to 32
+  // here by zero queries, and the matrix has 32 elements to spare.)
+  const int k32 = (l.dim + 31) & ~31, ldq = k32 + 4, fr = lane & 15, fk = lane >> 4;
+  const int rr = r0 + wave * 16 + fr;
+  const unsigned short* w = l.w_q + ((size_t)h * l.rank + (rr < r1 ? rr : r1 - 1)) * l.dim + fk * 8;
+  bf16x8 wf[8];  // (dim is at most 256)
 #pragma unroll
-        for (int e = 0; e < 4; e++) {
-          s = __builtin_fmaf(__builtin_bit_cast(float, (unsigned)v[e] << 16), x[2 * e], s);
-          s = __builtin_fmaf(__builtin_bit_cast(float, (unsigned)v[e] & 0xffff0000u), x[2 * e + 1], s);
-        }
-      }
-      for (int o = 1; o < lpr; o <<= 1) s += __shfl_xor(s, o, 64);
-      if (k == 0 && r < r1) a.q[((size_t)b * g.H + h) * row_w + r] = s;
+  for (int i = 0; i < 8; i++)
+    if (i * 32 < l.dim) __builtin_memcpy(&wf[i], w + i * 32, 16);
+  for (int i = tid; i < 16 * (k32 / 4); i += 256) {
+    const int b = i / (k32 / 4), c = i % (k32 / 4) * 4;
+    f32x4 v = {0.f, 0.f, 0.f, 0.f};
+    if (b < a.B && c < l.dim) v = *(const f32x4*)(a.proj + (size_t)b * a.ldp + g.cq + h * g.D + c);
+    *(f32x4*)(lat_lds + b * ldq + c) = v;
+  }
+  __syncthreads();
+  if (r0 + wave * 16 >= r1) return;
+  f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int i = 0; i < 8; i++)
+    if (i * 32 < l.dim) {
+      float v[8];
+      read8(lat_lds + fr * ldq + i * 32 + fk * 8, v);
+      bf16x8 hi, mid, lo;
+      split3(v, hi, mid, lo);
+      acc = mfma_bf16(hi, wf[i], mfma_bf16(mid, wf[i], mfma_bf16(lo, wf[i], acc)));
     }
+  if (rr < r1) {
+#pragma unroll
+    for (int e = 0; e < 4; e++)
+      if (fk * 4 + e < a.B) a.q[((size_t)(fk * 4 + e) * g.H + h) * row_w + rr] = acc[e];
   }
 }
 
@@ -242,15 +243,63 @@ __global__ __launch_bounds__(256) void k_latent_attn(const LatStep a) {
   float* p_s = (float*)(k_s + KT * ld);  // [16][LP]
   const int nh = g.H - h0 < LAT_HEADS ? g.H - h0 : LAT_HEADS;
   const float* q = a.q + ((size_t)b * g.H + h0) * row_w;
-  for (int i = tid; i < LAT_HEADS * w32; i += 256) {
-    const int h = i / w32, c = i % w32;
-    q_s[h * ld + c] = kv_from<T>(h < nh && c < row_w ? q[(size_t)h * row_w + c] : 0.f);
-  }
   const StepSeq sq = a.seq[b];
   const LatRange rg = latent_range<T>(g, sq.pos);
   const int lo = split * rg.per, hi = lo + rg.per < rg.n ? lo + rg.per : rg.n;
   if (lo >= hi) return;  // (whole workgroup)
   const T* cache = (const T*)(sq.slab + a.rs.k);
+  // a tile's octets in row order, 256 at a time: thread t starts at (row tr0, octet tc0) and goes on by (dr, dc)
+  const int tr0 = tid / cpr, tc0 = tid % cpr, dr = 256 / cpr, dc = 256 % cpr;
+  constexpr int UN = sizeof(T) == 2 ? 9 : 5;  // octets in flight per thread
+  auto stage = [&](int t0, int n, int rows, const T* src, T* dst) {  // rows of LDS; those from n on are zero
+    int r = tr0, c = tc0;
+    while (true) {
+      Oct<T> v[UN];
+      int at[UN];
+#pragma unroll
+      for (int u = 0; u < UN; u++) {
+        at[u] = r < rows ? r * ld + c * 8 : -1;
+        v[u] = oct_zero<T>();
+        if (r < n && r < rows && c * 8 < row_w) v[u] = oct_load(src + (size_t)(t0 + r) * row_w + c * 8);
+        r += dr;
+        c += dc;
+        if (c >= cpr) {
+          c -= cpr;
+          r++;
+        }
+      }
+#pragma unroll
+      for (int u = 0; u < UN; u++)
+        if (at[u] >= 0) oct_store(dst + at[u], v[u]);
+      if (__all(r >= rows)) return;
+    }
+  };
+  {
+    constexpr int UQ = LAT_HEADS * LAT_MAX_ROW / 8 / 256;
+    int r = tr0, c = tc0, at[UQ];
+    float v[UQ][8];
+#pragma unroll
+    for (int u = 0; u < UQ; u++) {
+      at[u] = r < LAT_HEADS ? r * ld + c * 8 : -1;
+#pragma unroll
+      for (int e = 0; e < 8; e++) v[u][e] = 0.f;
+      if (r < nh && c * 8 < row_w) read8(q + (size_t)r * row_w + c * 8, v[u]);
+      r += dr;
+      c += dc;
+      if (c >= cpr) {
+        c -= cpr;
+        r++;
+      }
+    }
+#pragma unroll
+    for (int u = 0; u < UQ; u++)
+      if (at[u] >= 0) {
+        T t[8];
+#pragma unroll
+        for (int e = 0; e < 8; e++) t[e] = kv_from<T>(v[u][e]);
+        __builtin_memcpy(q_s + at[u], t, sizeof t);
+      }
+  }
   f32x4 o[NT];
 #pragma unroll
   for (int j = 0; j < NT; j++) o[j] = f32x4{0.f, 0.f, 0.f, 0.f};
@@ -262,10 +311,7 @@ __global__ __launch_bounds__(256) void k_latent_attn(const LatStep a) {
   }
   for (int t0 = lo; t0 < hi; t0 += KT) {
     __syncthreads();  // the previous tile has been read
-    for (int i = tid; i < KT * cpr; i += 256) {
-      const int r = i / cpr, c = i % cpr * 8;
-      oct_store(k_s + r * ld + c, t0 + r < hi && c < row_w ? oct_load(cache + (size_t)(t0 + r) * row_w + c) : oct_zero<T>());
-    }
+    stage(t0, hi - t0, KT, cache, k_s);
     __syncthreads();
     if (wave < KT / 16) {
       const f32x4 s = mma_rows(q_s + fr * ld, k_s + (wave * 16 + fr) * ld, w32, f32x4{0.f, 0.f, 0.f, 0.f});
@@ -325,42 +371,66 @@ __global__ __launch_bounds__(256) void k_latent_value(const LatStep a) {
   const LatRange rg = latent_range<T>(g, a.seq[b].pos);
   const int active = (rg.n + rg.per - 1) / rg.per, pw = l.rank + 2;
   const float* part = a.part + ((size_t)b * g.H + h) * LAT_SPLITS * pw;
-  float w[LAT_SPLITS], top = -INFINITY, den = 0.f;
+  int lpr = 1;  // lanes per weight row
+  while (lpr < 64 && lpr * 8 < l.rank) lpr <<= 1;
+  const int rows = 64 / lpr, sub = lane / lpr, k0 = lane % lpr * 8;
+  const unsigned short* wv = l.w_kv + (size_t)(g.H * l.dim + h * g.V) * l.ldl;
+  // a wave's LAT_VSLICE / 4 rows, `rows` at a time: their first octets are on their way while the splits are merged
+  constexpr int RW = LAT_VSLICE / 4;
+  i32x4 wf[RW];
+  const int kf = k0 < l.ldl ? k0 : 0;
+#pragma unroll
+  for (int j = 0; j < RW; j++) {
+    const int v = v0 + wave * RW + j * rows + sub;
+    if (j * rows < RW) wf[j] = *(const i32x4*)(wv + (size_t)(v < v1 ? v : v1 - 1) * l.ldl + kf);
+  }
+  float w[LAT_SPLITS], ds[LAT_SPLITS], top = -INFINITY, den = 0.f;
+#pragma unroll
+  for (int s = 0; s < LAT_SPLITS; s++) {  // (requests without branches; a split that is not there counts nothing)
+    const float* p = part + (size_t)s * pw + l.rank;
+    w[s] = p[0];
+    ds[s] = p[1];
+  }
 #pragma unroll
   for (int s = 0; s < LAT_SPLITS; s++) {
-    w[s] = s < active ? part[(size_t)s * pw + l.rank] : -INFINITY;
+    w[s] = s < active ? w[s] : -INFINITY;
     top = fmaxf(top, w[s]);
   }
 #pragma unroll
   for (int s = 0; s < LAT_SPLITS; s++) {
     w[s] = __expf(w[s] - top);
-    if (s < active) den = __builtin_fmaf(part[(size_t)s * pw + l.rank + 1], w[s], den);
+    den = __builtin_fmaf(s < active ? ds[s] : 0.f, w[s], den);
   }
-  for (int i = tid; i < l.rank; i += 256) {
-    float o = 0.f;
+  const float inv = 1.0f / den;
+  for (int i = tid; i < l.ldl; i += 256) {
+    float p[LAT_SPLITS], o = 0.f;
 #pragma unroll
-    for (int s = 0; s < LAT_SPLITS; s++)
-      if (s < active) o = __builtin_fmaf(part[(size_t)s * pw + i], w[s], o);
-    x[i] = o / den;
+    for (int s = 0; s < LAT_SPLITS; s++) p[s] = part[(size_t)s * pw + (i < l.rank ? i : 0)];
+#pragma unroll
+    for (int s = 0; s < LAT_SPLITS; s++) o = __builtin_fmaf(s < active ? p[s] : 0.f, w[s], o);
+    x[i] = i < l.rank ? o * inv : 0.f;
   }
-  int lpr = 1;  // lanes per weight row
-  while (lpr < 64 && lpr * 8 < l.rank) lpr <<= 1;
-  const int rows = 64 / lpr, sub = lane / lpr;
-  const unsigned short* wv = l.w_kv + (size_t)(g.H * l.dim + h * g.V) * l.ldl;
   __syncthreads();
-  for (int n = v0; n < v1; n += 4 * rows) {
-    const int v = n + wave * rows + sub;
-    float s = 0.f;
-    if (v < v1)
-      for (int k = lane % lpr * 8; k < l.rank; k += lpr * 8) {
-        float f[8], xv[8];
-        kv_load8(wv + (size_t)v * l.ldl + k, f);
-        read8(x + k, xv);
 #pragma unroll
-        for (int e = 0; e < 8; e++) s = __builtin_fmaf(f[e], xv[e], s);
+  for (int j = 0; j < RW; j++) {
+    if (j * rows >= RW) break;
+    const int v = v0 + wave * RW + j * rows + sub;
+    float s = 0.f;
+    for (int k = k0; k < l.ldl; k += lpr * 8) {  // (one round up to 512 latent columns; the padding is zero on both sides)
+      if (k != k0) wf[j] = *(const i32x4*)(wv + (size_t)(v < v1 ? v : v1 - 1) * l.ldl + k);
+      float xv[8];
+      read8(x + k, xv);
+#pragma unroll
+      for (int e = 0; e < 4; e++) {
+        s = __builtin_fmaf(__builtin_bit_cast(float, (unsigned)wf[j][e] << 16), xv[2 * e], s);
+        s = __builtin_fmaf(__builtin_bit_cast(float, (unsigned)wf[j][e] & 0xffff0000u), xv[2 * e + 1], s);
       }
-    for (int o = 1; o < lpr; o <<= 1) s += __shfl_xor(s, o, 64);
-    if (lane % lpr == 0 && v < v1) a.cat[(size_t)b * a.ldc + h * g.V + v] = s * g.out_scale;
+    }
+    if (lpr == 64)
+      s = wave_sum_f32(s);
+    else
+      for (int o = 1; o < lpr; o <<= 1) s += __shfl_xor(s, o, 64);
+    if (k0 == 0 && v < v1 && j * rows + sub < RW) a.cat[(size_t)b * a.ldc + h * g.V + v] = s * g.out_scale;
   }
 }
 
@@ -385,7 +455,7 @@ inline int launch_latent_attn(crabml_hip_device* dev, crabml_hip_device::ProfRec
 }
 template <typename T>
 inline void launch_latent_query(hipStream_t st, crabml_hip_device::ProfRec* rec, const LatStep& a) {
-  const size_t fl = (size_t)a.B * a.la.dim > (size_t)a.la.rot ? (size_t)a.B * a.la.dim : (size_t)a.la.rot;
+  const size_t fl = 16 * (align_up((size_t)a.la.dim, 32) + 4);  // (at least the 256 of a whole turn table)
   launch_k(st, rec, k_latent_query<T>, dim3(a.at.H * ((a.la.rank + LAT_SLICE - 1) / LAT_SLICE) + a.B), dim3(256), fl * sizeof(float), a);
 }
 template <typename T>
