@@ -157,8 +157,7 @@ __global__ __launch_bounds__(64 * WGM * WGN) void k_gemm_bf16(const GemmBf16 g, 
     // their way through LDS, so that a thread has sixteen requests out.
     constexpr int UNITS = HR * BN / 8 / NT, UG = 2;
     static_assert(UNITS % UG == 0, "units come in pairs");
-    typedef const float __attribute__((address_space(4))) constant;
-    constant *coef = (constant*)(size_t)g.sm.coef, *inw = (constant*)(size_t)g.sm.in;
+    const_f32 *coef = (const_f32*)(size_t)g.sm.coef, *inw = (const_f32*)(size_t)g.sm.in;
 #pragma unroll 1
     for (int h = 0; h < BM / HR; h++) {
 #pragma unroll
@@ -209,18 +208,17 @@ __global__ __launch_bounds__(64 * WGM * WGN) void k_gemm_bf16(const GemmBf16 g, 
               if (g.bias) y[k] += *(const f32x4*)(g.bias + col[u] + 4 * k);
             }
 #pragma unroll
-            for (int t = 0; t < 4; t++)
-              if (t < g.sm.n) {
-                constant* c = coef + t * HC_ROW;
+            for (int t = 0; t < 4; t++) {
+              const_f32* c = coef + t * HC_ROW;
 #pragma unroll
-                for (int k = 0; k < 2; k++) {
-                  f32x4 v = c[HC_MAX] * y[k];
+              for (int k = 0; k < 2; k++) {
+                f32x4 v = c[HC_MAX] * y[k];
 #pragma unroll
-                  for (int s = 0; s < 4; s++) v += c[s] * old[u][k][s];
-                  *(f32x4*)(xs[u] + t * g.sm.stride + 4 * k) = v;
-                  n[k] += inw[t] * v;
-                }
+                for (int s = 0; s < 4; s++) v += c[s] * old[u][k][s];
+                if (t < g.sm.n) *(f32x4*)(xs[u] + t * g.sm.stride + 4 * k) = v;
+                n[k] += inw[t] * v;
               }
+            }
             float v[8];
 #pragma unroll
             for (int k = 0; k < 2; k++) {
@@ -268,7 +266,10 @@ __global__ __launch_bounds__(64 * WGM * WGN) void k_gemm_bf16(const GemmBf16 g, 
           for (int k = 0; k < 8; k += 4) {
             f32x4 y = *(const f32x4*)(lc + r * LC + c + k) * f;
             if (g.bias) y += *(const f32x4*)(g.bias + col + k);
-            const f32x4 n = stream_mix(g.sm, g.x + (size_t)row * g.ldx + col + k, y), gain = *(const f32x4*)(g.gain_next + col + k);
+            f32x4 old[HC_MAX];
+            float* xs = g.x + (size_t)row * g.ldx + col + k;
+            stream_load(g.sm, xs, old);
+            const f32x4 n = stream_apply(g.sm, xs, old, y), gain = *(const f32x4*)(g.gain_next + col + k);
 #pragma unroll
             for (int e = 0; e < 4; e++) {
               sq = __builtin_fmaf(n[e], n[e], sq);

@@ -43,12 +43,14 @@ struct ActRanges {  // columns [end[i-1], end[i]) take activation kind[i]
 struct StreamMix {
   int n = 0;
   size_t stride = 0;            // floats between the streams
-  const float* coef = nullptr;  // [n][HC_ROW]: row t = mix[0 .. HC_MAX)[t] (zeros from n on), out[t]
-  const float* in = nullptr;    // [n]: of the sublayer that comes next
+  const float* coef = nullptr;  // [HC_MAX][HC_ROW]: row t = mix[0 .. HC_MAX)[t], out[t]; zeros from n on, both ways
+  const float* in = nullptr;    // [HC_MAX]: of the sublayer that comes next
 };
+// (constant address space: scalar loads, which no store can be taken to change)
+typedef const float __attribute__((address_space(4))) const_f32;
+// x: an element (or a vector of neighbours) of stream 0
 template <typename V>
-__device__ __forceinline__ V stream_mix(const StreamMix& m, float* x, V y) {  // x: this element (or vector of neighbours) of stream 0
-  V old[HC_MAX], u = V{};
+__device__ __forceinline__ void stream_load(const StreamMix& m, const float* x, V (&old)[HC_MAX]) {
   // (four at a time without a branch each -- past the last stream the first one again, with a zero coefficient)
 #pragma unroll
   for (int s = 0; s < 4; s++) old[s] = *(const V*)(x + (s < m.n ? s : 0) * m.stride);
@@ -58,12 +60,28 @@ __device__ __forceinline__ V stream_mix(const StreamMix& m, float* x, V y) {  //
 #pragma unroll
     for (int s = 4; s < HC_MAX; s++) old[s] = *(const V*)(x + (s < m.n ? s : 0) * m.stride);
   }
-  // (constant address space: scalar loads, which the stores below cannot be taken to change)
-  typedef const float __attribute__((address_space(4))) constant;
-  constant *coef = (constant*)(size_t)m.coef, *in = (constant*)(size_t)m.in;
+}
+template <typename V>
+__device__ __forceinline__ V stream_apply(const StreamMix& m, float* x, const V (&old)[HC_MAX], V y) {
+  const_f32 *coef = (const_f32*)(size_t)m.coef, *in = (const_f32*)(size_t)m.in;
+  V u = V{};
+  if (m.n <= 4) {  // (all coefficients in one go)
+    V v[4];
+#pragma unroll
+    for (int t = 0; t < 4; t++) {
+      v[t] = coef[t * HC_ROW + HC_MAX] * y;
+#pragma unroll
+      for (int s = 0; s < 4; s++) v[t] += coef[t * HC_ROW + s] * old[s];
+      u += in[t] * v[t];
+    }
+#pragma unroll
+    for (int t = 0; t < 4; t++)
+      if (t < m.n) *(V*)(x + t * m.stride) = v[t];
+    return u;
+  }
 #pragma unroll 1
   for (int t = 0; t < m.n; t++) {
-    constant* c = coef + t * HC_ROW;
+    const_f32* c = coef + t * HC_ROW;
     V v = c[HC_MAX] * y;
 #pragma unroll
     for (int s = 0; s < HC_MAX; s++) v += c[s] * old[s];
@@ -133,9 +151,7 @@ template <int OUT>
 __device__ __forceinline__ void gemv_out(const GemvBf16& a, int row, int b, float v) {
   float* o = a.out + (size_t)b * a.ldo + row;
   if constexpr (OUT == GEMV_OUT_STORE) *o = v;
-  if constexpr (OUT == GEMV_OUT_ACT || OUT == GEMV_OUT_STREAMS) v += a.bias ? a.bias[row] : 0.f;
-  if constexpr (OUT == GEMV_OUT_ACT) *o = act_ranges(v, row, a.act);
-  if constexpr (OUT == GEMV_OUT_STREAMS) a.u[(size_t)b * a.ldo + row] = stream_mix(a.sm, o, v);
+  if constexpr (OUT == GEMV_OUT_ACT) *o = act_ranges(a.bias ? v + a.bias[row] : v, row, a.act);
   if constexpr (OUT == GEMV_OUT_RESIDUAL) {
     float s = *o + v;
     if (a.add_rows) s += a.add_rows[(size_t)b * a.ld_add + row];
@@ -144,6 +160,18 @@ __device__ __forceinline__ void gemv_out(const GemvBf16& a, int row, int b, floa
   }
   if constexpr (OUT == GEMV_OUT_XIELU) *o = xielu_apply(v, a.xielu[0], a.xielu[1]);
   if constexpr (OUT == GEMV_OUT_SOFTCAP) *o = soft_cap(v, a.cap);
+}
+
+// GEMV_OUT_STREAMS: what the thread that will have (row, b) needs, requested ahead of the products
+struct StreamElem {
+  float old[HC_MAX], bias = 0.f;
+};
+__device__ __forceinline__ void stream_elem_load(const GemvBf16& a, int row, int b, StreamElem& e) {
+  stream_load(a.sm, a.out + (size_t)b * a.ldo + row, e.old);
+  if (a.bias) e.bias = a.bias[row];
+}
+__device__ __forceinline__ void stream_elem_out(const GemvBf16& a, int row, int b, const StreamElem& e, float v) {
+  a.u[(size_t)b * a.ldo + row] = stream_apply(a.sm, a.out + (size_t)b * a.ldo + row, e.old, v + e.bias);
 }
 
 #define GEMV_BF16_LDS_FLOATS 8192  // rhs elements staged at a time, all rows together: a cut segment is a multiple of the steps in flight
@@ -174,6 +202,13 @@ __global__ __launch_bounds__(256) void k_gemv_bf16(const GemvBf16 a) {
     }
   };
   request(0);
+  StreamElem elem;  // of lane r NB + b
+  const int my_row = row0 + lane / NB, my_b = b0 + lane % NB;
+  const bool mine = OUT == GEMV_OUT_STREAMS && lane < R * NB && my_row < a.N && my_b < a.nb;
+  if constexpr (OUT == GEMV_OUT_STREAMS) {
+    static_assert(R * NB <= 64, "a lane per result");
+    if (mine) stream_elem_load(a, my_row, my_b, elem);
+  }
   float acc[R][NB];
 #pragma unroll
   for (int r = 0; r < R; r++)
@@ -287,6 +322,18 @@ __global__ __launch_bounds__(256) void k_gemv_bf16(const GemvBf16 a) {
       }
     return;
   }
+  if constexpr (OUT == GEMV_OUT_STREAMS) {
+    float y = 0.f;
+#pragma unroll
+    for (int r = 0; r < R; r++)
+#pragma unroll
+      for (int b = 0; b < NB; b++) {
+        const float v = wave_sum_f32(acc[r][b]) * scale[b];
+        y = lane == r * NB + b ? v : y;
+      }
+    if (mine) stream_elem_out(a, my_row, my_b, elem, y);
+    return;
+  }
 #pragma unroll
   for (int r = 0; r < R; r++)
 #pragma unroll
@@ -353,6 +400,14 @@ __global__ __launch_bounds__(512) void k_gemv16_bf16(const GemvBf16 a) {
   };
   const int n = a.K / 64;
   if (wave < n) request(wave * 64);
+  StreamElem elem[(RT + 1) / 2];  // of this thread's results: element tid + 512 i of the tile
+  if constexpr (OUT == GEMV_OUT_STREAMS) {
+#pragma unroll
+    for (int i = 0; i < (RT + 1) / 2; i++) {
+      const int j = tid + i * 512, b = (j >> 4) & 15, row = row0 + (j >> 8) * 16 + (j & 15);
+      if (j < RT * 256 && b < a.nb && row < a.N) stream_elem_load(a, row, b, elem[i]);
+    }
+  }
   float tail = 1.f, sq = 0.f;
   if constexpr (IN == GEMV_IN_SPLIT) {
     float s = 0.f;
@@ -441,6 +496,19 @@ __global__ __launch_bounds__(512) void k_gemv16_bf16(const GemvBf16 a) {
         up *= scale[b];
       }
       if (b < a.nb && row < a.N) a.out[(size_t)b * a.ldo + row / 2] = gelu_tanh(gate) * up;
+    }
+    return;
+  }
+  if constexpr (OUT == GEMV_OUT_STREAMS) {
+#pragma unroll
+    for (int i = 0; i < (RT + 1) / 2; i++) {
+      const int j = tid + i * 512, t = j >> 8, b = (j >> 4) & 15, r = j & 15, row = row0 + t * 16 + r;
+      if (j < RT * 256 && b < a.nb && row < a.N) {
+        float v = 0.f;
+#pragma unroll
+        for (int w = 0; w < W; w++) v += tile[w][t][b * LD + r];
+        stream_elem_out(a, row, b, elem[i], v);
+      }
     }
     return;
   }

@@ -188,11 +188,12 @@ int pack_connection(Ctx* c, const crabml_hip_buf* in, const crabml_hip_buf* out,
   if (!c->cfg.streams) {  // a plain residual: one stream that keeps itself
     h.in = o = m = c->ones;
   } else {
-    CH_TRY(pack_vector(c, in, "a connection's input weights", n, &h.in));
+    CH_TRY(dalloc_n(c, HC_MAX, &h.in));
+    CH_TRY(pack_into(c, in, "a connection's input weights", n, h.in));
     CH_TRY(pack_vector(c, out, "a connection's output weights", n, &o));
     CH_TRY(pack_vector(c, mix, "a connection's mixing matrix", n * n, &m));
   }
-  CH_TRY(dalloc_n(c, n * HC_ROW, &h.coef));
+  CH_TRY(dalloc_n(c, HC_MAX * HC_ROW, &h.coef));
   k_pack_connection<<<1, 1, 0, c->dev->stream>>>(m, o, (int)n, h.coef);
   CH_HIP(c->dev, hipGetLastError());
   return 0;
