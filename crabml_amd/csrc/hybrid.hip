@@ -531,6 +531,7 @@ int latent_step(Ctx* c, const Run& run, int B, bool prof) {
   m.B = B;
   m.ldp = L.n_in;
   m.ldc = L.ldc;
+  m.splits = latent_splits(B, L.at.H);
   hipStream_t st = c->dev->stream;
   {
     Prof p(c->dev, prof, ST_STEP + ST_LAT, (double)L.at.H * L.la.rank * L.la.dim * 2);

@@ -89,9 +89,8 @@ __global__ __launch_bounds__(256) void k_latent_append(const MixRows<T> a) {
 
 // ---- decode step ---------------------------------------------------------------------------------------------------------------------
 #define LAT_HEADS 16       // query heads per workgroup: the rows of a matrix instruction
-#define LAT_SPLITS 16      // workgroups that share a sequence's cached rows
+#define LAT_SPLITS 16      // most workgroups that share a sequence's cached rows
 #define LAT_SLICE 64       // latent columns per workgroup of k_latent_query
-#define LAT_VSLICE 32      // value columns per workgroup of k_latent_value
 #define LAT_MAX_ROW 768    // rank + rot
 template <typename T>
 struct LatTile {
@@ -107,18 +106,19 @@ struct LatStep {
   float* part = nullptr;        // [B][H][LAT_SPLITS][rank + 2]: unnormalized sums, maximum, denominator
   float* cat = nullptr;         // [B][ldc]
   int B = 0, ldp = 0, ldc = 0;
+  int splits = LAT_SPLITS;
 };
 // rows that are there, rows per split
 struct LatRange {
   int n, per;
 };
 template <typename T>
-__device__ __forceinline__ LatRange latent_range(const AttnGeom& g, int pos) {
+__device__ __forceinline__ LatRange latent_range(const AttnGeom& g, int splits, int pos) {
   constexpr int KT = LatTile<T>::KT;
   LatRange r;
   r.n = g.window && pos >= g.span ? g.span : pos % g.span + 1;
   const int tiles = (r.n + KT - 1) / KT;
-  r.per = (tiles + LAT_SPLITS - 1) / LAT_SPLITS * KT;
+  r.per = (tiles + splits - 1) / splits * KT;
   return r;
 }
 
@@ -244,7 +244,7 @@ __global__ __launch_bounds__(256) void k_latent_attn(const LatStep a) {
   const int nh = g.H - h0 < LAT_HEADS ? g.H - h0 : LAT_HEADS;
   const float* q = a.q + ((size_t)b * g.H + h0) * row_w;
   const StepSeq sq = a.seq[b];
-  const LatRange rg = latent_range<T>(g, sq.pos);
+  const LatRange rg = latent_range<T>(g, a.splits, sq.pos);
   const int lo = split * rg.per, hi = lo + rg.per < rg.n ? lo + rg.per : rg.n;
   if (lo >= hi) return;  // (whole workgroup)
   const T* cache = (const T*)(sq.slab + a.rs.k);
@@ -359,24 +359,24 @@ __global__ __launch_bounds__(256) void k_latent_attn(const LatStep a) {
   }
 }
 
-// grid: (H * slices of the value columns, B)
-template <typename T>
+// grid: (H * slices of VS value columns, B); SP: splits
+template <typename T, int SP, int VS>
 __global__ __launch_bounds__(256) void k_latent_value(const LatStep a) {
   __shared__ __attribute__((aligned(16))) float x[LAT_MAX_ROW];
   const AttnGeom& g = a.at;
   const LatGeom& l = a.la;
   const int tid = threadIdx.x, lane = tid & 63, wave = wave_in_wg(), b = blockIdx.y;
-  const int slices = (g.V + LAT_VSLICE - 1) / LAT_VSLICE, h = blockIdx.x / slices, v0 = blockIdx.x % slices * LAT_VSLICE;
-  const int v1 = v0 + LAT_VSLICE < g.V ? v0 + LAT_VSLICE : g.V;
-  const LatRange rg = latent_range<T>(g, a.seq[b].pos);
+  const int slices = (g.V + VS - 1) / VS, h = blockIdx.x / slices, v0 = blockIdx.x % slices * VS;
+  const int v1 = v0 + VS < g.V ? v0 + VS : g.V;
+  const LatRange rg = latent_range<T>(g, SP, a.seq[b].pos);
   const int active = (rg.n + rg.per - 1) / rg.per, pw = l.rank + 2;
   const float* part = a.part + ((size_t)b * g.H + h) * LAT_SPLITS * pw;
   int lpr = 1;  // lanes per weight row
   while (lpr < 64 && lpr * 8 < l.rank) lpr <<= 1;
   const int rows = 64 / lpr, sub = lane / lpr, k0 = lane % lpr * 8;
   const unsigned short* wv = l.w_kv + (size_t)(g.H * l.dim + h * g.V) * l.ldl;
-  // a wave's LAT_VSLICE / 4 rows, `rows` at a time: their first octets are on their way while the splits are merged
-  constexpr int RW = LAT_VSLICE / 4;
+  // a wave's VS / 4 rows, `rows` at a time: their first octets are on their way while the splits are merged
+  constexpr int RW = VS / 4;
   i32x4 wf[RW];
   const int kf = k0 < l.ldl ? k0 : 0;
 #pragma unroll
@@ -384,30 +384,30 @@ __global__ __launch_bounds__(256) void k_latent_value(const LatStep a) {
     const int v = v0 + wave * RW + j * rows + sub;
     if (j * rows < RW) wf[j] = *(const i32x4*)(wv + (size_t)(v < v1 ? v : v1 - 1) * l.ldl + kf);
   }
-  float w[LAT_SPLITS], ds[LAT_SPLITS], top = -INFINITY, den = 0.f;
+  float w[SP], ds[SP], top = -INFINITY, den = 0.f;
 #pragma unroll
-  for (int s = 0; s < LAT_SPLITS; s++) {  // (requests without branches; a split that is not there counts nothing)
+  for (int s = 0; s < SP; s++) {  // (requests without branches; a split that is not there counts nothing)
     const float* p = part + (size_t)s * pw + l.rank;
     w[s] = p[0];
     ds[s] = p[1];
   }
 #pragma unroll
-  for (int s = 0; s < LAT_SPLITS; s++) {
+  for (int s = 0; s < SP; s++) {
     w[s] = s < active ? w[s] : -INFINITY;
     top = fmaxf(top, w[s]);
   }
 #pragma unroll
-  for (int s = 0; s < LAT_SPLITS; s++) {
+  for (int s = 0; s < SP; s++) {
     w[s] = __expf(w[s] - top);
     den = __builtin_fmaf(s < active ? ds[s] : 0.f, w[s], den);
   }
   const float inv = 1.0f / den;
   for (int i = tid; i < l.ldl; i += 256) {
-    float p[LAT_SPLITS], o = 0.f;
+    float p[SP], o = 0.f;
 #pragma unroll
-    for (int s = 0; s < LAT_SPLITS; s++) p[s] = part[(size_t)s * pw + (i < l.rank ? i : 0)];
+    for (int s = 0; s < SP; s++) p[s] = part[(size_t)s * pw + (i < l.rank ? i : 0)];
 #pragma unroll
-    for (int s = 0; s < LAT_SPLITS; s++) o = __builtin_fmaf(s < active ? p[s] : 0.f, w[s], o);
+    for (int s = 0; s < SP; s++) o = __builtin_fmaf(s < active ? p[s] : 0.f, w[s], o);
     x[i] = i < l.rank ? o * inv : 0.f;
   }
   __syncthreads();
@@ -434,6 +434,8 @@ __global__ __launch_bounds__(256) void k_latent_value(const LatStep a) {
   }
 }
 
+// half as many splits once the chip is full: every split's sums pass through memory
+inline int latent_splits(int B, int H) { return B * H >= 512 ? LAT_SPLITS / 2 : LAT_SPLITS; }
 template <typename T>
 inline size_t latent_attn_lds(const LatGeom& l) {
   const size_t ld = align_up((size_t)(l.rank + l.rot), 32) + LatTile<T>::PAD;
@@ -443,7 +445,7 @@ template <typename T, int NT>
 inline int launch_latent_attn_t(crabml_hip_device* dev, crabml_hip_device::ProfRec* rec, const LatStep& a) {
   const size_t lds = latent_attn_lds<T>(a.la);
   CH_HIP(dev, raise_dyn_lds(dev, (const void*)k_latent_attn<T, NT>, (int)lds));
-  launch_k(dev->stream, rec, k_latent_attn<T, NT>, dim3(LAT_SPLITS, (a.at.H + LAT_HEADS - 1) / LAT_HEADS, a.B), dim3(256), lds, a);
+  launch_k(dev->stream, rec, k_latent_attn<T, NT>, dim3(a.splits, (a.at.H + LAT_HEADS - 1) / LAT_HEADS, a.B), dim3(256), lds, a);
   return 0;
 }
 template <typename T>
@@ -460,7 +462,10 @@ inline void launch_latent_query(hipStream_t st, crabml_hip_device::ProfRec* rec,
 }
 template <typename T>
 inline void launch_latent_value(hipStream_t st, crabml_hip_device::ProfRec* rec, const LatStep& a) {
-  launch_k(st, rec, k_latent_value<T>, dim3(a.at.H * ((a.at.V + LAT_VSLICE - 1) / LAT_VSLICE), a.B), dim3(256), 0, a);
+  if (a.splits == LAT_SPLITS)
+    launch_k(st, rec, k_latent_value<T, LAT_SPLITS, 32>, dim3(a.at.H * ((a.at.V + 31) / 32), a.B), dim3(256), 0, a);
+  else
+    launch_k(st, rec, k_latent_value<T, LAT_SPLITS / 2, 64>, dim3(a.at.H * ((a.at.V + 63) / 64), a.B), dim3(256), 0, a);
 }
 
 }  // namespace crabml_hip

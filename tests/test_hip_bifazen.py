@@ -191,6 +191,20 @@ def test_unequal_batch_against_each_alone(ca, hdev, models, name, f32):
     close(got, [w[-2] for w in want], f32)
 
 
+@pytest.mark.parametrize("f32", [True, False])
+def test_many_heads_times_many_sequences(ca, hdev, tmp_path, f32):
+    """enough (head, sequence) pairs to fill the chip: the decode attention of latents then runs in fewer, longer pieces"""
+    c = sb.config(48, 60, [sb.latent(36, 16, 8, 24, 72, 400, 32)], streams=2)
+    m = Model(c, tmp_path / "m", seed=2)
+    r = m.runner(ca, hdev, f32)
+    toks = [m.tokens(20 + 41 * i, seed=300 + i) for i in range(15)]
+    want = [m.oracle(t) for t in toks]
+    seqs = [r.open() for _ in toks]
+    r.step([(s, t[:-3], []) for s, t in zip(seqs, toks)])
+    for k in (3, 2, 1):
+        close(r.step([(s, [t[-k]], [0]) for s, t in zip(seqs, toks)]), [w[-k] for w in want], f32)
+
+
 def test_rows_of_a_batch_do_not_change_each_other(ca, hdev, models):
     m = models("plain")
     r = m.runner(ca, hdev, True)
