@@ -300,7 +300,6 @@ int build_layer(Ctx* c, const crabml_hip_hybrid_layer_t& s, Layer& L) {
     la.dim = (int)dimp;
     la.rot = (int)rotp;
     la.rank_true = (int)rank;
-    la.rot_true = (int)rot;
     la.ldl = up(rank, 64);
     CH_TRY(pack_matrix(c, s.attn_q, "attn_q", H * s.attn_dim, W, L.w_in, ldw, a.cq, s.attn_dim, D, 0, 0, 0, s.attn_dim + rot, 0));
     if (rot) CH_TRY(pack_matrix(c, s.attn_q, "attn_q", H * rot, W, L.w_in, ldw, a.cq + dimp, rot, D, 0, 0, 0, s.attn_dim + rot, s.attn_dim));

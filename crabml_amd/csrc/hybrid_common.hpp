@@ -103,7 +103,7 @@ __host__ __device__ inline int attn_first(const AttnGeom& g, int pos) {
 // products of the latent, its second part is shared.  A cache row is [rank, rot].
 struct LatGeom {
   int rank = 0, dim = 0, rot = 0;  // padded to 8
-  int rank_true = 0, rot_true = 0;
+  int rank_true = 0;               // what the latent's norm averages over
   int ldl = 0;                     // rank padded to 64: the latent as a row operand
   int cc = 0, cr = 0;              // columns of the projected row: latent, shared key part
   const float* norm = nullptr;     // [rank]

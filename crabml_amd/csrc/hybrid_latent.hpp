@@ -314,7 +314,8 @@ __global__ __launch_bounds__(256) void k_latent_attn(const LatStep a) {
     stage(t0, hi - t0, KT, cache, k_s);
     __syncthreads();
     if (wave < KT / 16) {
-      const f32x4 s = mma_rows(q_s + fr * ld, k_s + (wave * 16 + fr) * ld, w32, f32x4{0.f, 0.f, 0.f, 0.f});
+      f32x4 s = {0.f, 0.f, 0.f, 0.f};
+      for (int k = 0; k < w32; k += 32) s = mma_rows(q_s + fr * ld + k, k_s + (wave * 16 + fr) * ld + k, 32, s);
 #pragma unroll
       for (int e = 0; e < 4; e++) p_s[(fk * 4 + e) * LP + wave * 16 + fr] = t0 + wave * 16 + fr < hi ? s[e] * g.scale : -INFINITY;
     }
